@@ -251,6 +251,8 @@ class PlainOps:
         g, u = gate_up[:, :inner].to(self.work), gate_up[:, inner:].to(self.work)
         if act is None:
             out.copy_((g * torch.sigmoid(g) * u).to(out.dtype))
+        elif act == "relu":
+            out.copy_((torch.clamp(g, min=0.0) * u).to(out.dtype))
         elif act == "gelu_tanh":
             out.copy_((0.5 * g * (1.0 + torch.tanh(0.7978845608028654 * (g + 0.044715 * g * g * g))) * u).to(out.dtype))
         else:
@@ -444,20 +446,107 @@ class PlainOps:
     def _unit(self, x, eps):
         return x / torch.sqrt((x * x).mean(dim=-1, keepdim=True) + eps)
 
-    def norm_add_rmsnorm(self, residual, delta, post_weight, post_eps, weight, eps, out, rows=None, store_residual=True):
+    def _unit_groups(self, x, eps, groups):
+        return self._unit(x.reshape(x.shape[0], groups, -1), eps).reshape(x.shape)
+
+    def norm_add_rmsnorm(self, residual, delta, post_weight, post_eps, weight, eps, out, rows=None, store_residual=True,
+                         post_groups=1, groups=1):
         x = (residual if rows is None else residual[rows.long()]).to(self.work)
         if delta is not None:
             d = (delta if rows is None else delta[rows.long()]).to(self.work)
             if post_weight is not None:
-                d = self._unit(d, post_eps) * post_weight.to(self.work)
+                d = self._unit_groups(d, post_eps, post_groups) * post_weight.to(self.work)
             x = x + d
         if store_residual and delta is not None:
             assert rows is None
             residual.copy_(x.to(torch.float32))
             x = residual.to(self.work)
         if weight is not None:
-            x = self._unit(x, eps) * weight.to(self.work)
+            x = self._unit_groups(x, eps, groups) * weight.to(self.work)
         out.copy_(x.to(out.dtype))
+        return out
+
+    def rotation_table(self, positions, rates, magnitude, out):
+        angles = positions.to(torch.float32)[:, None] * rates.to(torch.float32)[None, :]      # float32 angles
+        out.copy_(magnitude * torch.cat([angles.cos(), angles.sin()], dim=1))
+        return out
+
+    def _turn_heads(self, x, table, dims):
+        """x [T, heads, d]: the first `dims` coordinates turn by the rows of `table` ([cosines | sines])."""
+        half = dims // 2
+        if not half:
+            return x
+        cos, sin = table[:, None, :half].to(self.work), table[:, None, half:].to(self.work)
+        a, b = x[..., :half], x[..., half:dims]
+        return torch.cat([a * cos - b * sin, b * cos + a * sin, x[..., dims:]], dim=-1)
+
+    def head_norm_rotate_store(self, qkv, table, dims, slots, k_pages, v_pages, n_q, n_k, n_v, d, dv, q_norm, k_norm,
+                               norm_values, first, share, eps):
+        n_tokens = qkv.shape[0]
+        x = qkv.to(self.work)
+        q = x[:, :n_q * d].reshape(n_tokens, n_q, d)
+        k = x[:, n_q * d:(n_q + n_k) * d].reshape(n_tokens, n_k, d)
+        v = x[:, (n_q + n_k) * d:(n_q + n_k) * d + n_v * dv].reshape(n_tokens, n_v, dv)
+        if q_norm is not None:
+            q = self._unit(q, eps) * q_norm.to(self.work)
+        if k_norm is not None:
+            k = self._unit(k, eps) * k_norm.to(self.work)
+        q, k = self._turn_heads(q, table, dims), self._turn_heads(k, table, dims)
+        if norm_values:
+            v = self._unit(v, eps)
+        if share is not None:
+            s = share.to(self.work).reshape(())
+            v = (1.0 - s) * v + s * first.to(self.work).reshape(v.shape)
+        k, v = k.to(qkv.dtype), v.to(qkv.dtype)
+        qkv[:, :n_q * d] = q.reshape(n_tokens, -1).to(qkv.dtype)
+        qkv[:, n_q * d:(n_q + n_k) * d] = k.reshape(n_tokens, -1)
+        qkv[:, (n_q + n_k) * d:(n_q + n_k) * d + n_v * dv] = v.reshape(n_tokens, -1)
+        if slots is not None:
+            page_size = k_pages.shape[2]
+            for t in range(n_tokens):
+                slot = int(slots[t])
+                if slot >= 0:
+                    page, off = divmod(slot, page_size)
+                    k_pages[page, :, off, :] = k[t]
+                    v_pages[page, :, :, off] = v[t]
+
+    def talking_attention(self, qkv, out, k_pages, v_pages, positions, entry_of_token, block_table, n_q, n_kv, head_dim,
+                          value_dim, scale, talk, max_position=None, batch=None):
+        page_size, group = k_pages.shape[2], n_q // n_kv
+        for t in range(qkv.shape[0]):
+            if int(entry_of_token[t]) < 0:
+                continue
+            table = block_table[int(entry_of_token[t])]
+            keys = range(int(positions[t]) + 1)
+            pages, offs = [int(table[j // page_size]) for j in keys], [j % page_size for j in keys]
+            k = k_pages[pages, :, offs, :].to(self.work).repeat_interleave(group, dim=1)
+            v = v_pages[pages, :, :, offs].to(self.work).repeat_interleave(group, dim=1)
+            q = qkv[t, :n_q * head_dim].reshape(n_q, head_dim).to(self.work)
+            weights = talk.to(self.work) @ torch.softmax(torch.einsum("hd,khd->hk", q, k) * scale, dim=-1)
+            out[t] = torch.einsum("hk,khd->hd", weights, v).reshape(-1).to(out.dtype)
+        return out
+
+    def retention(self, qkvg, table, dims, decays, state, cu_q, first_position, state_slots, out, heads, d, dv, eps):
+        w = self.work
+        n_tokens = qkvg.shape[0]
+        x = qkvg.to(w)
+        q = self._turn_heads(x[:, :heads * d].reshape(n_tokens, heads, d), table, dims)
+        k = self._turn_heads(x[:, heads * d:2 * heads * d].reshape(n_tokens, heads, d), table, dims) * d ** -0.5
+        v = x[:, 2 * heads * d:2 * heads * d + heads * dv].reshape(n_tokens, heads, dv)
+        g = x[:, 2 * heads * d + heads * dv:2 * heads * (d + dv)]
+        for e in range(cu_q.numel() - 1):
+            lo, hi = int(cu_q[e]), int(cu_q[e + 1])
+            if hi <= lo:
+                continue
+            slot = int(state_slots[e])
+            S = state[slot, :heads * dv * d].to(w).reshape(heads, dv, d)
+            if int(first_position[e]) == 0:
+                S = torch.zeros_like(S)
+            for t in range(lo, hi):
+                S = decays.to(w)[:, None, None] * S + v[t][:, :, None] * k[t][:, None, :]
+                o = self._unit(torch.einsum("hvd,hd->hv", S, q[t]), eps).reshape(-1)
+                out[t] = (o * (g[t] * torch.sigmoid(g[t]))).to(out.dtype)
+            state[slot, :heads * dv * d] = S.reshape(-1).to(state.dtype)
         return out
 
     def norm_rotate_store(self, qkv, bias, positions, rates, dims, slots, k_pages, v_pages, n_q, n_k, n_v, d, dv,

@@ -6,7 +6,9 @@ from .napadra import NapadraConfig
 from .dolidra import DolidraConfig
 from .bokulorn import BokulornConfig
 from .zomavik import ZomavikConfig
+from .gafonex import GafonexConfig
 
 __all__ = ["ConfigError", "ModelConfig", "read_config_json", "Architecture", "architecture_name",
            "get_architecture", "load_config", "register_architecture", "registered_architectures",
-           "Qwen2Config", "NapadraConfig", "DolidraConfig", "BokulornConfig", "ZomavikConfig"]
+           "Qwen2Config", "NapadraConfig", "DolidraConfig", "BokulornConfig", "ZomavikConfig",
+           "GafonexConfig"]

@@ -227,8 +227,9 @@ skinny_gemm_kernel(const bf16_t* __restrict__ A, int lda, int k_chunk, const bf1
         continue;
       }
       if (bias && !partial && n + r < n_out) sum0 += bias[n + r];
-      // gate_act 1: the tanh form of GELU in place of silu.
+      // gate_act 1: the tanh form of GELU in place of silu; 2: max(z, 0).
       v[r] = !GATED ? sum0
+             : gate_act == 2 ? fmaxf(sum0, 0.f) * sum1
              : gate_act == 1 ? 0.5f * sum0 * (1.0f + tanhf(0.7978845608028654f * (sum0 + 0.044715f * sum0 * sum0 * sum0))) * sum1
                              : sum0 / (1.0f + __expf(-sum0)) * sum1;
     }
@@ -339,14 +340,14 @@ static int pick_waves(const void* A, int lda, const void* W, const void* bias, v
 }
 
 // M <= 64; K, lda multiples of 8; pointers 16-byte aligned; with `gated` N is even and C is [M, N/2]
-// (gated 1: silu(gate) * up; 2: the tanh form of GELU in place of silu).
+// (gated 1: silu(gate) * up; 2: the tanh form of GELU in place of silu; 3: max(gate, 0)).
 // col_blocks: blocks of sixteen output columns per workgroup, 0 = the launcher's choice (see column_blocks).
 extern "C" int ta_gemm_skinny_bf16(const void* A, int lda, const void* W, const void* bias, void* C, int ldc,
                                    int M, int N, int K, int out_dtype, int gated, int col_blocks, hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;
   if (M > 64 || (K & 7) || (lda & 7) || (gated && (N & 1))) return -1;
   const int mb = (M + 15) / 16;
-#define GO(MBV) (gated ? pick_waves<MBV, true>(A, lda, W, bias, C, ldc, M, N, K, out_dtype, stream, col_blocks, gated == 2) \
+#define GO(MBV) (gated ? pick_waves<MBV, true>(A, lda, W, bias, C, ldc, M, N, K, out_dtype, stream, col_blocks, gated - 1) \
                        : pick_waves<MBV, false>(A, lda, W, bias, C, ldc, M, N, K, out_dtype, stream, col_blocks))
   switch (mb) {
     case 1: return GO(1);

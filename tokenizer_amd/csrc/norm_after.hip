@@ -526,3 +526,161 @@ extern "C" int ta_norm_add_rmsnorm(void* residual, const void* delta, const void
 #undef GO
   return LAUNCH_STATUS();
 }
+
+// ---------------------------------------------------------------------------------------------------------------
+// The norm behind a sub-layer, the add and the next norm as above, with both norms over groups: the row falls into
+// `post_groups` (`groups`) equal runs of neighbours, each divided by its own root mean square.
+
+// 1 / rms of every group from the squares that `part` holds (entry i: the sum over `unit` neighbours): wave w adds up
+// groups w, w + 4, ...; everybody meets before and behind.
+__device__ __forceinline__ void na_group_rms(const float* part, float* inv, int hidden, int unit, int groups, float eps) {
+  const int lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE;
+  const int size = hidden / groups, entries = size / unit;
+  __syncthreads();
+  for (int g = wave; g < groups; g += NA_THREADS / WAVE) {
+    float sq = 0.f;
+    for (int i = lane; i < entries; i += WAVE) sq += part[(size_t)g * entries + i];
+    sq = wave_sum(sq);
+    if (lane == 0) inv[g] = 1.0f / sqrtf(sq / (float)size + eps);
+  }
+  __syncthreads();
+}
+
+// Rows and groups that are multiples of 4, rows of up to CHUNKS * 1,024 elements.  Dynamic LDS: hidden / 4 floats and
+// room for the larger number of groups.
+template <typename TD, typename TO, int CHUNKS>
+__global__ void __launch_bounds__(NA_THREADS)
+group_norm_add_vec_kernel(float* __restrict__ residual, const TD* __restrict__ delta, const float* __restrict__ post_weight,
+                          float post_eps, int post_groups, const float* __restrict__ weight, float eps, int groups,
+                          TO* __restrict__ out, const int* __restrict__ rows, int hidden, int store_residual) {
+  extern __shared__ float na_part[];
+  float* inv = na_part + hidden / 4;
+  const int i = blockIdx.x;
+  const int r = rows ? rows[i] : i;
+  float* res = residual + (size_t)r * hidden;
+  float4 x[CHUNKS], d[CHUNKS], behind_w[CHUNKS], next_w[CHUNKS];
+#pragma unroll
+  for (int c = 0; c < CHUNKS; ++c) {
+    const int h = min((c * NA_THREADS + (int)threadIdx.x) * 4, hidden - 4);
+    x[c] = na_ld4(res + h);
+    d[c] = delta ? na_ld4(delta + (size_t)r * hidden + h) : make_float4(0.f, 0.f, 0.f, 0.f);
+    behind_w[c] = post_weight ? na_ld4(post_weight + h) : make_float4(1.f, 1.f, 1.f, 1.f);
+    next_w[c] = weight ? na_ld4(weight + h) : make_float4(1.f, 1.f, 1.f, 1.f);
+  }
+  if (post_weight) {
+#pragma unroll
+    for (int c = 0; c < CHUNKS; ++c) {
+      const int e = c * NA_THREADS + threadIdx.x;
+      if (e * 4 < hidden) na_part[e] = na_sq4(d[c]);
+    }
+    na_group_rms(na_part, inv, hidden, 4, post_groups, post_eps);
+  }
+#pragma unroll
+  for (int c = 0; c < CHUNKS; ++c) {
+    const int h = (c * NA_THREADS + (int)threadIdx.x) * 4;
+    if (h >= hidden) continue;
+    const float f = post_weight ? inv[h / (hidden / post_groups)] : 1.f;
+    x[c].x += d[c].x * f * behind_w[c].x; x[c].y += d[c].y * f * behind_w[c].y;
+    x[c].z += d[c].z * f * behind_w[c].z; x[c].w += d[c].w * f * behind_w[c].w;
+    if (store_residual) na_st4(res + h, x[c]);
+  }
+  if (weight) {
+    __syncthreads();                                         // the first norm's factors have been read
+#pragma unroll
+    for (int c = 0; c < CHUNKS; ++c) {
+      const int e = c * NA_THREADS + threadIdx.x;
+      if (e * 4 < hidden) na_part[e] = na_sq4(x[c]);
+    }
+    na_group_rms(na_part, inv, hidden, 4, groups, eps);
+  }
+  TO* dst = out + (size_t)i * hidden;
+#pragma unroll
+  for (int c = 0; c < CHUNKS; ++c) {
+    const int h = (c * NA_THREADS + (int)threadIdx.x) * 4;
+    if (h >= hidden) continue;
+    const float f = weight ? inv[h / (hidden / groups)] : 1.f;
+    na_st4(dst + h, make_float4(x[c].x * f * next_w[c].x, x[c].y * f * next_w[c].y, x[c].z * f * next_w[c].z,
+                                x[c].w * f * next_w[c].w));
+  }
+}
+
+// Any other row: an element a step, read again for every pass; a group's squares are added up by one wave.  Dynamic
+// LDS: room for both norms' factors.
+template <typename TD, typename TO>
+__global__ void __launch_bounds__(NA_THREADS)
+group_norm_add_kernel(float* __restrict__ residual, const TD* __restrict__ delta, const float* __restrict__ post_weight,
+                      float post_eps, int post_groups, const float* __restrict__ weight, float eps, int groups,
+                      TO* __restrict__ out, const int* __restrict__ rows, int hidden, int store_residual) {
+  extern __shared__ float na_part[];
+  float* inv_d = na_part;
+  float* inv_x = na_part + post_groups;
+  const int i = blockIdx.x, lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE;
+  const int r = rows ? rows[i] : i;
+  float* res = residual + (size_t)r * hidden;
+  const TD* del = delta ? delta + (size_t)r * hidden : nullptr;
+  const int size_d = hidden / post_groups, size_x = hidden / groups;
+  if (post_weight) {
+    for (int g = wave; g < post_groups; g += NA_THREADS / WAVE) {
+      float sq = 0.f;
+      for (int h = lane; h < size_d; h += WAVE) { const float v = ld(del + g * size_d + h); sq += v * v; }
+      sq = wave_sum(sq);
+      if (lane == 0) inv_d[g] = 1.0f / sqrtf(sq / (float)size_d + post_eps);
+    }
+  }
+  __syncthreads();
+  auto at = [&](int h) {
+    float v = res[h];
+    if (del) v += post_weight ? ld(del + h) * inv_d[h / size_d] * post_weight[h] : ld(del + h);
+    return v;
+  };
+  if (weight) {
+    for (int g = wave; g < groups; g += NA_THREADS / WAVE) {
+      float sq = 0.f;
+      for (int h = lane; h < size_x; h += WAVE) { const float v = at(g * size_x + h); sq += v * v; }
+      sq = wave_sum(sq);
+      if (lane == 0) inv_x[g] = 1.0f / sqrtf(sq / (float)size_x + eps);
+    }
+  }
+  __syncthreads();
+  TO* dst = out + (size_t)i * hidden;
+  for (int h = threadIdx.x; h < hidden; h += NA_THREADS) {
+    const float v = at(h);
+    if (store_residual) res[h] = v;
+    na_store(dst + h, weight ? v * inv_x[h / size_x] * weight[h] : v);
+  }
+}
+
+// As ta_norm_add_rmsnorm, with the number of groups of each norm.
+extern "C" int ta_group_norm_add(void* residual, const void* delta, const void* post_weight, float post_eps, int post_groups,
+                                 const void* weight, float eps, int groups, void* out, const void* rows, int n_rows,
+                                 int hidden, int store_residual, int delta_dtype, int out_dtype, hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  if (hidden <= 0 || post_groups <= 0 || groups <= 0 || hidden % post_groups || hidden % groups) return -1;
+  if (post_weight && !delta) return -1;
+  const int most = post_groups > groups ? post_groups : groups;
+  if (post_groups + groups > 12 * 1024) return -1;           // (what LDS holds of factors)
+  const bool aligned = (((uintptr_t)residual | (uintptr_t)delta | (uintptr_t)post_weight | (uintptr_t)weight | (uintptr_t)out) & 15) == 0;
+  const bool vec = aligned && hidden <= 8192 && (hidden / post_groups) % 4 == 0 && (hidden / groups) % 4 == 0;
+  const size_t lds = sizeof(float) * (vec ? (size_t)hidden / 4 + most : (size_t)post_groups + groups);
+#define GROUP_VEC(TD, TO, CH)                                                                                            \
+    group_norm_add_vec_kernel<TD, TO, CH><<<n_rows, NA_THREADS, lds, stream>>>(                                           \
+        (float*)residual, (const TD*)delta, (const float*)post_weight, post_eps, post_groups, (const float*)weight, eps,  \
+        groups, (TO*)out, (const int*)rows, hidden, store_residual)
+#define GROUP_GO(TD, TO)                                                                                                 \
+  do {                                                                                                                   \
+    if (vec) {                                                                                                           \
+      if (hidden <= 1024) GROUP_VEC(TD, TO, 1); else if (hidden <= 2048) GROUP_VEC(TD, TO, 2);                            \
+      else if (hidden <= 4096) GROUP_VEC(TD, TO, 4); else GROUP_VEC(TD, TO, 8);                                           \
+    } else                                                                                                               \
+      group_norm_add_kernel<TD, TO><<<n_rows, NA_THREADS, lds, stream>>>(                                                 \
+          (float*)residual, (const TD*)delta, (const float*)post_weight, post_eps, post_groups, (const float*)weight,     \
+          eps, groups, (TO*)out, (const int*)rows, hidden, store_residual);                                               \
+  } while (0)
+  if (delta_dtype == DT_F32 && out_dtype == DT_F32) GROUP_GO(float, float);
+  else if (delta_dtype == DT_BF16 && out_dtype == DT_BF16) GROUP_GO(bf16_t, bf16_t);
+  else if (delta_dtype == DT_BF16 && out_dtype == DT_F32) GROUP_GO(bf16_t, float);
+  else return -1;
+#undef GROUP_GO
+#undef GROUP_VEC
+  return LAUNCH_STATUS();
+}

@@ -120,3 +120,118 @@ extern "C" int ta_norm_rotate_store(void* qkv, int row_stride, const void* bias,
         (bf16_t*)k_pages, (bf16_t*)v_pages, n_q, n_k, n_v, d, dv, page_size, (const float*)q_norm, (const float*)k_norm, eps);
   return LAUNCH_STATUS();
 }
+
+// table[t] = [cosines | sines] (each rot / 2 floats) of positions[t] * rates[i], formed and taken in float, times magnitude.
+__global__ void __launch_bounds__(RP_THREADS)
+rotation_table_kernel(const int* __restrict__ positions, const float* __restrict__ rates, float magnitude, int half,
+                      float* __restrict__ table, int total) {
+  const int idx = blockIdx.x * RP_THREADS + threadIdx.x;
+  if (idx >= total) return;
+  const int t = idx / half, i = idx - t * half;
+  float s, c;
+  sincosf((float)positions[t] * rates[i], &s, &c);
+  table[(size_t)t * 2 * half + i] = magnitude * c;
+  table[(size_t)t * 2 * half + half + i] = magnitude * s;
+}
+
+// A wave a head of a token.  Rows of qkv as above: n_q query heads and n_k key heads of d elements, n_v value heads of dv.
+// q_norm / k_norm (float [d], or null): the head is divided by its root mean square (eps inside the root) and multiplied
+// by the weight; then the first `rot` coordinates turn by the token's row of `table` ([cosines | sines]).  norm_values:
+// a value head is divided by its root mean square; share (float [1], or null): it becomes (1 - share) v + share * first,
+// first[t * first_stride + ...] being the token's value heads of another layer.  Heads go back into their rows, keys and
+// values also into their pages (slots as above), rounded once.
+template <typename T, int PER>
+__global__ void __launch_bounds__(RP_THREADS)
+head_norm_rotate_store_kernel(T* __restrict__ qkv, int row_stride, const float* __restrict__ table, int rot,
+                              const int* __restrict__ slots, T* __restrict__ k_pages, T* __restrict__ v_pages, int n_q,
+                              int n_k, int n_v, int d, int dv, int page_size, const float* __restrict__ q_norm,
+                              const float* __restrict__ k_norm, int norm_values, const T* __restrict__ first,
+                              int first_stride, const float* __restrict__ share, float eps) {
+  __shared__ float row_s[RP_THREADS / WAVE][PER * WAVE];
+  const int t = blockIdx.x, lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE;
+  const int head = blockIdx.y * (RP_THREADS / WAVE) + wave;
+  if (head >= n_q + n_k + n_v) return;                       // (nobody waits for anybody in this kernel)
+  const bool value = head >= n_q + n_k, key = !value && head >= n_q;
+  const int h = value ? head - n_q - n_k : key ? head - n_q : head, n = value ? dv : d;
+  T* row = qkv + (size_t)t * row_stride + (value ? (size_t)(n_q + n_k) * d + (size_t)h * dv : (size_t)head * d);
+  const float* weight = value ? nullptr : key ? k_norm : q_norm;
+  const T* other = (value && share) ? first + (size_t)t * first_stride + (size_t)h * dv : nullptr;
+  const int slot = slots ? slots[t] : -1, half = rot / 2;
+  float x[PER], w[PER], o[PER], c[PER], s[PER], sq = 0.f;
+#pragma unroll
+  for (int r = 0; r < PER; ++r) {
+    const int i = lane + r * WAVE;
+    x[r] = i < n ? ld(row + i) : 0.f;
+    w[r] = (weight && i < n) ? weight[i] : 1.f;
+    o[r] = (other && i < n) ? ld(other + i) : 0.f;
+    const bool turns = !value && i < rot;
+    c[r] = turns ? table[(size_t)t * rot + (i < half ? i : i - half)] : 1.f;
+    s[r] = turns ? table[(size_t)t * rot + half + (i < half ? i : i - half)] : 0.f;
+  }
+  const float mix = other ? share[0] : 0.f;
+  if (weight || (value && norm_values)) {
+#pragma unroll
+    for (int r = 0; r < PER; ++r) sq = fmaf(x[r], x[r], sq);
+    const float inv = 1.0f / sqrtf(wave_sum(sq) / (float)n + eps);
+#pragma unroll
+    for (int r = 0; r < PER; ++r) x[r] *= inv * w[r];
+  }
+  if (other) {
+#pragma unroll
+    for (int r = 0; r < PER; ++r) x[r] = (1.0f - mix) * x[r] + mix * o[r];
+  }
+  if (!value && half > 0) {
+    // A coordinate's partner lies with another lane: through the wave's own row in LDS.
+#pragma unroll
+    for (int r = 0; r < PER; ++r) row_s[wave][lane + r * WAVE] = x[r];
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int r = 0; r < PER; ++r) {
+      const int i = lane + r * WAVE;
+      if (i >= rot) continue;
+      const float with = row_s[wave][i < half ? i + half : i - half];
+      x[r] = i < half ? x[r] * c[r] - with * s[r] : x[r] * c[r] + with * s[r];
+    }
+  }
+  const int page = slot >= 0 ? slot / page_size : 0, off = slot >= 0 ? slot % page_size : 0;
+#pragma unroll
+  for (int r = 0; r < PER; ++r) {
+    const int i = lane + r * WAVE;
+    if (i >= n) continue;
+    st(row + i, x[r]);
+    if (slot < 0) continue;
+    if (key) st(k_pages + (((size_t)page * n_k + h) * page_size + off) * d + i, x[r]);
+    if (value) st(v_pages + (((size_t)page * n_v + h) * dv + i) * page_size + off, x[r]);
+  }
+}
+
+extern "C" int ta_rotation_table(const void* positions, const void* rates, float magnitude, int rot, void* table,
+                                 int n_tokens, hipStream_t stream) {
+  if (n_tokens <= 0 || rot <= 0) return 0;
+  const long total = (long)n_tokens * (rot / 2);
+  if (rot % 2 || total > 0x7fffffffL - RP_THREADS) return -1;
+  rotation_table_kernel<<<(unsigned)((total + RP_THREADS - 1) / RP_THREADS), RP_THREADS, 0, stream>>>(
+      (const int*)positions, (const float*)rates, magnitude, rot / 2, (float*)table, (int)total);
+  return LAUNCH_STATUS();
+}
+
+extern "C" int ta_head_norm_rotate_store(void* qkv, int row_stride, const void* table, int rot, const void* slots, void* k_pages,
+                                         void* v_pages, int n_tokens, int n_q, int n_k, int n_v, int d, int dv, int page_size,
+                                         const void* q_norm, const void* k_norm, int norm_values, const void* first,
+                                         int first_stride, const void* share, float eps, int dtype, hipStream_t stream) {
+  if (n_tokens <= 0) return 0;
+  if (rot < 0 || rot % 2 || rot > d || d <= 0 || dv <= 0 || n_q < 0 || n_k < 0 || n_v < 0 || n_q + n_k + n_v <= 0) return -1;
+  if ((rot > 0 && !table) || (share && !first) || d > 8 * WAVE || dv > 8 * WAVE) return -1;
+  const int waves = RP_THREADS / WAVE, most = d > dv ? d : dv;
+  dim3 grid(n_tokens, (n_q + n_k + n_v + waves - 1) / waves);
+#define STORE(TT, PP) head_norm_rotate_store_kernel<TT, PP><<<grid, RP_THREADS, 0, stream>>>((TT*)qkv, row_stride,          \
+      (const float*)table, rot, (const int*)slots, (TT*)k_pages, (TT*)v_pages, n_q, n_k, n_v, d, dv, page_size,              \
+      (const float*)q_norm, (const float*)k_norm, norm_values, (const TT*)first, first_stride, (const float*)share, eps)
+#define STORES(TT) if (most <= WAVE) STORE(TT, 1); else if (most <= 2 * WAVE) STORE(TT, 2);                                  \
+                   else if (most <= 4 * WAVE) STORE(TT, 4); else STORE(TT, 8)
+  if (dtype == DT_F32) { STORES(float); } else { STORES(bf16_t); }
+#undef STORES
+#undef STORE
+  return LAUNCH_STATUS();
+}

@@ -188,13 +188,16 @@ __global__ void side_gate_kernel(const T* __restrict__ gate, const T* __restrict
   }
 }
 
-// out[t, j] = gelu_tanh(in[t, j]) * in[t, inner + j].
-template <typename T>
-__global__ void gelu_gate_kernel(const T* __restrict__ in, T* __restrict__ out, int inner, size_t total) {
+template <bool RELU>
+__device__ __forceinline__ float rt_gate_act(float z) { return RELU ? fmaxf(z, 0.f) : rt_gelu_tanh(z); }
+
+// out[t, j] = act(in[t, j]) * in[t, inner + j]: gelu_tanh, or (RELU) max(z, 0).
+template <typename T, bool RELU>
+__global__ void named_gate_kernel(const T* __restrict__ in, T* __restrict__ out, int inner, size_t total) {
   for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total; idx += (size_t)gridDim.x * blockDim.x) {
     const size_t t = idx / inner;
     const int j = (int)(idx - t * inner);
-    st(out + idx, rt_gelu_tanh(ld(in + t * 2 * inner + j)) * ld(in + t * 2 * inner + inner + j));
+    st(out + idx, rt_gate_act<RELU>(ld(in + t * 2 * inner + j)) * ld(in + t * 2 * inner + inner + j));
   }
 }
 
@@ -235,8 +238,9 @@ __global__ void expert_gate_vec_kernel(const bf16_t* __restrict__ gate_up, const
   }
 }
 
-// gelu_gate for bfloat16 rows whose length is a multiple of 8: sixteen bytes of gate and of up per thread.
-__global__ void gelu_gate_vec_kernel(const bf16_t* __restrict__ in, bf16_t* __restrict__ out, int inner8, size_t total8) {
+// The same for bfloat16 rows whose length is a multiple of 8: sixteen bytes of gate and of up per thread.
+template <bool RELU>
+__global__ void named_gate_vec_kernel(const bf16_t* __restrict__ in, bf16_t* __restrict__ out, int inner8, size_t total8) {
   for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total8; idx += (size_t)gridDim.x * blockDim.x) {
     const size_t t = idx / inner8, j = idx - t * inner8;
     const uint4* row = reinterpret_cast<const uint4*>(in) + t * 2 * inner8;
@@ -244,7 +248,7 @@ __global__ void gelu_gate_vec_kernel(const bf16_t* __restrict__ in, bf16_t* __re
     rt_unpack8(row[j], g);
     rt_unpack8(row[inner8 + j], u);
 #pragma unroll
-    for (int k = 0; k < 8; ++k) v[k] = rt_gelu_tanh(g[k]) * u[k];
+    for (int k = 0; k < 8; ++k) v[k] = rt_gate_act<RELU>(g[k]) * u[k];
     reinterpret_cast<uint4*>(out)[idx] = rt_pack8(v);
   }
 }
@@ -313,18 +317,27 @@ extern "C" int ta_side_gate(const void* gate, const void* table, int table_width
   return LAUNCH_STATUS();
 }
 
-extern "C" int ta_gelu_gate(const void* in, void* out, int n_tokens, int inner, int dtype, hipStream_t stream) {
+template <bool RELU>
+static int launch_named_gate(const void* in, void* out, int n_tokens, int inner, int dtype, hipStream_t stream) {
   const size_t total = (size_t)n_tokens * inner;
   if (total == 0) return 0;
   if (dtype == DT_BF16 && inner % 8 == 0 && (((uintptr_t)in | (uintptr_t)out) & 15) == 0) {
-    gelu_gate_vec_kernel<<<rt_blocks(total / 8), 256, 0, stream>>>((const bf16_t*)in, (bf16_t*)out, inner / 8, total / 8);
+    named_gate_vec_kernel<RELU><<<rt_blocks(total / 8), 256, 0, stream>>>((const bf16_t*)in, (bf16_t*)out, inner / 8, total / 8);
     return LAUNCH_STATUS();
   }
   if (dtype == DT_F32)
-    gelu_gate_kernel<float><<<rt_blocks(total), 256, 0, stream>>>((const float*)in, (float*)out, inner, total);
+    named_gate_kernel<float, RELU><<<rt_blocks(total), 256, 0, stream>>>((const float*)in, (float*)out, inner, total);
   else
-    gelu_gate_kernel<bf16_t><<<rt_blocks(total), 256, 0, stream>>>((const bf16_t*)in, (bf16_t*)out, inner, total);
+    named_gate_kernel<bf16_t, RELU><<<rt_blocks(total), 256, 0, stream>>>((const bf16_t*)in, (bf16_t*)out, inner, total);
   return LAUNCH_STATUS();
+}
+
+extern "C" int ta_gelu_gate(const void* in, void* out, int n_tokens, int inner, int dtype, hipStream_t stream) {
+  return launch_named_gate<false>(in, out, n_tokens, inner, dtype, stream);
+}
+
+extern "C" int ta_relu_gate(const void* in, void* out, int n_tokens, int inner, int dtype, hipStream_t stream) {
+  return launch_named_gate<true>(in, out, n_tokens, inner, dtype, stream);
 }
 
 // ---------------------------------------------------------------------------------------------------------------

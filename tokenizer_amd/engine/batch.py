@@ -82,6 +82,8 @@ class StepContext:
     max_position: int                # largest position in the batch
     page_size: int
     n_wanted: int = -1               # wanted places of the real entries (the leading rows of the step's logits)
+    shared: dict = dataclasses.field(default_factory=dict, repr=False, compare=False)   # what a layer leaves for later
+    #                                  layers of the same forward (emptied when a forward starts)
 
 
 def build_context(entries: list[StepEntry], manager, device, table_width: int | None = None,

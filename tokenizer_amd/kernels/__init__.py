@@ -158,7 +158,9 @@ class Ops:
                      "ta_sigmoid_head_gate", "ta_route_top", "ta_expert_gate", "ta_side_gate", "ta_gelu_gate", "ta_norm_side_norm", "ta_route_rows", "ta_expert_slots", "ta_grouped_gemm_bf16", "ta_expert_combine",
                      "ta_add_pair_rmsnorm", "ta_latent_store", "ta_rotate_tails", "ta_head_linear", "ta_short_conv_silu",
                      "ta_delta_scan", "ta_route_sigmoid", "ta_route_rows_sigmoid", "ta_expert_act", "ta_relu2",
-                     "ta_add_terms_rmsnorm", "ta_scale_cap", "ta_route_scores", "ta_selective_scan", "ta_route_rows_scores"):
+                     "ta_add_terms_rmsnorm", "ta_scale_cap", "ta_route_scores", "ta_selective_scan", "ta_route_rows_scores",
+                     "ta_rotation_table", "ta_head_norm_rotate_store", "ta_group_norm_add", "ta_relu_gate",
+                     "ta_talking_attention_generic", "ta_retention_scan"):
             getattr(self.lib, name).restype = ctypes.c_int
         self.lib.ta_grouped_gemm_bf16.argtypes = [ctypes.c_void_p, ctypes.c_int, ctypes.c_void_p, ctypes.c_void_p, ctypes.c_int,
                                                   ctypes.c_int, ctypes.c_void_p, ctypes.c_long, ctypes.c_int, ctypes.c_void_p,
@@ -592,11 +594,13 @@ class Ops:
 
     def norm_add_rmsnorm(self, residual: torch.Tensor, delta: torch.Tensor | None, post_weight: torch.Tensor | None,
                          post_eps: float, weight: torch.Tensor | None, eps: float, out: torch.Tensor,
-                         rows: torch.Tensor | None = None, store_residual: bool = True) -> torch.Tensor:
+                         rows: torch.Tensor | None = None, store_residual: bool = True, post_groups: int = 1,
+                         groups: int = 1) -> torch.Tensor:
         """The norm behind a sub-layer, the residual add and the norm before the next one in one kernel:
         x = residual + delta / sqrt(mean(delta^2) + post_eps) * post_weight (delta as it is without `post_weight`,
         nothing without `delta`), stored back into `residual` unless `rows` selects a subset or `store_residual` is
-        off; out = x / sqrt(mean(x^2) + eps) * weight, or x itself without `weight`.
+        off; out = x / sqrt(mean(x^2) + eps) * weight, or x itself without `weight`.  `post_groups`, `groups`: the norm on
+        delta (on x) is over so many equal runs of neighbours, each divided by its own root mean square.
 
         residual float32 [T, H]; delta [T, H] float32 or bfloat16; weights float32 [H]; rows int32 or None; out
         [rows, H] in delta's dtype or float32."""
@@ -613,6 +617,14 @@ class Ops:
         if rows is not None:
             _need(rows.dtype == torch.int32 and not store_residual, "a row subset (int32) never stores the residual")
         delta_code = _code(delta.dtype) if delta is not None else _code(out.dtype)
+        if post_groups != 1 or groups != 1:
+            _need(post_groups > 0 and groups > 0 and hidden % post_groups == 0 and hidden % groups == 0,
+                  "the groups are equal parts of the row")
+            self._check(self.lib.ta_group_norm_add(
+                _ptr(residual), _ptr(delta), _ptr(post_weight if delta is not None else None), ctypes.c_float(post_eps), post_groups,
+                _ptr(weight), ctypes.c_float(eps), groups, _ptr(out), _ptr(rows), n_rows, hidden,
+                int(store_residual and delta is not None), delta_code, _code(out.dtype), self._stream()), "group_norm_add")
+            return out
         self._check(self.lib.ta_norm_add_rmsnorm(_ptr(residual), _ptr(delta), _ptr(post_weight), ctypes.c_float(post_eps),
                                                  _ptr(weight), ctypes.c_float(eps), _ptr(out), _ptr(rows), n_rows, hidden,
                                                  int(store_residual and delta is not None), delta_code, _code(out.dtype),
@@ -683,6 +695,51 @@ class Ops:
             _ptr(qkv), qkv.stride(0), _ptr(bias), _ptr(positions), _ptr(rates if dims else None), dims, _ptr(slots),
             _ptr(k_pages), _ptr(v_pages), n_tokens, n_q, n_k, n_v, d, dv, page_size, _ptr(q_norm), _ptr(k_norm),
             ctypes.c_float(eps), _code(qkv.dtype), self._stream()), "norm_rotate_store")
+
+    def rotation_table(self, positions: torch.Tensor, rates: torch.Tensor, magnitude: float, out: torch.Tensor) -> torch.Tensor:
+        """out [T, 2 R] float32: the cosines, then the sines, of positions[t] * rates[i] (float32 angles, accurate sine and
+        cosine), times `magnitude`.  positions int32 [T], rates float32 [R]."""
+        _dev(positions, rates, out)
+        n_tokens, pairs = positions.numel(), rates.numel()
+        _need(positions.dtype == torch.int32 and rates.dtype == torch.float32 and out.dtype == torch.float32
+              and tuple(out.shape) == (n_tokens, 2 * pairs), "rotation_table operands do not fit")
+        self._check(self.lib.ta_rotation_table(_ptr(positions), _ptr(rates), ctypes.c_float(magnitude), 2 * pairs, _ptr(out),
+                                               n_tokens, self._stream()), "rotation_table")
+        return out
+
+    def head_norm_rotate_store(self, qkv: torch.Tensor, table: torch.Tensor | None, dims: int, slots: torch.Tensor | None,
+                               k_pages: torch.Tensor | None, v_pages: torch.Tensor | None, n_q: int, n_k: int, n_v: int, d: int,
+                               dv: int, q_norm: torch.Tensor | None, k_norm: torch.Tensor | None, norm_values: bool,
+                               first: torch.Tensor | None, share: torch.Tensor | None, eps: float) -> None:
+        """In place on rows of `qkv` ([T, >= (n_q + n_k) d + n_v dv]: query heads, key heads, value heads), head by head:
+        an RMS norm with weight `q_norm` / `k_norm` (float32 [d], the same for every head), then the rotation of the first
+        `dims` coordinates by the token's row of `table` (float32 [T, dims], see `rotation_table`); values to unit RMS
+        (`norm_values`), then (1 - share) v + share * first with `first` [T, n_v dv] (rows may lie apart) and share float32
+        [1].  Keys and values are written at `slots` into their pages (layouts as in `norm_rotate_store`)."""
+        _dev(qkv, table, slots, k_pages, v_pages, q_norm, k_norm, share)
+        n_tokens, width = qkv.shape
+        _need(width >= (n_q + n_k) * d + n_v * dv and qkv.stride(1) == 1, "qkv is narrower than its heads")
+        _need(dims % 2 == 0 and 0 <= dims <= d and 0 < d <= 512 and 0 < dv <= 512, "head sizes the kernel does not take")
+        _need(dims == 0 or (table is not None and table.dtype == torch.float32 and tuple(table.shape) == (n_tokens, dims)),
+              "the rotation's table is float32 [T, dims]")
+        for norm in (q_norm, k_norm):
+            _need(norm is None or (norm.dtype == torch.float32 and norm.numel() == d), "the heads' norm weights are float32 [d]")
+        _need((first is None) == (share is None), "values to take in come with their share")
+        if first is not None:
+            _need(first.is_cuda and first.dtype == qkv.dtype and tuple(first.shape) == (n_tokens, n_v * dv) and first.stride(1) == 1,
+                  "the values to take in are [T, n_v dv] of qkv's dtype")
+            _need(share.dtype == torch.float32 and share.numel() == 1, "the share is float32 [1]")
+        page_size = 1
+        if slots is not None:
+            _need(slots.dtype == torch.int32 and slots.numel() == n_tokens, "slots must be int32 [T]")
+            _need(k_pages is not None and v_pages is not None, "slots without pages")
+            _need(k_pages.dtype == qkv.dtype and v_pages.dtype == qkv.dtype, "pages must have the dtype of qkv")
+            page_size = self._page_size(k_pages, v_pages, n_k, d, dv, n_v)
+        self._check(self.lib.ta_head_norm_rotate_store(
+            _ptr(qkv), qkv.stride(0), _ptr(table if dims else None), dims, _ptr(slots), _ptr(k_pages), _ptr(v_pages), n_tokens,
+            n_q, n_k, n_v, d, dv, page_size, _ptr(q_norm), _ptr(k_norm), int(bool(norm_values)), _ptr(first),
+            0 if first is None else first.stride(0), _ptr(share), ctypes.c_float(eps), _code(qkv.dtype), self._stream()),
+            "head_norm_rotate_store")
 
     def differential_heads(self, mixed: torch.Tensor, lam: torch.Tensor, eps: float, out_scale: float, n_heads: int,
                            group: int, dv: int, out: torch.Tensor) -> torch.Tensor:
@@ -894,14 +951,15 @@ class Ops:
     def silu_gate(self, gate_up: torch.Tensor, out: torch.Tensor, act: tuple | None = None) -> torch.Tensor:
         """out = silu(gate_up[:, :I]) * gate_up[:, I:].  gate_up [T, 2I]; out [T, I].  With `act` = (alpha, limit,
         shift): g' = min(g, limit), u' = clamp(u, -limit, limit), out = g' * sigmoid(alpha g') * (u' + shift); with
-        `act` = "gelu_tanh": out = 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))) * u."""
+        `act` = "gelu_tanh": out = 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))) * u; "relu": out = max(g, 0) * u."""
         _dev(gate_up, out)
         n_tokens, two_inner = gate_up.shape
         _need(two_inner % 2 == 0 and tuple(out.shape) == (n_tokens, two_inner // 2) and out.dtype == gate_up.dtype,
               "silu_gate shapes do not fit")
-        if act == "gelu_tanh":
-            self._check(self.lib.ta_gelu_gate(_ptr(gate_up), _ptr(out), n_tokens, two_inner // 2, _code(out.dtype),
-                                              self._stream()), "gelu_gate")
+        if isinstance(act, str):
+            _need(act in ("gelu_tanh", "relu"), f"unknown gated activation {act!r}")
+            gate = self.lib.ta_gelu_gate if act == "gelu_tanh" else self.lib.ta_relu_gate
+            self._check(gate(_ptr(gate_up), _ptr(out), n_tokens, two_inner // 2, _code(out.dtype), self._stream()), act)
             return out
         if act is not None:
             alpha, limit, shift = act
@@ -1100,6 +1158,34 @@ class Ops:
             split_keys, splits, 0 if chunk is None else int(chunk), _ptr(slopes), _ptr(sinks),
             int(keep_first) if kept_splits else 0, kept_splits, n_kv if value_heads is None else int(value_heads),
             ctypes.c_float(softcap or 0.0), self._stream()), "decode_attention")
+        return out
+
+    def talking_attention(self, qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
+                          positions: torch.Tensor, entry_of_token: torch.Tensor, block_table: torch.Tensor, n_q: int, n_kv: int,
+                          head_dim: int, value_dim: int, scale: float, talk: torch.Tensor, max_position: int | None = None,
+                          batch=None) -> torch.Tensor:
+        """Causal attention whose heads' softmax weights are mixed: head h's weights become sum_g talk[h, g] weight_g and
+        meet the values of head h's own kv head.  Operands as in `paged_attention`; talk float32 [n_q, n_q]; out
+        [T, n_q value_dim].  Scores, weights and the mix are float32."""
+        _dev(qkv, out, k_pages, v_pages, positions, entry_of_token, block_table, talk)
+        n_tokens = qkv.shape[0]
+        _need(qkv.shape[1] >= n_q * head_dim and qkv.stride(1) == 1, "qkv is narrower than the query heads")
+        _need(tuple(out.shape) == (n_tokens, n_q * value_dim) and out.dtype == qkv.dtype, "attention output shape")
+        _need(k_pages.dtype == qkv.dtype and v_pages.dtype == qkv.dtype, "pages must have the dtype of qkv")
+        page_size = self._page_size(k_pages, v_pages, n_kv, head_dim, value_dim)
+        _need(positions.dtype == torch.int32 and positions.numel() == n_tokens, "positions must be int32 [T]")
+        _need(entry_of_token.dtype == torch.int32 and entry_of_token.numel() == n_tokens, "entry_of_token must be int32 [T]")
+        _need(block_table.dtype == torch.int32 and block_table.dim() == 2, "block_table must be int32 [E, P]")
+        _need(n_kv > 0 and n_q % n_kv == 0 and n_q <= 128, "query heads are a multiple of kv heads, at most 128")
+        _need(talk.dtype == torch.float32 and tuple(talk.shape) == (n_q, n_q), "the heads' mix is float32 [n_q, n_q]")
+        _need(0 < head_dim <= 512 and 0 < value_dim, "head sizes up to 512 are supported")
+        if max_position is not None:
+            _need(max_position // page_size < block_table.shape[1], "block table is too narrow for the positions")
+        stats = torch.empty((n_tokens, n_q, 2), dtype=torch.float32, device=qkv.device)
+        self._check(self.lib.ta_talking_attention_generic(
+            _ptr(qkv), qkv.stride(0), _ptr(out), _ptr(k_pages), _ptr(v_pages), _ptr(positions), _ptr(entry_of_token),
+            _ptr(block_table), block_table.shape[1], _ptr(stats), _ptr(talk), n_tokens, n_q, n_kv, head_dim, value_dim, page_size,
+            ctypes.c_float(scale), _code(qkv.dtype), self._stream()), "talking_attention")
         return out
 
     # --------------------------------------------------------------------- linear
@@ -1302,7 +1388,7 @@ class Ops:
         if out is None:
             out = torch.empty((m, inner), dtype=x.dtype, device=x.device)
         _need(tuple(out.shape) == (m, inner) and out.dtype == x.dtype and out.is_contiguous(), "gated output shape")
-        if act is not None and act != "gelu_tanh":
+        if act is not None and not isinstance(act, str):
             return self.silu_gate(self.linear(x, weight), out, act=act)
         if (x.dtype == torch.bfloat16 and m <= self.SKINNY_ROWS and x.shape[1] % 8 == 0 and (m == 1 or x.stride(0) % 8 == 0)
                 and not (self.use_library_gemm and m > self.FUSED_ROWS
@@ -1314,7 +1400,7 @@ class Ops:
             _need(k % 8 == 0 and lda % 8 == 0, "bfloat16 products need K and the row stride to be multiples of 8")
             _need(x.data_ptr() % 16 == 0 and weight.data_ptr() % 16 == 0, "operands must be 16-byte aligned")
             self._check(self.lib.ta_gemm_skinny_bf16(_ptr(x), lda, _ptr(weight), None, _ptr(out), inner, m, 2 * inner,
-                                                     k, _BF16, 2 if act == "gelu_tanh" else 1, self.skinny_column_blocks,
+                                                     k, _BF16, {None: 1, "gelu_tanh": 2, "relu": 3}[act], self.skinny_column_blocks,
                                                      self._stream()), "linear_silu_gate")
             return out
         return self.silu_gate(self.linear(x, weight), out, act=act)
@@ -1567,6 +1653,35 @@ class Ops:
         self._check(self.lib.ta_head_norm_gate(_ptr(read), _ptr(weight), _ptr(gate_rows), gate_rows.shape[1], gate_offset,
                                                ctypes.c_float(eps), n_tokens, heads, dv, _ptr(out), _code(out.dtype),
                                                self._stream()), "head_norm_gate")
+        return out
+
+    # ------------------------------------------------------------------- retention
+    def retention(self, qkvg: torch.Tensor, table: torch.Tensor | None, dims: int, decays: torch.Tensor, state: torch.Tensor,
+                  cu_q: torch.Tensor, first_position: torch.Tensor, state_slots: torch.Tensor, out: torch.Tensor, heads: int,
+                  d: int, dv: int, eps: float) -> torch.Tensor:
+        """The retention recurrence over every entry's rows, from and into the entries' state rows, with the rotation in
+        front and the heads' norm and gate behind: per head S <- c S + k v^T, o = S^T q, out = o / rms(o) * silu(g).
+
+        qkvg [T, >= 2 heads d + 2 heads dv]: q, k (heads of d), v and g (heads of dv) side by side; the first `dims`
+        coordinates of q and k turn by `table` (float32 [T, dims], see `rotation_table`), k is multiplied by d^(-1/2);
+        decays float32 [heads]; state float32 [slots, heads dv d] (S transposed; an entry whose first position is 0 starts
+        from zeros); out [T, heads dv] of qkvg's dtype."""
+        _dev(qkvg, table, decays, state, cu_q, first_position, state_slots, out)
+        n_tokens = qkvg.shape[0]
+        _need(qkvg.stride(1) == 1 and qkvg.shape[1] >= 2 * heads * (d + dv), "q, k, v, g do not fit the rows")
+        _need(dims % 2 == 0 and 0 <= dims <= d, "the rotation covers an even number of a head's coordinates")
+        _need(dims == 0 or (table is not None and table.dtype == torch.float32 and tuple(table.shape) == (n_tokens, dims)),
+              "the rotation's table is float32 [T, dims]")
+        _need(decays.dtype == torch.float32 and decays.numel() == heads, "decays float32 [heads]")
+        _need(state.dtype == torch.float32 and state.dim() == 2 and state.shape[1] >= heads * d * dv, "state rows are too short")
+        _need(tuple(out.shape) == (n_tokens, heads * dv) and out.dtype == qkvg.dtype, "out [T, heads dv] of qkvg's dtype")
+        _need(0 < d <= 256 and 0 < dv <= 256, "heads of up to 256 coordinates and 256 values are supported")
+        n_entries = cu_q.numel() - 1
+        _need(first_position.numel() == n_entries == state_slots.numel(), "one first position and slot per entry")
+        self._check(self.lib.ta_retention_scan(
+            _ptr(qkvg), qkvg.stride(0), _ptr(table if dims else None), dims, _ptr(decays), _ptr(state), ctypes.c_long(state.shape[1]),
+            _ptr(cu_q), _ptr(first_position), _ptr(state_slots), _ptr(out), n_entries, heads, d, dv, ctypes.c_float(eps),
+            0x7fffffff, _code(qkvg.dtype), self._stream()), "retention_scan")
         return out
 
     # ------------------------------------------------------------------- sampling

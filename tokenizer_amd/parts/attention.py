@@ -38,7 +38,11 @@ class GQAttention(Mixer):
     [n_kv d] over all query rows at once and over all key rows at once, before the rotation) and `head_gate`
     (head h's output times sigmoid(W_g x)_h, W_g = `gate_proj.weight` [n_heads, hidden], read from the mixer's
     input; the gate's rows ride in the joined projection) and `softcap` c (a scaled score s becomes c tanh(s / c)
-    before the softmax); `sink` joins these too.  For the kernels the maps of differential heads are
+    before the softmax); `sink` joins these too; `qk_norm` "head" (an RMS norm of every query and key head on its own, one
+    weight `q_norm` / `k_norm` [d] for all heads), `value_norm` (every value head brought to unit RMS, no weight),
+    `value_mix` (see `MixerSpec`; the share is the tensor `vmix`, one number) and `talking` (behind the softmax the heads'
+    weights are mixed, head h's becoming sum_g talk[h, g] weight_g with the tensor `talk` [H, H], and then meet the
+    values of head h's own kv head).  For the kernels the maps of differential heads are
     heads of their own: the query rows are reordered at load time to (kv head, map, head within the group), so
     that map m of kv head g is key head 2 g + m in the ordinary grouping, and key heads 2 g and 2 g + 1 read
     value head g (`value_heads`).
@@ -82,7 +86,7 @@ class GQAttention(Mixer):
     @staticmethod
     def _is_extended(spec: MixerSpec) -> bool:
         return (spec.differential is not None or bool(spec.keep_first) or spec.qk_norm is not None or spec.head_gate
-                or spec.softcap is not None or (spec.position is not None and spec.position.kind == "rope_partial"))
+                or spec.softcap is not None or spec.value_norm or spec.value_mix is not None or spec.talking or (spec.position is not None and spec.position.kind == "rope_partial"))
 
     def _build_extended(self, spec: MixerSpec, tensors: dict[str, torch.Tensor], runtime: Runtime) -> None:
         if not spec.own_kv or spec.chunk is not None or spec.distance_bias is not None or spec.out_bias:
@@ -92,8 +96,21 @@ class GQAttention(Mixer):
             raise ValueError("a sink belongs to one softmax a head, not to the two maps of a differential head")
         if spec.softcap is not None and not spec.softcap > 0:
             raise ValueError(f"a cap on the scores is positive, found {spec.softcap}")
-        if spec.qk_norm not in (None, "whole"):
-            raise ValueError(f"qk_norm {spec.qk_norm!r}: known is \"whole\"")
+        if spec.qk_norm not in (None, "whole", "head"):
+            raise ValueError(f"qk_norm {spec.qk_norm!r}: known are \"whole\" and \"head\"")
+        if spec.value_mix not in (None, "give", "take"):
+            raise ValueError(f"value_mix {spec.value_mix!r}: known are \"give\" and \"take\"")
+        # (Norms of single heads and whatever changes the values run in a store kernel of their own.)
+        self.head_wise = spec.qk_norm == "head" or spec.value_norm or spec.value_mix is not None
+        self.value_norm, self.value_mix, self.talk = spec.value_norm, spec.value_mix, None
+        if self.head_wise and (spec.qkv_bias or spec.differential is not None or spec.qk_norm == "whole"):
+            raise ValueError("norms of single heads and changed values do not combine with biases, differential maps or a norm "
+                             "over the whole projection")
+        if spec.talking:
+            if spec.differential is not None or spec.sink or spec.softcap is not None or spec.window is not None:
+                raise ValueError("mixed heads do not combine with differential maps, sinks, capped scores or windows")
+            self.talk = tensors["talk"].to(torch.float32).contiguous()
+        self.share = tensors["vmix"].to(torch.float32).reshape(1).contiguous() if spec.value_mix is not None else None
         H, G, d, dv, hidden = self.n_q, self.n_kv, self.d, self.dv, spec.hidden_size
         self.maps = 2 if spec.differential is not None else 1
         self.group = H // G
@@ -123,7 +140,9 @@ class GQAttention(Mixer):
             pair = lambda a, b: torch.exp((tensors[a].to(torch.float32) * tensors[b].to(torch.float32)).sum())
             self.lam = (pair("lq1", "lk1") - pair("lq2", "lk2") + float(spec.differential)).reshape(1).contiguous()
             self.out_scale = 1.0 - float(spec.differential)
-        self.q_norm = by_kv_head(tensors["q_norm"]).to(torch.float32).contiguous() if spec.qk_norm else None
+        self.q_norm = None
+        if spec.qk_norm:
+            self.q_norm = (by_kv_head(tensors["q_norm"]) if spec.qk_norm == "whole" else tensors["q_norm"]).to(torch.float32).contiguous()
         self.k_norm = tensors["k_norm"].to(torch.float32).contiguous() if spec.qk_norm else None
         self.head_gate, self.eps = spec.head_gate, float(spec.eps)
         # (A sink and a cap on the scores are handed to the attention kernels only where a layer has them.)
@@ -167,8 +186,13 @@ class GQAttention(Mixer):
             for name in ("lq1", "lk1", "lq2", "lk2"):
                 out[name] = TensorSpec((spec.head_dim,), role="vector", std=0.1)
         if spec.qk_norm is not None:
-            out["q_norm"] = TensorSpec((q_out,), init="ones", role="vector")
-            out["k_norm"] = TensorSpec((kv_out,), init="ones", role="vector")
+            head = spec.qk_norm == "head"
+            out["q_norm"] = TensorSpec((spec.head_dim if head else q_out,), init="ones", role="vector")
+            out["k_norm"] = TensorSpec((spec.head_dim if head else kv_out,), init="ones", role="vector")
+        if spec.value_mix is not None:
+            out["vmix"] = TensorSpec((), role="vector", std=0.3)
+        if spec.talking:
+            out["talk"] = TensorSpec((spec.n_heads, spec.n_heads), init="eye", role="vector")
         if spec.head_gate:
             out["gate_proj.weight"] = TensorSpec((spec.n_heads, hidden))
         return out
@@ -232,8 +256,24 @@ class GQAttention(Mixer):
         ops = self.runtime.ops
         heads, key_heads = self.n_q * self.maps, self.n_kv * self.maps
         qkv = ops.linear(x, self.w_qkv, self.b_qkv)           # bias joins the float accumulator
-        self.position.encode_and_store(qkv, None, heads, key_heads, self.d, ctx, cache, value_dim=self.dv,
-                                       value_heads=self.n_kv, q_norm=self.q_norm, k_norm=self.k_norm, eps=self.eps)
+        if self.head_wise:
+            take = None
+            if self.value_mix == "take":
+                take = (ctx.shared["values"], self.share)
+            self.position.encode_heads(qkv, heads, key_heads, self.d, ctx, cache, self.dv, q_norm=self.q_norm,
+                                       k_norm=self.k_norm, norm_values=self.value_norm, take=take, eps=self.eps)
+            if self.value_mix == "give":                      # (the values as they were stored, where their rows hold them)
+                at = (heads + key_heads) * self.d
+                ctx.shared["values"] = qkv[:, at:at + self.n_kv * self.dv]
+        else:
+            self.position.encode_and_store(qkv, None, heads, key_heads, self.d, ctx, cache, value_dim=self.dv,
+                                           value_heads=self.n_kv, q_norm=self.q_norm, k_norm=self.k_norm, eps=self.eps)
+        if self.talk is not None:
+            mixed = torch.empty((x.shape[0], heads * self.dv), dtype=x.dtype, device=x.device)
+            ops.talking_attention(qkv, mixed, cache.k_pages, cache.v_pages, ctx.positions, ctx.entry_of_token,
+                                  ctx.block_tables[cache.group], heads, key_heads, self.d, self.dv, self.scale, self.talk,
+                                  max_position=ctx.max_position, batch=ctx)
+            return ops.linear(mixed, self.w_o)
         mixed = torch.empty((x.shape[0], heads * self.dv), dtype=x.dtype, device=x.device)
         ops.paged_attention(qkv, mixed, cache.k_pages, cache.v_pages, ctx.positions, ctx.entry_of_token,
                             ctx.block_tables[cache.group], heads, key_heads, self.d, self.window, self.scale,

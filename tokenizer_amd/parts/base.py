@@ -108,7 +108,7 @@ class Part:
 class NormFold:
     """A norm in the form the fused products take into their prologue: y = x / sqrt(mean(x^2) + eps) * weight,
     with `weight` float32 [H] on the device.  A norm of that form says so through `Norm.fold()`, whatever its
-    class and however it derives the weight from its tensors."""
+    class and however it derives the weight from its tensors.  (A norm over groups of coordinates is not of that form.)"""
     weight: torch.Tensor
     eps: float
 
@@ -200,17 +200,26 @@ class NormedDelta:
     stands (a block's per-layer token input): an object with `fused(residual, delta, weight, eps, out, rows)`, which
     does the add, its own addition and the next norm in one kernel or returns None, and `settle(residual, delta)`,
     which adds this term to the stream, works its own addition out step by step and returns it as a `NormedDelta`
-    without a `side`."""
+    without a `side`.
 
-    def __init__(self, ops, rows: torch.Tensor, weight: torch.Tensor, eps: float, side=None):
-        self.ops, self.rows, self.weight, self.eps, self.side = ops, rows, weight, float(eps), side
+    `groups`: the rows' coordinates form so many equal runs of neighbours, each brought to unit RMS on its own."""
+
+    def __init__(self, ops, rows: torch.Tensor, weight: torch.Tensor, eps: float, side=None, groups: int = 1):
+        self.ops, self.rows, self.weight, self.eps, self.side, self.groups = ops, rows, weight, float(eps), side, int(groups)
+
+    def join(self, residual: torch.Tensor, weight, eps: float, out: torch.Tensor, rows=None, store_residual: bool = True,
+             groups: int = 1) -> torch.Tensor:
+        """The stream with this term added (stored back unless told not to), normalised by `weight` over `groups` groups
+        (as it is where `weight` is None) into `out`."""
+        more = {} if self.groups == 1 and groups == 1 else {"post_groups": self.groups, "groups": groups}
+        return self.ops.norm_add_rmsnorm(residual, self.rows, self.weight, self.eps, weight, eps, out, rows,
+                                         store_residual=store_residual, **more)
 
     def resolve(self) -> torch.Tensor:
         if self.side is not None:
             raise ValueError("a term with an addition behind it that reads the stream cannot stand alone: hand it to a norm")
         zero = torch.zeros((self.rows.shape[0], self.rows.shape[1]), dtype=torch.float32, device=self.rows.device)
-        out = torch.empty_like(zero)
-        return self.ops.norm_add_rmsnorm(zero, self.rows, self.weight, self.eps, None, 0.0, out, store_residual=False)
+        return self.join(zero, None, 0.0, torch.empty_like(zero), store_residual=False)
 
 
 class SumDelta:

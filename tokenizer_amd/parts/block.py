@@ -209,3 +209,60 @@ class _TokenInput:
         gated = torch.empty_like(gate)
         ops.side_gate(gate, block.side_table, self.token_ids, block.side_offset, block.side_dim, gated)
         return NormedDelta(ops, ops.linear(gated, block.side_proj), block.side_norm, block.eps)
+
+
+@BLOCKS.register("post_norm")
+class PostNormBlock(Block):
+    """x + s1 * norm1(mixer(x)), then + s2 * norm2(feed_forward(.)): every sub-layer reads the stream itself (in the
+    compute dtype) and is normalised behind; (option `layer_scale`) a learned scale per coordinate on each normalised
+    output (the block's own tensors `ls1`, `ls2` [width]).  The layer's two norms are the ones behind the sub-layers, RMS
+    norms with a weight, over groups of coordinates or the whole row.
+
+    The stream is float32.  A sub-layer's output is handed on as a `NormedDelta` whose weight is norm times scale: one
+    kernel brings it to unit RMS, weighs it, adds it to the stream and leaves the sum in the compute dtype for the next
+    sub-layer (or normalised, behind the last layer)."""
+    graph_safe = True
+
+    @staticmethod
+    def tensor_specs(layer) -> dict:
+        width, out = int(layer.options["width"]), {}
+        if layer.options.get("layer_scale"):
+            if layer.mixer is not None:
+                out["ls1"] = TensorSpec((width,), init="ones", role="vector")
+            if layer.feed_forward is not None:
+                out["ls2"] = TensorSpec((width,), init="ones", role="vector")
+        return out
+
+    def __init__(self, mixer_norm, mixer, feed_forward_norm, feed_forward, layer, tensors, runtime):
+        self.mixer_norm, self.mixer = mixer_norm, mixer
+        self.feed_forward_norm, self.feed_forward = feed_forward_norm, feed_forward
+        self.runtime = runtime
+
+        def weight_of(norm, name):
+            if norm is None:
+                return None
+            weight = norm.weight.to(torch.float32)
+            return (weight * tensors[name].to(torch.float32) if layer.options.get("layer_scale") else weight).contiguous()
+        self.after_mixer = weight_of(mixer_norm, "ls1")
+        self.after_feed_forward = weight_of(feed_forward_norm, "ls2")
+
+    def _input(self, residual, delta):
+        """The stream with what is still to be added to it (stored back), in the compute dtype."""
+        ops = self.runtime.ops
+        out = torch.empty(residual.shape, dtype=self.runtime.dtype, device=residual.device)
+        if isinstance(delta, NormedDelta):
+            if delta.side is not None:
+                delta = delta.side.settle(residual, delta)
+            return delta.join(residual, None, 0.0, out)
+        return ops.norm_add_rmsnorm(residual, None if delta is None else as_tensor(delta), None, 0.0, None, 0.0, out)
+
+    def forward(self, residual, delta, ctx, cache):
+        ops = self.runtime.ops
+        for part, norm, weight in ((self.mixer, self.mixer_norm, self.after_mixer),
+                                   (self.feed_forward, self.feed_forward_norm, self.after_feed_forward)):
+            if part is None:
+                continue
+            x = self._input(residual, delta)
+            out = part.forward(x, ctx, cache) if part is self.mixer else part.forward(x, ctx)
+            delta = NormedDelta(ops, out, weight, norm.eps, groups=norm.groups)
+        return delta

@@ -19,10 +19,11 @@ class GatedDense(FeedForward):
 
 
     def __init__(self, spec: FeedForwardSpec, tensors: dict[str, torch.Tensor], runtime: Runtime):
-        if spec.activation not in ("silu", "capped_swish", "gelu_tanh"):
-            raise ValueError(f"gated_dense knows the activations silu, gelu_tanh and capped_swish, not {spec.activation!r}")
+        if spec.activation not in ("silu", "capped_swish", "gelu_tanh", "relu"):
+            raise ValueError(f"gated_dense knows the activations silu, gelu_tanh, relu and capped_swish, not {spec.activation!r}")
         self.spec, self.runtime = spec, runtime
-        self.gelu = spec.activation == "gelu_tanh"     # 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))) in place of silu
+        # In place of silu: "gelu_tanh", 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))), or "relu", max(g, 0).
+        self.named = spec.activation if spec.activation in ("gelu_tanh", "relu") else None
         # capped_swish: g' = min(g, limit), u' = clamp(u, -limit, limit); g' * sigmoid(alpha g') * (u' + shift).
         # (silu is alpha 1, no limit, shift 0, and keeps the kernels written for it.)
         self.act = None
@@ -49,7 +50,7 @@ class GatedDense(FeedForward):
                 "down_proj.weight": TensorSpec((spec.hidden_size, spec.intermediate_size))}
 
     def repeatable(self):
-        if self.gelu:
+        if self.named:
             return None
         return Repeatable(("gated_dense", self.act), (self.w_gate_up, self.w_down))
 
@@ -58,7 +59,7 @@ class GatedDense(FeedForward):
         down product added straight into the residual stream."""
         ops = self.runtime.ops
         fold = norm.fold() if delta is None else None      # the norm says whether it has the form the kernel computes
-        if fold is None or self.act is not None or self.gelu or not _can_fuse(ops, residual, self.runtime.dtype):
+        if fold is None or self.act is not None or self.named or not _can_fuse(ops, residual, self.runtime.dtype):
             # The output is handed on as a delta: a down product whose K is cut over workgroups may stay in
             # parts, and the norm that takes it next adds them in its own kernel.
             return self._run(norm.apply(residual, delta), pending=getattr(ops, "takes_pending", False))
@@ -74,8 +75,8 @@ class GatedDense(FeedForward):
 
     def _run(self, x, pending: bool):
         ops = self.runtime.ops
-        if self.gelu:
-            act = ops.linear_silu_gate(x, self.w_gate_up, act="gelu_tanh")
+        if self.named:
+            act = ops.linear_silu_gate(x, self.w_gate_up, act=self.named)
         elif self.act is None:
             act = ops.linear_silu_gate(x, self.w_gate_up)
         elif _can_fuse(ops, x, self.runtime.dtype) and x.shape[1] % 8 == 0:

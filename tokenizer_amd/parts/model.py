@@ -267,6 +267,8 @@ class DecoderModel:
     def forward(self, ctx, layer_caches: list[LayerCache]) -> torch.Tensor:
         """Run the tokens of `ctx` through the schedule; float32 logits [len(want_rows), vocab]."""
         ops = self.runtime.ops
+        if getattr(ctx, "shared", None):
+            ctx.shared.clear()                     # what the last forward's layers left for each other
         residual = self.embed(ctx)
         delta = None
         both = None

@@ -96,10 +96,30 @@ def scaled_rates(theta: float, dims: int, scaling: dict | None) -> torch.Tensor:
     return torch.tensor(rates, dtype=torch.float64).to(torch.float32)
 
 
+def yarn_rates(theta: float, dims: int, scaling: dict) -> tuple[torch.Tensor, float]:
+    """(float32 [dims / 2] rates, the factor on every cosine and sine) of a rotation stretched to longer contexts
+    (`scaling`: factor, original, fast, slow; Peng et al., "YaRN: Efficient Context Window Extension of Large Language
+    Models").  The pair that turns n times in `original` positions has the index at(n) = dims ln(original / (2 pi n)) /
+    (2 ln theta); from lo = max(floor(at(fast)), 0) to hi = min(ceil(at(slow)), dims - 1) the rate goes over from f_i to
+    f_i / factor linearly in i; the amplitude is 0.1 ln(factor) + 1.  Worked out in float64."""
+    factor, original, fast, slow = (float(scaling[key]) for key in ("factor", "original", "fast", "slow"))
+
+    def at(turns: float) -> float:
+        return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(float(theta)))
+
+    lo, hi = max(math.floor(at(fast)), 0), min(math.ceil(at(slow)), dims - 1)
+    rates = []
+    for i in range(dims // 2):
+        f = float(theta) ** (-2.0 * i / dims)
+        slowed = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+        rates.append(f / factor * slowed + f * (1.0 - slowed))
+    return torch.tensor(rates, dtype=torch.float64).to(torch.float32), 0.1 * math.log(factor) + 1.0
+
+
 @POSITIONS.register("rope_partial")
 class RotaryPartial(PositionEncoding):
     """Rotation of the first `dims` coordinates of every query and key head (options `dims`, even and at most the
-    head size; `scaling`, see `scaled_rates`): coordinate i < dims / 2 is paired with coordinate i + dims / 2 and the
+    head size; `scaling`, see `scaled_rates` and, where it names `fast` and `slow`, `yarn_rates`): coordinate i < dims / 2 is paired with coordinate i + dims / 2 and the
     pair turns by the angle position * f_i; the coordinates from `dims` on pass unchanged.  There is no table of
     positions: the kernel forms the angle in float32 from the position and the rate and takes its accurate sine and
     cosine, so positions are bounded by nothing here.  Keys are stored after the rotation.
@@ -113,12 +133,43 @@ class RotaryPartial(PositionEncoding):
         self.dims = int(spec.options.get("dims", spec.head_dim))
         if self.dims % 2 or not 0 <= self.dims <= spec.head_dim:
             raise ValueError(f"a rotation over {self.dims} of {spec.head_dim} coordinates")
-        self.rates = scaled_rates(spec.theta, self.dims, spec.options.get("scaling")).to(runtime.device).contiguous()
+        scaling, self.magnitude = spec.options.get("scaling") or {}, 1.0     # (the factor on cosines and sines)
+        if "fast" in scaling and self.dims:
+            rates, self.magnitude = yarn_rates(spec.theta, self.dims, scaling)
+        else:
+            rates = scaled_rates(spec.theta, self.dims, scaling or None)
+        self.rates = rates.to(runtime.device).contiguous()
+        self.name = ("rotation", self.dims, float(spec.theta), tuple(sorted(scaling.items())))
+
+    def angles(self, ctx) -> torch.Tensor | None:
+        """float32 [tokens, dims]: the cosines, then the sines, of this step's positions times the rates (times the
+        magnitude), made once a step for all layers that rotate alike; None where nothing turns."""
+        if not self.dims:
+            return None
+        table = ctx.shared.get(self.name)
+        if table is None:
+            table = torch.empty((ctx.positions.numel(), self.dims), dtype=torch.float32, device=self.rates.device)
+            ctx.shared[self.name] = self.runtime.ops.rotation_table(ctx.positions, self.rates, self.magnitude, table)
+        return table
+
+    def encode_heads(self, qkv, n_q, n_kv, head_dim, ctx, cache, value_dim, q_norm=None, k_norm=None, norm_values=False,
+                     take=None, eps=0.0):
+        """As `encode_and_store` for rows without a bias, with norms of every head on its own before the rotation (weights
+        `q_norm`, `k_norm` [head_dim] for all heads) and, for value heads, `norm_values` (unit RMS, no weight) and then
+        `take` = (rows, share): v becomes (1 - share) v + share * rows."""
+        slots = ctx.slots[cache.group] if cache.writes else None
+        rows, share = take if take is not None else (None, None)
+        self.runtime.ops.head_norm_rotate_store(qkv, self.angles(ctx), self.dims, slots,
+                                                cache.k_pages if slots is not None else None,
+                                                cache.v_pages if slots is not None else None, n_q, n_kv, n_kv, head_dim,
+                                                value_dim, q_norm, k_norm, norm_values, rows, share, eps)
 
     def encode_and_store(self, qkv, bias, n_q, n_kv, head_dim, ctx, cache, value_dim=None, value_heads=None,
                          q_norm=None, k_norm=None, eps=0.0):
         """Rows of `qkv`: n_q query heads and n_kv key heads of `head_dim`, then `value_heads` (n_kv if None) value
         heads of `value_dim`; whatever lies behind them in a row is left alone."""
+        if self.magnitude != 1.0:
+            raise ValueError("a rotation with a magnitude is applied head by head (`encode_heads`)")
         slots = ctx.slots[cache.group] if cache.writes and n_kv else None
         self.runtime.ops.norm_rotate_store(qkv, bias, ctx.positions, self.rates, self.dims, slots,
                                            cache.k_pages if slots is not None else None,

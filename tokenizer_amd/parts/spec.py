@@ -118,7 +118,13 @@ class MixerSpec:
     keep_first: int = 0           # with a window: keys at positions below this stay visible to every later query
     differential: float | None = None   # c: two score maps per head over the same values, o = a1 - lambda a2 with
     #                               lambda = exp(lq1.lk1) - exp(lq2.lk2) + c, o brought to unit RMS per head, times 1 - c
-    qk_norm: str | None = None    # "whole": RMS norm with a weight over all query rows at once (and all key rows), before rotation
+    qk_norm: str | None = None    # before rotation: "whole": RMS norm with a weight over all query rows at once (and all
+    #                               key rows); "head": over each head's coordinates, one weight [head_dim] for all heads
+    value_norm: bool = False      # each value head is brought to unit RMS (no weight) before it is cached
+    value_mix: str | None = None  # "give": later layers of the model may take in this layer's values; "take": the values
+    #                               become (1 - s) v + s v' with v' the giving layer's values of the same token, s learned
+    talking: bool = False         # the heads' softmax weights are mixed with each other by a learned [heads, heads] matrix
+    decays: tuple[float, ...] = ()   # retention: each head's decay of its state from token to token
     head_gate: bool = False       # each head's output times sigmoid of one number projected from the mixer's input
     q_rank: int = 0               # latent attention: width of the normalised latent the queries are projected up from
     kv_rank: int = 0              # latent attention: width of the normalised latent that keys and values are projected
@@ -140,7 +146,7 @@ class FeedForwardSpec:
     kind: str                     # "gated_dense", ...
     hidden_size: int
     intermediate_size: int = 0
-    activation: str = "silu"      # "silu", "gelu_tanh", or "capped_swish" with the three numbers below
+    activation: str = "silu"      # "silu", "gelu_tanh", "relu", or "capped_swish" with the three numbers below
     act_alpha: float = 1.0        # g * sigmoid(alpha g)
     act_limit: float | None = None  # g is cut at +limit, the other branch at +-limit
     act_up_shift: float = 0.0     # added to the other branch before the product
