@@ -18,7 +18,7 @@ share a prefix of 1,024 ids, with the prefix cache) and prints one JSON line for
 
 times the prompt attention kernel alone on a portion of TOKENS tokens after C cached ones.
 
-    python bench.py --design napadra|dolidra|bokulorn|zomavik [--size 0.5b|1.5b|7b] [--layers N] [--batch B] [--steps K]
+    python bench.py --design napadra|dolidra|bokulorn|zomavik|gafonex [--size 0.5b|1.5b|7b] [--layers N] [--batch B] [--steps K]
 
 times a prefill of 2,048 tokens and decoding at batch B of a Napadra model whose layers have the sizes of the
 Qwen2.5 model named (width, heads, feed-forward and vocabulary; its layers alternate attention, attention on the
@@ -362,19 +362,41 @@ def zomavik_config(sizes: dict, layers: int, experts: int = 8, top: int = 2) -> 
             "embedding": {"scale": 1.0}, "logit_scale": 1.0, "logit_softcap": 30.0, "loop": loop, "layers": out}
 
 
+def gafonex_config(sizes: dict, layers: int) -> dict:
+    """A Gafonex configuration with the layer sizes of a Qwen2 one: every fourth layer (the third, the seventh, ...) is an
+    attention with Qwen2's heads (values as wide as keys, the whole head rotated with slowed long waves, values taken in
+    from the first), the others a retention with as many heads of the same size; every layer has a dense feed-forward of
+    Qwen2's inner width; norms over two groups."""
+    width, heads, kv_heads = sizes["hidden_size"], sizes["num_attention_heads"], sizes["num_key_value_heads"]
+    d, base = width // heads, float(sizes.get("rope_theta", 1e6))
+    mlp = {"kind": "dense", "ff": sizes["intermediate_size"]}
+    attention = {"heads": heads, "kv_heads": kv_heads, "dim": d, "vdim": d, "scale": d ** -0.5, "v_mix": True,
+                 "rot": {"dims": d, "base": base, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    retention = {"heads": heads, "dim": d, "vdim": d, "decay": [1.0 - 2.0 ** (-5.0 - h % 8) for h in range(heads)],
+                 "rot": {"dims": d, "base": base}}
+    out = [{"type": "attention", "mixer": attention, "mlp": mlp} if index % 4 == 2 else
+           {"type": "retention", "mixer": retention, "mlp": mlp} for index in range(layers)]
+    return {"architecture": "Gafonex", "vocab": sizes["vocab_size"], "width": width, "norm": {"eps": 1e-6, "groups": 2},
+            "logit_softcap": 30.0, "layers": out}
+
+
 def run_design(args, sizes: dict) -> dict:
-    """Prefill and decode throughput of the named design beside its closest neighbour (Qwen2; for Zomavik, Bokulorn, whose layers also set a recurrence with
+    """Prefill and decode throughput of the named design beside its closest neighbour (Qwen2; for Gafonex, Napadra, whose layers
+    mix attention with a recurrence over a matrix of state a head; for Zomavik, Bokulorn, whose layers also set a recurrence with
     its state in the request's slot beside attention and routed experts; for Bokulorn, Dolidra, whose
     layers also mix attention with routed experts) at equal layer sizes and number of layer runs."""
     import torch
-    from tokenizer_amd.config import BokulornConfig, DolidraConfig, NapadraConfig, Qwen2Config, ZomavikConfig
+    from tokenizer_amd.config import BokulornConfig, DolidraConfig, GafonexConfig, NapadraConfig, Qwen2Config, ZomavikConfig
     from tokenizer_amd.engine import random_model
     layers = args.layers or 8
     steps = min(args.steps, 256)
-    beside = {"bokulorn": "dolidra", "zomavik": "bokulorn"}.get(args.design, "qwen2")
+    beside = {"bokulorn": "dolidra", "zomavik": "bokulorn", "gafonex": "napadra"}.get(args.design, "qwen2")
     record = {"design": args.design, "beside": beside, "size": args.size, "layers": layers, "dtype": args.dtype,
               "prompt_len": PROMPT_LEN, "batch": args.batch, "decode_steps": steps, "data": "synthetic (random weights)"}
-    if args.design == "zomavik":
+    if args.design == "gafonex":
+        configs = {"gafonex": lambda: GafonexConfig.from_dict(gafonex_config(sizes, layers)),
+                   "napadra": lambda: NapadraConfig.from_dict(napadra_config(sizes, layers))}
+    elif args.design == "zomavik":
         # (Two of Zomavik's layers run twice: `layers` counts the runs, so that both models run as many layers a token.)
         configs = {"zomavik": lambda: ZomavikConfig.from_dict(zomavik_config(sizes, max(2, layers - 2))),
                    "bokulorn": lambda: BokulornConfig.from_dict(bokulorn_config(sizes, layers))}
@@ -499,9 +521,9 @@ def main() -> int:
     parser.add_argument("--layers", type=int, default=None)
     parser.add_argument("--size", default="0.5b", choices=["0.5b", "1.5b", "7b"],
                         help="layer sizes of the decode benchmark (the default is the one the record is for)")
-    parser.add_argument("--design", default=None, choices=["napadra", "dolidra", "bokulorn", "zomavik"],
+    parser.add_argument("--design", default=None, choices=["napadra", "dolidra", "bokulorn", "zomavik", "gafonex"],
                         help="time this design beside its closest neighbour at equal layer sizes (prefill and decode)")
-    parser.add_argument("--only", default=None, choices=["napadra", "dolidra", "bokulorn", "zomavik", "qwen2"], help="with --design: one of the two models")
+    parser.add_argument("--only", default=None, choices=["napadra", "dolidra", "bokulorn", "zomavik", "gafonex", "qwen2"], help="with --design: one of the two models")
     parser.add_argument("--peaks", action="store_true", help="measure what the device reaches in HBM reads and bf16 products")
     parser.add_argument("--workload", default=None, choices=["mixed-1.5b", "mixed-0.5b", "prefix-7b"],
                         help="run a serving workload through the scheduler instead of the decode benchmark")

@@ -133,3 +133,587 @@ extern "C" int ta_talking_attention_generic(const void* q, int q_stride, void* o
 #undef GO
   return LAUNCH_STATUS();
 }
+
+// ---------------------------------------------------------------------------------------------------------------
+// The matrix-core form for bfloat16.  The mix commutes with the product with the values: with
+// A_g = sum_j p_g(j) V(j) over the values of ALL kv heads side by side (W = n_kv dv numbers), head h's output is
+// sum_g talk[h, g] times A_g's part at h's own kv head.  So every head is an ordinary softmax over its own keys against
+// values W wide, in one walk over the keys, and the mix is a small product at the end (`talking_finish_kernel`), in float.
+// The value pages hold exactly these wide values: a page's [n_kv, dv, page_size] read as [W, page_size].
+// Both kernels leave, per (token, part of its keys, head), the unnormalised sums [W] with the maximum and the sum of
+// exponentials they stand under: part_o float [items, parts, n_q, W], part_ml float [items, parts, n_q, 2].
+
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef float floatx4 __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ bf16x8 tk_zero8() {
+  bf16x8 z;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) z[i] = (__bf16)0.0f;
+  return z;
+}
+
+// Single tokens.  A workgroup a (part of the keys, token), all heads and all value columns: first the scores of every
+// head over the part (a wave a kv head's block of 32 keys at a time, up to sixteen heads the N side of the instruction)
+// into LDS, then maximum, exponentials and sum head by head, then O^T = V^T P^T, a wave sixteen of the W value rows at
+// a time for all heads.  The values of a wave's next rows are asked for while it works on the current ones, the first
+// before the scores.  HB: blocks of sixteen heads.  d a multiple of 8 up to 256; split_keys a multiple of 32 up to 256.
+// Dynamic LDS: 16 HB rows of (split_keys + 4) floats, then 16 HB rows of (split_keys + 8) bfloat16.
+#define TKD_BLOCKS 8
+template <int NW, int HB>
+__global__ void __launch_bounds__(NW * WAVE)
+talking_decode_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ k_pages,
+                      const bf16_t* __restrict__ vt_pages, const int* __restrict__ rows, const int* __restrict__ positions,
+                      const int* __restrict__ entry_of_token, const int* __restrict__ block_table, int table_stride,
+                      float* __restrict__ part_o, float* __restrict__ part_ml, int n_q, int n_kv, int d, int wide,
+                      int page_size, float scale, int split_keys, int splits) {
+  HELD(q, q_stride, k_pages, vt_pages, rows, positions, entry_of_token, block_table, table_stride, part_o, part_ml, n_q,
+       n_kv, d, wide, page_size, scale, split_keys, splits);
+  extern __shared__ __attribute__((aligned(16))) char tkd_lds[];
+  const int s_ld = split_keys + 4, p_ld = split_keys + 8;
+  float* s_s = reinterpret_cast<float*>(tkd_lds);
+  bf16_t* p_s = reinterpret_cast<bf16_t*>(tkd_lds + sizeof(float) * 16 * HB * s_ld);
+  const int split = blockIdx.x, item = blockIdx.y;
+  const int t = rows ? scalar_int(rows + item) : item;
+  if (t < 0) return;                                       // a row that only fills the list up
+  const int lane = threadIdx.x & 63, wave = wave_index(), col = lane & 15, g = lane >> 4;
+  const int* table = block_table + (size_t)(entry_of_token ? scalar_int(entry_of_token + t) : t) * table_stride;
+  const int pos = scalar_int(positions + t), first = split * split_keys, last = min(pos, first + split_keys - 1);
+  const size_t part = (size_t)item * splits + split;
+  if (first > pos) {                                       // no key of the token lies here
+    for (int h = threadIdx.x; h < n_q; h += NW * WAVE) {
+      part_ml[(part * n_q + h) * 2] = -INFINITY;
+      part_ml[(part * n_q + h) * 2 + 1] = 0.f;
+    }
+    return;
+  }
+  const int blocks = (last - first) / 32 + 1, group = n_q / n_kv, head_blocks = (group + 15) / 16;
+  union VFrag { uint4 bits; bf16x8 v; };
+  // Rows rb * 16 .. + 15 of the wide values over the part's keys: lane (col, g) has row col, keys 8 g .. 8 g + 7 of a block.
+  auto load_values = [&](VFrag (&vf)[TKD_BLOCKS], int rb) {
+    const int row = min(rb * 16 + col, wide - 1);          // (a row past the last repeats it and is not written)
+#pragma unroll
+    for (int b = 0; b < TKD_BLOCKS; ++b) {
+      vf[b].bits = make_uint4(0, 0, 0, 0);
+      if (b >= blocks) continue;
+      const int kb = first + 32 * b;
+      const bool there1 = kb + 16 <= last;                 // (a half without keys borrows the other's page; its values are zeroed)
+      const int page0 = scalar_int(table + kb / page_size), page1 = scalar_int(table + (there1 ? kb + 16 : kb) / page_size);
+      const uint32_t at = ((uint32_t)((g >> 1) ? page1 : page0) * wide + row) * page_size + (kb + 16 * (g >> 1)) % page_size + 8 * (g & 1);
+      vf[b].bits = *reinterpret_cast<const uint4*>(vt_pages + at);
+    }
+  };
+  const int row_blocks = (wide + 15) / 16;
+  VFrag vf[TKD_BLOCKS], vn[TKD_BLOCKS];
+  if (wave < row_blocks) load_values(vf, wave);
+  // Scores.
+  for (int unit = wave; unit < n_kv * blocks; unit += NW) {
+    const int kvh = unit % n_kv, kb = first + 32 * (unit / n_kv);
+    const bool there1 = kb + 16 <= last;
+    const int page0 = scalar_int(table + kb / page_size), page1 = scalar_int(table + (there1 ? kb + 16 : kb) / page_size);
+    const bf16_t* k0 = k_pages + (((size_t)page0 * n_kv + kvh) * page_size + kb % page_size + col) * d + 8 * g;
+    const bf16_t* k1 = k_pages + (((size_t)page1 * n_kv + kvh) * page_size + (there1 ? kb + 16 : kb) % page_size + col) * d + 8 * g;
+    for (int hb = 0; hb < head_blocks; ++hb) {
+      const int head = kvh * group + hb * 16 + col;
+      const bool has = hb * 16 + col < group;
+      const bf16_t* qr = q + (size_t)t * q_stride + (size_t)(has ? head : 0) * d + 8 * g;
+      floatx4 st[2] = {(floatx4){0.f, 0.f, 0.f, 0.f}, (floatx4){0.f, 0.f, 0.f, 0.f}};
+      for (int ks0 = 0; ks0 * 32 < d; ks0 += 4) {
+        bf16x8 kf0[4], kf1[4], qf[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int at = (ks0 + i) * 32;
+          const bool in = at + 8 * g < d;
+          kf0[i] = kf1[i] = qf[i] = tk_zero8();
+          if (in) {
+            kf0[i] = *reinterpret_cast<const bf16x8*>(k0 + at);
+            kf1[i] = *reinterpret_cast<const bf16x8*>(k1 + at);
+          }
+          if (in && has) qf[i] = *reinterpret_cast<const bf16x8*>(qr + at);
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          st[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf0[i], qf[i], st[0], 0, 0, 0);
+          st[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf1[i], qf[i], st[1], 0, 0, 0);
+        }
+      }
+      if (has) {
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+          const int key = kb + 16 * u + 4 * g;
+          float4 s;
+          s.x = key <= last ? st[u][0] * scale : -INFINITY;
+          s.y = key + 1 <= last ? st[u][1] * scale : -INFINITY;
+          s.z = key + 2 <= last ? st[u][2] * scale : -INFINITY;
+          s.w = key + 3 <= last ? st[u][3] * scale : -INFINITY;
+          *reinterpret_cast<float4*>(s_s + (size_t)head * s_ld + key - first) = s;
+        }
+      }
+    }
+  }
+  __syncthreads();
+  // Maximum, exponentials and sum: a wave a head.  (Key 0 of the part is seen, so every maximum is a number.)
+  for (int h = wave; h < 16 * HB; h += NW) {
+    float s[TKD_BLOCKS / 2], m = -INFINITY, l = 0.f;
+#pragma unroll
+    for (int i = 0; i < TKD_BLOCKS / 2; ++i) {
+      const int j = lane + 64 * i;
+      s[i] = (h < n_q && j < 32 * blocks) ? s_s[(size_t)h * s_ld + j] : -INFINITY;
+      m = fmaxf(m, s[i]);
+    }
+    m = wave_max(m);
+#pragma unroll
+    for (int i = 0; i < TKD_BLOCKS / 2; ++i) {
+      const int j = lane + 64 * i;
+      const float p = s[i] == -INFINITY ? 0.f : __expf(s[i] - m);
+      l += p;
+      if (j < 32 * blocks) st(p_s + (size_t)h * p_ld + j, p);
+    }
+    l = wave_sum(l);
+    if (lane == 0 && h < n_q) {
+      part_ml[(part * n_q + h) * 2] = m;
+      part_ml[(part * n_q + h) * 2 + 1] = l;
+    }
+  }
+  __syncthreads();
+  // The wide values.
+  for (int rb = wave; rb < row_blocks; rb += NW) {
+    const bool more = rb + NW < row_blocks;
+    if (more) load_values(vn, rb + NW);
+    floatx4 acc[HB];
+#pragma unroll
+    for (int hb = 0; hb < HB; ++hb) acc[hb] = (floatx4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int b = 0; b < TKD_BLOCKS; ++b) {
+      if (b >= blocks) continue;
+      const int left = last - (first + 32 * b + 8 * g);    // the lane's keys that exist: 0 .. left; slots nobody wrote may hold anything
+      if (left < 7) {
+        uint4 v = vf[b].bits;
+        if (left < 0) v.x = 0; else if (left < 1) v.x &= 0xffffu;
+        if (left < 2) v.y = 0; else if (left < 3) v.y &= 0xffffu;
+        if (left < 4) v.z = 0; else if (left < 5) v.z &= 0xffffu;
+        if (left < 6) v.w = 0; else v.w &= 0xffffu;
+        vf[b].bits = v;
+      }
+#pragma unroll
+      for (int hb = 0; hb < HB; ++hb) {
+        const bf16x8 pf = *reinterpret_cast<const bf16x8*>(p_s + (size_t)(hb * 16 + col) * p_ld + 32 * b + 8 * g);
+        acc[hb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[b].v, pf, acc[hb], 0, 0, 0);
+      }
+    }
+    const int row = rb * 16 + 4 * g;
+#pragma unroll
+    for (int hb = 0; hb < HB; ++hb) {
+      const int head = hb * 16 + col;
+      if (head >= n_q) continue;
+      float* dst = part_o + (part * n_q + head) * wide + row;
+      if (wide % 4 == 0) {
+        if (row < wide) *reinterpret_cast<float4*>(dst) = make_float4(acc[hb][0], acc[hb][1], acc[hb][2], acc[hb][3]);
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (row + r < wide) dst[r] = acc[hb][r];
+      }
+    }
+    if (more) {
+#pragma unroll
+      for (int b = 0; b < TKD_BLOCKS; ++b) vf[b].bits = vn[b].bits;
+    }
+  }
+}
+
+// Prompt portions.  A workgroup a (tile of sixteen tokens, kv head, block of 4 HG of its query heads, slab of 16 VB of the
+// W value columns, part of the tile's keys); its four waves have HG heads each and walk the same blocks of KB keys, which
+// come from the pages once for all of them straight into LDS, two buffers deep (the next block is on its way while the
+// current one is worked on).  S^T = K Q^T and O^T = V^T P^T with 16x16x32 instructions, token index in `lane % 16`;
+// softmax online in float; a row block of ones beside V^T gives the probabilities' sums.  A fragment of the values is
+// read from LDS once for the wave's HG heads.
+// Keys in LDS: rows of DP (d filled up to a power of two) elements; the sixteen bytes that hold elements 8 p .. 8 p + 7 of
+// key k stand at place p ^ turn(k), so that rows read at once lie in different banks; a piece past d repeats the row's
+// last one and meets a query of zeros.  Values: runs of sixteen keys, 16 VB rows of 32 bytes each.
+template <int DP, int VB>
+struct TalkBlock {
+  static constexpr int KB = DP + 16 * VB > 256 ? 32 : 64;
+  static constexpr int RUNS = KB / 16, SHARE = 4 / RUNS;     // runs of sixteen keys; waves that share a run's loads
+  static constexpr int PIECES = DP / 8, KEYS_A_LOAD = 64 / PIECES, K_LOADS = 16 / KEYS_A_LOAD, V_LOADS = VB / 2;
+  static constexpr int K_ROW = 2 * DP, K_BYTES = KB * K_ROW, V_RUN = 32 * 16 * VB, BYTES = K_BYTES + RUNS * V_RUN;
+  __device__ static constexpr int turn(int key) { return ((key & 3) | ((key >> 1) & 4)) & (PIECES - 1); }
+};
+
+struct Whole { static constexpr bool value = true; };    // every key of the block is seen by every token of the tile
+struct Edge { static constexpr bool value = false; };
+
+template <int DP, int VB, int HG>
+__global__ void __launch_bounds__(4 * WAVE, 2)
+talking_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ k_pages,
+                       const bf16_t* __restrict__ vt_pages, const int* __restrict__ tiles, int n_tiles,
+                       const int* __restrict__ cu_q, const int* __restrict__ first_position,
+                       const int* __restrict__ block_table, int table_stride, float* __restrict__ part_o,
+                       float* __restrict__ part_ml, int n_q, int n_kv, int d, int wide, int page_size, float scale,
+                       int slabs, int key_splits) {
+  typedef TalkBlock<DP, VB> B;
+  constexpr int KS = DP / 32, KB = B::KB, HALVES = KB / 32;
+  HELD(q, q_stride, k_pages, vt_pages, tiles, n_tiles, cu_q, first_position, block_table, table_stride, part_o, part_ml,
+       n_q, n_kv, d, wide, page_size, scale, slabs, key_splits);
+  extern __shared__ __attribute__((aligned(16))) char tkp_lds[];
+  const int lane = threadIdx.x & 63, wave = wave_index(), col = lane & 15, g = lane >> 4;
+  const int group = n_q / n_kv, head_blocks = (group + 4 * HG - 1) / (4 * HG);
+  // Late tiles first: they see the most keys.
+  int which = blockIdx.x;
+  const int split = which % key_splits; which /= key_splits;
+  const int slab = which % slabs; which /= slabs;
+  const int hb = which % head_blocks; which /= head_blocks;
+  const int kvh = which % n_kv; which /= n_kv;
+  const int tile_index = n_tiles - 1 - which;
+  const int first_head = hb * 4 * HG + wave * HG, heads_here = max(0, min(HG, group - first_head));
+  const int head0 = kvh * group + first_head;
+  const int entry = scalar_int(tiles + 2 * tile_index), offset = scalar_int(tiles + 2 * tile_index + 1);
+  const int entry_row = scalar_int(cu_q + entry), next_row = scalar_int(cu_q + entry + 1);
+  const int entry_position = scalar_int(first_position + entry);
+  HELD(entry_row, next_row, entry_position);
+  const int row0 = entry_row + offset, n_valid = min(16, next_row - row0);
+  if (n_valid <= 0) return;                                // a tile that only fills the list up
+  const int p0 = entry_position + offset, hi = p0 + n_valid - 1;
+  const int my_pos = p0 + min(col, n_valid - 1), my_row = row0 + min(col, n_valid - 1);
+  const int* table = block_table + (size_t)entry * table_stride;
+  // This workgroup's blocks: a run of whole turns of the walk.
+  const int turns = hi / KB + 1, each = (turns + key_splits - 1) / key_splits;
+  const int begin = split * each * KB, end = min(hi, begin + each * KB - 1);
+  bf16x8 qf[HG][KS];
+  floatx4 acc[HG][VB], l[HG];
+  float m[HG];
+#pragma unroll
+  for (int h = 0; h < HG; ++h) {
+    m[h] = -INFINITY;
+    l[h] = (floatx4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int db = 0; db < VB; ++db) acc[h][db] = (floatx4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const int d0 = ks * 32 + 8 * g;
+      qf[h][ks] = tk_zero8();
+      if (h < heads_here && d0 < d)
+        qf[h][ks] = *reinterpret_cast<const bf16x8*>(q + (size_t)my_row * q_stride + (size_t)(head0 + h) * d + d0);
+    }
+  }
+  // What a lane brings of a run: offsets worked out once.
+  const int run = wave % B::RUNS, share = wave / B::RUNS;
+  uint32_t k_from[B::K_LOADS], v_from[B::V_LOADS];
+#pragma unroll
+  for (int j = 0; j < B::K_LOADS; ++j) {
+    const int key = B::KEYS_A_LOAD * j + lane / B::PIECES, piece = (lane % B::PIECES) ^ B::turn(key);
+    k_from[j] = (uint32_t)(key * d + min(piece * 8, d - 8)) * 2;
+  }
+#pragma unroll
+  for (int j = 0; j < B::V_LOADS; ++j) {
+    const int row = min(slab * 16 * VB + 32 * j + (lane >> 1), wide - 1);
+    v_from[j] = (uint32_t)(row * page_size + (lane & 1) * 8) * 2;
+  }
+  const auto page_of = [&](int kb) {                       // (a run past the last key borrows the last key's page: its keys are masked)
+    return scalar_int(table + min(kb + 16 * run, hi) / page_size);
+  };
+  const auto fetch = [&](int kb, int page, char* buf) {
+    typedef const void __attribute__((address_space(1)))* from_t;
+    typedef void __attribute__((address_space(3)))* to_t;
+    const int slot = (kb + 16 * run) % page_size;
+    const char* k_run = reinterpret_cast<const char*>(k_pages + (((uint32_t)page * n_kv + kvh) * page_size + slot) * d);
+    const char* v_run = reinterpret_cast<const char*>(vt_pages + ((uint32_t)page * wide * page_size + slot));
+    char* k_to = buf + run * 16 * B::K_ROW;
+    char* v_to = buf + B::K_BYTES + run * B::V_RUN;
+#pragma unroll
+    for (int j = 0; j < B::K_LOADS; ++j)
+      if (B::SHARE == 1 || j % B::SHARE == share)
+        __builtin_amdgcn_global_load_lds((from_t)(k_run + k_from[j]), (to_t)(k_to + j * 1024), 16, 0, 0);
+#pragma unroll
+    for (int j = 0; j < B::V_LOADS; ++j)
+      if (B::SHARE == 1 || j % B::SHARE == share)
+        __builtin_amdgcn_global_load_lds((from_t)(v_run + v_from[j]), (to_t)(v_to + j * 1024), 16, 0, 0);
+  };
+  bf16x8 ones;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) ones[i] = (__bf16)1.0f;
+  const float c = scale * 1.4426950408889634f;
+  const int turned = B::turn((col & 3) | ((col >> 2) & 1) << 3);     // of the lane's keys: the same in every instruction
+  const auto block = [&](const char* buf, int kb, auto full) {
+    constexpr bool FULL = decltype(full)::value;
+    float s[HG][KB / 4];
+#pragma unroll
+    for (int t = 0; t < 2 * HALVES; ++t) {
+      // Row r of the instruction is key 8 (r / 4) + 4 (t % 2) + r % 4 of its half of 32, whose score then lies in the lane
+      // group that holds that key in the second product (lane group g: keys 8 g .. 8 g + 7).
+      const int key = 32 * (t >> 1) + 8 * (col >> 2) + 4 * (t & 1) + (col & 3);
+      bf16x8 kf[KS];
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks)
+        kf[ks] = *reinterpret_cast<const bf16x8*>(buf + key * B::K_ROW + ((ks * 4 + g) ^ turned) * 16);
+#pragma unroll
+      for (int h = 0; h < HG; ++h) {
+        floatx4 st = (floatx4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) st = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks], qf[h][ks], st, 0, 0, 0);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int at = kb + 32 * (t >> 1) + 8 * g + 4 * (t & 1) + r;
+          s[h][t * 4 + r] = FULL || at <= my_pos ? st[r] : -INFINITY;
+        }
+      }
+    }
+    bf16x8 pf[HG][HALVES];
+#pragma unroll
+    for (int h = 0; h < HG; ++h) {
+      float mx = s[h][0];
+#pragma unroll
+      for (int i = 1; i < KB / 4; ++i) mx = __builtin_elementwise_maximum(mx, s[h][i]);
+      mx = __builtin_elementwise_maximum(mx, __shfl_xor(mx, 16, WAVE));
+      mx = __builtin_elementwise_maximum(mx, __shfl_xor(mx, 32, WAVE));
+      const float m_new = __builtin_elementwise_maximum(m[h], mx);
+      const float mc = (m_new == -INFINITY) ? 0.f : m_new * c;         // (no key seen yet: exp2 of inf - inf would be NaN)
+      if (__any(m_new > m[h])) {                            // rescale only when some token's maximum moved
+        const float corr = __builtin_amdgcn_exp2f(m[h] * c - mc);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) l[h][r] *= corr;
+#pragma unroll
+        for (int db = 0; db < VB; ++db)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) acc[h][db][r] *= corr;
+        m[h] = m_new;
+      }
+#pragma unroll
+      for (int i = 0; i < KB / 4; ++i)
+        pf[h][i >> 3][i & 7] = (__bf16)__builtin_amdgcn_exp2f(fmaf(s[h][i], c, -mc));
+    }
+#pragma unroll
+    for (int u = 0; u < HALVES; ++u) {
+#pragma unroll
+      for (int h = 0; h < HG; ++h) l[h] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf[h][u], l[h], 0, 0, 0);
+#pragma unroll
+      for (int db = 0; db < VB; ++db) {
+        bf16x8 vf = *reinterpret_cast<const bf16x8*>(buf + B::K_BYTES + (2 * u + (g >> 1)) * B::V_RUN + (db * 16 + col) * 32 + (g & 1) * 16);
+        if (!FULL) {                                        // slots nobody wrote may hold anything: 0 * NaN must stay 0
+#pragma unroll
+          for (int i = 0; i < 8; ++i)
+            if (kb + 32 * u + 8 * g + i > hi) vf[i] = (__bf16)0.0f;
+        }
+#pragma unroll
+        for (int h = 0; h < HG; ++h) acc[h][db] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[h][u], acc[h][db], 0, 0, 0);
+      }
+    }
+  };
+  // Turn by turn: ask for the next block into the buffer that the turn before read, work on the current one, wait for
+  // what was asked for, meet.  The page of the block after the next is looked up meanwhile.
+  int cur = 0, kb = begin;
+  if (kb <= end) fetch(kb, page_of(kb), tkp_lds);
+  int next_page = page_of(kb + KB);
+  __builtin_amdgcn_s_waitcnt(0x0F70);                       // all that this wave fetched has arrived (vmcnt 0)
+  __syncthreads();
+#define TALK_TURN(KIND)                                                              \
+  {                                                                                  \
+    if (kb + KB <= end) fetch(kb + KB, next_page, tkp_lds + (cur ^ 1) * B::BYTES);   \
+    next_page = page_of(kb + 2 * KB);                                                \
+    if (heads_here > 0) block(tkp_lds + cur * B::BYTES, kb, KIND{});                 \
+    __builtin_amdgcn_s_waitcnt(0x0F70);                                              \
+    __syncthreads();                                                                 \
+    cur ^= 1;                                                                        \
+  }
+  for (; kb <= end && kb + KB - 1 <= p0; kb += KB) TALK_TURN(Whole)
+  for (; kb <= end; kb += KB) TALK_TURN(Edge)
+#undef TALK_TURN
+  if (col >= n_valid) return;
+#pragma unroll
+  for (int h = 0; h < HG; ++h) {
+    if (h >= heads_here) break;
+    const size_t at = (((size_t)tile_index * 16 + col) * key_splits + split) * n_q + head0 + h;
+    if (slab == 0 && g == 0) {
+      part_ml[at * 2] = m[h] * scale;                       // in units of the scaled scores
+      part_ml[at * 2 + 1] = l[h][0];
+    }
+#pragma unroll
+    for (int db = 0; db < VB; ++db) {
+      const int row = slab * 16 * VB + db * 16 + 4 * g;
+      float* dst = part_o + at * wide + row;
+      if (wide % 4 == 0) {
+        if (row < wide) *reinterpret_cast<float4*>(dst) = make_float4(acc[h][db][0], acc[h][db][1], acc[h][db][2], acc[h][db][3]);
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (row + r < wide) dst[r] = acc[h][db][r];
+      }
+    }
+  }
+}
+
+// The parts of every head brought together and the heads mixed: a workgroup a (item, kv head, 64 value columns).  Wave w
+// makes A_g for g = w, w + NW, ... (a lane a column; parts under their common maximum, over the common sum) into LDS,
+// then head h = w, w + NW, ... of the kv head's group, sum_g talk[h, g] A_g.  Items are rows (`rows`, or themselves), or,
+// with `tiles`, (tile, token of the tile).  Dynamic LDS: n_q rows of 64 floats.
+template <int NW>
+__global__ void __launch_bounds__(NW * WAVE)
+talking_finish_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, const float* __restrict__ talk,
+                      const int* __restrict__ rows, const int* __restrict__ tiles, const int* __restrict__ cu_q,
+                      bf16_t* __restrict__ out, int n_q, int n_kv, int dv, int parts) {
+  extern __shared__ float tkf_lds[];
+  const int item = blockIdx.x, kvh = blockIdx.y, lane = threadIdx.x & 63, wave = wave_index();
+  int t = rows ? scalar_int(rows + item) : item;
+  if (t < 0) return;
+  if (tiles) {
+    const int tile = item >> 4, token = item & 15;
+    const int entry = scalar_int(tiles + 2 * tile), row0 = scalar_int(cu_q + entry) + scalar_int(tiles + 2 * tile + 1);
+    if (token >= scalar_int(cu_q + entry + 1) - row0) return;
+    t = row0 + token;
+  }
+  const int wide = n_kv * dv, group = n_q / n_kv, i = blockIdx.z * WAVE + lane;
+  const bool live = i < dv;
+  const size_t base = (size_t)item * parts * n_q;
+  const float* src = part_o + base * wide + (size_t)kvh * dv + (live ? i : 0);
+  for (int g = wave; g < n_q; g += NW) {
+    float a = 0.f;
+    if (parts == 1) {
+      const float inv = 1.0f / part_ml[(base + g) * 2 + 1];
+      a = src[(size_t)g * wide] * inv;
+    } else {
+      float m = -INFINITY, l = 0.f;
+      for (int p0 = 0; p0 < parts; p0 += WAVE) m = fmaxf(m, p0 + lane < parts ? part_ml[(base + (size_t)(p0 + lane) * n_q + g) * 2] : -INFINITY);
+      m = wave_max(m);
+      for (int p0 = 0; p0 < parts; p0 += WAVE) {
+        // Lane p: what part p's sums are multiplied by.
+        float f = 0.f;
+        if (p0 + lane < parts) {
+          const float* ml = part_ml + (base + (size_t)(p0 + lane) * n_q + g) * 2;
+          f = ml[0] == -INFINITY ? 0.f : __expf(ml[0] - m);
+          l = fmaf(f, ml[1], l);
+        }
+        const int count = min(WAVE, parts - p0);
+        const float* from = src + (size_t)p0 * n_q * wide + (size_t)g * wide;
+        for (int p = 0; p < count; p += 16) {
+          float v[16];
+#pragma unroll
+          for (int x = 0; x < 16; ++x) {
+            // (A part without keys left its sums unwritten: whatever lies there is passed over by selection.)
+            const int at = min(p + x, count - 1);
+            v[x] = from[(size_t)at * n_q * wide];
+          }
+#pragma unroll
+          for (int x = 0; x < 16; ++x) {
+            const float w = p + x < count ? __shfl(f, (p + x) & 63, WAVE) : 0.f;
+            a += w == 0.f ? 0.f : w * v[x];
+          }
+        }
+      }
+      a /= wave_sum(l);
+    }
+    tkf_lds[g * WAVE + lane] = a;
+  }
+  __syncthreads();
+  for (int r = wave; r < group; r += NW) {
+    const int h = kvh * group + r;
+    float o = 0.f;
+    for (int g = 0; g < n_q; ++g) o = fmaf(talk[(size_t)h * n_q + g], tkf_lds[g * WAVE + lane], o);
+    if (live) st(out + (size_t)t * n_q * dv + (size_t)h * dv + i, o);
+  }
+}
+
+static int launch_finish(const void* part_o, const void* part_ml, const void* talk, const void* rows, const void* tiles,
+                         const void* cu_q, void* out, int items, int n_q, int n_kv, int dv, int parts, hipStream_t stream) {
+  dim3 grid(items, n_kv, (dv + WAVE - 1) / WAVE);
+  const size_t lds = sizeof(float) * n_q * WAVE;
+#define FINISH(NWV) talking_finish_kernel<NWV><<<grid, NWV * WAVE, lds, stream>>>((const float*)part_o, (const float*)part_ml, \
+      (const float*)talk, (const int*)rows, (const int*)tiles, (const int*)cu_q, (bf16_t*)out, n_q, n_kv, dv, parts)
+  if (parts > 2 || items <= 64) FINISH(16); else FINISH(4);
+#undef FINISH
+  return LAUNCH_STATUS();
+}
+
+// A launch that wants more dynamic LDS than every kernel may have says so first.
+static int allow_lds(const void* kernel, int bytes) {
+  if (bytes <= 48 * 1024) return 0;
+  return (int)hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
+}
+
+// Whether the matrix-core kernels take these sizes.
+static bool talking_fits(int n_q, int n_kv, int d, int dv, int page_size) {
+  return n_kv > 0 && n_q > 0 && n_q % n_kv == 0 && n_q <= 64 && d >= 8 && d <= 256 && d % 8 == 0 && dv > 0 && page_size % 16 == 0 &&
+         (long)n_kv * dv <= 65536;
+}
+
+// Single tokens: items are the rows of `rows` (or every row); entry_of_token null: row e is entry e.  part_o float
+// [n_items, splits, n_q, n_kv dv], part_ml float [n_items, splits, n_q, 2].  Returns -2 for sizes without an instance.
+extern "C" int ta_talking_decode_bf16(const void* q, int q_stride, void* out, const void* k_pages, const void* vt_pages,
+                                      const void* rows, const void* positions, const void* entry_of_token,
+                                      const void* block_table, int table_stride, void* part_o, void* part_ml, const void* talk,
+                                      int n_items, int n_q, int n_kv, int d, int dv, int page_size, float scale, int split_keys,
+                                      int splits, hipStream_t stream) {
+  if (n_items <= 0) return 0;
+  if (!talking_fits(n_q, n_kv, d, dv, page_size) || q_stride % 8) return -2;
+  if (split_keys < 32 || split_keys % 32 || split_keys > 32 * TKD_BLOCKS || splits < 1 || splits > 0x7ffffff || n_items > 65535) return -1;
+  const int wide = n_kv * dv, hb = (n_q + 15) / 16;
+  dim3 grid(splits, n_items);
+#define DECODE(NWV, HBV)                                                                                                 \
+  const int lds = 16 * HBV * (4 * (split_keys + 4) + 2 * (split_keys + 8));       /* at most 101 KB */                    \
+  if (const int bad = allow_lds(reinterpret_cast<const void*>(&talking_decode_kernel<NWV, HBV>), lds)) return bad;         \
+  talking_decode_kernel<NWV, HBV><<<grid, NWV * WAVE, lds, stream>>>(                                                     \
+      (const bf16_t*)q, q_stride, (const bf16_t*)k_pages, (const bf16_t*)vt_pages, (const int*)rows, (const int*)positions, \
+      (const int*)entry_of_token, (const int*)block_table, table_stride, (float*)part_o, (float*)part_ml, n_q, n_kv, d, wide, \
+      page_size, scale, split_keys, splits)
+#define DECODES(HBV) if (wide >= 256) { DECODE(8, HBV); } else { DECODE(4, HBV); }
+  if (hb <= 1) { DECODES(1); } else if (hb <= 2) { DECODES(2); } else { DECODES(4); }
+#undef DECODES
+#undef DECODE
+  const int status = LAUNCH_STATUS();
+  if (status) return status;
+  return launch_finish(part_o, part_ml, talk, rows, nullptr, nullptr, out, n_items, n_q, n_kv, dv, splits, stream);
+}
+
+// What a launch over `n_tiles` tiles that reach `reach` keys is cut into: slabs of the value columns (16 * *blocks columns
+// each), and parts of the keys (a few tiles behind a long context would leave the device idle).
+static void talking_plan(int n_tiles, int n_q, int n_kv, int d, int dv, int reach, int* blocks, int* slabs, int* heads, int* parts) {
+  const int wide = n_kv * dv, group = n_q / n_kv;
+  *blocks = wide <= 64 ? 4 : wide <= 128 ? 8 : 16;
+  *slabs = (wide + 16 * *blocks - 1) / (16 * *blocks);
+  *heads = (group > 4 && d <= 128) ? 2 : 1;
+  const long groups = (long)n_tiles * n_kv * ((group + 4 * *heads - 1) / (4 * *heads)) * *slabs;
+  int cut = 1;
+  while (cut < 16 && groups * cut < 512 && reach / (cut * 2) >= 256) cut *= 2;
+  *parts = cut;
+}
+
+extern "C" int ta_talking_prefill_parts(int n_tiles, int n_q, int n_kv, int d, int dv, int reach) {
+  if (n_tiles <= 0 || n_kv <= 0 || n_q % n_kv) return 1;
+  int blocks, slabs, heads, parts;
+  talking_plan(n_tiles, n_q, n_kv, d, dv, reach, &blocks, &slabs, &heads, &parts);
+  return parts;
+}
+
+// Prompt portions: tiles [n_tiles, 2] = (entry, offset of the tile's first token inside the entry's tokens).  part_o float
+// [n_tiles * 16, parts, n_q, n_kv dv], part_ml float [n_tiles * 16, parts, n_q, 2] with `parts` as
+// ta_talking_prefill_parts says.  Returns -2 for sizes without an instance.
+extern "C" int ta_talking_prefill_bf16(const void* q, int q_stride, void* out, const void* k_pages, const void* vt_pages,
+                                       const void* tiles, int n_tiles, const void* cu_q, const void* first_position,
+                                       const void* block_table, int table_stride, void* part_o, void* part_ml, const void* talk,
+                                       int n_q, int n_kv, int d, int dv, int page_size, float scale, int reach, hipStream_t stream) {
+  if (n_tiles <= 0) return 0;
+  if (!talking_fits(n_q, n_kv, d, dv, page_size) || q_stride % 8) return -2;
+  int blocks, slabs, heads, parts;
+  talking_plan(n_tiles, n_q, n_kv, d, dv, reach, &blocks, &slabs, &heads, &parts);
+  const int wide = n_kv * dv, group = n_q / n_kv;
+  const long total = (long)n_tiles * n_kv * ((group + 4 * heads - 1) / (4 * heads)) * slabs * parts;
+  if (total > 0x7fffffffL || (long)n_tiles * 16 > 0x7fffffffL) return -1;
+#define PREFILL(DPV, VBV, HGV)                                                                                            \
+  {                                                                                                                       \
+  if (const int bad = allow_lds(reinterpret_cast<const void*>(&talking_prefill_kernel<DPV, VBV, HGV>),                     \
+                                2 * TalkBlock<DPV, VBV>::BYTES)) return bad;                                              \
+  talking_prefill_kernel<DPV, VBV, HGV><<<(unsigned)total, 4 * WAVE, 2 * TalkBlock<DPV, VBV>::BYTES, stream>>>(             \
+      (const bf16_t*)q, q_stride, (const bf16_t*)k_pages, (const bf16_t*)vt_pages, (const int*)tiles, n_tiles,             \
+      (const int*)cu_q, (const int*)first_position, (const int*)block_table, table_stride, (float*)part_o,                 \
+      (float*)part_ml, n_q, n_kv, d, wide, page_size, scale, slabs, parts);                                                \
+  }
+#define PREFILL_H(DPV, VBV) if (heads == 2) PREFILL(DPV, VBV, 2) else PREFILL(DPV, VBV, 1)
+#define PREFILL_V(DPV) if (blocks == 4) { PREFILL_H(DPV, 4); } else if (blocks == 8) { PREFILL_H(DPV, 8); } else { PREFILL_H(DPV, 16); }
+  if (d <= 32) { PREFILL_V(32); } else if (d <= 64) { PREFILL_V(64); } else if (d <= 128) { PREFILL_V(128); }
+  else if (blocks == 4) PREFILL(256, 4, 1) else if (blocks == 8) PREFILL(256, 8, 1) else PREFILL(256, 16, 1)
+#undef PREFILL_V
+#undef PREFILL_H
+#undef PREFILL
+  const int status = LAUNCH_STATUS();
+  if (status) return status;
+  return launch_finish(part_o, part_ml, talk, nullptr, tiles, cu_q, out, n_tiles * 16, n_q, n_kv, dv, parts, stream);
+}

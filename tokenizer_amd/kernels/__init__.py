@@ -160,7 +160,8 @@ class Ops:
                      "ta_delta_scan", "ta_route_sigmoid", "ta_route_rows_sigmoid", "ta_expert_act", "ta_relu2",
                      "ta_add_terms_rmsnorm", "ta_scale_cap", "ta_route_scores", "ta_selective_scan", "ta_route_rows_scores",
                      "ta_rotation_table", "ta_head_norm_rotate_store", "ta_group_norm_add", "ta_relu_gate",
-                     "ta_talking_attention_generic", "ta_retention_scan"):
+                     "ta_talking_attention_generic", "ta_talking_decode_bf16", "ta_talking_prefill_bf16",
+                     "ta_talking_prefill_parts", "ta_retention_scan"):
             getattr(self.lib, name).restype = ctypes.c_int
         self.lib.ta_grouped_gemm_bf16.argtypes = [ctypes.c_void_p, ctypes.c_int, ctypes.c_void_p, ctypes.c_void_p, ctypes.c_int,
                                                   ctypes.c_int, ctypes.c_void_p, ctypes.c_long, ctypes.c_int, ctypes.c_void_p,
@@ -1181,12 +1182,53 @@ class Ops:
         _need(0 < head_dim <= 512 and 0 < value_dim, "head sizes up to 512 are supported")
         if max_position is not None:
             _need(max_position // page_size < block_table.shape[1], "block table is too narrow for the positions")
+        if (qkv.dtype == torch.bfloat16 and self.use_fast_attention and head_dim % 8 == 0 and head_dim <= 256 and n_q <= 64
+                and page_size % 16 == 0 and qkv.stride(0) % 8 == 0 and qkv.data_ptr() % 16 == 0):
+            reach = block_table.shape[1] * page_size if max_position is None else int(max_position) + 1
+            reach = -(-reach // self.PLAN_KEYS) * self.PLAN_KEYS
+            args = (qkv, out, k_pages, v_pages, positions, entry_of_token, block_table, n_q, n_kv, head_dim, value_dim, page_size,
+                    scale, talk, reach)
+            if batch is None:
+                return self._talking_decode(*args)
+            if batch.q_tiles.numel() == 0:
+                return self._talking_decode(*args, identity_entries=batch.n_tokens == block_table.shape[0])
+            _need(batch.n_tokens == n_tokens and batch.cu_q.numel() == block_table.shape[0] + 1,
+                  "the batch description does not belong to these tokens")
+            n_tiles = batch.q_tiles.shape[0]
+            parts = self.lib.ta_talking_prefill_parts(n_tiles, n_q, n_kv, head_dim, value_dim, reach)
+            part_o = torch.empty((n_tiles * 16, parts, n_q, n_kv * value_dim), dtype=torch.float32, device=qkv.device)
+            part_ml = torch.empty((n_tiles * 16, parts, n_q, 2), dtype=torch.float32, device=qkv.device)
+            self._check(self.lib.ta_talking_prefill_bf16(
+                _ptr(qkv), qkv.stride(0), _ptr(out), _ptr(k_pages), _ptr(v_pages), _ptr(batch.q_tiles), n_tiles, _ptr(batch.cu_q),
+                _ptr(batch.first_position), _ptr(block_table), block_table.shape[1], _ptr(part_o), _ptr(part_ml), _ptr(talk), n_q,
+                n_kv, head_dim, value_dim, page_size, ctypes.c_float(scale), reach, self._stream()), "talking_prefill")
+            if batch.decode_rows.numel():
+                self._talking_decode(*args, rows=batch.decode_rows)
+            return out
         stats = torch.empty((n_tokens, n_q, 2), dtype=torch.float32, device=qkv.device)
         self._check(self.lib.ta_talking_attention_generic(
             _ptr(qkv), qkv.stride(0), _ptr(out), _ptr(k_pages), _ptr(v_pages), _ptr(positions), _ptr(entry_of_token),
             _ptr(block_table), block_table.shape[1], _ptr(stats), _ptr(talk), n_tokens, n_q, n_kv, head_dim, value_dim, page_size,
             ctypes.c_float(scale), _code(qkv.dtype), self._stream()), "talking_attention")
         return out
+
+    def _talking_decode(self, qkv, out, k_pages, v_pages, positions, entry_of_token, block_table, n_q, n_kv, head_dim, value_dim,
+                        page_size, scale, talk, reach, rows=None, identity_entries=False):
+        """Single tokens of `talking_attention`: the keys cut over workgroups in parts of 64 to 256."""
+        n_items = qkv.shape[0] if rows is None else rows.numel()
+        split_keys = min(256, max(64, -(-reach // max(1, self.talking_workgroups // max(1, n_items)))))
+        split_keys = -(-split_keys // 32) * 32
+        splits = -(-reach // split_keys)
+        part_o = torch.empty((n_items, splits, n_q, n_kv * value_dim), dtype=torch.float32, device=qkv.device)
+        part_ml = torch.empty((n_items, splits, n_q, 2), dtype=torch.float32, device=qkv.device)
+        self._check(self.lib.ta_talking_decode_bf16(
+            _ptr(qkv), qkv.stride(0), _ptr(out), _ptr(k_pages), _ptr(v_pages), _ptr(rows), _ptr(positions),
+            _ptr(None if identity_entries and rows is None else entry_of_token), _ptr(block_table), block_table.shape[1],
+            _ptr(part_o), _ptr(part_ml), _ptr(talk), n_items, n_q, n_kv, head_dim, value_dim, page_size, ctypes.c_float(scale),
+            split_keys, splits, self._stream()), "talking_decode")
+        return out
+
+    talking_workgroups = 512      # what the single tokens' split of the keys aims at
 
     # --------------------------------------------------------------------- linear
     takes_pending = True      # `linear(pending=True)` and `add_rmsnorm` with a `PendingSum` exist here
