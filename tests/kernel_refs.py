@@ -526,7 +526,11 @@ class PlainOps:
             out[t] = torch.einsum("hk,khd->hd", weights, v).reshape(-1).to(out.dtype)
         return out
 
-    def retention(self, qkvg, table, dims, decays, state, cu_q, first_position, state_slots, out, heads, d, dv, eps):
+    def decay_powers(self, decays):
+        return decays
+
+    def retention(self, qkvg, table, dims, decays, powers, state, cu_q, first_position, state_slots, out, heads, d, dv, eps,
+                  single_rows=False):
         w = self.work
         n_tokens = qkvg.shape[0]
         x = qkvg.to(w)

@@ -161,7 +161,7 @@ class Ops:
                      "ta_add_terms_rmsnorm", "ta_scale_cap", "ta_route_scores", "ta_selective_scan", "ta_route_rows_scores",
                      "ta_rotation_table", "ta_head_norm_rotate_store", "ta_group_norm_add", "ta_relu_gate",
                      "ta_talking_attention_generic", "ta_talking_decode_bf16", "ta_talking_prefill_bf16",
-                     "ta_talking_prefill_parts", "ta_retention_scan"):
+                     "ta_talking_prefill_parts", "ta_retention_scan", "ta_retention_chunked"):
             getattr(self.lib, name).restype = ctypes.c_int
         self.lib.ta_grouped_gemm_bf16.argtypes = [ctypes.c_void_p, ctypes.c_int, ctypes.c_void_p, ctypes.c_void_p, ctypes.c_int,
                                                   ctypes.c_int, ctypes.c_void_p, ctypes.c_long, ctypes.c_int, ctypes.c_void_p,
@@ -1698,16 +1698,27 @@ class Ops:
         return out
 
     # ------------------------------------------------------------------- retention
-    def retention(self, qkvg: torch.Tensor, table: torch.Tensor | None, dims: int, decays: torch.Tensor, state: torch.Tensor,
-                  cu_q: torch.Tensor, first_position: torch.Tensor, state_slots: torch.Tensor, out: torch.Tensor, heads: int,
-                  d: int, dv: int, eps: float) -> torch.Tensor:
+    RETENTION_CHUNK = 64         # tokens a chunk
+    RETENTION_TOKENS = 8         # entries of more rows than this run in chunks (bfloat16; the 32-bit path walks them all)
+
+    @classmethod
+    def decay_powers(cls, decays: torch.Tensor) -> torch.Tensor:
+        """float32 [heads, 65]: c^0 .. c^64 of every head's decay, worked out in float64, for `retention`."""
+        c = decays.detach().to("cpu", torch.float64)
+        return torch.stack([c ** n for n in range(cls.RETENTION_CHUNK + 1)], dim=1).to(torch.float32).to(decays.device).contiguous()
+
+    def retention(self, qkvg: torch.Tensor, table: torch.Tensor | None, dims: int, decays: torch.Tensor, powers: torch.Tensor,
+                  state: torch.Tensor, cu_q: torch.Tensor, first_position: torch.Tensor, state_slots: torch.Tensor,
+                  out: torch.Tensor, heads: int, d: int, dv: int, eps: float, single_rows: bool = False) -> torch.Tensor:
         """The retention recurrence over every entry's rows, from and into the entries' state rows, with the rotation in
         front and the heads' norm and gate behind: per head S <- c S + k v^T, o = S^T q, out = o / rms(o) * silu(g).
 
         qkvg [T, >= 2 heads d + 2 heads dv]: q, k (heads of d), v and g (heads of dv) side by side; the first `dims`
         coordinates of q and k turn by `table` (float32 [T, dims], see `rotation_table`), k is multiplied by d^(-1/2);
-        decays float32 [heads]; state float32 [slots, heads dv d] (S transposed; an entry whose first position is 0 starts
-        from zeros); out [T, heads dv] of qkvg's dtype."""
+        decays float32 [heads], powers as `decay_powers` makes them; state float32 [slots, heads dv d] (S transposed; an entry whose first position is 0 starts
+        from zeros); out [T, heads dv] of qkvg's dtype.  `single_rows`: every entry brings one row.
+
+        Entries of a few rows walk token by token; longer bfloat16 ones run in chunks side by side."""
         _dev(qkvg, table, decays, state, cu_q, first_position, state_slots, out)
         n_tokens = qkvg.shape[0]
         _need(qkvg.stride(1) == 1 and qkvg.shape[1] >= 2 * heads * (d + dv), "q, k, v, g do not fit the rows")
@@ -1720,10 +1731,21 @@ class Ops:
         _need(0 < d <= 256 and 0 < dv <= 256, "heads of up to 256 coordinates and 256 values are supported")
         n_entries = cu_q.numel() - 1
         _need(first_position.numel() == n_entries == state_slots.numel(), "one first position and slot per entry")
+        most = self.RETENTION_TOKENS
+        chunked = qkvg.dtype == torch.bfloat16 and not single_rows and n_tokens > most
         self._check(self.lib.ta_retention_scan(
             _ptr(qkvg), qkvg.stride(0), _ptr(table if dims else None), dims, _ptr(decays), _ptr(state), ctypes.c_long(state.shape[1]),
             _ptr(cu_q), _ptr(first_position), _ptr(state_slots), _ptr(out), n_entries, heads, d, dv, ctypes.c_float(eps),
-            0x7fffffff, _code(qkvg.dtype), self._stream()), "retention_scan")
+            most if chunked else 0x7fffffff, _code(qkvg.dtype), self._stream()), "retention_scan")
+        if chunked:
+            _need(powers.is_cuda and powers.dtype == torch.float32 and powers.is_contiguous()
+                  and tuple(powers.shape) == (heads, self.RETENTION_CHUNK + 1), "powers float32 [heads, 65]")
+            max_chunks = n_tokens // self.RETENTION_CHUNK + n_entries
+            scratch = torch.empty((max_chunks, heads, dv, d), dtype=torch.float32, device=qkvg.device)
+            self._check(self.lib.ta_retention_chunked(
+                _ptr(qkvg), qkvg.stride(0), _ptr(table if dims else None), dims, _ptr(powers), _ptr(state),
+                ctypes.c_long(state.shape[1]), _ptr(cu_q), _ptr(first_position), _ptr(state_slots), _ptr(scratch), _ptr(out),
+                n_entries, max_chunks, heads, d, dv, ctypes.c_float(eps), most, self._stream()), "retention_chunked")
         return out
 
     # ------------------------------------------------------------------- sampling

@@ -35,6 +35,7 @@ class Retention(Mixer):
         if fill:
             self.w_in = torch.cat([self.w_in, self.w_in.new_zeros((fill, self.w_in.shape[1]))], dim=0).contiguous()
         self.decays = torch.tensor(spec.decays, dtype=torch.float32, device=runtime.device)
+        self.powers = runtime.ops.decay_powers(self.decays)
         position = spec.position or PositionSpec("rope_partial", head_dim=self.d, theta=1.0, options={"dims": 0})
         if position.kind != "rope_partial":
             raise ValueError(f"retention turns its queries and keys by the partial rotation, not {position.kind!r}")
@@ -57,6 +58,7 @@ class Retention(Mixer):
             raise ValueError("the recurrent mixer needs its state in the request's slot")
         qkvg = ops.linear(x, self.w_in)
         mixed = torch.empty((x.shape[0], self.heads * self.dv), dtype=x.dtype, device=x.device)
-        ops.retention(qkvg, self.position.angles(ctx), self.position.dims, self.decays, cache.state, ctx.cu_q,
-                      ctx.first_position, ctx.state_slots, mixed, self.heads, self.d, self.dv, self.eps)
+        ops.retention(qkvg, self.position.angles(ctx), self.position.dims, self.decays, self.powers, cache.state, ctx.cu_q,
+                      ctx.first_position, ctx.state_slots, mixed, self.heads, self.d, self.dv, self.eps,
+                      single_rows=ctx.q_tiles.numel() == 0)
         return ops.linear(mixed, self.w_o)
