@@ -138,7 +138,7 @@ extern "C" int ta_talking_attention_generic(const void* q, int q_stride, void* o
 // The matrix-core form for bfloat16.  The mix commutes with the product with the values: with
 // A_g = sum_j p_g(j) V(j) over the values of ALL kv heads side by side (W = n_kv dv numbers), head h's output is
 // sum_g talk[h, g] times A_g's part at h's own kv head.  So every head is an ordinary softmax over its own keys against
-// values W wide, in one walk over the keys, and the mix is a small product at the end (`talking_finish_kernel`), in float.
+// values W wide, in one walk over the keys, and the mix is a small product at the end (`talking_mix_kernel`), in float.
 // The value pages hold exactly these wide values: a page's [n_kv, dv, page_size] read as [W, page_size].
 // Both kernels leave, per (token, part of its keys, head), the unnormalised sums [W] with the maximum and the sum of
 // exponentials they stand under: part_o float [items, parts, n_q, W], part_ml float [items, parts, n_q, 2].
@@ -152,6 +152,33 @@ __device__ __forceinline__ bf16x8 tk_zero8() {
   for (int i = 0; i < 8; ++i) z[i] = (__bf16)0.0f;
   return z;
 }
+
+// Over the sixteen lanes of a row (lanes 16 i .. 16 i + 15), in every lane of the row: rotations within the row, which cost no
+// trip through LDS.
+#define TK_ROR(x, n) __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), 0x120 | (n), 0xF, 0xF, false))
+__device__ __forceinline__ float tk_row_sum16(float x) {
+  x += TK_ROR(x, 8);
+  x += TK_ROR(x, 4);
+  x += TK_ROR(x, 2);
+  x += TK_ROR(x, 1);
+  return x;
+}
+__device__ __forceinline__ float tk_row_max16(float x) {
+  x = fmaxf(x, TK_ROR(x, 8));
+  x = fmaxf(x, TK_ROR(x, 4));
+  x = fmaxf(x, TK_ROR(x, 2));
+  x = fmaxf(x, TK_ROR(x, 1));
+  return x;
+}
+
+// Where a key's page and slot lie; page sizes are powers of two as a rule, and a division costs thirty scalar instructions.
+struct TalkPages {
+  int size, shift;
+  __device__ __forceinline__ explicit TalkPages(int page_size)
+      : size(page_size), shift((page_size & (page_size - 1)) ? -1 : 31 - __builtin_clz(page_size)) {}
+  __device__ __forceinline__ int page(int key) const { return shift >= 0 ? key >> shift : key / size; }
+  __device__ __forceinline__ int slot(int key) const { return shift >= 0 ? key & (size - 1) : key % size; }
+};
 
 // Single tokens.  A workgroup a (part of the keys, token), all heads and all value columns: first the scores of every
 // head over the part (a wave a kv head's block of 32 keys at a time, up to sixteen heads the N side of the instruction)
@@ -187,6 +214,7 @@ talking_decode_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* 
     }
     return;
   }
+  const TalkPages pages(page_size);
   const int blocks = (last - first) / 32 + 1, group = n_q / n_kv, head_blocks = (group + 15) / 16;
   union VFrag { uint4 bits; bf16x8 v; };
   // Rows rb * 16 .. + 15 of the wide values over the part's keys: lane (col, g) has row col, keys 8 g .. 8 g + 7 of a block.
@@ -198,8 +226,9 @@ talking_decode_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* 
       if (b >= blocks) continue;
       const int kb = first + 32 * b;
       const bool there1 = kb + 16 <= last;                 // (a half without keys borrows the other's page; its values are zeroed)
-      const int page0 = scalar_int(table + kb / page_size), page1 = scalar_int(table + (there1 ? kb + 16 : kb) / page_size);
-      const uint32_t at = ((uint32_t)((g >> 1) ? page1 : page0) * wide + row) * page_size + (kb + 16 * (g >> 1)) % page_size + 8 * (g & 1);
+      const int page0 = scalar_int(table + pages.page(kb)), page1 = scalar_int(table + pages.page(there1 ? kb + 16 : kb));
+      const int slot0 = pages.slot(kb), slot1 = pages.slot(kb + 16);
+      const uint32_t at = ((uint32_t)((g >> 1) ? page1 : page0) * wide + row) * page_size + ((g >> 1) ? slot1 : slot0) + 8 * (g & 1);
       vf[b].bits = *reinterpret_cast<const uint4*>(vt_pages + at);
     }
   };
@@ -210,9 +239,9 @@ talking_decode_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* 
   for (int unit = wave; unit < n_kv * blocks; unit += NW) {
     const int kvh = unit % n_kv, kb = first + 32 * (unit / n_kv);
     const bool there1 = kb + 16 <= last;
-    const int page0 = scalar_int(table + kb / page_size), page1 = scalar_int(table + (there1 ? kb + 16 : kb) / page_size);
-    const bf16_t* k0 = k_pages + (((size_t)page0 * n_kv + kvh) * page_size + kb % page_size + col) * d + 8 * g;
-    const bf16_t* k1 = k_pages + (((size_t)page1 * n_kv + kvh) * page_size + (there1 ? kb + 16 : kb) % page_size + col) * d + 8 * g;
+    const int page0 = scalar_int(table + pages.page(kb)), page1 = scalar_int(table + pages.page(there1 ? kb + 16 : kb));
+    const bf16_t* k0 = k_pages + (((size_t)page0 * n_kv + kvh) * page_size + pages.slot(kb) + col) * d + 8 * g;
+    const bf16_t* k1 = k_pages + (((size_t)page1 * n_kv + kvh) * page_size + pages.slot(there1 ? kb + 16 : kb) + col) * d + 8 * g;
     for (int hb = 0; hb < head_blocks; ++hb) {
       const int head = kvh * group + hb * 16 + col;
       const bool has = hb * 16 + col < group;
@@ -252,25 +281,29 @@ talking_decode_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* 
     }
   }
   __syncthreads();
-  // Maximum, exponentials and sum: a wave a head.  (Key 0 of the part is seen, so every maximum is a number.)
-  for (int h = wave; h < 16 * HB; h += NW) {
-    float s[TKD_BLOCKS / 2], m = -INFINITY, l = 0.f;
+  // Maximum, exponentials and sum: sixteen lanes a head.  (Key 0 of the part is seen, so every maximum is a number.)
+  for (int h0 = wave * 4; h0 < 16 * HB; h0 += NW * 4) {
+    const int h = h0 + g;
+    const bool live = h < n_q;
+    const float* row = s_s + (size_t)h * s_ld + col;
+    float s[2 * TKD_BLOCKS], m = -INFINITY, l = 0.f;
 #pragma unroll
-    for (int i = 0; i < TKD_BLOCKS / 2; ++i) {
-      const int j = lane + 64 * i;
-      s[i] = (h < n_q && j < 32 * blocks) ? s_s[(size_t)h * s_ld + j] : -INFINITY;
+    for (int i = 0; i < 2 * TKD_BLOCKS; ++i) {
+      s[i] = -INFINITY;
+      if (i < 2 * blocks && live) s[i] = row[16 * i];
       m = fmaxf(m, s[i]);
     }
-    m = wave_max(m);
+    m = tk_row_max16(m);
+    bf16_t* to = p_s + (size_t)h * p_ld + col;
 #pragma unroll
-    for (int i = 0; i < TKD_BLOCKS / 2; ++i) {
-      const int j = lane + 64 * i;
+    for (int i = 0; i < 2 * TKD_BLOCKS; ++i) {
+      if (i >= 2 * blocks) continue;
       const float p = s[i] == -INFINITY ? 0.f : __expf(s[i] - m);
       l += p;
-      if (j < 32 * blocks) st(p_s + (size_t)h * p_ld + j, p);
+      st(to + 16 * i, p);
     }
-    l = wave_sum(l);
-    if (lane == 0 && h < n_q) {
+    l = tk_row_sum16(l);
+    if (col == 0 && live) {
       part_ml[(part * n_q + h) * 2] = m;
       part_ml[(part * n_q + h) * 2 + 1] = l;
     }
@@ -409,13 +442,14 @@ talking_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t*
     const int row = min(slab * 16 * VB + 32 * j + (lane >> 1), wide - 1);
     v_from[j] = (uint32_t)(row * page_size + (lane & 1) * 8) * 2;
   }
+  const TalkPages pages(page_size);
   const auto page_of = [&](int kb) {                       // (a run past the last key borrows the last key's page: its keys are masked)
-    return scalar_int(table + min(kb + 16 * run, hi) / page_size);
+    return scalar_int(table + pages.page(min(kb + 16 * run, hi)));
   };
   const auto fetch = [&](int kb, int page, char* buf) {
     typedef const void __attribute__((address_space(1)))* from_t;
     typedef void __attribute__((address_space(3)))* to_t;
-    const int slot = (kb + 16 * run) % page_size;
+    const int slot = pages.slot(kb + 16 * run);
     const char* k_run = reinterpret_cast<const char*>(k_pages + (((uint32_t)page * n_kv + kvh) * page_size + slot) * d);
     const char* v_run = reinterpret_cast<const char*>(vt_pages + ((uint32_t)page * wide * page_size + slot));
     char* k_to = buf + run * 16 * B::K_ROW;
@@ -542,84 +576,164 @@ talking_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t*
   }
 }
 
-// The parts of every head brought together and the heads mixed: a workgroup a (item, kv head, 64 value columns).  Wave w
-// makes A_g for g = w, w + NW, ... (a lane a column; parts under their common maximum, over the common sum) into LDS,
-// then head h = w, w + NW, ... of the kv head's group, sum_g talk[h, g] A_g.  Items are rows (`rows`, or themselves), or,
-// with `tiles`, (tile, token of the tile).  Dynamic LDS: n_q rows of 64 floats.
-template <int NW>
-__global__ void __launch_bounds__(NW * WAVE)
-talking_finish_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, const float* __restrict__ talk,
-                      const int* __restrict__ rows, const int* __restrict__ tiles, const int* __restrict__ cu_q,
-                      bf16_t* __restrict__ out, int n_q, int n_kv, int dv, int parts) {
-  extern __shared__ float tkf_lds[];
-  const int item = blockIdx.x, kvh = blockIdx.y, lane = threadIdx.x & 63, wave = wave_index();
-  int t = rows ? scalar_int(rows + item) : item;
-  if (t < 0) return;
-  if (tiles) {
-    const int tile = item >> 4, token = item & 15;
-    const int entry = scalar_int(tiles + 2 * tile), row0 = scalar_int(cu_q + entry) + scalar_int(tiles + 2 * tile + 1);
-    if (token >= scalar_int(cu_q + entry + 1) - row0) return;
-    t = row0 + token;
+// The heads mixed: out of head h = sum_g talk[h, g] A_g at h's own kv head, float products on the matrix cores (16x16x4): the
+// sixteen heads of a block are the M side, sixteen value columns the N side, the heads g the contraction; lane (col, grp)
+// has row `col` of the talk table and column `col` of the A_g for g = 4 s + grp.  STEPS: steps of four heads g.
+#define TK_MFMA32(a, b, c) __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0)
+
+// The output row of item `item` (-1: none): rows, or with `tiles` (tile, token of the tile).
+__device__ __forceinline__ int talking_row(int item, const int* rows, const int* tiles, const int* cu_q) {
+  if (!tiles) return rows ? scalar_int(rows + item) : item;
+  const int tile = item >> 4, token = item & 15;
+  const int entry = scalar_int(tiles + 2 * tile), row0 = scalar_int(cu_q + entry) + scalar_int(tiles + 2 * tile + 1);
+  return token < scalar_int(cu_q + entry + 1) - row0 ? row0 + token : -1;
+}
+
+__device__ __forceinline__ void talking_store(bf16_t* out, const floatx4& acc, int row, int n_q, int dv, int head0, int heads,
+                                              int column, int grp) {
+#pragma unroll
+  for (int r = 0; r < 4; ++r)
+    if (4 * grp + r < heads && column < dv)
+      st(out + (size_t)row * n_q * dv + (size_t)(head0 + 4 * grp + r) * dv + column, acc[r]);
+}
+
+// Keys in one part: a wave four items one after another, for one (kv head, block of sixteen of its heads) and all its value
+// columns.
+template <int STEPS>
+__global__ void __launch_bounds__(4 * WAVE)
+talking_mix_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, const float* __restrict__ talk,
+                   const int* __restrict__ rows, const int* __restrict__ tiles, const int* __restrict__ cu_q,
+                   bf16_t* __restrict__ out, int items, int n_q, int n_kv, int dv) {
+  const int lane = threadIdx.x & 63, wave = wave_index(), col = lane & 15, grp = lane >> 4;
+  const int group = n_q / n_kv, head_blocks = (group + 15) / 16, wide = n_kv * dv;
+  const int kvh = blockIdx.y / head_blocks, first = (blockIdx.y - kvh * head_blocks) * 16, heads = min(16, group - first);
+  const int head0 = kvh * group + first;
+  float t[STEPS];
+#pragma unroll
+  for (int s = 0; s < STEPS; ++s) {
+    const int g = 4 * s + grp;
+    t[s] = (col < heads && g < n_q) ? talk[(size_t)(head0 + col) * n_q + g] : 0.f;
   }
-  const int wide = n_kv * dv, group = n_q / n_kv, i = blockIdx.z * WAVE + lane;
-  const bool live = i < dv;
-  const size_t base = (size_t)item * parts * n_q;
-  const float* src = part_o + base * wide + (size_t)kvh * dv + (live ? i : 0);
-  for (int g = wave; g < n_q; g += NW) {
-    float a = 0.f;
-    if (parts == 1) {
-      const float inv = 1.0f / part_ml[(base + g) * 2 + 1];
-      a = src[(size_t)g * wide] * inv;
-    } else {
-      float m = -INFINITY, l = 0.f;
-      for (int p0 = 0; p0 < parts; p0 += WAVE) m = fmaxf(m, p0 + lane < parts ? part_ml[(base + (size_t)(p0 + lane) * n_q + g) * 2] : -INFINITY);
-      m = wave_max(m);
-      for (int p0 = 0; p0 < parts; p0 += WAVE) {
-        // Lane p: what part p's sums are multiplied by.
-        float f = 0.f;
-        if (p0 + lane < parts) {
-          const float* ml = part_ml + (base + (size_t)(p0 + lane) * n_q + g) * 2;
-          f = ml[0] == -INFINITY ? 0.f : __expf(ml[0] - m);
-          l = fmaf(f, ml[1], l);
-        }
-        const int count = min(WAVE, parts - p0);
-        const float* from = src + (size_t)p0 * n_q * wide + (size_t)g * wide;
-        for (int p = 0; p < count; p += 16) {
-          float v[16];
+  for (int x = 0; x < 4; ++x) {
+    const int item = (blockIdx.x * 4 + wave) * 4 + x;
+    if (item >= items) break;
+    const int row = talking_row(item, rows, tiles, cu_q);
+    if (row < 0) continue;
+    float inv[STEPS];
 #pragma unroll
-          for (int x = 0; x < 16; ++x) {
-            // (A part without keys left its sums unwritten: whatever lies there is passed over by selection.)
-            const int at = min(p + x, count - 1);
-            v[x] = from[(size_t)at * n_q * wide];
-          }
+    for (int s = 0; s < STEPS; ++s) inv[s] = 4 * s + grp < n_q ? 1.0f / part_ml[((size_t)item * n_q + 4 * s + grp) * 2 + 1] : 0.f;
+    for (int c0 = 0; c0 < dv; c0 += 64) {
+      float a[4][STEPS];
 #pragma unroll
-          for (int x = 0; x < 16; ++x) {
-            const float w = p + x < count ? __shfl(f, (p + x) & 63, WAVE) : 0.f;
-            a += w == 0.f ? 0.f : w * v[x];
-          }
+      for (int cb = 0; cb < 4; ++cb) {
+        const int column = c0 + 16 * cb + col;
+#pragma unroll
+        for (int s = 0; s < STEPS; ++s) {
+          a[cb][s] = 0.f;
+          if (4 * s + grp < n_q && column < dv) a[cb][s] = part_o[((size_t)item * n_q + 4 * s + grp) * wide + (size_t)kvh * dv + column];
         }
       }
-      a /= wave_sum(l);
+#pragma unroll
+      for (int cb = 0; cb < 4; ++cb) {
+        floatx4 acc = (floatx4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < STEPS; ++s) acc = TK_MFMA32(t[s], a[cb][s] * inv[s], acc);
+        talking_store(out, acc, row, n_q, dv, head0, heads, c0 + 16 * cb + col, grp);
+      }
     }
-    tkf_lds[g * WAVE + lane] = a;
+  }
+}
+
+// Keys in several parts: a workgroup an (item, kv head and block of sixteen of its heads, sixteen value columns).  First every
+// head's maximum and sum over the parts; then wave w brings parts w, w + NW, ... together under them and mixes what it has
+// (the mix is linear), and the waves' results are added up in LDS.
+template <int STEPS, int NW>
+__global__ void __launch_bounds__(NW * WAVE)
+talking_merge_mix_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, const float* __restrict__ talk,
+                         const int* __restrict__ rows, const int* __restrict__ tiles, const int* __restrict__ cu_q,
+                         bf16_t* __restrict__ out, int n_q, int n_kv, int dv, int parts) {
+  __shared__ float m_s[4 * STEPS], inv_s[4 * STEPS];
+  __shared__ float sum_s[NW][4][WAVE];
+  const int item = blockIdx.x, lane = threadIdx.x & 63, wave = wave_index(), col = lane & 15, grp = lane >> 4;
+  const int row = talking_row(item, rows, tiles, cu_q);
+  if (row < 0) return;
+  const int group = n_q / n_kv, head_blocks = (group + 15) / 16, wide = n_kv * dv;
+  const int kvh = blockIdx.y / head_blocks, first = (blockIdx.y - kvh * head_blocks) * 16, heads = min(16, group - first);
+  const int head0 = kvh * group + first, column = blockIdx.z * 16 + col;
+  const size_t base = (size_t)item * parts * n_q;
+  const float2* ml = reinterpret_cast<const float2*>(part_ml) + base;
+  float t[STEPS];
+#pragma unroll
+  for (int s = 0; s < STEPS; ++s) {
+    const int g = 4 * s + grp;
+    t[s] = (col < heads && g < n_q) ? talk[(size_t)(head0 + col) * n_q + g] : 0.f;
+  }
+  // Sixteen lanes a head: lane `col` parts col, col + 16, ...
+  for (int g0 = wave * 4; g0 < n_q; g0 += NW * 4) {
+    const int g = g0 + grp;
+    float m = -INFINITY, l = 0.f;
+    for (int p = col; p < parts; p += 16) {
+      const float2 x = g < n_q ? ml[(size_t)p * n_q + g] : make_float2(-INFINITY, 0.f);
+      const float top = fmaxf(m, x.x);
+      if (x.x != -INFINITY) { l = (m == -INFINITY ? 0.f : l * __expf(m - top)) + x.y * __expf(x.x - top); m = top; }
+    }
+    const float big = tk_row_max16(m);
+    l = tk_row_sum16(m == -INFINITY ? 0.f : l * __expf(m - big));
+    if (col == 0 && g < n_q) { m_s[g] = big; inv_s[g] = 1.0f / l; }
   }
   __syncthreads();
-  for (int r = wave; r < group; r += NW) {
-    const int h = kvh * group + r;
-    float o = 0.f;
-    for (int g = 0; g < n_q; ++g) o = fmaf(talk[(size_t)h * n_q + g], tkf_lds[g * WAVE + lane], o);
-    if (live) st(out + (size_t)t * n_q * dv + (size_t)h * dv + i, o);
+  float a[STEPS], m[STEPS], inv[STEPS];
+#pragma unroll
+  for (int s = 0; s < STEPS; ++s) {
+    const bool in = 4 * s + grp < n_q;
+    a[s] = 0.f;
+    m[s] = in ? m_s[4 * s + grp] : 0.f;
+    inv[s] = in ? inv_s[4 * s + grp] : 0.f;
   }
+  const float* src = part_o + base * wide + (size_t)kvh * dv + min(column, dv - 1);
+  for (int p = wave; p < parts; p += NW) {
+    float v[STEPS];
+    float2 x[STEPS];
+#pragma unroll
+    for (int s = 0; s < STEPS; ++s) {
+      const int g = min(4 * s + grp, n_q - 1);
+      x[s] = ml[(size_t)p * n_q + g];
+      v[s] = src[((size_t)p * n_q + g) * wide];
+    }
+#pragma unroll
+    for (int s = 0; s < STEPS; ++s)       // (a part without keys left its sums unwritten: passed over by selection)
+      a[s] += x[s].x == -INFINITY || 4 * s + grp >= n_q ? 0.f : __expf(x[s].x - m[s]) * v[s];
+  }
+  floatx4 acc = (floatx4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int s = 0; s < STEPS; ++s) acc = TK_MFMA32(t[s], a[s] * inv[s], acc);
+#pragma unroll
+  for (int r = 0; r < 4; ++r) sum_s[wave][r][lane] = acc[r];
+  __syncthreads();
+  if (wave > 0) return;
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    acc[r] = 0.f;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) acc[r] += sum_s[w][r][lane];
+  }
+  talking_store(out, acc, row, n_q, dv, head0, heads, column, grp);
 }
 
 static int launch_finish(const void* part_o, const void* part_ml, const void* talk, const void* rows, const void* tiles,
                          const void* cu_q, void* out, int items, int n_q, int n_kv, int dv, int parts, hipStream_t stream) {
-  dim3 grid(items, n_kv, (dv + WAVE - 1) / WAVE);
-  const size_t lds = sizeof(float) * n_q * WAVE;
-#define FINISH(NWV) talking_finish_kernel<NWV><<<grid, NWV * WAVE, lds, stream>>>((const float*)part_o, (const float*)part_ml, \
-      (const float*)talk, (const int*)rows, (const int*)tiles, (const int*)cu_q, (bf16_t*)out, n_q, n_kv, dv, parts)
-  if (parts > 2 || items <= 64) FINISH(16); else FINISH(4);
+  const int blocks = n_kv * ((n_q / n_kv + 15) / 16);
+#define MIX(SV) talking_mix_kernel<SV><<<dim3((items + 15) / 16, blocks), 4 * WAVE, 0, stream>>>((const float*)part_o,          \
+      (const float*)part_ml, (const float*)talk, (const int*)rows, (const int*)tiles, (const int*)cu_q, (bf16_t*)out, items,    \
+      n_q, n_kv, dv)
+#define MERGE(SV) talking_merge_mix_kernel<SV, 8><<<dim3(items, blocks, (dv + 15) / 16), 8 * WAVE, 0, stream>>>(                \
+      (const float*)part_o, (const float*)part_ml, (const float*)talk, (const int*)rows, (const int*)tiles, (const int*)cu_q,   \
+      (bf16_t*)out, n_q, n_kv, dv, parts)
+#define FINISH(SV) if (parts == 1) MIX(SV); else MERGE(SV)
+  if (n_q <= 16) { FINISH(4); } else if (n_q <= 32) { FINISH(8); } else { FINISH(16); }
 #undef FINISH
+#undef MERGE
+#undef MIX
   return LAUNCH_STATUS();
 }
 

@@ -339,12 +339,12 @@ retention_chunk_carry_kernel(float* __restrict__ state, size_t state_stride, con
   float x = first_position[e] == 0 ? 0.f : *mine;
   const size_t step = (size_t)heads * plane;
   float* src = local + ((size_t)base * heads + h) * plane + idx;
-  for (int c0 = 0; c0 < count; c0 += 8) {
-    float now[8];
+  for (int c0 = 0; c0 < count; c0 += 16) {
+    float now[16];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) now[i] = c0 + i < count ? src[(size_t)(c0 + i) * step] : 0.f;
+    for (int i = 0; i < 16; ++i) now[i] = c0 + i < count ? src[(size_t)(c0 + i) * step] : 0.f;
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
+    for (int i = 0; i < 16; ++i) {
       if (c0 + i >= count) continue;
       src[(size_t)(c0 + i) * step] = x;
       x = fmaf(c0 + i == count - 1 ? rest : whole, x, now[i]);
