@@ -135,13 +135,7 @@ extern "C" int ta_talking_attention_generic(const void* q, int q_stride, void* o
 }
 
 // ---------------------------------------------------------------------------------------------------------------
-// The matrix-core form for bfloat16.  The mix commutes with the product with the values: with
-// A_g = sum_j p_g(j) V(j) over the values of ALL kv heads side by side (W = n_kv dv numbers), head h's output is
-// sum_g talk[h, g] times A_g's part at h's own kv head.  So every head is an ordinary softmax over its own keys against
-// values W wide, in one walk over the keys, and the mix is a small product at the end (`talking_mix_kernel`), in float.
-// The value pages hold exactly these wide values: a page's [n_kv, dv, page_size] read as [W, page_size].
-// Both kernels leave, per (token, part of its keys, head), the unnormalised sums [W] with the maximum and the sum of
-// exponentials they stand under: part_o float [items, parts, n_q, W], part_ml float [items, parts, n_q, 2].
+// The matrix-core form for bfloat16.
 
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float floatx4 __attribute__((ext_vector_type(4)));
@@ -180,46 +174,167 @@ struct TalkPages {
   __device__ __forceinline__ int slot(int key) const { return shift >= 0 ? key & (size - 1) : key % size; }
 };
 
-// Single tokens.  A workgroup a (part of the keys, token), all heads and all value columns: first the scores of every
-// head over the part (a wave a kv head's block of 32 keys at a time, up to sixteen heads the N side of the instruction)
-// into LDS, then maximum, exponentials and sum head by head, then O^T = V^T P^T, a wave sixteen of the W value rows at
-// a time for all heads.  The values of a wave's next rows are asked for while it works on the current ones, the first
-// before the scores.  HB: blocks of sixteen heads.  d a multiple of 8 up to 256; split_keys a multiple of 32 up to 256.
-// Dynamic LDS: 16 HB rows of (split_keys + 4) floats, then 16 HB rows of (split_keys + 8) bfloat16.
+// Single tokens, in two passes over the keys' parts, since a part's weights can be mixed once every head's maximum and sum over
+// all parts are known: the scores of every part from its keys, then the mixed weights of every part onto its values.
+// d a multiple of 8 up to 256; split_keys a multiple of 32 up to 256.
 #define TKD_BLOCKS 8
-template <int NW, int HB>
-__global__ void __launch_bounds__(NW * WAVE)
-talking_decode_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ k_pages,
-                      const bf16_t* __restrict__ vt_pages, const int* __restrict__ rows, const int* __restrict__ positions,
-                      const int* __restrict__ entry_of_token, const int* __restrict__ block_table, int table_stride,
-                      float* __restrict__ part_o, float* __restrict__ part_ml, int n_q, int n_kv, int d, int wide,
-                      int page_size, float scale, int split_keys, int splits) {
-  HELD(q, q_stride, k_pages, vt_pages, rows, positions, entry_of_token, block_table, table_stride, part_o, part_ml, n_q,
-       n_kv, d, wide, page_size, scale, split_keys, splits);
-  extern __shared__ __attribute__((aligned(16))) char tkd_lds[];
-  const int s_ld = split_keys + 4, p_ld = split_keys + 8;
-  float* s_s = reinterpret_cast<float*>(tkd_lds);
-  bf16_t* p_s = reinterpret_cast<bf16_t*>(tkd_lds + sizeof(float) * 16 * HB * s_ld);
-  const int split = blockIdx.x, item = blockIdx.y;
+
+// A workgroup a (part of the keys, kv head and block of sixteen of its heads, token): scores, a wave a block of 32 keys at a
+// time (the heads the N side of the instruction), through LDS to exponentials under the part's own maximum.
+// e: float [items, splits, n_q, split_keys]; part_ml: float [items, splits, n_q, 2], maximum and sum (-inf and 0 for a part
+// past the token).
+__global__ void __launch_bounds__(4 * WAVE)
+talking_scores_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ k_pages,
+                      const int* __restrict__ rows, const int* __restrict__ positions, const int* __restrict__ entry_of_token,
+                      const int* __restrict__ block_table, int table_stride, float* __restrict__ e, float* __restrict__ part_ml,
+                      int n_q, int n_kv, int d, int page_size, float scale, int split_keys, int splits) {
+  HELD(q, q_stride, k_pages, rows, positions, entry_of_token, block_table, table_stride, e, part_ml, n_q, n_kv, d, page_size,
+       scale, split_keys, splits);
+  __shared__ __attribute__((aligned(16))) float s_s[16][32 * TKD_BLOCKS + 4];
+  const int split = blockIdx.x, item = blockIdx.z;
   const int t = rows ? scalar_int(rows + item) : item;
   if (t < 0) return;                                       // a row that only fills the list up
   const int lane = threadIdx.x & 63, wave = wave_index(), col = lane & 15, g = lane >> 4;
   const int* table = block_table + (size_t)(entry_of_token ? scalar_int(entry_of_token + t) : t) * table_stride;
   const int pos = scalar_int(positions + t), first = split * split_keys, last = min(pos, first + split_keys - 1);
+  const int group = n_q / n_kv, head_blocks = (group + 15) / 16;
+  const int kvh = blockIdx.y / head_blocks, hb = blockIdx.y - kvh * head_blocks;
+  const int heads = min(16, group - hb * 16), head0 = kvh * group + hb * 16;
   const size_t part = (size_t)item * splits + split;
-  if (first > pos) {                                       // no key of the token lies here
-    for (int h = threadIdx.x; h < n_q; h += NW * WAVE) {
-      part_ml[(part * n_q + h) * 2] = -INFINITY;
-      part_ml[(part * n_q + h) * 2 + 1] = 0.f;
+  if (first > pos) {
+    if ((int)threadIdx.x < heads) {
+      part_ml[(part * n_q + head0 + threadIdx.x) * 2] = -INFINITY;
+      part_ml[(part * n_q + head0 + threadIdx.x) * 2 + 1] = 0.f;
     }
     return;
   }
   const TalkPages pages(page_size);
-  const int blocks = (last - first) / 32 + 1, group = n_q / n_kv, head_blocks = (group + 15) / 16;
+  const int blocks = (last - first) / 32 + 1;
+  const bool has = col < heads;
+  const bf16_t* qr = q + (size_t)t * q_stride + (size_t)(head0 + (has ? col : 0)) * d + 8 * g;
+  for (int b = wave; b < blocks; b += 4) {
+    const int kb = first + 32 * b;
+    const bool there1 = kb + 16 <= last;                   // (a half without keys borrows the other's page; its scores are masked)
+    const int kb1 = there1 ? kb + 16 : kb;
+    const int page0 = scalar_int(table + pages.page(kb)), page1 = scalar_int(table + pages.page(kb1));
+    const bf16_t* k0 = k_pages + (((size_t)page0 * n_kv + kvh) * page_size + pages.slot(kb) + col) * d + 8 * g;
+    const bf16_t* k1 = k_pages + (((size_t)page1 * n_kv + kvh) * page_size + pages.slot(kb1) + col) * d + 8 * g;
+    floatx4 st[2] = {(floatx4){0.f, 0.f, 0.f, 0.f}, (floatx4){0.f, 0.f, 0.f, 0.f}};
+    for (int ks0 = 0; ks0 * 32 < d; ks0 += 4) {
+      bf16x8 kf0[4], kf1[4], qf[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int at = (ks0 + i) * 32;
+        const bool in = at + 8 * g < d;
+        kf0[i] = kf1[i] = qf[i] = tk_zero8();
+        if (in) {
+          kf0[i] = *reinterpret_cast<const bf16x8*>(k0 + at);
+          kf1[i] = *reinterpret_cast<const bf16x8*>(k1 + at);
+        }
+        if (in && has) qf[i] = *reinterpret_cast<const bf16x8*>(qr + at);
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        st[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf0[i], qf[i], st[0], 0, 0, 0);
+        st[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf1[i], qf[i], st[1], 0, 0, 0);
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const int key = kb + 16 * u + 4 * g;
+      float4 s;
+      s.x = key <= last ? st[u][0] * scale : -INFINITY;
+      s.y = key + 1 <= last ? st[u][1] * scale : -INFINITY;
+      s.z = key + 2 <= last ? st[u][2] * scale : -INFINITY;
+      s.w = key + 3 <= last ? st[u][3] * scale : -INFINITY;
+      *reinterpret_cast<float4*>(&s_s[col][key - first]) = s;
+    }
+  }
+  __syncthreads();
+  // Maximum, exponentials and sum: sixteen lanes a head, four heads a wave.  (The part's first key is seen, so every maximum
+  // is a number.)
+  const int h = wave * 4 + g;
+  float s[2 * TKD_BLOCKS], m = -INFINITY, l = 0.f;
+#pragma unroll
+  for (int i = 0; i < 2 * TKD_BLOCKS; ++i) {
+    s[i] = i < 2 * blocks ? s_s[h][col + 16 * i] : -INFINITY;
+    m = fmaxf(m, s[i]);
+  }
+  m = tk_row_max16(m);
+  float* to = e + (part * n_q + head0 + h) * split_keys + col;
+#pragma unroll
+  for (int i = 0; i < 2 * TKD_BLOCKS; ++i) {
+    if (i >= 2 * blocks) continue;
+    const float p = s[i] == -INFINITY ? 0.f : __expf(s[i] - m);
+    l += p;
+    if (h < heads) to[16 * i] = p;
+  }
+  l = tk_row_sum16(l);
+  if (col == 0 && h < heads) {
+    part_ml[(part * n_q + head0 + h) * 2] = m;
+    part_ml[(part * n_q + head0 + h) * 2 + 1] = l;
+  }
+}
+
+#define TK_MFMA32(a, b, c) __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0)
+
+// Every head's maximum over the parts and one over its sum under it, into m_s and inv_s: sixteen lanes a head, lane `col` parts
+// col, col + 16, ....  ml: (maximum, sum) of part 0 of the item.
+template <int NW>
+__device__ __forceinline__ void talking_totals(const float2* __restrict__ ml, int n_q, int parts, float* m_s, float* inv_s,
+                                               int wave, int col, int grp) {
+  for (int g0 = wave * 4; g0 < n_q; g0 += NW * 4) {
+    const int g = min(g0 + grp, n_q - 1);
+    float m = -INFINITY, l = 0.f;
+    for (int p0 = col; p0 < parts; p0 += 64) {
+      float2 x[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) x[i] = p0 + 16 * i < parts ? ml[(size_t)(p0 + 16 * i) * n_q + g] : make_float2(-INFINITY, 0.f);
+      float top = m;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) top = fmaxf(top, x[i].x);
+      if (top == -INFINITY) continue;
+      l = m == -INFINITY ? 0.f : l * __expf(m - top);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) l += x[i].x == -INFINITY ? 0.f : x[i].y * __expf(x[i].x - top);
+      m = top;
+    }
+    const float big = tk_row_max16(m);
+    l = tk_row_sum16(m == -INFINITY ? 0.f : l * __expf(m - big));
+    if (col == 0 && g0 + grp < n_q) { m_s[g] = big; inv_s[g] = 1.0f / l; }
+  }
+}
+
+// A workgroup a (part, kv head and block of sixteen of its heads, token): the part's weights of all heads g (exponentials times
+// what brings them under the heads' totals), mixed by the rows of the talk table (float products on the matrix cores: heads
+// the M side, sixteen keys the N side, g the contraction), rounded to bfloat16 once, onto the kv head's values.  part_o: float
+// [items, splits, n_q, dv], plain sums (nothing where the part lies past the token).
+template <int STEPS>
+__global__ void __launch_bounds__(4 * WAVE)
+talking_values_kernel(const float* __restrict__ e, const float* __restrict__ part_ml, const float* __restrict__ talk,
+                      const bf16_t* __restrict__ vt_pages, const int* __restrict__ rows, const int* __restrict__ positions,
+                      const int* __restrict__ entry_of_token, const int* __restrict__ block_table, int table_stride,
+                      float* __restrict__ part_o, int n_q, int n_kv, int dv, int page_size, int split_keys, int splits) {
+  HELD(e, part_ml, talk, vt_pages, rows, positions, entry_of_token, block_table, table_stride, part_o, n_q, n_kv, dv, page_size,
+       split_keys, splits);
+  __shared__ float m_s[4 * STEPS], inv_s[4 * STEPS];
+  __shared__ __attribute__((aligned(16))) bf16_t w_s[16][32 * TKD_BLOCKS + 8];
+  const int split = blockIdx.x, item = blockIdx.z;
+  const int t = rows ? scalar_int(rows + item) : item;
+  if (t < 0) return;
+  const int lane = threadIdx.x & 63, wave = wave_index(), col = lane & 15, g = lane >> 4;
+  const int* table = block_table + (size_t)(entry_of_token ? scalar_int(entry_of_token + t) : t) * table_stride;
+  const int pos = scalar_int(positions + t), first = split * split_keys, last = min(pos, first + split_keys - 1);
+  if (first > pos) return;
+  const int group = n_q / n_kv, head_blocks = (group + 15) / 16;
+  const int kvh = blockIdx.y / head_blocks, hb = blockIdx.y - kvh * head_blocks;
+  const int heads = min(16, group - hb * 16), head0 = kvh * group + hb * 16;
+  const TalkPages pages(page_size);
+  const int blocks = (last - first) / 32 + 1;
   union VFrag { uint4 bits; bf16x8 v; };
-  // Rows rb * 16 .. + 15 of the wide values over the part's keys: lane (col, g) has row col, keys 8 g .. 8 g + 7 of a block.
+  // Value rows rb * 16 .. + 15 over the part's keys: lane (col, g) has row col, keys 8 g .. 8 g + 7 of a block of 32.
   auto load_values = [&](VFrag (&vf)[TKD_BLOCKS], int rb) {
-    const int row = min(rb * 16 + col, wide - 1);          // (a row past the last repeats it and is not written)
+    const int row = min(rb * 16 + col, dv - 1);            // (a row past the last repeats it and is not written)
 #pragma unroll
     for (int b = 0; b < TKD_BLOCKS; ++b) {
       vf[b].bits = make_uint4(0, 0, 0, 0);
@@ -228,94 +343,51 @@ talking_decode_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* 
       const bool there1 = kb + 16 <= last;                 // (a half without keys borrows the other's page; its values are zeroed)
       const int page0 = scalar_int(table + pages.page(kb)), page1 = scalar_int(table + pages.page(there1 ? kb + 16 : kb));
       const int slot0 = pages.slot(kb), slot1 = pages.slot(kb + 16);
-      const uint32_t at = ((uint32_t)((g >> 1) ? page1 : page0) * wide + row) * page_size + ((g >> 1) ? slot1 : slot0) + 8 * (g & 1);
+      const uint32_t at = (((uint32_t)((g >> 1) ? page1 : page0) * n_kv + kvh) * dv + row) * page_size + ((g >> 1) ? slot1 : slot0) + 8 * (g & 1);
       vf[b].bits = *reinterpret_cast<const uint4*>(vt_pages + at);
     }
   };
-  const int row_blocks = (wide + 15) / 16;
-  VFrag vf[TKD_BLOCKS], vn[TKD_BLOCKS];
-  if (wave < row_blocks) load_values(vf, wave);
-  // Scores.
-  for (int unit = wave; unit < n_kv * blocks; unit += NW) {
-    const int kvh = unit % n_kv, kb = first + 32 * (unit / n_kv);
-    const bool there1 = kb + 16 <= last;
-    const int page0 = scalar_int(table + pages.page(kb)), page1 = scalar_int(table + pages.page(there1 ? kb + 16 : kb));
-    const bf16_t* k0 = k_pages + (((size_t)page0 * n_kv + kvh) * page_size + pages.slot(kb) + col) * d + 8 * g;
-    const bf16_t* k1 = k_pages + (((size_t)page1 * n_kv + kvh) * page_size + pages.slot(there1 ? kb + 16 : kb) + col) * d + 8 * g;
-    for (int hb = 0; hb < head_blocks; ++hb) {
-      const int head = kvh * group + hb * 16 + col;
-      const bool has = hb * 16 + col < group;
-      const bf16_t* qr = q + (size_t)t * q_stride + (size_t)(has ? head : 0) * d + 8 * g;
-      floatx4 st[2] = {(floatx4){0.f, 0.f, 0.f, 0.f}, (floatx4){0.f, 0.f, 0.f, 0.f}};
-      for (int ks0 = 0; ks0 * 32 < d; ks0 += 4) {
-        bf16x8 kf0[4], kf1[4], qf[4];
+  const int row_blocks = (dv + 15) / 16;
+  VFrag vf[TKD_BLOCKS];
+  if (wave < row_blocks) load_values(vf, wave);            // on their way while the weights are made
+  const size_t part = (size_t)item * splits + split;
+  const float* src = e + part * n_q * split_keys;
+  float a[STEPS];                                          // the talk table's rows of this block of heads
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int at = (ks0 + i) * 32;
-          const bool in = at + 8 * g < d;
-          kf0[i] = kf1[i] = qf[i] = tk_zero8();
-          if (in) {
-            kf0[i] = *reinterpret_cast<const bf16x8*>(k0 + at);
-            kf1[i] = *reinterpret_cast<const bf16x8*>(k1 + at);
-          }
-          if (in && has) qf[i] = *reinterpret_cast<const bf16x8*>(qr + at);
-        }
+  for (int s = 0; s < STEPS; ++s) {
+    const int gg = 4 * s + g;
+    a[s] = (col < heads && gg < n_q) ? talk[(size_t)(head0 + col) * n_q + gg] : 0.f;
+  }
+  // A wave's first block of sixteen keys is asked for beside the totals.
+  const int key_blocks = 2 * blocks;
+  float x[STEPS];
+  auto load_weights = [&](int kb16) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          st[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf0[i], qf[i], st[0], 0, 0, 0);
-          st[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf1[i], qf[i], st[1], 0, 0, 0);
-        }
-      }
-      if (has) {
+    for (int s = 0; s < STEPS; ++s) x[s] = 4 * s + g < n_q ? src[(size_t)(4 * s + g) * split_keys + 16 * kb16 + col] : 0.f;
+  };
+  if (wave < key_blocks) load_weights(wave);
+  talking_totals<4>(reinterpret_cast<const float2*>(part_ml) + (size_t)item * splits * n_q, n_q, splits, m_s, inv_s, wave, col, g);
+  float mine[STEPS];                                       // (maximum of this part, asked for with the totals)
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {
-          const int key = kb + 16 * u + 4 * g;
-          float4 s;
-          s.x = key <= last ? st[u][0] * scale : -INFINITY;
-          s.y = key + 1 <= last ? st[u][1] * scale : -INFINITY;
-          s.z = key + 2 <= last ? st[u][2] * scale : -INFINITY;
-          s.w = key + 3 <= last ? st[u][3] * scale : -INFINITY;
-          *reinterpret_cast<float4*>(s_s + (size_t)head * s_ld + key - first) = s;
-        }
-      }
-    }
+  for (int s = 0; s < STEPS; ++s) mine[s] = part_ml[(part * n_q + min(4 * s + g, n_q - 1)) * 2];
+  __syncthreads();
+#pragma unroll
+  for (int s = 0; s < STEPS; ++s) {
+    const int gg = min(4 * s + g, n_q - 1);
+    mine[s] = 4 * s + g < n_q ? __expf(mine[s] - m_s[gg]) * inv_s[gg] : 0.f;
+  }
+  for (int kb16 = wave; kb16 < key_blocks; kb16 += 4) {
+    if (kb16 != wave) load_weights(kb16);
+    floatx4 w = (floatx4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < STEPS; ++s) w = TK_MFMA32(a[s], x[s] * mine[s], w);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) st(&w_s[4 * g + r][16 * kb16 + col], w[r]);      // (rows past the last head hold zeros)
   }
   __syncthreads();
-  // Maximum, exponentials and sum: sixteen lanes a head.  (Key 0 of the part is seen, so every maximum is a number.)
-  for (int h0 = wave * 4; h0 < 16 * HB; h0 += NW * 4) {
-    const int h = h0 + g;
-    const bool live = h < n_q;
-    const float* row = s_s + (size_t)h * s_ld + col;
-    float s[2 * TKD_BLOCKS], m = -INFINITY, l = 0.f;
-#pragma unroll
-    for (int i = 0; i < 2 * TKD_BLOCKS; ++i) {
-      s[i] = -INFINITY;
-      if (i < 2 * blocks && live) s[i] = row[16 * i];
-      m = fmaxf(m, s[i]);
-    }
-    m = tk_row_max16(m);
-    bf16_t* to = p_s + (size_t)h * p_ld + col;
-#pragma unroll
-    for (int i = 0; i < 2 * TKD_BLOCKS; ++i) {
-      if (i >= 2 * blocks) continue;
-      const float p = s[i] == -INFINITY ? 0.f : __expf(s[i] - m);
-      l += p;
-      st(to + 16 * i, p);
-    }
-    l = tk_row_sum16(l);
-    if (col == 0 && live) {
-      part_ml[(part * n_q + h) * 2] = m;
-      part_ml[(part * n_q + h) * 2 + 1] = l;
-    }
-  }
-  __syncthreads();
-  // The wide values.
-  for (int rb = wave; rb < row_blocks; rb += NW) {
-    const bool more = rb + NW < row_blocks;
-    if (more) load_values(vn, rb + NW);
-    floatx4 acc[HB];
-#pragma unroll
-    for (int hb = 0; hb < HB; ++hb) acc[hb] = (floatx4){0.f, 0.f, 0.f, 0.f};
+  for (int rb = wave; rb < row_blocks; rb += 4) {
+    if (rb != wave) load_values(vf, rb);
+    floatx4 acc = (floatx4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int b = 0; b < TKD_BLOCKS; ++b) {
       if (b >= blocks) continue;
@@ -328,34 +400,61 @@ talking_decode_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t* 
         if (left < 6) v.w = 0; else v.w &= 0xffffu;
         vf[b].bits = v;
       }
-#pragma unroll
-      for (int hb = 0; hb < HB; ++hb) {
-        const bf16x8 pf = *reinterpret_cast<const bf16x8*>(p_s + (size_t)(hb * 16 + col) * p_ld + 32 * b + 8 * g);
-        acc[hb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[b].v, pf, acc[hb], 0, 0, 0);
-      }
+      const bf16x8 pf = *reinterpret_cast<const bf16x8*>(&w_s[col][32 * b + 8 * g]);
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[b].v, pf, acc, 0, 0, 0);
     }
     const int row = rb * 16 + 4 * g;
-#pragma unroll
-    for (int hb = 0; hb < HB; ++hb) {
-      const int head = hb * 16 + col;
-      if (head >= n_q) continue;
-      float* dst = part_o + (part * n_q + head) * wide + row;
-      if (wide % 4 == 0) {
-        if (row < wide) *reinterpret_cast<float4*>(dst) = make_float4(acc[hb][0], acc[hb][1], acc[hb][2], acc[hb][3]);
+    if (col < heads) {
+      float* dst = part_o + (part * n_q + head0 + col) * dv + row;
+      if (dv % 4 == 0) {
+        if (row < dv) *reinterpret_cast<float4*>(dst) = make_float4(acc[0], acc[1], acc[2], acc[3]);
       } else {
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          if (row + r < wide) dst[r] = acc[hb][r];
+          if (row + r < dv) dst[r] = acc[r];
       }
-    }
-    if (more) {
-#pragma unroll
-      for (int b = 0; b < TKD_BLOCKS; ++b) vf[b].bits = vn[b].bits;
     }
   }
 }
 
-// Prompt portions.  A workgroup a (tile of sixteen tokens, kv head, block of 4 HG of its query heads, slab of 16 VB of the
+// out[t, i] = the sum of part_o[item, p, i] over the parts with keys of the token.  A workgroup an (item, 64 of its n_q dv
+// outputs); its waves share the parts.
+#define TKS_WAVES 4
+__global__ void __launch_bounds__(TKS_WAVES * WAVE)
+talking_sum_kernel(const float* __restrict__ part_o, const int* __restrict__ rows, const int* __restrict__ positions,
+                   bf16_t* __restrict__ out, int outputs, int split_keys, int splits) {
+  __shared__ float sum_s[TKS_WAVES][WAVE];
+  const int item = blockIdx.y, lane = threadIdx.x & 63, wave = wave_index(), i = blockIdx.x * WAVE + lane;
+  const int t = rows ? scalar_int(rows + item) : item;
+  if (t < 0) return;
+  const int parts = min(splits, scalar_int(positions + t) / split_keys + 1);
+  const float* src = part_o + (size_t)item * splits * outputs + min(i, outputs - 1);
+  float sum = 0.f;
+  for (int p0 = wave; p0 < parts; p0 += TKS_WAVES * 8) {
+    float v[8];
+#pragma unroll
+    for (int x = 0; x < 8; ++x) v[x] = p0 + TKS_WAVES * x < parts ? src[(size_t)(p0 + TKS_WAVES * x) * outputs] : 0.f;
+#pragma unroll
+    for (int x = 0; x < 8; ++x) sum += v[x];
+  }
+  sum_s[wave][lane] = sum;
+  __syncthreads();
+  if (wave > 0 || i >= outputs) return;
+  sum = 0.f;
+#pragma unroll
+  for (int w = 0; w < TKS_WAVES; ++w) sum += sum_s[w][lane];
+  st(out + (size_t)t * outputs + i, sum);
+}
+
+// Prompt portions, in one walk over the keys: the mix commutes with the product with the values.  With A_g = sum_j p_g(j) V(j)
+// over the values of ALL kv heads side by side (W = n_kv dv numbers), head h's output is sum_g talk[h, g] times A_g's part at
+// h's own kv head.  So every head is an ordinary softmax over its own keys against values W wide, and the mix is a small
+// product at the end (`talking_mix_kernel`), in float.  The value pages hold exactly these wide values: a page's
+// [n_kv, dv, page_size] read as [W, page_size].  The kernel leaves, per (token, part of its keys, head), the unnormalised sums
+// [W] with the maximum and the sum of exponentials they stand under: part_o float [items, parts, n_q, W], part_ml float
+// [items, parts, n_q, 2].
+//
+// A workgroup a (tile of sixteen tokens, kv head, block of 4 HG of its query heads, slab of 16 VB of the
 // W value columns, part of the tile's keys); its four waves have HG heads each and walk the same blocks of KB keys, which
 // come from the pages once for all of them straight into LDS, two buffers deep (the next block is on its way while the
 // current one is worked on).  S^T = K Q^T and O^T = V^T P^T with 16x16x32 instructions, token index in `lane % 16`;
@@ -576,165 +675,86 @@ talking_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t*
   }
 }
 
-// The heads mixed: out of head h = sum_g talk[h, g] A_g at h's own kv head, float products on the matrix cores (16x16x4): the
-// sixteen heads of a block are the M side, sixteen value columns the N side, the heads g the contraction; lane (col, grp)
-// has row `col` of the talk table and column `col` of the A_g for g = 4 s + grp.  STEPS: steps of four heads g.
-#define TK_MFMA32(a, b, c) __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0)
-
-// The output row of item `item` (-1: none): rows, or with `tiles` (tile, token of the tile).
-__device__ __forceinline__ int talking_row(int item, const int* rows, const int* tiles, const int* cu_q) {
-  if (!tiles) return rows ? scalar_int(rows + item) : item;
-  const int tile = item >> 4, token = item & 15;
-  const int entry = scalar_int(tiles + 2 * tile), row0 = scalar_int(cu_q + entry) + scalar_int(tiles + 2 * tile + 1);
-  return token < scalar_int(cu_q + entry + 1) - row0 ? row0 + token : -1;
-}
-
-__device__ __forceinline__ void talking_store(bf16_t* out, const floatx4& acc, int row, int n_q, int dv, int head0, int heads,
-                                              int column, int grp) {
-#pragma unroll
-  for (int r = 0; r < 4; ++r)
-    if (4 * grp + r < heads && column < dv)
-      st(out + (size_t)row * n_q * dv + (size_t)(head0 + 4 * grp + r) * dv + column, acc[r]);
-}
-
-// Keys in one part: a wave four items one after another, for one (kv head, block of sixteen of its heads) and all its value
-// columns.
+// The parts of every head brought together and the heads mixed: out of head h = sum_g talk[h, g] A_g at h's own kv head, float
+// products on the matrix cores (16x16x4): the sixteen heads of a block are the M side, sixteen value columns the N side, the
+// heads g the contraction; lane (col, grp) has row `col` of the talk table and column `col` of the A_g for g = 4 s + grp.
+// STEPS: steps of four heads g.  A wave four tokens of a tile one after another, for one (kv head, block of sixteen of its
+// heads) and all its value columns.
 template <int STEPS>
 __global__ void __launch_bounds__(4 * WAVE)
 talking_mix_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, const float* __restrict__ talk,
-                   const int* __restrict__ rows, const int* __restrict__ tiles, const int* __restrict__ cu_q,
-                   bf16_t* __restrict__ out, int items, int n_q, int n_kv, int dv) {
-  const int lane = threadIdx.x & 63, wave = wave_index(), col = lane & 15, grp = lane >> 4;
+                   const int* __restrict__ tiles, const int* __restrict__ cu_q, bf16_t* __restrict__ out, int n_q, int n_kv,
+                   int dv, int parts) {
+  const int lane = threadIdx.x & 63, wave = wave_index(), col = lane & 15, grp = lane >> 4, tile = blockIdx.x;
   const int group = n_q / n_kv, head_blocks = (group + 15) / 16, wide = n_kv * dv;
   const int kvh = blockIdx.y / head_blocks, first = (blockIdx.y - kvh * head_blocks) * 16, heads = min(16, group - first);
   const int head0 = kvh * group + first;
+  const int entry = scalar_int(tiles + 2 * tile), row0 = scalar_int(cu_q + entry) + scalar_int(tiles + 2 * tile + 1);
+  const int n_valid = min(16, scalar_int(cu_q + entry + 1) - row0);
   float t[STEPS];
 #pragma unroll
   for (int s = 0; s < STEPS; ++s) {
     const int g = 4 * s + grp;
     t[s] = (col < heads && g < n_q) ? talk[(size_t)(head0 + col) * n_q + g] : 0.f;
   }
-  for (int x = 0; x < 4; ++x) {
-    const int item = (blockIdx.x * 4 + wave) * 4 + x;
-    if (item >= items) break;
-    const int row = talking_row(item, rows, tiles, cu_q);
-    if (row < 0) continue;
-    float inv[STEPS];
+  for (int token = 4 * wave; token < min(n_valid, 4 * wave + 4); ++token) {
+    const size_t base = ((size_t)tile * 16 + token) * parts * n_q;
+    const float2* ml = reinterpret_cast<const float2*>(part_ml) + base;
+    float m[STEPS], l[STEPS];
 #pragma unroll
-    for (int s = 0; s < STEPS; ++s) inv[s] = 4 * s + grp < n_q ? 1.0f / part_ml[((size_t)item * n_q + 4 * s + grp) * 2 + 1] : 0.f;
+    for (int s = 0; s < STEPS; ++s) {
+      const float2 x = ml[min(4 * s + grp, n_q - 1)];
+      m[s] = x.x;                                          // (the first part always has keys)
+      l[s] = x.y;
+    }
+    for (int p = 1; p < parts; ++p) {
+#pragma unroll
+      for (int s = 0; s < STEPS; ++s) {
+        const float2 x = ml[(size_t)p * n_q + min(4 * s + grp, n_q - 1)];
+        const float top = fmaxf(m[s], x.x);
+        l[s] = l[s] * __expf(m[s] - top) + (x.x == -INFINITY ? 0.f : x.y * __expf(x.x - top));
+        m[s] = top;
+      }
+    }
+#pragma unroll
+    for (int s = 0; s < STEPS; ++s) l[s] = 1.0f / l[s];
+    const float* src = part_o + base * wide + (size_t)kvh * dv;
     for (int c0 = 0; c0 < dv; c0 += 64) {
       float a[4][STEPS];
 #pragma unroll
-      for (int cb = 0; cb < 4; ++cb) {
-        const int column = c0 + 16 * cb + col;
+      for (int cb = 0; cb < 4; ++cb)
+#pragma unroll
+        for (int s = 0; s < STEPS; ++s) a[cb][s] = 0.f;
+      for (int p = 0; p < parts; ++p) {
+        float f[STEPS];
 #pragma unroll
         for (int s = 0; s < STEPS; ++s) {
-          a[cb][s] = 0.f;
-          if (4 * s + grp < n_q && column < dv) a[cb][s] = part_o[((size_t)item * n_q + 4 * s + grp) * wide + (size_t)kvh * dv + column];
+          const float top = ml[(size_t)p * n_q + min(4 * s + grp, n_q - 1)].x;
+          f[s] = 4 * s + grp >= n_q || top == -INFINITY ? 0.f : __expf(top - m[s]) * l[s];
+        }
+#pragma unroll
+        for (int cb = 0; cb < 4; ++cb) {
+          const float* from = src + (size_t)p * n_q * wide + min(c0 + 16 * cb + col, dv - 1);
+          float v[STEPS];
+#pragma unroll
+          for (int s = 0; s < STEPS; ++s) v[s] = from[(size_t)min(4 * s + grp, n_q - 1) * wide];
+#pragma unroll
+          for (int s = 0; s < STEPS; ++s) a[cb][s] += f[s] == 0.f ? 0.f : f[s] * v[s];   // (unwritten sums of a part without keys: by selection)
         }
       }
 #pragma unroll
       for (int cb = 0; cb < 4; ++cb) {
         floatx4 acc = (floatx4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int s = 0; s < STEPS; ++s) acc = TK_MFMA32(t[s], a[cb][s] * inv[s], acc);
-        talking_store(out, acc, row, n_q, dv, head0, heads, c0 + 16 * cb + col, grp);
+        for (int s = 0; s < STEPS; ++s) acc = TK_MFMA32(t[s], a[cb][s], acc);
+        const int column = c0 + 16 * cb + col;
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (4 * grp + r < heads && column < dv)
+            st(out + (size_t)(row0 + token) * n_q * dv + (size_t)(head0 + 4 * grp + r) * dv + column, acc[r]);
       }
     }
   }
-}
-
-// Keys in several parts: a workgroup an (item, kv head and block of sixteen of its heads, sixteen value columns).  First every
-// head's maximum and sum over the parts; then wave w brings parts w, w + NW, ... together under them and mixes what it has
-// (the mix is linear), and the waves' results are added up in LDS.
-template <int STEPS, int NW>
-__global__ void __launch_bounds__(NW * WAVE)
-talking_merge_mix_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, const float* __restrict__ talk,
-                         const int* __restrict__ rows, const int* __restrict__ tiles, const int* __restrict__ cu_q,
-                         bf16_t* __restrict__ out, int n_q, int n_kv, int dv, int parts) {
-  __shared__ float m_s[4 * STEPS], inv_s[4 * STEPS];
-  __shared__ float sum_s[NW][4][WAVE];
-  const int item = blockIdx.x, lane = threadIdx.x & 63, wave = wave_index(), col = lane & 15, grp = lane >> 4;
-  const int row = talking_row(item, rows, tiles, cu_q);
-  if (row < 0) return;
-  const int group = n_q / n_kv, head_blocks = (group + 15) / 16, wide = n_kv * dv;
-  const int kvh = blockIdx.y / head_blocks, first = (blockIdx.y - kvh * head_blocks) * 16, heads = min(16, group - first);
-  const int head0 = kvh * group + first, column = blockIdx.z * 16 + col;
-  const size_t base = (size_t)item * parts * n_q;
-  const float2* ml = reinterpret_cast<const float2*>(part_ml) + base;
-  float t[STEPS];
-#pragma unroll
-  for (int s = 0; s < STEPS; ++s) {
-    const int g = 4 * s + grp;
-    t[s] = (col < heads && g < n_q) ? talk[(size_t)(head0 + col) * n_q + g] : 0.f;
-  }
-  // Sixteen lanes a head: lane `col` parts col, col + 16, ...
-  for (int g0 = wave * 4; g0 < n_q; g0 += NW * 4) {
-    const int g = g0 + grp;
-    float m = -INFINITY, l = 0.f;
-    for (int p = col; p < parts; p += 16) {
-      const float2 x = g < n_q ? ml[(size_t)p * n_q + g] : make_float2(-INFINITY, 0.f);
-      const float top = fmaxf(m, x.x);
-      if (x.x != -INFINITY) { l = (m == -INFINITY ? 0.f : l * __expf(m - top)) + x.y * __expf(x.x - top); m = top; }
-    }
-    const float big = tk_row_max16(m);
-    l = tk_row_sum16(m == -INFINITY ? 0.f : l * __expf(m - big));
-    if (col == 0 && g < n_q) { m_s[g] = big; inv_s[g] = 1.0f / l; }
-  }
-  __syncthreads();
-  float a[STEPS], m[STEPS], inv[STEPS];
-#pragma unroll
-  for (int s = 0; s < STEPS; ++s) {
-    const bool in = 4 * s + grp < n_q;
-    a[s] = 0.f;
-    m[s] = in ? m_s[4 * s + grp] : 0.f;
-    inv[s] = in ? inv_s[4 * s + grp] : 0.f;
-  }
-  const float* src = part_o + base * wide + (size_t)kvh * dv + min(column, dv - 1);
-  for (int p = wave; p < parts; p += NW) {
-    float v[STEPS];
-    float2 x[STEPS];
-#pragma unroll
-    for (int s = 0; s < STEPS; ++s) {
-      const int g = min(4 * s + grp, n_q - 1);
-      x[s] = ml[(size_t)p * n_q + g];
-      v[s] = src[((size_t)p * n_q + g) * wide];
-    }
-#pragma unroll
-    for (int s = 0; s < STEPS; ++s)       // (a part without keys left its sums unwritten: passed over by selection)
-      a[s] += x[s].x == -INFINITY || 4 * s + grp >= n_q ? 0.f : __expf(x[s].x - m[s]) * v[s];
-  }
-  floatx4 acc = (floatx4){0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-  for (int s = 0; s < STEPS; ++s) acc = TK_MFMA32(t[s], a[s] * inv[s], acc);
-#pragma unroll
-  for (int r = 0; r < 4; ++r) sum_s[wave][r][lane] = acc[r];
-  __syncthreads();
-  if (wave > 0) return;
-#pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    acc[r] = 0.f;
-#pragma unroll
-    for (int w = 0; w < NW; ++w) acc[r] += sum_s[w][r][lane];
-  }
-  talking_store(out, acc, row, n_q, dv, head0, heads, column, grp);
-}
-
-static int launch_finish(const void* part_o, const void* part_ml, const void* talk, const void* rows, const void* tiles,
-                         const void* cu_q, void* out, int items, int n_q, int n_kv, int dv, int parts, hipStream_t stream) {
-  const int blocks = n_kv * ((n_q / n_kv + 15) / 16);
-#define MIX(SV) talking_mix_kernel<SV><<<dim3((items + 15) / 16, blocks), 4 * WAVE, 0, stream>>>((const float*)part_o,          \
-      (const float*)part_ml, (const float*)talk, (const int*)rows, (const int*)tiles, (const int*)cu_q, (bf16_t*)out, items,    \
-      n_q, n_kv, dv)
-#define MERGE(SV) talking_merge_mix_kernel<SV, 8><<<dim3(items, blocks, (dv + 15) / 16), 8 * WAVE, 0, stream>>>(                \
-      (const float*)part_o, (const float*)part_ml, (const float*)talk, (const int*)rows, (const int*)tiles, (const int*)cu_q,   \
-      (bf16_t*)out, n_q, n_kv, dv, parts)
-#define FINISH(SV) if (parts == 1) MIX(SV); else MERGE(SV)
-  if (n_q <= 16) { FINISH(4); } else if (n_q <= 32) { FINISH(8); } else { FINISH(16); }
-#undef FINISH
-#undef MERGE
-#undef MIX
-  return LAUNCH_STATUS();
 }
 
 // A launch that wants more dynamic LDS than every kernel may have says so first.
@@ -749,32 +769,30 @@ static bool talking_fits(int n_q, int n_kv, int d, int dv, int page_size) {
          (long)n_kv * dv <= 65536;
 }
 
-// Single tokens: items are the rows of `rows` (or every row); entry_of_token null: row e is entry e.  part_o float
-// [n_items, splits, n_q, n_kv dv], part_ml float [n_items, splits, n_q, 2].  Returns -2 for sizes without an instance.
+// Single tokens: items are the rows of `rows` (or every row); entry_of_token null: row e is entry e.  e float
+// [n_items, splits, n_q, split_keys], part_ml float [n_items, splits, n_q, 2], part_o float [n_items, splits, n_q, dv].
+// Returns -2 for sizes without an instance.
 extern "C" int ta_talking_decode_bf16(const void* q, int q_stride, void* out, const void* k_pages, const void* vt_pages,
                                       const void* rows, const void* positions, const void* entry_of_token,
-                                      const void* block_table, int table_stride, void* part_o, void* part_ml, const void* talk,
-                                      int n_items, int n_q, int n_kv, int d, int dv, int page_size, float scale, int split_keys,
-                                      int splits, hipStream_t stream) {
+                                      const void* block_table, int table_stride, void* e, void* part_ml, void* part_o,
+                                      const void* talk, int n_items, int n_q, int n_kv, int d, int dv, int page_size, float scale,
+                                      int split_keys, int splits, hipStream_t stream) {
   if (n_items <= 0) return 0;
   if (!talking_fits(n_q, n_kv, d, dv, page_size) || q_stride % 8) return -2;
   if (split_keys < 32 || split_keys % 32 || split_keys > 32 * TKD_BLOCKS || splits < 1 || splits > 0x7ffffff || n_items > 65535) return -1;
-  const int wide = n_kv * dv, hb = (n_q + 15) / 16;
-  dim3 grid(splits, n_items);
-#define DECODE(NWV, HBV)                                                                                                 \
-  const int lds = 16 * HBV * (4 * (split_keys + 4) + 2 * (split_keys + 8));       /* at most 101 KB */                    \
-  if (const int bad = allow_lds(reinterpret_cast<const void*>(&talking_decode_kernel<NWV, HBV>), lds)) return bad;         \
-  talking_decode_kernel<NWV, HBV><<<grid, NWV * WAVE, lds, stream>>>(                                                     \
-      (const bf16_t*)q, q_stride, (const bf16_t*)k_pages, (const bf16_t*)vt_pages, (const int*)rows, (const int*)positions, \
-      (const int*)entry_of_token, (const int*)block_table, table_stride, (float*)part_o, (float*)part_ml, n_q, n_kv, d, wide, \
-      page_size, scale, split_keys, splits)
-#define DECODES(HBV) if (wide >= 256) { DECODE(8, HBV); } else { DECODE(4, HBV); }
-  if (hb <= 1) { DECODES(1); } else if (hb <= 2) { DECODES(2); } else { DECODES(4); }
-#undef DECODES
-#undef DECODE
-  const int status = LAUNCH_STATUS();
-  if (status) return status;
-  return launch_finish(part_o, part_ml, talk, rows, nullptr, nullptr, out, n_items, n_q, n_kv, dv, splits, stream);
+  dim3 grid(splits, n_kv * ((n_q / n_kv + 15) / 16), n_items);
+  talking_scores_kernel<<<grid, 4 * WAVE, 0, stream>>>((const bf16_t*)q, q_stride, (const bf16_t*)k_pages, (const int*)rows,
+      (const int*)positions, (const int*)entry_of_token, (const int*)block_table, table_stride, (float*)e, (float*)part_ml, n_q,
+      n_kv, d, page_size, scale, split_keys, splits);
+#define VALUES(SV) talking_values_kernel<SV><<<grid, 4 * WAVE, 0, stream>>>((const float*)e, (const float*)part_ml,          \
+      (const float*)talk, (const bf16_t*)vt_pages, (const int*)rows, (const int*)positions, (const int*)entry_of_token,      \
+      (const int*)block_table, table_stride, (float*)part_o, n_q, n_kv, dv, page_size, split_keys, splits)
+  if (n_q <= 16) VALUES(4); else if (n_q <= 32) VALUES(8); else VALUES(16);
+#undef VALUES
+  const int outputs = n_q * dv;
+  talking_sum_kernel<<<dim3((outputs + WAVE - 1) / WAVE, n_items), TKS_WAVES * WAVE, 0, stream>>>((const float*)part_o,
+      (const int*)rows, (const int*)positions, (bf16_t*)out, outputs, split_keys, splits);
+  return LAUNCH_STATUS();
 }
 
 // What a launch over `n_tiles` tiles that reach `reach` keys is cut into: slabs of the value columns (16 * *blocks columns
@@ -829,5 +847,10 @@ extern "C" int ta_talking_prefill_bf16(const void* q, int q_stride, void* out, c
 #undef PREFILL
   const int status = LAUNCH_STATUS();
   if (status) return status;
-  return launch_finish(part_o, part_ml, talk, nullptr, tiles, cu_q, out, n_tiles * 16, n_q, n_kv, dv, parts, stream);
+  const dim3 grid(n_tiles, n_kv * ((group + 15) / 16));
+#define MIX(SV) talking_mix_kernel<SV><<<grid, 4 * WAVE, 0, stream>>>((const float*)part_o, (const float*)part_ml,             \
+      (const float*)talk, (const int*)tiles, (const int*)cu_q, (bf16_t*)out, n_q, n_kv, dv, parts)
+  if (n_q <= 16) MIX(4); else if (n_q <= 32) MIX(8); else MIX(16);
+#undef MIX
+  return LAUNCH_STATUS();
 }

@@ -1216,15 +1216,16 @@ class Ops:
                         page_size, scale, talk, reach, rows=None, identity_entries=False):
         """Single tokens of `talking_attention`: the keys cut over workgroups in parts of 64 to 256."""
         n_items = qkv.shape[0] if rows is None else rows.numel()
-        split_keys = min(256, max(64, -(-reach // max(1, self.talking_workgroups // max(1, n_items)))))
+        split_keys = min(256, max(64, -(-reach // max(1, self.talking_workgroups // max(1, n_items * n_kv)))))
         split_keys = -(-split_keys // 32) * 32
         splits = -(-reach // split_keys)
-        part_o = torch.empty((n_items, splits, n_q, n_kv * value_dim), dtype=torch.float32, device=qkv.device)
+        e = torch.empty((n_items, splits, n_q, split_keys), dtype=torch.float32, device=qkv.device)
         part_ml = torch.empty((n_items, splits, n_q, 2), dtype=torch.float32, device=qkv.device)
+        part_o = torch.empty((n_items, splits, n_q, value_dim), dtype=torch.float32, device=qkv.device)
         self._check(self.lib.ta_talking_decode_bf16(
             _ptr(qkv), qkv.stride(0), _ptr(out), _ptr(k_pages), _ptr(v_pages), _ptr(rows), _ptr(positions),
             _ptr(None if identity_entries and rows is None else entry_of_token), _ptr(block_table), block_table.shape[1],
-            _ptr(part_o), _ptr(part_ml), _ptr(talk), n_items, n_q, n_kv, head_dim, value_dim, page_size, ctypes.c_float(scale),
+            _ptr(e), _ptr(part_ml), _ptr(part_o), _ptr(talk), n_items, n_q, n_kv, head_dim, value_dim, page_size, ctypes.c_float(scale),
             split_keys, splits, self._stream()), "talking_decode")
         return out
 
