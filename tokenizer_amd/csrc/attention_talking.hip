@@ -678,81 +678,80 @@ talking_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t*
 // The parts of every head brought together and the heads mixed: out of head h = sum_g talk[h, g] A_g at h's own kv head, float
 // products on the matrix cores (16x16x4): the sixteen heads of a block are the M side, sixteen value columns the N side, the
 // heads g the contraction; lane (col, grp) has row `col` of the talk table and column `col` of the A_g for g = 4 s + grp.
-// STEPS: steps of four heads g.  A wave four tokens of a tile one after another, for one (kv head, block of sixteen of its
-// heads) and all its value columns.
+// STEPS: steps of four heads g.  A wave a token, for one (kv head, block of sixteen of its heads) and all its value columns;
+// four workgroups a tile.
 template <int STEPS>
 __global__ void __launch_bounds__(4 * WAVE)
 talking_mix_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, const float* __restrict__ talk,
                    const int* __restrict__ tiles, const int* __restrict__ cu_q, bf16_t* __restrict__ out, int n_q, int n_kv,
                    int dv, int parts) {
-  const int lane = threadIdx.x & 63, wave = wave_index(), col = lane & 15, grp = lane >> 4, tile = blockIdx.x;
+  const int lane = threadIdx.x & 63, wave = wave_index(), col = lane & 15, grp = lane >> 4;
+  const int tile = blockIdx.x >> 2, token = 4 * (blockIdx.x & 3) + wave;
   const int group = n_q / n_kv, head_blocks = (group + 15) / 16, wide = n_kv * dv;
   const int kvh = blockIdx.y / head_blocks, first = (blockIdx.y - kvh * head_blocks) * 16, heads = min(16, group - first);
   const int head0 = kvh * group + first;
   const int entry = scalar_int(tiles + 2 * tile), row0 = scalar_int(cu_q + entry) + scalar_int(tiles + 2 * tile + 1);
-  const int n_valid = min(16, scalar_int(cu_q + entry + 1) - row0);
+  if (token >= scalar_int(cu_q + entry + 1) - row0) return;
   float t[STEPS];
 #pragma unroll
   for (int s = 0; s < STEPS; ++s) {
     const int g = 4 * s + grp;
     t[s] = (col < heads && g < n_q) ? talk[(size_t)(head0 + col) * n_q + g] : 0.f;
   }
-  for (int token = 4 * wave; token < min(n_valid, 4 * wave + 4); ++token) {
-    const size_t base = ((size_t)tile * 16 + token) * parts * n_q;
-    const float2* ml = reinterpret_cast<const float2*>(part_ml) + base;
-    float m[STEPS], l[STEPS];
+  const size_t base = ((size_t)tile * 16 + token) * parts * n_q;
+  const float2* ml = reinterpret_cast<const float2*>(part_ml) + base;
+  float m[STEPS], l[STEPS];
+#pragma unroll
+  for (int s = 0; s < STEPS; ++s) {
+    const float2 x = ml[min(4 * s + grp, n_q - 1)];
+    m[s] = x.x;                                          // (the first part always has keys)
+    l[s] = x.y;
+  }
+  for (int p = 1; p < parts; ++p) {
 #pragma unroll
     for (int s = 0; s < STEPS; ++s) {
-      const float2 x = ml[min(4 * s + grp, n_q - 1)];
-      m[s] = x.x;                                          // (the first part always has keys)
-      l[s] = x.y;
+      const float2 x = ml[(size_t)p * n_q + min(4 * s + grp, n_q - 1)];
+      const float top = fmaxf(m[s], x.x);
+      l[s] = l[s] * __expf(m[s] - top) + (x.x == -INFINITY ? 0.f : x.y * __expf(x.x - top));
+      m[s] = top;
     }
-    for (int p = 1; p < parts; ++p) {
+  }
+#pragma unroll
+  for (int s = 0; s < STEPS; ++s) l[s] = 1.0f / l[s];
+  const float* src = part_o + base * wide + (size_t)kvh * dv;
+  for (int c0 = 0; c0 < dv; c0 += 64) {
+    float a[4][STEPS];
+#pragma unroll
+    for (int cb = 0; cb < 4; ++cb)
+#pragma unroll
+      for (int s = 0; s < STEPS; ++s) a[cb][s] = 0.f;
+    for (int p = 0; p < parts; ++p) {
+      float f[STEPS];
 #pragma unroll
       for (int s = 0; s < STEPS; ++s) {
-        const float2 x = ml[(size_t)p * n_q + min(4 * s + grp, n_q - 1)];
-        const float top = fmaxf(m[s], x.x);
-        l[s] = l[s] * __expf(m[s] - top) + (x.x == -INFINITY ? 0.f : x.y * __expf(x.x - top));
-        m[s] = top;
-      }
-    }
-#pragma unroll
-    for (int s = 0; s < STEPS; ++s) l[s] = 1.0f / l[s];
-    const float* src = part_o + base * wide + (size_t)kvh * dv;
-    for (int c0 = 0; c0 < dv; c0 += 64) {
-      float a[4][STEPS];
-#pragma unroll
-      for (int cb = 0; cb < 4; ++cb)
-#pragma unroll
-        for (int s = 0; s < STEPS; ++s) a[cb][s] = 0.f;
-      for (int p = 0; p < parts; ++p) {
-        float f[STEPS];
-#pragma unroll
-        for (int s = 0; s < STEPS; ++s) {
-          const float top = ml[(size_t)p * n_q + min(4 * s + grp, n_q - 1)].x;
-          f[s] = 4 * s + grp >= n_q || top == -INFINITY ? 0.f : __expf(top - m[s]) * l[s];
-        }
-#pragma unroll
-        for (int cb = 0; cb < 4; ++cb) {
-          const float* from = src + (size_t)p * n_q * wide + min(c0 + 16 * cb + col, dv - 1);
-          float v[STEPS];
-#pragma unroll
-          for (int s = 0; s < STEPS; ++s) v[s] = from[(size_t)min(4 * s + grp, n_q - 1) * wide];
-#pragma unroll
-          for (int s = 0; s < STEPS; ++s) a[cb][s] += f[s] == 0.f ? 0.f : f[s] * v[s];   // (unwritten sums of a part without keys: by selection)
-        }
+        const float top = ml[(size_t)p * n_q + min(4 * s + grp, n_q - 1)].x;
+        f[s] = 4 * s + grp >= n_q || top == -INFINITY ? 0.f : __expf(top - m[s]) * l[s];
       }
 #pragma unroll
       for (int cb = 0; cb < 4; ++cb) {
-        floatx4 acc = (floatx4){0.f, 0.f, 0.f, 0.f};
+        const float* from = src + (size_t)p * n_q * wide + min(c0 + 16 * cb + col, dv - 1);
+        float v[STEPS];
 #pragma unroll
-        for (int s = 0; s < STEPS; ++s) acc = TK_MFMA32(t[s], a[cb][s], acc);
-        const int column = c0 + 16 * cb + col;
+        for (int s = 0; s < STEPS; ++s) v[s] = from[(size_t)min(4 * s + grp, n_q - 1) * wide];
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
-          if (4 * grp + r < heads && column < dv)
-            st(out + (size_t)(row0 + token) * n_q * dv + (size_t)(head0 + 4 * grp + r) * dv + column, acc[r]);
+        for (int s = 0; s < STEPS; ++s) a[cb][s] += f[s] == 0.f ? 0.f : f[s] * v[s];   // (unwritten sums of a part without keys: by selection)
       }
+    }
+#pragma unroll
+    for (int cb = 0; cb < 4; ++cb) {
+      floatx4 acc = (floatx4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int s = 0; s < STEPS; ++s) acc = TK_MFMA32(t[s], a[cb][s], acc);
+      const int column = c0 + 16 * cb + col;
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (4 * grp + r < heads && column < dv)
+          st(out + (size_t)(row0 + token) * n_q * dv + (size_t)(head0 + 4 * grp + r) * dv + column, acc[r]);
     }
   }
 }
@@ -804,7 +803,7 @@ static void talking_plan(int n_tiles, int n_q, int n_kv, int d, int dv, int reac
   *heads = (group > 4 && d <= 128) ? 2 : 1;
   const long groups = (long)n_tiles * n_kv * ((group + 4 * *heads - 1) / (4 * *heads)) * *slabs;
   int cut = 1;
-  while (cut < 16 && groups * cut < 512 && reach / (cut * 2) >= 256) cut *= 2;
+  while (cut < 16 && groups * cut < 1024 && reach / (cut * 2) >= 256) cut *= 2;
   *parts = cut;
 }
 
@@ -847,7 +846,7 @@ extern "C" int ta_talking_prefill_bf16(const void* q, int q_stride, void* out, c
 #undef PREFILL
   const int status = LAUNCH_STATUS();
   if (status) return status;
-  const dim3 grid(n_tiles, n_kv * ((group + 15) / 16));
+  const dim3 grid(n_tiles * 4, n_kv * ((group + 15) / 16));
 #define MIX(SV) talking_mix_kernel<SV><<<grid, 4 * WAVE, 0, stream>>>((const float*)part_o, (const float*)part_ml,             \
       (const float*)talk, (const int*)tiles, (const int*)cu_q, (bf16_t*)out, n_q, n_kv, dv, parts)
   if (n_q <= 16) MIX(4); else if (n_q <= 32) MIX(8); else MIX(16);

@@ -206,6 +206,86 @@ head_norm_rotate_store_kernel(T* __restrict__ qkv, int row_stride, const float* 
   }
 }
 
+// The same for bfloat16 heads in whole pieces of eight elements (d, dv and rot / 2 multiples of 8, everything 16-byte aligned):
+// LPH lanes a head, a piece a lane, so a wave has 64 / LPH heads of a token; a head's sum of squares goes over its LPH lanes,
+// and the piece that turns together with a lane's lies with another of them.
+template <int LPH>
+__global__ void __launch_bounds__(RP_THREADS)
+head_norm_rotate_store_vec_kernel(bf16_t* __restrict__ qkv, int row_stride, const float* __restrict__ table, int rot,
+                                  const int* __restrict__ slots, bf16_t* __restrict__ k_pages, bf16_t* __restrict__ v_pages,
+                                  int n_q, int n_k, int n_v, int d, int dv, int page_size, const float* __restrict__ q_norm,
+                                  const float* __restrict__ k_norm, int norm_values, const bf16_t* __restrict__ first,
+                                  int first_stride, const float* __restrict__ share, float eps) {
+  const int t = blockIdx.x, lane = threadIdx.x & (WAVE - 1), piece = lane % LPH;
+  const int head = (blockIdx.y * RP_THREADS + threadIdx.x) / LPH;
+  const bool there = head < n_q + n_k + n_v;                 // (lanes without a head go along: they take part in the exchanges)
+  const bool value = head >= n_q + n_k, key = !value && head >= n_q;
+  const int h = value ? head - n_q - n_k : key ? head - n_q : head, n = value ? dv : d, i = piece * 8;
+  const bool in = there && i < n;
+  bf16_t* at = qkv + (size_t)t * row_stride + (value ? (size_t)(n_q + n_k) * d + (size_t)h * dv : (size_t)head * d) + i;
+  const float* weight = value ? nullptr : key ? k_norm : q_norm;
+  const int slot = slots ? slots[t] : -1, half = rot / 2;
+  const bool turns = in && !value && i < rot, upper = i >= half;
+  uint4 raw = make_uint4(0, 0, 0, 0), other = make_uint4(0, 0, 0, 0);
+  float4 w0 = make_float4(1.f, 1.f, 1.f, 1.f), w1 = w0, c0 = w0, c1 = w0, s0 = make_float4(0.f, 0.f, 0.f, 0.f), s1 = s0;
+  if (in) raw = *reinterpret_cast<const uint4*>(at);
+  if (in && value && share) other = *reinterpret_cast<const uint4*>(first + (size_t)t * first_stride + (size_t)h * dv + i);
+  if (in && weight) { w0 = *reinterpret_cast<const float4*>(weight + i); w1 = *reinterpret_cast<const float4*>(weight + i + 4); }
+  if (turns) {
+    const float4* cs = reinterpret_cast<const float4*>(table + (size_t)t * rot + (upper ? i - half : i));
+    c0 = cs[0];
+    c1 = cs[1];
+    s0 = cs[half / 4];
+    s1 = cs[half / 4 + 1];
+  }
+  float x[8] = {bf16_bits_to_float(raw.x & 0xffffu), bf16_bits_to_float(raw.x >> 16), bf16_bits_to_float(raw.y & 0xffffu),
+                bf16_bits_to_float(raw.y >> 16), bf16_bits_to_float(raw.z & 0xffffu), bf16_bits_to_float(raw.z >> 16),
+                bf16_bits_to_float(raw.w & 0xffffu), bf16_bits_to_float(raw.w >> 16)};
+  float sq = 0.f;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) sq = fmaf(x[e], x[e], sq);
+#pragma unroll
+  for (int off = LPH / 2; off > 0; off >>= 1) sq += __shfl_xor(sq, off, WAVE);
+  if (weight || (value && norm_values)) {
+    const float inv = 1.0f / sqrtf(sq / (float)n + eps);
+    const float w[8] = {w0.x, w0.y, w0.z, w0.w, w1.x, w1.y, w1.z, w1.w};
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x[e] *= inv * w[e];
+  }
+  if (value && share) {
+    const float mix = share[0];
+    const float o[8] = {bf16_bits_to_float(other.x & 0xffffu), bf16_bits_to_float(other.x >> 16), bf16_bits_to_float(other.y & 0xffffu),
+                        bf16_bits_to_float(other.y >> 16), bf16_bits_to_float(other.z & 0xffffu), bf16_bits_to_float(other.z >> 16),
+                        bf16_bits_to_float(other.w & 0xffffu), bf16_bits_to_float(other.w >> 16)};
+#pragma unroll
+    for (int e = 0; e < 8; ++e) x[e] = (1.0f - mix) * x[e] + mix * o[e];
+  }
+  if (half > 0) {
+    const int partner = turns ? lane + (upper ? -half : half) / 8 : lane;
+    const float c[8] = {c0.x, c0.y, c0.z, c0.w, c1.x, c1.y, c1.z, c1.w}, sn[8] = {s0.x, s0.y, s0.z, s0.w, s1.x, s1.y, s1.z, s1.w};
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float with = __shfl(x[e], partner, WAVE);
+      x[e] = x[e] * c[e] + (upper ? with : -with) * sn[e];
+    }
+  }
+  if (!in) return;
+  uint32_t packed[4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+    packed[e] = (uint32_t)float_to_bf16_bits(x[2 * e]) | ((uint32_t)float_to_bf16_bits(x[2 * e + 1]) << 16);
+  const uint4 out = make_uint4(packed[0], packed[1], packed[2], packed[3]);
+  *reinterpret_cast<uint4*>(at) = out;
+  if (slot < 0) return;
+  const int page = slot / page_size, off = slot % page_size;
+  if (key) *reinterpret_cast<uint4*>(k_pages + (((size_t)page * n_k + h) * page_size + off) * d + i) = out;
+  if (value) {
+    bf16_t* to = v_pages + (((size_t)page * n_v + h) * dv + i) * page_size + off;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) to[(size_t)e * page_size].bits = (uint16_t)(packed[e >> 1] >> (16 * (e & 1)));
+  }
+}
+
 extern "C" int ta_rotation_table(const void* positions, const void* rates, float magnitude, int rot, void* table,
                                  int n_tokens, hipStream_t stream) {
   if (n_tokens <= 0 || rot <= 0) return 0;
@@ -225,6 +305,18 @@ extern "C" int ta_head_norm_rotate_store(void* qkv, int row_stride, const void* 
   if ((rot > 0 && !table) || (share && !first) || d > 8 * WAVE || dv > 8 * WAVE) return -1;
   const int waves = RP_THREADS / WAVE, most = d > dv ? d : dv;
   dim3 grid(n_tokens, (n_q + n_k + n_v + waves - 1) / waves);
+  const uintptr_t bases = (uintptr_t)qkv | (uintptr_t)table | (uintptr_t)k_pages | (uintptr_t)q_norm | (uintptr_t)k_norm |
+                          (share ? (uintptr_t)first : 0);
+  if (dtype == DT_BF16 && d % 8 == 0 && dv % 8 == 0 && rot % 16 == 0 && row_stride % 8 == 0 && most <= 256 && (bases & 15) == 0 &&
+      (!share || first_stride % 8 == 0)) {
+#define STORE_VEC(LL) head_norm_rotate_store_vec_kernel<LL><<<dim3(n_tokens, ((n_q + n_k + n_v) * LL + RP_THREADS - 1) / RP_THREADS), \
+      RP_THREADS, 0, stream>>>((bf16_t*)qkv, row_stride, (const float*)table, rot, (const int*)slots, (bf16_t*)k_pages,       \
+      (bf16_t*)v_pages, n_q, n_k, n_v, d, dv, page_size, (const float*)q_norm, (const float*)k_norm, norm_values,             \
+      (const bf16_t*)first, first_stride, (const float*)share, eps)
+    if (most <= 64) STORE_VEC(8); else if (most <= 128) STORE_VEC(16); else STORE_VEC(32);
+#undef STORE_VEC
+    return LAUNCH_STATUS();
+  }
 #define STORE(TT, PP) head_norm_rotate_store_kernel<TT, PP><<<grid, RP_THREADS, 0, stream>>>((TT*)qkv, row_stride,          \
       (const float*)table, rot, (const int*)slots, (TT*)k_pages, (TT*)v_pages, n_q, n_k, n_v, d, dv, page_size,              \
       (const float*)q_norm, (const float*)k_norm, norm_values, (const TT*)first, first_stride, (const float*)share, eps)
