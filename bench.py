@@ -371,7 +371,7 @@ def gafonex_config(sizes: dict, layers: int) -> dict:
     d, base = width // heads, float(sizes.get("rope_theta", 1e6))
     mlp = {"kind": "dense", "ff": sizes["intermediate_size"]}
     attention = {"heads": heads, "kv_heads": kv_heads, "dim": d, "vdim": d, "scale": d ** -0.5, "v_mix": True,
-                 "rot": {"dims": d, "base": base, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+                 "rot": {"dims": d, "base": base, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
     retention = {"heads": heads, "dim": d, "vdim": d, "decay": [1.0 - 2.0 ** (-5.0 - h % 8) for h in range(heads)],
                  "rot": {"dims": d, "base": base}}
     out = [{"type": "attention", "mixer": attention, "mlp": mlp} if index % 4 == 2 else

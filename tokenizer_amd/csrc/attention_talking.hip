@@ -343,7 +343,8 @@ talking_values_kernel(const float* __restrict__ e, const float* __restrict__ par
       const bool there1 = kb + 16 <= last;                 // (a half without keys borrows the other's page; its values are zeroed)
       const int page0 = scalar_int(table + pages.page(kb)), page1 = scalar_int(table + pages.page(there1 ? kb + 16 : kb));
       const int slot0 = pages.slot(kb), slot1 = pages.slot(kb + 16);
-      const uint32_t at = (((uint32_t)((g >> 1) ? page1 : page0) * n_kv + kvh) * dv + row) * page_size + ((g >> 1) ? slot1 : slot0) + 8 * (g & 1);
+      const uint32_t at = (((uint32_t)((g >> 1) ? page1 : page0) * n_kv + kvh) * dv + row) * page_size +
+                          ((g >> 1) ? slot1 : slot0) + 8 * (g & 1);
       vf[b].bits = *reinterpret_cast<const uint4*>(vt_pages + at);
     }
   };
@@ -621,7 +622,8 @@ talking_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, const bf16_t*
       for (int h = 0; h < HG; ++h) l[h] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf[h][u], l[h], 0, 0, 0);
 #pragma unroll
       for (int db = 0; db < VB; ++db) {
-        bf16x8 vf = *reinterpret_cast<const bf16x8*>(buf + B::K_BYTES + (2 * u + (g >> 1)) * B::V_RUN + (db * 16 + col) * 32 + (g & 1) * 16);
+        bf16x8 vf = *reinterpret_cast<const bf16x8*>(buf + B::K_BYTES + (2 * u + (g >> 1)) * B::V_RUN +
+                                                     (db * 16 + col) * 32 + (g & 1) * 16);
         if (!FULL) {                                        // slots nobody wrote may hold anything: 0 * NaN must stay 0
 #pragma unroll
           for (int i = 0; i < 8; ++i)

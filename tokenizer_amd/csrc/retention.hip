@@ -360,7 +360,8 @@ template <int DB, int VB, bool VEC>
 __global__ void __launch_bounds__(4 * WAVE)
 retention_chunk_read_kernel(const bf16_t* __restrict__ qkvg, int row_stride, const float* __restrict__ table, int rot,
                             const float* __restrict__ powers, const int* __restrict__ cu_q, int n_entries,
-                            const int* __restrict__ first_position, const float* __restrict__ start, bf16_t* __restrict__ out, int heads, int d,
+                            const int* __restrict__ first_position, const float* __restrict__ start,
+                            bf16_t* __restrict__ out, int heads, int d,
                             int dv, float eps, int most) {
   extern __shared__ __attribute__((aligned(16))) float rc_lds[];
   constexpr int LDK = rc_ld_rows(16 * DB), LDQ = LDK > rc_ld_rows(RC_L) ? LDK : rc_ld_rows(RC_L), LDV = rc_ld_lines(16 * VB);
