@@ -33,26 +33,29 @@ class PlainOps:
         return out
 
     # ------------------------------------------------------------ attention over a cached latent
-    def _turn(self, x, positions, rates):
-        """Coordinate j < n/2 of the last axis with coordinate j + n/2, by position * rates[j] (float32 angles)."""
+    def _turn(self, x, positions, rates, neighbours=False):
+        """Coordinate j < n/2 of the last axis with coordinate j + n/2 (or 2j with 2j + 1), by position * rates[j] (float32 angles)."""
         half = x.shape[-1] // 2
         angles = positions.to(torch.float32)[:, None] * rates.to(torch.float32)[None, :]
         cos, sin = angles.cos().to(self.work), angles.sin().to(self.work)
         while cos.dim() < x.dim():
             cos, sin = cos.unsqueeze(1), sin.unsqueeze(1)
+        if neighbours:
+            a, b = x[..., 0::2], x[..., 1::2]
+            return torch.stack([a * cos - b * sin, b * cos + a * sin], dim=-1).flatten(-2)
         a, b = x[..., :half], x[..., half:]
         return torch.cat([a * cos - b * sin, b * cos + a * sin], dim=-1)
 
     def latent_store(self, rows, q_offset, q_rank, q_norm, kv_offset, kv_rank, kv_norm, rot_dim, rates, eps, positions,
-                     slots, k_pages, v_pages, latent_q):
+                     slots, k_pages, v_pages, latent_q, neighbours=False):
         x = rows.to(self.work)
         latent_q.copy_((self._unit(x[:, q_offset:q_offset + q_rank], eps) * q_norm.to(self.work)).to(latent_q.dtype))
+        if slots is None:
+            return
         kept = self._unit(x[:, kv_offset:kv_offset + kv_rank], eps) * kv_norm.to(self.work)
         if rot_dim:
             tail = x[:, kv_offset + kv_rank:kv_offset + kv_rank + rot_dim]
-            kept = torch.cat([kept, self._turn(tail, positions, rates)], dim=1)
-        if slots is None:
-            return
+            kept = torch.cat([kept, self._turn(tail, positions, rates, neighbours)], dim=1)
         page_size = k_pages.shape[2]
         kept = kept.to(k_pages.dtype)
         for t in range(rows.shape[0]):
@@ -71,9 +74,10 @@ class PlainOps:
             out[:, at:at + n] = (a @ weight[h].to(self.work).t()).to(out.dtype)
         return out
 
-    def rotate_tails(self, q, heads, head_width, tail_offset, dims, rates, positions, out, out_head_stride, out_offset):
+    def rotate_tails(self, q, heads, head_width, tail_offset, dims, rates, positions, out, out_head_stride, out_offset,
+                     neighbours=False):
         x = q.to(self.work).reshape(q.shape[0], heads, head_width)[:, :, tail_offset:tail_offset + dims]
-        turned = self._turn(x, positions, rates).to(out.dtype)
+        turned = self._turn(x, positions, rates, neighbours).to(out.dtype)
         for h in range(heads):
             at = h * out_head_stride + out_offset
             out[:, at:at + dims] = turned[:, h]
@@ -156,7 +160,7 @@ class PlainOps:
         return x
 
     def route_scores(self, logits, correction, n_experts, n_groups, keep_groups, chosen, weights, softmax=False,
-                     group_max=False, gate=None):
+                     group_max=False, gate=None, renormalize=True):
         top = chosen.shape[1]
         z = logits.to(torch.float32)
         s = torch.softmax(z[:, :n_experts], dim=-1) if softmax else torch.sigmoid(z[:, :n_experts])
@@ -171,7 +175,7 @@ class PlainOps:
         ids = torch.topk(choice, top, dim=-1).indices
         picked = torch.gather(s, 1, ids)
         chosen.copy_(ids.to(torch.int32))
-        weights.copy_(picked / (picked.sum(-1, keepdim=True) + 1e-20))
+        weights.copy_(picked / (picked.sum(-1, keepdim=True) + 1e-20) if renormalize else picked)
         if gate is not None:
             gate.copy_(torch.sigmoid(z[:, n_experts]))
 
@@ -586,6 +590,24 @@ class PlainOps:
                 k_pages[page, :, off, :] = keys[t]
                 v_pages[page, :, :, off] = values[t]
 
+    def temper_store(self, qkv, positions, coef, every, slots, k_pages, v_pages, n_q, n_k, d, dv, tied):
+        n_tokens = qkv.shape[0]
+        steps = torch.div(positions.long() + 1, every, rounding_mode="floor").to(torch.float32)
+        factor = 1.0 + coef * torch.log(steps + 1.0)
+        qkv[:, :n_q * d] = (qkv[:, :n_q * d].to(self.work) * factor.to(self.work)[:, None]).to(qkv.dtype)
+        if slots is None:
+            return
+        page_size = k_pages.shape[2]
+        keys = qkv[:, n_q * d:(n_q + n_k) * d].reshape(n_tokens, n_k, d)
+        values = keys if tied else qkv[:, (n_q + n_k) * d:(n_q + n_k) * d + n_k * dv].reshape(n_tokens, n_k, dv)
+        for t in range(n_tokens):
+            slot = int(slots[t])
+            if slot < 0:
+                continue
+            page, off = divmod(slot, page_size)
+            k_pages[page, :, off, :] = keys[t]
+            v_pages[page, :, :, off] = values[t]
+
     def differential_heads(self, mixed, lam, eps, out_scale, n_heads, group, dv, out):
         n_tokens = mixed.shape[0]
         maps = mixed.to(self.work).reshape(n_tokens, n_heads // group, 2, group, dv)
@@ -613,7 +635,7 @@ class PlainOps:
         chosen.copy_(ids.to(torch.int32))
         weights.copy_(torch.softmax(values, dim=-1))
 
-    def expert_gate(self, gate_up, chosen, weights, n_experts, inner, shared, out, shared_weight=None):
+    def expert_gate(self, gate_up, chosen, weights, n_experts, inner, shared, out, shared_weight=None, weigh_input=False):
         n_tokens = gate_up.shape[0]
         x = gate_up.to(self.work)
         out.zero_()
@@ -621,6 +643,8 @@ class PlainOps:
         factor = torch.zeros((n_tokens, n_experts), dtype=self.work)
         factor.scatter_(1, chosen.long(), weights.to(self.work))
         g, u = routed[:, :, 0], routed[:, :, 1]
+        if weigh_input:
+            g, u, factor = factor[:, :, None] * g, factor[:, :, None] * u, torch.ones_like(factor)
         out[:, :n_experts * inner] = (factor[:, :, None] * (g * torch.sigmoid(g) * u)).reshape(n_tokens, -1).to(out.dtype)
         if shared:
             g, u = x[:, n_experts * 2 * inner:n_experts * 2 * inner + shared], x[:, n_experts * 2 * inner + shared:]

@@ -176,7 +176,7 @@ __global__ void expert_combine_kernel(const float* __restrict__ rows, const int*
     if (shared && shared_weight) sum *= shared_weight[t];
     for (int k = 0; k < top; ++k) {
       const int slot = slot_of[t * top + k];
-      if (slot >= 0) sum = fmaf(weights[t * top + k], rows[(size_t)slot * hidden + h], sum);
+      if (slot >= 0) sum = fmaf(weights ? weights[t * top + k] : 1.f, rows[(size_t)slot * hidden + h], sum);
     }
     st(out + idx, sum);
   }

@@ -8,8 +8,8 @@
 
 // rows: [n_tokens, row_stride].  latent_q[t, :] = rows[t, q_offset : q_offset + q_rank] / rms * q_norm.  The kept row
 // of a token is [c | turned tail]: c = rows[t, kv_offset : kv_offset + kv_rank] / rms * kv_norm, and the rot
-// coordinates behind it in `rows` with coordinate i < rot / 2 and coordinate i + rot / 2 turned by the angle
-// position * rates[i] (float).  It goes into key page [n_pages, 1, page_size, kv_rank + rot] at the token's slot and,
+// coordinates behind it in `rows` with coordinate i < rot / 2 and coordinate i + rot / 2 (neighbours: coordinates 2 i and
+// 2 i + 1) turned by the angle position * rates[i] (float).  It goes into key page [n_pages, 1, page_size, kv_rank + rot] at the token's slot and,
 // transposed inside a page, into value page [n_pages, 1, kv_rank + rot, page_size].  slots null or a negative slot:
 // nothing is stored.  A workgroup a token.
 template <typename T>
@@ -17,7 +17,7 @@ __global__ void __launch_bounds__(LT_THREADS)
 latent_store_kernel(const T* __restrict__ rows, int row_stride, int q_offset, int q_rank, const float* __restrict__ q_norm,
                     int kv_offset, int kv_rank, const float* __restrict__ kv_norm, int rot, const float* __restrict__ rates,
                     float eps, const int* __restrict__ positions, const int* __restrict__ slots, T* __restrict__ k_pages,
-                    T* __restrict__ v_pages, int page_size, T* __restrict__ latent_q) {
+                    T* __restrict__ v_pages, int page_size, T* __restrict__ latent_q, int neighbours) {
   __shared__ float scratch[16];
   const int t = blockIdx.x;
   const T* row = rows + (size_t)t * row_stride;
@@ -45,22 +45,24 @@ latent_store_kernel(const T* __restrict__ rows, int row_stride, int q_offset, in
   for (int i = threadIdx.x; i < half; i += LT_THREADS) {
     float s, c;
     sincosf(position * rates[i], &s, &c);
-    const float a = ld(tail + i), b = ld(tail + half + i);
+    const int one = neighbours ? 2 * i : i, other = neighbours ? 2 * i + 1 : half + i;
+    const float a = ld(tail + one), b = ld(tail + other);
     const float lo = a * c - b * s, hi = b * c + a * s;
-    st(k_row + kv_rank + i, lo);
-    st(k_row + kv_rank + half + i, hi);
-    st(v_col + (size_t)(kv_rank + i) * page_size, lo);
-    st(v_col + (size_t)(kv_rank + half + i) * page_size, hi);
+    st(k_row + kv_rank + one, lo);
+    st(k_row + kv_rank + other, hi);
+    st(v_col + (size_t)(kv_rank + one) * page_size, lo);
+    st(v_col + (size_t)(kv_rank + other) * page_size, hi);
   }
 }
 
 // out[t, h * out_stride + out_offset + i] for i < rot: the rot coordinates of q[t, h * head_width + tail_offset ...]
-// with coordinate i < rot / 2 and coordinate i + rot / 2 turned by position * rates[i].
+// with coordinate i < rot / 2 and coordinate i + rot / 2 (neighbours: coordinates 2 i and 2 i + 1) turned by
+// position * rates[i].
 template <typename T>
 __global__ void __launch_bounds__(LT_THREADS)
 rotate_tails_kernel(const T* __restrict__ q, int q_stride, int heads, int head_width, int tail_offset, int rot,
                     const float* __restrict__ rates, const int* __restrict__ positions, T* __restrict__ out, int out_row,
-                    int out_stride, int out_offset) {
+                    int out_stride, int out_offset, int neighbours) {
   const int t = blockIdx.x, half = rot / 2;
   const float position = (float)positions[t];
   for (int idx = threadIdx.x; idx < heads * half; idx += LT_THREADS) {
@@ -69,9 +71,10 @@ rotate_tails_kernel(const T* __restrict__ q, int q_stride, int heads, int head_w
     sincosf(position * rates[i], &s, &c);
     const T* src = q + (size_t)t * q_stride + (size_t)h * head_width + tail_offset;
     T* dst = out + (size_t)t * out_row + (size_t)h * out_stride + out_offset;
-    const float a = ld(src + i), b = ld(src + half + i);
-    st(dst + i, a * c - b * s);
-    st(dst + half + i, b * c + a * s);
+    const int one = neighbours ? 2 * i : i, other = neighbours ? 2 * i + 1 : half + i;
+    const float a = ld(src + one), b = ld(src + other);
+    st(dst + one, a * c - b * s);
+    st(dst + other, b * c + a * s);
   }
 }
 
@@ -219,13 +222,13 @@ head_linear_skinny_kernel(const bf16_t* __restrict__ x, int x_row, int x_stride,
 extern "C" int ta_latent_store(const void* rows, int row_stride, int q_offset, int q_rank, const void* q_norm, int kv_offset,
                                int kv_rank, const void* kv_norm, int rot, const void* rates, float eps, const void* positions,
                                const void* slots, void* k_pages, void* v_pages, int page_size, void* latent_q, int n_tokens,
-                               int dtype, hipStream_t stream) {
+                               int neighbours, int dtype, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
-  if (q_rank <= 0 || kv_rank <= 0 || rot < 0 || (rot & 1) || (rot > 0 && !rates) || (slots && (!k_pages || !v_pages || page_size <= 0)))
+  if (q_rank <= 0 || kv_rank <= 0 || rot < 0 || (rot & 1) || (rot > 0 && !rates) || (slots && (!k_pages || !v_pages || !kv_norm || page_size <= 0)))
     return -1;
 #define LS(TT) latent_store_kernel<TT><<<n_tokens, LT_THREADS, 0, stream>>>((const TT*)rows, row_stride, q_offset, q_rank, \
     (const float*)q_norm, kv_offset, kv_rank, (const float*)kv_norm, rot, (const float*)rates, eps, (const int*)positions, \
-    (const int*)slots, (TT*)k_pages, (TT*)v_pages, page_size, (TT*)latent_q)
+    (const int*)slots, (TT*)k_pages, (TT*)v_pages, page_size, (TT*)latent_q, neighbours)
   if (dtype == DT_F32) LS(float); else LS(bf16_t);
 #undef LS
   return LAUNCH_STATUS();
@@ -233,11 +236,11 @@ extern "C" int ta_latent_store(const void* rows, int row_stride, int q_offset, i
 
 extern "C" int ta_rotate_tails(const void* q, int q_stride, int heads, int head_width, int tail_offset, int rot,
                                const void* rates, const void* positions, void* out, int out_row, int out_stride,
-                               int out_offset, int n_tokens, int dtype, hipStream_t stream) {
+                               int out_offset, int n_tokens, int neighbours, int dtype, hipStream_t stream) {
   if (n_tokens <= 0 || rot == 0) return 0;
   if (rot < 0 || (rot & 1) || heads <= 0 || tail_offset + rot > head_width) return -1;
 #define RT(TT) rotate_tails_kernel<TT><<<n_tokens, LT_THREADS, 0, stream>>>((const TT*)q, q_stride, heads, head_width, \
-    tail_offset, rot, (const float*)rates, (const int*)positions, (TT*)out, out_row, out_stride, out_offset)
+    tail_offset, rot, (const float*)rates, (const int*)positions, (TT*)out, out_row, out_stride, out_offset, neighbours)
   if (dtype == DT_F32) RT(float); else RT(bf16_t);
 #undef RT
   return LAUNCH_STATUS();

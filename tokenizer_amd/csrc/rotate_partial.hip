@@ -121,6 +121,98 @@ extern "C" int ta_norm_rotate_store(void* qkv, int row_stride, const void* bias,
   return LAUNCH_STATUS();
 }
 
+// Rows of qkv as above without a bias: n_q query heads and n_k key heads of d elements, then n_k value heads of dv (tied: no
+// value heads, the keys are the values too and dv = d).  The query heads are multiplied by
+// 1 + coef * ln(floor((position + 1) / every) + 1), formed in float, and go back into their rows; keys and values go into
+// their pages as they are.  A workgroup a token.
+template <typename T>
+__global__ void __launch_bounds__(RP_THREADS)
+temper_store_kernel(T* __restrict__ qkv, int row_stride, const int* __restrict__ positions, float coef, int every,
+                    const int* __restrict__ slots, T* __restrict__ k_pages, T* __restrict__ v_pages, int n_q, int n_k, int d,
+                    int dv, int page_size, int tied) {
+  const int t = blockIdx.x;
+  T* row = qkv + (size_t)t * row_stride;
+  const int steps = (positions[t] + 1) / every;
+  if (steps > 0 && coef != 0.f) {                            // (before the first step the factor is 1)
+    const float factor = 1.f + coef * logf((float)steps + 1.f);
+    for (int i = threadIdx.x; i < n_q * d; i += RP_THREADS) st(row + i, ld(row + i) * factor);
+  }
+  const int slot = slots ? slots[t] : -1;
+  if (slot < 0) return;
+  const int page = slot / page_size, off = slot % page_size;
+  const T* keys = row + n_q * d;
+  const T* values = tied ? keys : keys + n_k * d;
+  for (int i = threadIdx.x; i < n_k * d; i += RP_THREADS)
+    k_pages[(((size_t)page * n_k + i / d) * page_size + off) * d + i % d] = keys[i];
+  for (int i = threadIdx.x; i < n_k * dv; i += RP_THREADS)    // head i / dv, coordinate i % dv: one line of a transposed page
+    v_pages[((size_t)page * n_k * dv + i) * page_size + off] = values[i];
+}
+
+// The same for bfloat16 rows in whole pieces of eight elements (d and dv multiples of 8, everything 16-byte aligned): a
+// thread a piece; the pieces of a token lie over grid.y workgroups.
+__global__ void __launch_bounds__(RP_THREADS)
+temper_store_vec_kernel(bf16_t* __restrict__ qkv, int row_stride, const int* __restrict__ positions, float coef, int every,
+                        const int* __restrict__ slots, bf16_t* __restrict__ k_pages, bf16_t* __restrict__ v_pages, int n_q,
+                        int n_k, int d, int dv, int page_size, int tied) {
+  HELD(qkv, row_stride, positions, coef, every, slots, k_pages, v_pages, n_q, n_k, d, dv, page_size, tied);
+  const int t = blockIdx.x, i = (blockIdx.y * RP_THREADS + threadIdx.x) * 8;
+  const int q_size = n_q * d, k_size = n_k * d, used = q_size + k_size + (tied ? 0 : n_k * dv);
+  if (i >= used) return;
+  bf16_t* at = qkv + (size_t)t * row_stride + i;
+  const uint4 raw = *reinterpret_cast<const uint4*>(at);
+  const int position = scalar_int(positions + t), slot = slots ? scalar_int(slots + t) : -1;
+  if (i < q_size) {
+    const int steps = (position + 1) / every;
+    if (steps == 0 || coef == 0.f) return;
+    const float factor = 1.f + coef * logf((float)steps + 1.f);
+    const uint32_t in[4] = {raw.x, raw.y, raw.z, raw.w};
+    uint32_t out[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      out[e] = (uint32_t)float_to_bf16_bits(bf16_bits_to_float(in[e] & 0xffffu) * factor) |
+               ((uint32_t)float_to_bf16_bits(bf16_bits_to_float(in[e] >> 16) * factor) << 16);
+    *reinterpret_cast<uint4*>(at) = make_uint4(out[0], out[1], out[2], out[3]);
+    return;
+  }
+  if (slot < 0) return;
+  const int page = slot / page_size, off = slot % page_size;
+  const bool key = i < q_size + k_size;
+  if (key) {
+    const int j = i - q_size;
+    *reinterpret_cast<uint4*>(k_pages + (((size_t)page * n_k + j / d) * page_size + off) * d + j % d) = raw;
+  }
+  if (!key || tied) {
+    const int j = i - q_size - (tied ? 0 : k_size);           // head j / dv, coordinate j % dv
+    bf16_t* to = v_pages + ((size_t)page * n_k * dv + j) * page_size + off;
+    const uint32_t in[4] = {raw.x, raw.y, raw.z, raw.w};
+#pragma unroll
+    for (int e = 0; e < 8; ++e) to[(size_t)e * page_size].bits = (uint16_t)(in[e >> 1] >> (16 * (e & 1)));
+  }
+}
+
+extern "C" int ta_temper_store(void* qkv, int row_stride, const void* positions, float coef, int every, const void* slots,
+                               void* k_pages, void* v_pages, int n_tokens, int n_q, int n_k, int d, int dv, int page_size,
+                               int tied, int dtype, hipStream_t stream) {
+  if (n_tokens <= 0) return 0;
+  if (every < 1 || d <= 0 || dv <= 0 || n_q <= 0 || n_k < 0 || page_size <= 0 || (tied && dv != d) ||
+      (slots && (!k_pages || !v_pages)))
+    return -1;
+  const int used = (n_q + n_k) * d + (tied ? 0 : n_k * dv);
+  if (used > row_stride) return -1;
+  if (dtype == DT_BF16 && d % 8 == 0 && dv % 8 == 0 && row_stride % 8 == 0 &&
+      (((uintptr_t)qkv | (uintptr_t)k_pages | (uintptr_t)v_pages) & 15) == 0) {
+    temper_store_vec_kernel<<<dim3(n_tokens, (used / 8 + RP_THREADS - 1) / RP_THREADS), RP_THREADS, 0, stream>>>(
+        (bf16_t*)qkv, row_stride, (const int*)positions, coef, every, (const int*)slots, (bf16_t*)k_pages, (bf16_t*)v_pages,
+        n_q, n_k, d, dv, page_size, tied);
+    return LAUNCH_STATUS();
+  }
+#define TEMPER(TT) temper_store_kernel<TT><<<n_tokens, RP_THREADS, 0, stream>>>((TT*)qkv, row_stride, (const int*)positions, \
+      coef, every, (const int*)slots, (TT*)k_pages, (TT*)v_pages, n_q, n_k, d, dv, page_size, tied)
+  if (dtype == DT_F32) TEMPER(float); else TEMPER(bf16_t);
+#undef TEMPER
+  return LAUNCH_STATUS();
+}
+
 // table[t] = [cosines | sines] (each rot / 2 floats) of positions[t] * rates[i], formed and taken in float, times magnitude.
 __global__ void __launch_bounds__(RP_THREADS)
 rotation_table_kernel(const int* __restrict__ positions, const float* __restrict__ rates, float magnitude, int half,

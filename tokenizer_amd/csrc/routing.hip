@@ -143,11 +143,13 @@ route_rows_kernel(const T* __restrict__ x, int lda, const T* __restrict__ router
 // gate_up: [n_tokens, n_experts * 2 * inner + 2 * shared], expert e's gate rows then its up rows, the shared expert
 // last.  out: [n_tokens, columns] with columns >= n_experts * inner + shared: out[t, e * inner + i] =
 // w * silu(gate) * up for an expert the token chose with weight w, 0 for the others; the shared expert's columns
-// with weight 1 (or shared_weight[t], float, where given); columns beyond are 0.
+// with weight 1 (or shared_weight[t], float, where given); columns beyond are 0.  weigh_input: silu(w * gate) * (w * up)
+// instead (the expert is handed its row times w).
 template <typename T>
 __global__ void expert_gate_kernel(const T* __restrict__ gate_up, const int* __restrict__ chosen,
                                    const float* __restrict__ weights, int top, int n_experts, int inner, int shared,
-                                   int columns, T* __restrict__ out, size_t total, const float* __restrict__ shared_weight) {
+                                   int columns, T* __restrict__ out, size_t total, const float* __restrict__ shared_weight,
+                                   int weigh_input) {
   const int in_stride = n_experts * 2 * inner + 2 * shared;
   for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total; idx += (size_t)gridDim.x * blockDim.x) {
     const size_t t = idx / columns;
@@ -160,7 +162,8 @@ __global__ void expert_gate_kernel(const T* __restrict__ gate_up, const int* __r
       for (int k = 0; k < top; ++k)
         if (chosen[t * top + k] == e) w += weights[t * top + k];
       if (w != 0.f) {
-        const float g = ld(row + (size_t)e * 2 * inner + i), u = ld(row + (size_t)e * 2 * inner + inner + i);
+        float g = ld(row + (size_t)e * 2 * inner + i), u = ld(row + (size_t)e * 2 * inner + inner + i);
+        if (weigh_input) { g *= w; u *= w; w = 1.f; }
         value = w * (g / (1.0f + expf(-g)) * u);
       }
     } else if (c < n_experts * inner + shared) {
@@ -206,7 +209,7 @@ __global__ void named_gate_kernel(const T* __restrict__ in, T* __restrict__ out,
 __global__ void expert_gate_vec_kernel(const bf16_t* __restrict__ gate_up, const int* __restrict__ chosen,
                                        const float* __restrict__ weights, int top, int n_experts, int inner, int shared,
                                        int columns, bf16_t* __restrict__ out, size_t total8,
-                                       const float* __restrict__ shared_weight) {
+                                       const float* __restrict__ shared_weight, int weigh_input) {
   const int in_stride = n_experts * 2 * inner + 2 * shared, columns8 = columns / 8;
   for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total8; idx += (size_t)gridDim.x * blockDim.x) {
     const size_t t = idx / columns8;
@@ -230,8 +233,12 @@ __global__ void expert_gate_vec_kernel(const bf16_t* __restrict__ gate_up, const
       float g[8], u[8], v[8];
       rt_unpack8(*reinterpret_cast<const uint4*>(g_at), g);
       rt_unpack8(*reinterpret_cast<const uint4*>(g_at + up_off), u);
+      const float before = weigh_input ? w : 1.f, behind = weigh_input ? 1.f : w;
 #pragma unroll
-      for (int k = 0; k < 8; ++k) v[k] = w * (g[k] / (1.0f + expf(-g[k])) * u[k]);
+      for (int k = 0; k < 8; ++k) {
+        const float z = before * g[k];
+        v[k] = behind * (z / (1.0f + expf(-z)) * (before * u[k]));
+      }
       packed = rt_pack8(v);
     }
     *reinterpret_cast<uint4*>(out + t * columns + c) = packed;
@@ -250,6 +257,42 @@ __global__ void named_gate_vec_kernel(const bf16_t* __restrict__ in, bf16_t* __r
 #pragma unroll
     for (int k = 0; k < 8; ++k) v[k] = rt_gate_act<RELU>(g[k]) * u[k];
     reinterpret_cast<uint4*>(out)[idx] = rt_pack8(v);
+  }
+}
+
+// Rows sorted by expert: gate_up [slots, 2 * inner], out [slots, inner]: for pair p (token p / top, its pick p % top) in slot
+// slot_of[p], out[slot] = silu(w * gate) * (w * up) with w = weights[p].  Slots of no pair are not written.
+template <typename T>
+__global__ void expert_gate_slots_kernel(const T* __restrict__ gate_up, const int* __restrict__ slot_of,
+                                         const float* __restrict__ weights, int inner, T* __restrict__ out, size_t total) {
+  for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total; idx += (size_t)gridDim.x * blockDim.x) {
+    const size_t p = idx / inner;
+    const int i = (int)(idx - p * inner);
+    if (slot_of[p] < 0) continue;
+    const size_t slot = slot_of[p];
+    const float w = weights[p], g = w * ld(gate_up + slot * 2 * inner + i), u = w * ld(gate_up + slot * 2 * inner + inner + i);
+    st(out + slot * inner + i, g / (1.0f + expf(-g)) * u);
+  }
+}
+
+__global__ void expert_gate_slots_vec_kernel(const bf16_t* __restrict__ gate_up, const int* __restrict__ slot_of,
+                                             const float* __restrict__ weights, int inner8, bf16_t* __restrict__ out,
+                                             size_t total8) {
+  for (size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x; idx < total8; idx += (size_t)gridDim.x * blockDim.x) {
+    const size_t p = idx / inner8, j = idx - p * inner8;
+    if (slot_of[p] < 0) continue;
+    const size_t slot = slot_of[p];
+    const float w = weights[p];
+    const uint4* row = reinterpret_cast<const uint4*>(gate_up) + slot * 2 * inner8;
+    float g[8], u[8], v[8];
+    rt_unpack8(row[j], g);
+    rt_unpack8(row[inner8 + j], u);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      const float z = w * g[k];
+      v[k] = z / (1.0f + expf(-z)) * (w * u[k]);
+    }
+    reinterpret_cast<uint4*>(out)[slot * inner8 + j] = rt_pack8(v);
   }
 }
 
@@ -284,22 +327,41 @@ extern "C" int ta_route_rows(const void* x, int lda, const void* router, int n_t
 
 extern "C" int ta_expert_gate(const void* gate_up, const void* chosen, const void* weights, int n_tokens, int top,
                               int n_experts, int inner, int shared, int columns, void* out, int dtype,
-                              const void* shared_weight, hipStream_t stream) {
+                              const void* shared_weight, int weigh_input, hipStream_t stream) {
   const size_t total = (size_t)n_tokens * columns;
   if (total == 0) return 0;
-  if (columns < n_experts * inner + shared) return -1;
+  if (columns < n_experts * inner + shared || (weigh_input && shared)) return -1;
   if (dtype == DT_BF16 && inner % 8 == 0 && shared % 8 == 0 && columns % 8 == 0 &&
       (((uintptr_t)gate_up | (uintptr_t)out) & 15) == 0) {
     expert_gate_vec_kernel<<<rt_blocks(total / 8), 256, 0, stream>>>((const bf16_t*)gate_up, (const int*)chosen,
-        (const float*)weights, top, n_experts, inner, shared, columns, (bf16_t*)out, total / 8, (const float*)shared_weight);
+        (const float*)weights, top, n_experts, inner, shared, columns, (bf16_t*)out, total / 8, (const float*)shared_weight,
+        weigh_input);
     return LAUNCH_STATUS();
   }
   if (dtype == DT_F32)
     expert_gate_kernel<float><<<rt_blocks(total), 256, 0, stream>>>((const float*)gate_up, (const int*)chosen,
-        (const float*)weights, top, n_experts, inner, shared, columns, (float*)out, total, (const float*)shared_weight);
+        (const float*)weights, top, n_experts, inner, shared, columns, (float*)out, total, (const float*)shared_weight,
+        weigh_input);
   else
     expert_gate_kernel<bf16_t><<<rt_blocks(total), 256, 0, stream>>>((const bf16_t*)gate_up, (const int*)chosen,
-        (const float*)weights, top, n_experts, inner, shared, columns, (bf16_t*)out, total, (const float*)shared_weight);
+        (const float*)weights, top, n_experts, inner, shared, columns, (bf16_t*)out, total, (const float*)shared_weight,
+        weigh_input);
+  return LAUNCH_STATUS();
+}
+
+extern "C" int ta_expert_gate_slots(const void* gate_up, const void* slot_of, const void* weights, int n_pairs, int inner,
+                                    void* out, int dtype, hipStream_t stream) {
+  const size_t total = (size_t)n_pairs * inner;
+  if (n_pairs <= 0 || inner <= 0) return 0;
+  if (dtype == DT_BF16 && inner % 8 == 0 && (((uintptr_t)gate_up | (uintptr_t)out) & 15) == 0)
+    expert_gate_slots_vec_kernel<<<rt_blocks(total / 8), 256, 0, stream>>>((const bf16_t*)gate_up, (const int*)slot_of,
+        (const float*)weights, inner / 8, (bf16_t*)out, total / 8);
+  else if (dtype == DT_F32)
+    expert_gate_slots_kernel<float><<<rt_blocks(total), 256, 0, stream>>>((const float*)gate_up, (const int*)slot_of,
+        (const float*)weights, inner, (float*)out, total);
+  else
+    expert_gate_slots_kernel<bf16_t><<<rt_blocks(total), 256, 0, stream>>>((const bf16_t*)gate_up, (const int*)slot_of,
+        (const float*)weights, inner, (bf16_t*)out, total);
   return LAUNCH_STATUS();
 }
 
@@ -355,7 +417,7 @@ extern "C" int ta_relu_gate(const void* in, void* out, int n_tokens, int inner, 
 // the same values); `store` says whether this wave writes the token's results.
 __device__ __forceinline__ void rs_choose(float* choice, const float* score, float* worth, int lane, int n_experts,
                                           int n_groups, int keep, int top, bool store, int* __restrict__ chosen_row,
-                                          float* __restrict__ weights_row, bool group_max = false) {
+                                          float* __restrict__ weights_row, bool group_max = false, bool renormalize = true) {
   if (n_groups > 0) {
     const int per = n_experts / n_groups;
     for (int g = lane; g < n_groups; g += WAVE) {
@@ -405,7 +467,7 @@ __device__ __forceinline__ void rs_choose(float* choice, const float* score, flo
     last = best_at;
     last_value = best;
   }
-  if (store && lane < top) weights_row[lane] = mine / (total + 1e-20f);
+  if (store && lane < top) weights_row[lane] = renormalize ? mine / (total + 1e-20f) : mine;
 }
 
 __global__ void __launch_bounds__(256)
@@ -432,11 +494,11 @@ route_sigmoid_kernel(const float* __restrict__ logits, const float* __restrict__
 // The same choice from scores of either kind.  logits: float rows of `stride` numbers, the experts' first.  softmax: the
 // scores are the softmax over all experts (else sigmoid); correction may be null; group_max: a group is worth its
 // largest choice score (else the sum of its two largest); gate (float [n_tokens] or null) gets sigmoid of the number
-// behind the experts' logits in the row.  A wave a token.
+// behind the experts' logits in the row.  raw: the weights are the chosen scores themselves, not over their sum.  A wave a token.
 __global__ void __launch_bounds__(256)
 route_scores_kernel(const float* __restrict__ logits, int stride, const float* __restrict__ correction, int n_tokens,
                     int n_experts, int n_groups, int keep, int top, int softmax, int group_max, int* __restrict__ chosen,
-                    float* __restrict__ weights, float* __restrict__ gate) {
+                    float* __restrict__ weights, float* __restrict__ gate, int raw) {
   extern __shared__ float rs_scratch[];
   const int lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE;
   const int slot = blockIdx.x * (blockDim.x / WAVE) + wave;
@@ -462,7 +524,7 @@ route_scores_kernel(const float* __restrict__ logits, int stride, const float* _
   if (gate && live && lane == 0) gate[t] = 1.0f / (1.0f + expf(-row[n_experts]));
   __syncthreads();
   rs_choose(choice, score, worth, lane, n_experts, n_groups, keep, top, live, chosen + (size_t)t * top,
-            weights + (size_t)t * top, group_max != 0);
+            weights + (size_t)t * top, group_max != 0, raw == 0);
 }
 
 // The router's product and the choice in one kernel, a token a workgroup (few rows: a decode step): as route_rows_kernel
@@ -472,7 +534,8 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 route_rows_sigmoid_kernel(const T* __restrict__ x, int lda, const T* __restrict__ router, const float* __restrict__ correction,
                           int hidden, int n_experts, int n_groups, int keep, int top, int* __restrict__ chosen,
-                          float* __restrict__ weights, int softmax = 0, int group_max = 0, float* __restrict__ gate = nullptr) {
+                          float* __restrict__ weights, int softmax = 0, int group_max = 0, float* __restrict__ gate = nullptr,
+                          int raw = 0) {
   constexpr int N = RtVec<T>::N;
   extern __shared__ float rs_scratch[];
   float* choice = rs_scratch;
@@ -531,7 +594,7 @@ route_rows_sigmoid_kernel(const T* __restrict__ x, int lda, const T* __restrict_
     __syncthreads();
   }
   rs_choose(choice, score, worth, lane, n_experts, n_groups, keep, top, wave == 0, chosen + (size_t)t * top,
-            weights + (size_t)t * top, group_max != 0);
+            weights + (size_t)t * top, group_max != 0, raw == 0);
 }
 
 // up: [n_tokens, n_experts * inner]; out: [n_tokens, columns], columns >= n_experts * inner:
@@ -614,21 +677,21 @@ extern "C" int ta_route_sigmoid(const void* logits, const void* correction, int 
 
 extern "C" int ta_route_scores(const void* logits, int stride, const void* correction, int n_tokens, int n_experts,
                                int n_groups, int keep, int top, int softmax, int group_max, void* chosen, void* weights,
-                               void* gate, hipStream_t stream) {
+                               void* gate, int raw, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
   if (top <= 0 || top > n_experts || top > WAVE || n_experts > RS_MAX_EXPERTS || n_groups < 0) return -1;
   if (stride < n_experts + (gate ? 1 : 0)) return -1;
   if (n_groups > 0 && (n_experts % n_groups || keep <= 0 || keep > n_groups || keep * (n_experts / n_groups) < top)) return -1;
   const size_t lds = (size_t)4 * (2 * n_experts + n_groups) * sizeof(float);
   route_scores_kernel<<<(n_tokens + 3) / 4, 256, lds, stream>>>((const float*)logits, stride, (const float*)correction,
-      n_tokens, n_experts, n_groups, keep, top, softmax, group_max, (int*)chosen, (float*)weights, (float*)gate);
+      n_tokens, n_experts, n_groups, keep, top, softmax, group_max, (int*)chosen, (float*)weights, (float*)gate, raw);
   return LAUNCH_STATUS();
 }
 
 // The same for scores of either kind (see route_scores_kernel): router [n_experts (+ 1 with a gate), hidden].
 extern "C" int ta_route_rows_scores(const void* x, int lda, const void* router, const void* correction, int n_tokens,
                                     int hidden, int n_experts, int n_groups, int keep, int top, int softmax, int group_max,
-                                    void* chosen, void* weights, void* gate, int dtype, hipStream_t stream) {
+                                    void* chosen, void* weights, void* gate, int raw, int dtype, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
   if (top <= 0 || top > n_experts || top > WAVE || n_groups < 0) return -1;
   if (n_groups > 0 && (n_experts % n_groups || keep <= 0 || keep > n_groups || keep * (n_experts / n_groups) < top)) return -1;
@@ -640,11 +703,11 @@ extern "C" int ta_route_rows_scores(const void* x, int lda, const void* router, 
   if (dtype == DT_F32)
     route_rows_sigmoid_kernel<float><<<n_tokens, 256, lds, stream>>>((const float*)x, lda, (const float*)router,
         (const float*)correction, hidden, n_experts, n_groups, keep, top, (int*)chosen, (float*)weights, softmax, group_max,
-        (float*)gate);
+        (float*)gate, raw);
   else
     route_rows_sigmoid_kernel<bf16_t><<<n_tokens, 256, lds, stream>>>((const bf16_t*)x, lda, (const bf16_t*)router,
         (const float*)correction, hidden, n_experts, n_groups, keep, top, (int*)chosen, (float*)weights, softmax, group_max,
-        (float*)gate);
+        (float*)gate, raw);
   return LAUNCH_STATUS();
 }
 

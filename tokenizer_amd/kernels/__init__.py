@@ -161,7 +161,8 @@ class Ops:
                      "ta_add_terms_rmsnorm", "ta_scale_cap", "ta_route_scores", "ta_selective_scan", "ta_route_rows_scores",
                      "ta_rotation_table", "ta_head_norm_rotate_store", "ta_group_norm_add", "ta_relu_gate",
                      "ta_talking_attention_generic", "ta_talking_decode_bf16", "ta_talking_prefill_bf16",
-                     "ta_talking_prefill_parts", "ta_retention_scan", "ta_retention_chunked"):
+                     "ta_talking_prefill_parts", "ta_retention_scan", "ta_retention_chunked", "ta_temper_store",
+                     "ta_expert_gate_slots"):
             getattr(self.lib, name).restype = ctypes.c_int
         self.lib.ta_grouped_gemm_bf16.argtypes = [ctypes.c_void_p, ctypes.c_int, ctypes.c_void_p, ctypes.c_void_p, ctypes.c_int,
                                                   ctypes.c_int, ctypes.c_void_p, ctypes.c_long, ctypes.c_int, ctypes.c_void_p,
@@ -302,18 +303,21 @@ class Ops:
     def latent_store(self, rows: torch.Tensor, q_offset: int, q_rank: int, q_norm: torch.Tensor, kv_offset: int, kv_rank: int,
                      kv_norm: torch.Tensor, rot_dim: int, rates: torch.Tensor | None, eps: float, positions: torch.Tensor,
                      slots: torch.Tensor | None, k_pages: torch.Tensor | None, v_pages: torch.Tensor | None,
-                     latent_q: torch.Tensor) -> None:
+                     latent_q: torch.Tensor, neighbours: bool = False) -> None:
         """latent_q[t] = rmsnorm(rows[t, q_offset : + q_rank]) * q_norm; the kept row of a token, [rmsnorm(rows[t,
         kv_offset : + kv_rank]) * kv_norm | the rot_dim coordinates behind them, coordinate i with i + rot_dim / 2 turned by
         positions[t] * rates[i]], goes into key pages [n_pages, 1, page_size, kv_rank + rot_dim] at slots[t] and,
         transposed within a page, into value pages [n_pages, 1, kv_rank + rot_dim, page_size] (slots None: nothing is
-        stored).  Norms and angles are float32."""
+        stored, and the rows need no such part: kv_norm may be None).  `neighbours`: coordinate 2i turns with 2i + 1.  Norms
+        and angles are float32."""
         _dev(rows, q_norm, kv_norm, rates, positions, slots, k_pages, v_pages, latent_q)
         n_tokens = rows.shape[0]
-        _need(rows.dim() == 2 and q_offset >= 0 and kv_offset >= 0 and q_offset + q_rank <= rows.shape[1]
-              and kv_offset + kv_rank + rot_dim <= rows.shape[1] and q_rank > 0 and kv_rank > 0, "the latents do not fit the rows")
-        _need(q_norm.dtype == torch.float32 and q_norm.numel() == q_rank and kv_norm.dtype == torch.float32
-              and kv_norm.numel() == kv_rank, "the latents' norm weights are float32")
+        _need(rows.dim() == 2 and rows.is_contiguous() and q_offset >= 0 and kv_offset >= 0 and q_offset + q_rank <= rows.shape[1]
+              and (slots is None or kv_offset + kv_rank + rot_dim <= rows.shape[1]) and q_rank > 0 and kv_rank > 0,
+              "the latents do not fit the rows")
+        _need(q_norm.dtype == torch.float32 and q_norm.numel() == q_rank and (slots is None or (
+            kv_norm is not None and kv_norm.dtype == torch.float32 and kv_norm.numel() == kv_rank)),
+              "the latents' norm weights are float32")
         _need(rot_dim >= 0 and rot_dim % 2 == 0 and (rot_dim == 0 or (rates is not None and rates.dtype == torch.float32
                                                                        and rates.numel() == rot_dim // 2)),
               "a rotation has an even number of coordinates and a float32 rate for each pair")
@@ -329,7 +333,7 @@ class Ops:
                                              _ptr(kv_norm), rot_dim, _ptr(rates), ctypes.c_float(eps), _ptr(positions),
                                              _ptr(slots), _ptr(k_pages if slots is not None else None),
                                              _ptr(v_pages if slots is not None else None), page_size, _ptr(latent_q),
-                                             n_tokens, _code(rows.dtype), self._stream()), "latent_store")
+                                             n_tokens, int(neighbours), _code(rows.dtype), self._stream()), "latent_store")
 
     def head_linear(self, x: torch.Tensor, x_offset: int, x_head_stride: int, weight: torch.Tensor, out: torch.Tensor,
                     out_offset: int, out_head_stride: int) -> torch.Tensor:
@@ -349,9 +353,11 @@ class Ops:
         return out
 
     def rotate_tails(self, q: torch.Tensor, heads: int, head_width: int, tail_offset: int, dims: int, rates: torch.Tensor,
-                     positions: torch.Tensor, out: torch.Tensor, out_head_stride: int, out_offset: int) -> torch.Tensor:
+                     positions: torch.Tensor, out: torch.Tensor, out_head_stride: int, out_offset: int,
+                     neighbours: bool = False) -> torch.Tensor:
         """out[t, h out_head_stride + out_offset + i], i < dims: coordinates tail_offset.. of head h of q [T, heads
-        head_width], coordinate i with i + dims / 2 turned by positions[t] * rates[i] (float32 angles)."""
+        head_width], coordinate i with i + dims / 2 (`neighbours`: 2i with 2i + 1) turned by positions[t] * rates[i]
+        (float32 angles)."""
         _dev(q, rates, positions, out)
         n_tokens = q.shape[0]
         _need(q.shape[1] >= heads * head_width and tail_offset >= 0 and tail_offset + dims <= head_width and dims % 2 == 0,
@@ -362,7 +368,7 @@ class Ops:
               and (heads - 1) * out_head_stride + out_offset + dims <= out.shape[1], "the tails do not fit the output")
         self._check(self.lib.ta_rotate_tails(_ptr(q), q.shape[1], heads, head_width, tail_offset, dims, _ptr(rates),
                                              _ptr(positions), _ptr(out), out.shape[1], out_head_stride, out_offset, n_tokens,
-                                             _code(q.dtype), self._stream()), "rotate_tails")
+                                             int(neighbours), _code(q.dtype), self._stream()), "rotate_tails")
         return out
 
     # ---------------------------------------------------- delta rule with a decay per key channel
@@ -493,11 +499,11 @@ class Ops:
 
     def route_scores(self, logits: torch.Tensor, correction: torch.Tensor | None, n_experts: int, n_groups: int,
                      keep_groups: int, chosen: torch.Tensor, weights: torch.Tensor, softmax: bool = False,
-                     group_max: bool = False, gate: torch.Tensor | None = None) -> None:
+                     group_max: bool = False, gate: torch.Tensor | None = None, renormalize: bool = True) -> None:
         """As `route_sigmoid`, from scores of either kind: float32 `logits` [T, >= n_experts] (the experts' first);
         `softmax`: s = softmax over all experts (else sigmoid); `correction` may be None; `group_max`: a group is worth
         its largest choice score (else its two largest); `gate` (float32 [T]) gets sigmoid of the number behind the
-        experts' logits in a row."""
+        experts' logits in a row; `renormalize` False: the weights are the chosen scores themselves."""
         _dev(logits, correction, chosen, weights, gate)
         n_tokens, top = logits.shape[0], chosen.shape[1]
         _need(logits.dtype == torch.float32 and logits.is_contiguous() and logits.shape[1] >= n_experts + (gate is not None),
@@ -511,7 +517,7 @@ class Ops:
                                 and keep_groups * (n_experts // n_groups) >= top), "the groups do not fit")
         self._check(self.lib.ta_route_scores(_ptr(logits), logits.shape[1], _ptr(correction), n_tokens, n_experts, int(n_groups),
                                              int(keep_groups), top, int(bool(softmax)), int(bool(group_max)), _ptr(chosen),
-                                             _ptr(weights), _ptr(gate), self._stream()), "route_scores")
+                                             _ptr(weights), _ptr(gate), int(not renormalize), self._stream()), "route_scores")
 
     def delta_scan(self, fresh: torch.Tensor, decay: torch.Tensor, neg_rate: torch.Tensor, rows: torch.Tensor, beta_offset: int,
                    state: torch.Tensor, cu_q: torch.Tensor, first_position: torch.Tensor, state_slots: torch.Tensor,
@@ -697,6 +703,30 @@ class Ops:
             _ptr(k_pages), _ptr(v_pages), n_tokens, n_q, n_k, n_v, d, dv, page_size, _ptr(q_norm), _ptr(k_norm),
             ctypes.c_float(eps), _code(qkv.dtype), self._stream()), "norm_rotate_store")
 
+    def temper_store(self, qkv: torch.Tensor, positions: torch.Tensor, coef: float, every: int, slots: torch.Tensor | None,
+                     k_pages: torch.Tensor | None, v_pages: torch.Tensor | None, n_q: int, n_k: int, d: int, dv: int,
+                     tied: bool = False) -> None:
+        """In place on rows of `qkv` ([T, >= (n_q + n_k) d + n_k dv]: query heads, key heads, value heads; `tied`: no value
+        heads, the keys are the values and dv = d): the query heads times 1 + coef ln(floor((position + 1) / every) + 1), a
+        float32 factor; keys and values written as they are at `slots` into key pages [n_pages, n_k, page_size, d] and
+        value pages [n_pages, n_k, dv, page_size]."""
+        _dev(positions, slots, k_pages, v_pages)
+        _need(qkv.is_cuda, "kernel operands must live on the GPU")
+        n_tokens, width = qkv.shape
+        _need(width >= (n_q + n_k) * d + (0 if tied else n_k * dv) and qkv.stride(1) == 1, "qkv is narrower than its heads")
+        _need(positions.dtype == torch.int32 and positions.numel() == n_tokens, "positions must be int32 [T]")
+        _need(every >= 1 and (not tied or dv == d), "the temperature steps every so many positions; tied values have the keys' size")
+        page_size = 1
+        if slots is not None:
+            _need(slots.dtype == torch.int32 and slots.numel() == n_tokens, "slots must be int32 [T]")
+            _need(k_pages is not None and v_pages is not None, "slots without pages")
+            _need(k_pages.dtype == qkv.dtype and v_pages.dtype == qkv.dtype, "pages must have the dtype of qkv")
+            page_size = self._page_size(k_pages, v_pages, n_k, d, dv)
+        self._check(self.lib.ta_temper_store(
+            _ptr(qkv), qkv.stride(0), _ptr(positions), ctypes.c_float(coef), int(every), _ptr(slots),
+            _ptr(k_pages if slots is not None else None), _ptr(v_pages if slots is not None else None), n_tokens, n_q, n_k, d,
+            dv, page_size, int(bool(tied)), _code(qkv.dtype), self._stream()), "temper_store")
+
     def rotation_table(self, positions: torch.Tensor, rates: torch.Tensor, magnitude: float, out: torch.Tensor) -> torch.Tensor:
         """out [T, 2 R] float32: the cosines, then the sines, of positions[t] * rates[i] (float32 angles, accurate sine and
         cosine), times `magnitude`.  positions int32 [T], rates float32 [R]."""
@@ -801,7 +831,7 @@ class Ops:
 
     def route_rows_scores(self, x: torch.Tensor, router: torch.Tensor, correction: torch.Tensor | None, n_experts: int,
                           n_groups: int, keep_groups: int, chosen: torch.Tensor, weights: torch.Tensor, softmax: bool = False,
-                          group_max: bool = False, gate: torch.Tensor | None = None) -> bool:
+                          group_max: bool = False, gate: torch.Tensor | None = None, renormalize: bool = True) -> bool:
         """`route_scores` of the float32 logits x @ router.T without leaving them in memory (router [n_experts, H], or with
         a gate [n_experts + 1, H], the gate's row last): product and choice in one kernel, a token a workgroup (for the few
         rows of a decode step).  Returns False for sizes the kernel does not take: the caller then forms the logits with
@@ -822,7 +852,7 @@ class Ops:
         status = self.lib.ta_route_rows_scores(_ptr(x), x.stride(0) if n_tokens > 1 else hidden, _ptr(router), _ptr(correction),
                                                n_tokens, hidden, n_experts, int(n_groups), int(keep_groups), top,
                                                int(bool(softmax)), int(bool(group_max)), _ptr(chosen), _ptr(weights),
-                                               _ptr(gate), _code(x.dtype), self._stream())
+                                               _ptr(gate), int(not renormalize), _code(x.dtype), self._stream())
         if status == -2:
             return False
         self._check(status, "route_rows_scores")
@@ -898,9 +928,10 @@ class Ops:
         return out
 
     def expert_combine(self, rows: torch.Tensor, slot_of: torch.Tensor, weights: torch.Tensor, shared: torch.Tensor | None,
-                       out: torch.Tensor, shared_weight: torch.Tensor | None = None) -> torch.Tensor:
-        """out[t] = shared[t] (if given; times shared_weight[t], float32 [T], if that is given) + sum over the token's picks of weights[t, k] * rows[slot_of[t top + k]]; rows
-        float32 [slots, H], weights float32 [T, top], shared and out [T, H] of one dtype."""
+                       out: torch.Tensor, shared_weight: torch.Tensor | None = None, weighted: bool = True) -> torch.Tensor:
+        """out[t] = shared[t] (if given; times shared_weight[t], float32 [T], if that is given) + sum over the token's picks of
+        weights[t, k] * rows[slot_of[t top + k]] (`weighted` False: of the rows as they are); rows float32 [slots, H], weights
+        float32 [T, top], shared and out [T, H] of one dtype."""
         _dev(rows, slot_of, weights, shared, out)
         n_tokens, top = weights.shape
         _need(rows.dtype == torch.float32 and rows.is_contiguous() and rows.shape[1] == out.shape[1], "rows are float32 [slots, H]")
@@ -911,15 +942,19 @@ class Ops:
         _dev(shared_weight)
         _need(shared_weight is None or (shared_weight.dtype == torch.float32 and shared_weight.numel() == n_tokens),
               "the shared expert's weights are float32 [T]")
-        self._check(self.lib.ta_expert_combine(_ptr(rows), _ptr(slot_of), _ptr(weights), n_tokens, top, _ptr(shared), _ptr(out),
+        self._check(self.lib.ta_expert_combine(_ptr(rows), _ptr(slot_of), _ptr(weights if weighted else None), n_tokens, top,
+                                               _ptr(shared), _ptr(out),
                                                out.shape[1], _code(out.dtype), _ptr(shared_weight), self._stream()), "expert_combine")
         return out
 
     def expert_gate(self, gate_up: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor, n_experts: int, inner: int,
-                    shared: int, out: torch.Tensor, shared_weight: torch.Tensor | None = None) -> torch.Tensor:
+                    shared: int, out: torch.Tensor, shared_weight: torch.Tensor | None = None,
+                    weigh_input: bool = False) -> torch.Tensor:
         """gate_up [T, n_experts 2 inner + 2 shared] (every expert's gate rows, then its up rows; the shared expert
         last) -> out [T, >= n_experts inner + shared]: weight * silu(gate) * up in the columns of the experts a token
-        chose, silu(gate) * up in the shared expert's (times shared_weight[t], float32 [T], if given), zero everywhere else."""
+        chose, silu(gate) * up in the shared expert's (times shared_weight[t], float32 [T], if given), zero everywhere else.
+        `weigh_input` (no shared expert): silu(weight * gate) * (weight * up) instead."""
+        _need(not (weigh_input and shared), "a weighted input without a shared expert")
         _dev(gate_up, chosen, weights, out, shared_weight)
         _need(shared_weight is None or (shared_weight.dtype == torch.float32 and shared_weight.numel() == gate_up.shape[0]),
               "the shared expert's weights are float32 [T]")
@@ -931,7 +966,20 @@ class Ops:
               and chosen.shape[0] == n_tokens and chosen.is_contiguous() and weights.is_contiguous(), "chosen and weights [T, top]")
         self._check(self.lib.ta_expert_gate(_ptr(gate_up), _ptr(chosen), _ptr(weights), n_tokens, chosen.shape[1], n_experts,
                                             inner, shared, out.shape[1], _ptr(out), _code(out.dtype), _ptr(shared_weight),
-                                            self._stream()), "expert_gate")
+                                            int(bool(weigh_input)), self._stream()), "expert_gate")
+        return out
+
+    def expert_gate_slots(self, gate_up: torch.Tensor, slot_of: torch.Tensor, weights: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+        """Rows sorted by expert (`expert_slots`): gate_up [slots, 2 inner], weights float32 [T, top] ->
+        out[slot_of[t top + k]] = silu(w gate) * (w up) with w = weights[t, k]; slots of no pair are left as they are."""
+        _dev(gate_up, slot_of, weights, out)
+        inner = gate_up.shape[1] // 2
+        _need(gate_up.is_contiguous() and out.is_contiguous() and gate_up.shape[1] == 2 * inner
+              and tuple(out.shape) == (gate_up.shape[0], inner) and out.dtype == gate_up.dtype, "gate_up [slots, 2 inner], out [slots, inner]")
+        _need(slot_of.dtype == torch.int32 and weights.dtype == torch.float32 and weights.is_contiguous()
+              and slot_of.numel() == weights.numel(), "slot_of int32 [T top], weights float32 [T, top]")
+        self._check(self.lib.ta_expert_gate_slots(_ptr(gate_up), _ptr(slot_of), _ptr(weights), weights.numel(), inner, _ptr(out),
+                                                  _code(out.dtype), self._stream()), "expert_gate_slots")
         return out
 
     def side_gate(self, gate: torch.Tensor, table: torch.Tensor, token_ids: torch.Tensor, offset: int, dim: int,

@@ -42,7 +42,9 @@ class GQAttention(Mixer):
     weight `q_norm` / `k_norm` [d] for all heads), `value_norm` (every value head brought to unit RMS, no weight),
     `value_mix` (see `MixerSpec`; the share is the tensor `vmix`, one number) and `talking` (behind the softmax the heads'
     weights are mixed, head h's becoming sum_g talk[h, g] weight_g with the tensor `talk` [H, H], and then meet the
-    values of head h's own kv head).  For the kernels the maps of differential heads are
+    values of head h's own kv head), `tied_values` (the values are the keys as projected, without a rotation: no value
+    projection) and `fixed_sink` c (every head's softmax has exp(c) added to its denominator: a sink that is a constant).
+    A position encoding of kind `query_temperature` takes the layer here too.  For the kernels the maps of differential heads are
     heads of their own: the query rows are reordered at load time to (kv head, map, head within the group), so
     that map m of kv head g is key head 2 g + m in the ordinary grouping, and key heads 2 g and 2 g + 1 read
     value head g (`value_heads`).
@@ -86,7 +88,9 @@ class GQAttention(Mixer):
     @staticmethod
     def _is_extended(spec: MixerSpec) -> bool:
         return (spec.differential is not None or bool(spec.keep_first) or spec.qk_norm is not None or spec.head_gate
-                or spec.softcap is not None or spec.value_norm or spec.value_mix is not None or spec.talking or (spec.position is not None and spec.position.kind == "rope_partial"))
+                or spec.softcap is not None or spec.value_norm or spec.value_mix is not None or spec.talking
+                or spec.tied_values or spec.fixed_sink is not None
+                or (spec.position is not None and spec.position.kind in ("rope_partial", "query_temperature")))
 
     def _build_extended(self, spec: MixerSpec, tensors: dict[str, torch.Tensor], runtime: Runtime) -> None:
         if not spec.own_kv or spec.chunk is not None or spec.distance_bias is not None or spec.out_bias:
@@ -94,6 +98,8 @@ class GQAttention(Mixer):
                              "the partial rotation do not combine with chunks, distance bias, borrowed keys or an output bias")
         if spec.sink and spec.differential is not None:
             raise ValueError("a sink belongs to one softmax a head, not to the two maps of a differential head")
+        if spec.sink and spec.fixed_sink is not None:
+            raise ValueError("a learned sink and a fixed one")
         if spec.softcap is not None and not spec.softcap > 0:
             raise ValueError(f"a cap on the scores is positive, found {spec.softcap}")
         if spec.qk_norm not in (None, "whole", "head"):
@@ -106,21 +112,26 @@ class GQAttention(Mixer):
         if self.head_wise and (spec.qkv_bias or spec.differential is not None or spec.qk_norm == "whole"):
             raise ValueError("norms of single heads and changed values do not combine with biases, differential maps or a norm "
                              "over the whole projection")
+        self.tied = spec.tied_values
+        if self.tied and (self.head_wise or spec.differential is not None or spec.qk_norm is not None or spec.qkv_bias
+                          or self.dv != self.d or (spec.position is not None and spec.position.kind != "query_temperature")):
+            raise ValueError("values that are the keys do not combine with biases, norms, differential maps, a rotation or "
+                             "value heads of another size")
         if spec.talking:
-            if spec.differential is not None or spec.sink or spec.softcap is not None or spec.window is not None:
+            if spec.differential is not None or spec.sink or spec.fixed_sink is not None or spec.softcap is not None or spec.window is not None:
                 raise ValueError("mixed heads do not combine with differential maps, sinks, capped scores or windows")
             self.talk = tensors["talk"].to(torch.float32).contiguous()
         self.share = tensors["vmix"].to(torch.float32).reshape(1).contiguous() if spec.value_mix is not None else None
         H, G, d, dv, hidden = self.n_q, self.n_kv, self.d, self.dv, spec.hidden_size
         self.maps = 2 if spec.differential is not None else 1
         self.group = H // G
-        q, k, v = tensors["q_proj.weight"], tensors["k_proj.weight"], tensors["v_proj.weight"]
+        q, k = tensors["q_proj.weight"], tensors["k_proj.weight"]
 
         def by_kv_head(rows):           # [H, maps, d, ...] -> (kv head, map, head within the group)
             tail = rows.shape[1:]
             return rows.reshape(G, self.group, self.maps, d, *tail).transpose(1, 2).reshape(H * self.maps * d, *tail)
 
-        joined = [by_kv_head(q) if self.maps > 1 else q, k, v]
+        joined = [by_kv_head(q) if self.maps > 1 else q, k] + ([] if self.tied else [tensors["v_proj.weight"]])
         self.gate_offset = sum(part.shape[0] for part in joined)
         if spec.head_gate:
             joined.append(tensors["gate_proj.weight"])
@@ -149,6 +160,8 @@ class GQAttention(Mixer):
         self.more = {}
         if spec.sink:
             self.more["sinks"] = tensors["sink"].to(torch.float32).contiguous()
+        if spec.fixed_sink is not None:
+            self.more["sinks"] = torch.full((H * self.maps,), float(spec.fixed_sink), dtype=torch.float32, device=runtime.device)
         if spec.softcap is not None:
             self.more["softcap"] = float(spec.softcap)
         self.w_o, self.b_o = tensors["o_proj.weight"], None
@@ -156,10 +169,13 @@ class GQAttention(Mixer):
         self.window = spec.window
         self.keep_first = int(spec.keep_first) if spec.window is not None else 0
         position = spec.position
+        if self.tied and position is None:
+            position = PositionSpec("query_temperature", head_dim=d, options={"coef": 0.0, "every": 1})
         if position is None or position.kind == "none":      # nothing turns: the same kernel with no coordinates to rotate
             position = PositionSpec("rope_partial", head_dim=d, theta=1.0, options={"dims": 0})
-        if position.kind != "rope_partial":
-            raise ValueError(f"these options store keys through the partial rotation's kernel, not {position.kind!r}")
+        if position.kind not in ("rope_partial", "query_temperature"):
+            raise ValueError(f"these options store keys through the partial rotation's or the query temperature's kernel, "
+                             f"not {position.kind!r}")
         self.position = POSITIONS.get(position.kind)(position, runtime)
         self.plain = False
 
@@ -171,8 +187,9 @@ class GQAttention(Mixer):
             q_out, kv_out = 2 * q_out, 2 * kv_out
         out = {"q_proj.weight": TensorSpec((q_out, hidden)), "o_proj.weight": TensorSpec((hidden, spec.n_heads * dv))}
         if spec.own_kv:
-            out.update({"k_proj.weight": TensorSpec((kv_out, hidden)),
-                        "v_proj.weight": TensorSpec((spec.n_kv_heads * dv, hidden))})
+            out["k_proj.weight"] = TensorSpec((kv_out, hidden))
+            if not spec.tied_values:
+                out["v_proj.weight"] = TensorSpec((spec.n_kv_heads * dv, hidden))
         if spec.qkv_bias:
             out["q_proj.bias"] = TensorSpec((q_out,), role="vector")
             if spec.own_kv:
@@ -267,7 +284,8 @@ class GQAttention(Mixer):
                 ctx.shared["values"] = qkv[:, at:at + self.n_kv * self.dv]
         else:
             self.position.encode_and_store(qkv, None, heads, key_heads, self.d, ctx, cache, value_dim=self.dv,
-                                           value_heads=self.n_kv, q_norm=self.q_norm, k_norm=self.k_norm, eps=self.eps)
+                                           value_heads=self.n_kv, q_norm=self.q_norm, k_norm=self.k_norm, eps=self.eps,
+                                           **({"tied_values": True} if self.tied else {}))
         if self.talk is not None:
             mixed = torch.empty((x.shape[0], heads * self.dv), dtype=x.dtype, device=x.device)
             ops.talking_attention(qkv, mixed, cache.k_pages, cache.v_pages, ctx.positions, ctx.entry_of_token,

@@ -62,8 +62,8 @@ class ParallelBlock(Block):
 
 @BLOCKS.register("parallel_scaled")
 class ScaledParallelBlock(Block):
-    """x + (s1 * mixer(norm1(x)) + s2 * feed_forward(norm2(x))): two norms of the same x, one for each sub-layer, and
-    (option `layer_scale`) a learned scale per coordinate on each output (the block's own tensors `ls1`, `ls2` [width]).
+    """x + (s1 * mixer(norm1(x)) + s2 * feed_forward(norm2(x))): two norms of the same x, one for each sub-layer (option
+    `one_norm`: the mixer's norm is the layer's norm and both sub-layers read its output), and (option `layer_scale`) a learned scale per coordinate on each output (the block's own tensors `ls1`, `ls2` [width]).
     The outputs are handed on as the terms of a `ScaledSum`: the next norm weights and adds them to the float32 stream
     and normalises the sum in one kernel.  Where both norms are of the form x / sqrt(mean(x^2) + eps) * w, that kernel
     also gives both normalised copies of the row at once.  A mixer may itself hand back a `ScaledSum` (two mixers
@@ -85,6 +85,7 @@ class ScaledParallelBlock(Block):
         self.mixer_norm, self.mixer = mixer_norm, mixer
         self.feed_forward_norm, self.feed_forward = feed_forward_norm, feed_forward
         self.runtime = runtime
+        self.one_norm = bool(layer.options.get("one_norm"))
         scaled = bool(layer.options.get("layer_scale"))
         self.mixer_scale = tensors["ls1"].to(torch.float32).contiguous() if scaled else None
         self.ff_scale = tensors["ls2"].to(torch.float32).contiguous() if scaled and feed_forward is not None else None
@@ -93,6 +94,9 @@ class ScaledParallelBlock(Block):
         """Both sub-layers' inputs from the stream and what is still to be added to it."""
         if self.feed_forward is None:
             return self.mixer_norm.apply(residual, delta), None
+        if self.one_norm:
+            h = self.mixer_norm.apply(residual, delta)
+            return h, h
         ops = self.runtime.ops
         first, second = self.mixer_norm.fold(), self.feed_forward_norm.fold()
         if first is not None and second is not None and hasattr(ops, "add_terms_rmsnorm") \

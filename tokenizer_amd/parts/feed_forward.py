@@ -146,7 +146,10 @@ class RoutedExperts(FeedForward):
     the chosen's sum (+ 1e-20).  `router` "softmax_all": the same with s = softmax over all experts and no correction;
     `group_worth` "max": a group is worth its largest choice score.  `shared_gate`: the shared expert's output times
     sigmoid(W_sg x), one number a token (tensor `shared.sg` [1, hidden]; its row rides behind the router's rows, so
-    the gate's logit is a float32 sum of the same product).  Logits, scores and weights are float32.
+    the gate's logit is a float32 sum of the same product).  Of the scored routers: `correction` False (no such tensor),
+    `renormalize` False (the weights are the chosen experts' s themselves); `weigh_input` (gated experts): an expert is
+    handed weight * x, so its gate and its up branch are both multiplied by the weight before the activation and what it
+    gives back is added as it is.  Logits, scores and weights are float32.
     """
     graph_safe = True
     GROUPED_FROM = 1024        # (token, expert) pairs from which the sorted form runs
@@ -164,7 +167,9 @@ class RoutedExperts(FeedForward):
         self.spec, self.runtime = spec, runtime
         self.n_experts, self.top_k = spec.n_experts, spec.top_k
         self.inner, self.shared = spec.intermediate_size, spec.shared_size
-        self.gated, self.sigmoid = spec.gated, spec.router == "sigmoid"
+        self.gated, self.sigmoid, self.weigh_input = spec.gated, spec.router == "sigmoid", spec.weigh_input
+        if self.weigh_input and (not self.gated or self.shared):
+            raise ValueError("a weighted input belongs to gated experts without a shared one here")
         self.scored = spec.router in ("sigmoid", "softmax_all")      # chosen by scores, weighted by them over their sum
         if not self.gated and self.shared:
             raise ValueError("ungated experts have no shared expert here")
@@ -175,7 +180,7 @@ class RoutedExperts(FeedForward):
         if self.shared_gate:          # the gate's row behind the experts' rows: its logit comes out of the same product
             self.w_router = torch.cat([self.w_router, tensors["shared.sg"].reshape(1, -1)], dim=0).contiguous()
         if self.scored:
-            self.correction = tensors["correction"].to(torch.float32).contiguous() if self.sigmoid else None
+            self.correction = tensors["correction"].to(torch.float32).contiguous() if self.sigmoid and spec.correction else None
             self.n_groups, self.keep_groups = int(spec.n_groups), int(spec.keep_groups)
             if self.n_groups and (self.n_experts % self.n_groups or not 0 < self.keep_groups <= self.n_groups
                                   or self.keep_groups * (self.n_experts // self.n_groups) < self.top_k):
@@ -203,7 +208,7 @@ class RoutedExperts(FeedForward):
     @staticmethod
     def tensor_specs(spec: FeedForwardSpec) -> dict[str, TensorSpec]:
         out = {"router": TensorSpec((spec.n_experts, spec.hidden_size), std=0.5)}
-        if spec.router == "sigmoid":
+        if spec.router == "sigmoid" and spec.correction:
             out["correction"] = TensorSpec((spec.n_experts,), role="vector", std=0.2)
         if spec.shared_gate and spec.shared_size:
             out["shared.sg"] = TensorSpec((1, spec.hidden_size), std=0.5)
@@ -221,7 +226,8 @@ class RoutedExperts(FeedForward):
         chosen = torch.empty((x.shape[0], self.top_k), dtype=torch.int32, device=x.device)
         weights = torch.empty((x.shape[0], self.top_k), dtype=torch.float32, device=x.device)
         shared_weight = None
-        if self.sigmoid and not self.shared_gate and self.spec.group_worth == "top2":
+        if self.sigmoid and self.correction is not None and self.spec.renormalize and not self.shared_gate \
+                and self.spec.group_worth == "top2":
             fused = getattr(ops, "route_rows_sigmoid", None)   # few rows: the router's product and the choice in one kernel
             if (fused is None or x.shape[0] > ops.ROUTE_ROWS_FUSED
                     or not fused(x, self.w_router, self.correction, self.n_groups, self.keep_groups, chosen, weights)):
@@ -231,6 +237,8 @@ class RoutedExperts(FeedForward):
             if self.shared_gate:
                 shared_weight = torch.empty((x.shape[0],), dtype=torch.float32, device=x.device)
             kind = dict(softmax=not self.sigmoid, group_max=self.spec.group_worth == "max", gate=shared_weight)
+            if not self.spec.renormalize:
+                kind["renormalize"] = False
             fused = getattr(ops, "route_rows_scores", None)    # few rows: the router's product and the choice in one kernel
             if (fused is None or x.shape[0] > ops.ROUTE_ROWS_FUSED
                     or not fused(x, self.w_router, self.correction, self.n_experts, self.n_groups, self.keep_groups, chosen,
@@ -248,7 +256,8 @@ class RoutedExperts(FeedForward):
         if self.gated and shared_weight is not None:
             ops.expert_gate(gate_up, chosen, weights, self.n_experts, self.inner, self.shared, act, shared_weight=shared_weight)
         elif self.gated:
-            ops.expert_gate(gate_up, chosen, weights, self.n_experts, self.inner, self.shared, act)
+            ops.expert_gate(gate_up, chosen, weights, self.n_experts, self.inner, self.shared, act,
+                            **({"weigh_input": True} if self.weigh_input else {}))
         else:
             ops.expert_act(gate_up, chosen, weights, self.n_experts, self.inner, act)
         return ops.linear(act, self.w_down)
@@ -262,7 +271,9 @@ class RoutedExperts(FeedForward):
         wide = (2 if self.gated else 1) * inner          # an expert's rows of the joined first matrix
         gate_up = ops.grouped_linear(x, row_of, tile_expert, bm, self.w_gate_up, wide * hidden, wide, hidden, torch.bfloat16)
         act = torch.empty((gate_up.shape[0], inner), dtype=x.dtype, device=x.device)
-        if self.gated:
+        if self.weigh_input:
+            ops.expert_gate_slots(gate_up, slot_of, weights, act)
+        elif self.gated:
             ops.silu_gate(gate_up, act)
         else:
             ops.relu2(gate_up, act)
@@ -273,4 +284,6 @@ class RoutedExperts(FeedForward):
         out = torch.empty((x.shape[0], hidden), dtype=x.dtype, device=x.device)
         if shared_weight is not None:
             return ops.expert_combine(rows, slot_of, weights, shared, out, shared_weight=shared_weight)
+        if self.weigh_input:              # (the weights are in the experts' rows already)
+            return ops.expert_combine(rows, slot_of, weights, shared, out, weighted=False)
         return ops.expert_combine(rows, slot_of, weights, shared, out)

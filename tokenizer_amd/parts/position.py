@@ -116,6 +116,29 @@ def yarn_rates(theta: float, dims: int, scaling: dict) -> tuple[torch.Tensor, fl
     return torch.tensor(rates, dtype=torch.float64).to(torch.float32), 0.1 * math.log(factor) + 1.0
 
 
+@POSITIONS.register("query_temperature")
+class QueryTemperature(PositionEncoding):
+    """No rotation: the query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1), a float32 factor
+    (options `coef` and `every`), and keys and values are stored as projected.  `tied_values`: the rows hold no value
+    heads, the keys are stored as the values too."""
+    graph_safe = True
+
+    def __init__(self, spec: PositionSpec, runtime: Runtime):
+        self.runtime, self.coef, self.every = runtime, float(spec.options["coef"]), int(spec.options["every"])
+        if self.every < 1:
+            raise ValueError(f"a query temperature that steps every {self.every} positions")
+
+    def encode_and_store(self, qkv, bias, n_q, n_kv, head_dim, ctx, cache, value_dim=None, value_heads=None,
+                         q_norm=None, k_norm=None, eps=0.0, tied_values=False):
+        if bias is not None or q_norm is not None or k_norm is not None or value_heads not in (None, n_kv):
+            raise ValueError("the query temperature does not combine with biases, normalised projections or shared value heads")
+        slots = ctx.slots[cache.group] if cache.writes and n_kv else None
+        self.runtime.ops.temper_store(qkv, ctx.positions, self.coef, self.every, slots,
+                                      cache.k_pages if slots is not None else None,
+                                      cache.v_pages if slots is not None else None, n_q, n_kv, head_dim,
+                                      head_dim if value_dim is None else value_dim, tied_values)
+
+
 @POSITIONS.register("rope_partial")
 class RotaryPartial(PositionEncoding):
     """Rotation of the first `dims` coordinates of every query and key head (options `dims`, even and at most the

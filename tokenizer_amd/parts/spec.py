@@ -123,6 +123,8 @@ class MixerSpec:
     value_norm: bool = False      # each value head is brought to unit RMS (no weight) before it is cached
     value_mix: str | None = None  # "give": later layers of the model may take in this layer's values; "take": the values
     #                               become (1 - s) v + s v' with v' the giving layer's values of the same token, s learned
+    tied_values: bool = False     # the values are the keys as projected: there is no value projection
+    fixed_sink: float | None = None   # exp of this number joins every head's softmax denominator (no key, no value)
     talking: bool = False         # the heads' softmax weights are mixed with each other by a learned [heads, heads] matrix
     decays: tuple[float, ...] = ()   # retention: each head's decay of its state from token to token
     head_gate: bool = False       # each head's output times sigmoid of one number projected from the mixer's input
@@ -158,6 +160,9 @@ class FeedForwardSpec:
     #                               scores s = sigmoid(logit), chosen by s + `correction` (a tensor, one number an
     #                               expert), weighted by s over the chosen's sum; "softmax_all": scores s = softmax
     #                               over all experts, chosen by s, weighted by s over the chosen's sum
+    correction: bool = True       # "sigmoid": False: no such tensor, chosen by s alone
+    renormalize: bool = True      # "sigmoid", "softmax_all": False: the weights are the chosen experts' s themselves
+    weigh_input: bool = False     # the weight multiplies what an expert is handed, not what it gives back
     n_groups: int = 0             # "sigmoid": experts form so many equal groups of neighbours (0: no groups) ...
     keep_groups: int = 0          # ... of which only the best so many (by the sum of a group's two largest choice
     #                               scores) can be chosen from
