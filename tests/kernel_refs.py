@@ -164,7 +164,8 @@ class PlainOps:
         top = chosen.shape[1]
         z = logits.to(torch.float32)
         s = torch.softmax(z[:, :n_experts], dim=-1) if softmax else torch.sigmoid(z[:, :n_experts])
-        choice = s if correction is None else s + correction.to(torch.float32)
+        # (Chosen by the score alone, without groups: by the logit, whose order is the same.)
+        choice = s + correction.to(torch.float32) if correction is not None else s if n_groups else z[:, :n_experts]
         if n_groups:
             per = n_experts // n_groups
             grouped = choice.reshape(-1, n_groups, per)

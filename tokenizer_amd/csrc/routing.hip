@@ -519,7 +519,8 @@ route_scores_kernel(const float* __restrict__ logits, int stride, const float* _
   for (int e = lane; e < n_experts; e += WAVE) {
     const float s = softmax ? expf(row[e] - top_logit) / total : 1.0f / (1.0f + expf(-row[e]));
     score[e] = s;
-    choice[e] = correction ? s + correction[e] : s;
+    // (Chosen by s alone, without groups: by the logit, whose order is the same and does not end where s rounds to 1.)
+    choice[e] = correction ? s + correction[e] : (n_groups > 0 ? s : row[e]);
   }
   if (gate && live && lane == 0) gate[t] = 1.0f / (1.0f + expf(-row[n_experts]));
   __syncthreads();
@@ -576,7 +577,7 @@ route_rows_sigmoid_kernel(const T* __restrict__ x, int lda, const T* __restrict_
       } else {
         const float s = 1.0f / (1.0f + expf(-sum));
         score[e] = s;
-        choice[e] = correction ? s + correction[e] : s;
+        choice[e] = correction ? s + correction[e] : (n_groups > 0 ? s : sum);
       }
     }
   }
@@ -587,9 +588,9 @@ route_rows_sigmoid_kernel(const T* __restrict__ x, int lda, const T* __restrict_
     for (int e = 0; e < n_experts; ++e) total += expf(score[e] - top_logit);
     __syncthreads();
     for (int e = threadIdx.x; e < n_experts; e += 256) {
-      const float s = expf(score[e] - top_logit) / total;
+      const float z = score[e], s = expf(z - top_logit) / total;
       score[e] = s;
-      choice[e] = correction ? s + correction[e] : s;
+      choice[e] = correction ? s + correction[e] : (n_groups > 0 ? s : z);
     }
     __syncthreads();
   }
