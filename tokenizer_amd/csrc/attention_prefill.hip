@@ -416,7 +416,8 @@ extern "C" int ta_prefill_attention_shared_bf16(const void* q, int q_stride, voi
                                                 const void* cu_q, const void* first_position,
                                                 const void* block_table, int table_stride, int n_q, int n_kv, int d,
                                                 int page_size, int window, float scale, int shape,
-                                                int key_splits, void* part_o, void* part_ml, hipStream_t stream);
+                                                int key_splits, void* part_o, void* part_ml, const void* sinks,
+                                                hipStream_t stream);
 
 // The shape in which the workgroup-shared kernel takes a launch (0: the per-wave kernel takes it), by what the
 // caller asked for and the launch's own plan.
@@ -449,7 +450,7 @@ extern "C" int ta_prefill_attention_key_splits(int n_tiles, int n_q, int n_kv, i
 // (float [n_q] or null): head h's score loses slopes[h] per position of distance; sinks (float [n_q] or null): exp(sinks[h])
 // joins the softmax's denominator.  keep_first > 0 (with a window): keys at positions below it stay visible behind the
 // window; n_v (a divisor of n_kv): the value pages hold n_v heads, key head g reads value head g / (n_kv / n_v).
-// With any of these the per-wave kernel runs, and the keys are not cut.
+// With any of these but the sinks the per-wave kernel runs, and the keys are not cut.
 extern "C" int ta_prefill_attention_bf16(const void* q, int q_stride, void* out, const void* k_pages,
                                          const void* vt_pages, const void* tiles, int n_tiles, const void* cu_q,
                                          const void* first_position, const void* block_table, int table_stride,
@@ -462,14 +463,14 @@ extern "C" int ta_prefill_attention_bf16(const void* q, int q_stride, void* out,
   if (n_v <= 0) n_v = n_kv;
   if (n_kv % n_v || keep_first < 0 || (keep_first > 0 && (window < 0 || chunk > 0 || slopes))) return -1;
   const PrefillExtras extra = {chunk, (const float*)slopes, (const float*)sinks, keep_first, n_v, softcap};
-  const bool plain = chunk <= 0 && !slopes && !sinks && keep_first == 0 && n_v == n_kv && !(softcap > 0.f);
+  const bool plain = chunk <= 0 && !slopes && keep_first == 0 && n_v == n_kv && !(softcap > 0.f);
   const int shape = plain ? shared_shape_for(n_tiles, n_q, n_kv, d, window, shared_shape, max_keys, waves, shared) : 0;
   if (shape) {
     const int parts = (part_o && part_ml)
         ? ta_prefill_attention_shared_key_splits(n_tiles, n_q, n_kv, planned_reach(max_keys, window), shape) : 1;
     const int status = ta_prefill_attention_shared_bf16(q, q_stride, out, k_pages, vt_pages, tiles, n_tiles, cu_q,
                                                         first_position, block_table, table_stride, n_q, n_kv, d,
-                                                        page_size, window, scale, shape, parts, part_o, part_ml, stream);
+                                                        page_size, window, scale, shape, parts, part_o, part_ml, sinks, stream);
     if (status != -2) return status;
   }
 #define CASE(DD, HG) case DD: return launch_prefill<DD, HG>(q, q_stride, out, k_pages, vt_pages, tiles, n_tiles, cu_q, \

@@ -244,7 +244,8 @@ __device__ __forceinline__ void shared_block(const char* buf, int kb, int col, i
   }
 }
 
-// Arguments as in prefill_attention_kernel.  Dynamic LDS: two blocks for each of the KG groups of four waves
+// Arguments as in prefill_attention_kernel (sinks: float [n_q] or null, exp(sinks[h]) joins the softmax's denominator; with
+// the keys cut over workgroups it rides in the first part).  Dynamic LDS: two blocks for each of the KG groups of four waves
 // (2 * KG * Staged<D>::BYTES).
 // KG = 2: two groups of four waves, each with the same heads, take the blocks in turn (group i the blocks i,
 // i + 2, ...) and merge their softmax states through LDS at the end: half as many turns for a long walk, for
@@ -256,7 +257,8 @@ prefill_attention_shared_kernel(const bf16_t* __restrict__ q, int q_stride, bf16
                                 const int* __restrict__ tiles, int n_tiles, const int* __restrict__ cu_q,
                                 const int* __restrict__ first_position, const int* __restrict__ block_table,
                                 int table_stride, int n_q, int n_kv, int page_size, int window, float scale_log2,
-                                int key_splits, float* __restrict__ part_o, float* __restrict__ part_ml) {
+                                int key_splits, float* __restrict__ part_o, float* __restrict__ part_ml,
+                                const float* __restrict__ sinks) {
   constexpr int KS = D / 32;
   constexpr int DB = D / 16;
   constexpr int NW = SHARED_WAVES;
@@ -412,6 +414,25 @@ prefill_attention_shared_kernel(const bf16_t* __restrict__ q, int q_stride, bf16
       m[h] = m_all;                                        // what the sums now stand under (a part hands it on)
     }
   }
+  // What the sums stand under, in the exponent's units (base 2).
+  float under[HG];
+#pragma unroll
+  for (int h = 0; h < HG; ++h) under[h] = (m[h] == -INFINITY) ? -INFINITY : m[h] * scale_log2;
+  if (sinks && split == 0) {
+    // The larger of the running maximum and the sink, so that neither overflows.
+#pragma unroll
+    for (int h = 0; h < HG; ++h) {
+      if (h >= heads_here) break;
+      const float sink = sinks[head0 + h] * 1.4426950408889634f, top = fmaxf(under[h], sink);
+      const float f = __builtin_amdgcn_exp2f(under[h] - top);
+      l[h][0] = l[h][0] * f + __builtin_amdgcn_exp2f(sink - top);
+#pragma unroll
+      for (int db = 0; db < DB; ++db)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) acc[h][db][r] *= f;
+      under[h] = top;
+    }
+  }
   if (key_splits > 1) {
     // This workgroup's part of the keys: the state goes out as it is, item (tile, token) x head x part, for the
     // kernel that merges the parts (maximum in natural units of the scaled scores, sum, unnormalised output).
@@ -421,7 +442,7 @@ prefill_attention_shared_kernel(const bf16_t* __restrict__ q, int q_stride, bf16
       if (col >= n_valid) continue;
       const size_t at = (((size_t)tile_index * 16 + col) * n_q + head0 + h) * key_splits + split;
       if (g == 0) {
-        part_ml[2 * at] = (m[h] == -INFINITY) ? -INFINITY : m[h] * scale_log2 * 0.6931471805599453f;
+        part_ml[2 * at] = under[h] * 0.6931471805599453f;
         part_ml[2 * at + 1] = l[h][0];
       }
 #pragma unroll
@@ -451,7 +472,7 @@ template <int D, int HG, int KG>
 static int launch_shared(const void* q, int q_stride, void* out, const void* k_pages, const void* vt_pages,
                          const void* tiles, int n_tiles, const void* cu_q, const void* first_position,
                          const void* block_table, int table_stride, int n_q, int n_kv, int page_size, int window,
-                         float scale, int key_splits, void* part_o, void* part_ml, hipStream_t stream) {
+                         float scale, int key_splits, void* part_o, void* part_ml, const void* sinks, hipStream_t stream) {
   const int group = n_q / n_kv;
   const long workgroups = (long)n_tiles * n_kv * ((group + HG * SHARED_WAVES - 1) / (HG * SHARED_WAVES)) * key_splits;
   if (workgroups > 0x7fffffffL) return -1;
@@ -466,7 +487,8 @@ static int launch_shared(const void* q, int q_stride, void* out, const void* k_p
   prefill_attention_shared_kernel<D, HG, KG><<<(unsigned)workgroups, SHARED_WAVES * KG * WAVE, lds, stream>>>(
       (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_pages, (const bf16_t*)vt_pages, (const int*)tiles,
       n_tiles, (const int*)cu_q, (const int*)first_position, (const int*)block_table, table_stride, n_q, n_kv, page_size,
-      window, scale * 1.4426950408889634f, key_splits, (float*)part_o, (float*)part_ml);
+      window, scale * 1.4426950408889634f, key_splits, (float*)part_o, (float*)part_ml,
+      (const float*)sinks);
   int status = LAUNCH_STATUS();
   if (status == 0 && key_splits > 1)
     status = ta_attention_merge_tiles(part_o, part_ml, tiles, n_tiles, cu_q, out, n_q, D, key_splits, stream);
@@ -550,13 +572,14 @@ extern "C" int ta_prefill_attention_shared_bf16(const void* q, int q_stride, voi
                                                 const void* cu_q, const void* first_position,
                                                 const void* block_table, int table_stride, int n_q, int n_kv, int d,
                                                 int page_size, int window, float scale, int shape,
-                                                int key_splits, void* part_o, void* part_ml, hipStream_t stream) {
+                                                int key_splits, void* part_o, void* part_ml, const void* sinks,
+                                                hipStream_t stream) {
   if (n_tiles <= 0) return 0;
   const int heads_per_wave = shape % 10, key_groups = shape / 10 + 1;
   if (n_kv <= 0 || n_q % n_kv || page_size % 16 || heads_per_wave < 1 || heads_per_wave > 2 || key_groups > 2) return -1;
   if (key_splits < 1 || key_splits > 64 || (key_splits > 1 && (!part_o || !part_ml))) return -1;
 #define GO(DD, HG, KG) return launch_shared<DD, HG, KG>(q, q_stride, out, k_pages, vt_pages, tiles, n_tiles, cu_q, \
-    first_position, block_table, table_stride, n_q, n_kv, page_size, window, scale, key_splits, part_o, part_ml, stream);
+    first_position, block_table, table_stride, n_q, n_kv, page_size, window, scale, key_splits, part_o, part_ml, sinks, stream);
 #define SIZE(DD) case DD: if (key_groups == 2) { if (heads_per_wave == 1) GO(DD, 1, 2) GO(DD, 2, 2) } \
     if (heads_per_wave == 1) GO(DD, 1, 1) GO(DD, 2, 1)
   switch (d) {

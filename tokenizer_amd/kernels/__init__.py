@@ -1099,7 +1099,7 @@ class Ops:
         for extra in (slopes, sinks):
             _need(extra is None or (extra.dtype == torch.float32 and extra.numel() == n_q), "slopes and sinks are float32 [n_q]")
         _need(chunk is None or chunk > 0, "a chunk has at least one position")
-        plain = value_dim == head_dim and chunk is None and slopes is None and sinks is None
+        plain = value_dim == head_dim and chunk is None and slopes is None     # (but for the sinks)
         value_heads = n_kv if value_heads is None else int(value_heads)
         keep_first = int(keep_first) if window is not None else 0
         _need(value_heads > 0 and n_kv % value_heads == 0 and keep_first >= 0, "value heads divide the key heads")
@@ -1123,7 +1123,7 @@ class Ops:
             args = (qkv, out, k_pages, v_pages, positions, entry_of_token, block_table, n_q, n_kv, head_dim,
                     page_size, window, scale, max_position)
             plain = plain and not softcap
-            extras = {} if plain else dict(chunk=chunk, slopes=slopes, sinks=sinks, keep_first=keep_first,
+            extras = {} if plain and sinks is None else dict(chunk=chunk, slopes=slopes, sinks=sinks, keep_first=keep_first,
                                            value_heads=value_heads, softcap=softcap)
             if batch is None:
                 return self._decode_attention(*args, **extras)
