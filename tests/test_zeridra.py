@@ -696,3 +696,59 @@ def test_one_norm_for_both_sub_layers_with_scales_on_their_outputs(backend, laye
     bound = 1e-5 if dtype == torch.float32 else 2e-2
     assert float((residual.double() - want).abs().max()) <= bound * float(want.abs().max())
     assert float((out.double() - plain.norm(want, final.double(), 1e-5)).abs().max()) <= bound * 4
+
+
+@pytest.mark.parametrize("backend", BACKENDS)
+@pytest.mark.parametrize("width", [40, 64, 52, 200, 1028, 2056, 4096, 4100])
+@pytest.mark.parametrize("count,scaled", [(1, False), (1, True), (2, True), (2, False), (3, True), (4, True)])
+def test_weighted_terms_onto_the_stream_and_the_norm(backend, width, count, scaled):
+    ops, device, dtype = ops_for(backend)
+    gen = torch.Generator().manual_seed(width + count)
+    n = 11
+    residual = torch.randn(n, width, generator=gen)
+    vectors = [1 + 0.4 * torch.randn(width, generator=gen) for _ in range(count + 2)]
+    terms = [(torch.randn(n, width, generator=gen).to(dtype), 0.5 + k, vectors[k] if scaled else None) for k in range(count)]
+    want = residual.double()
+    for rows, factor, scale in terms:
+        want = want + rows.double() * factor * (1.0 if scale is None else scale.double())
+    on = [(rows.to(device), factor, None if scale is None else scale.to(device)) for rows, factor, scale in terms]
+    bound = 2e-6 if dtype == torch.float32 else 1e-2
+    for rows_picked in (None, [3, 0, 10]):
+        stream = residual.clone().to(device)
+        out = torch.empty((n if rows_picked is None else 3, width), dtype=dtype, device=device)
+        second = torch.empty_like(out)
+        pick = None if rows_picked is None else torch.tensor(rows_picked, dtype=torch.int32, device=device)
+        ops.add_terms_rmsnorm(stream, on, vectors[-1].to(device), 1e-5, out, pick, store_residual=pick is None,
+                              weight2=vectors[-2].to(device), eps2=1e-3, out2=second)
+        x = want if rows_picked is None else want[rows_picked]
+        for got, weight, eps in ((out, vectors[-1], 1e-5), (second, vectors[-2], 1e-3)):
+            normed = plain.norm(x, weight.double(), eps)
+            assert float((got.double().cpu() - normed).abs().max()) <= bound * float(normed.abs().max())
+        kept = stream.double().cpu()
+        assert float((kept - (want if pick is None else residual.double())).abs().max()) <= 2e-6 * float(want.abs().max())
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("width", [64, 1024, 1028, 3584, 4096, 4104])
+@pytest.mark.parametrize("parts", [1, 3, 4, 5, 8, 13])
+@pytest.mark.parametrize("scaled", [True, False])
+def test_a_term_that_is_a_product_still_in_parts(width, parts, scaled):
+    from tokenizer_amd.kernels import PendingSum, get_ops
+    ops, device = get_ops(), torch.device("cuda:0")
+    gen = torch.Generator().manual_seed(width + parts)
+    n = 9
+    residual, rows = torch.randn(n, width, generator=gen), torch.randn(n, width, generator=gen).to(torch.bfloat16)
+    slabs = torch.randn(parts, n, width, generator=gen)
+    weight, one, two = (1 + 0.4 * torch.randn(width, generator=gen) for _ in range(3))
+    want = residual.double() + rows.double() * (one.double() if scaled else 1.0) + slabs.double().sum(0) * (two.double() if scaled else 1.0)
+    for rows_picked in (None, [8, 2]):
+        stream = residual.clone().to(device)
+        out = torch.empty((n if rows_picked is None else 2, width), dtype=torch.bfloat16, device=device)
+        terms = [(rows.to(device), 1.0, one.to(device) if scaled else None),
+                 (PendingSum(ops, slabs.to(device), None, torch.bfloat16), 1.0, two.to(device) if scaled else None)]
+        pick = None if rows_picked is None else torch.tensor(rows_picked, dtype=torch.int32, device=device)
+        ops.add_terms_rmsnorm(stream, terms, weight.to(device), 1e-5, out, pick, store_residual=pick is None)
+        normed = plain.norm(want if pick is None else want[rows_picked], weight.double(), 1e-5)
+        assert float((out.double().cpu() - normed).abs().max()) <= 1e-2 * float(normed.abs().max())
+        rough = 2e-6 if width <= 4096 else 1e-2              # (rows too long for that kernel: the parts are added into bfloat16 first)
+        assert pick is not None or float((stream.double().cpu() - want).abs().max()) <= rough * float(want.abs().max())

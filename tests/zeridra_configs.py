@@ -40,7 +40,7 @@ ZERIDRA = {
         _layer(_attention(4, 2, 16, 0.3, 0.4, 11), (6, 2, 24)), _layer(_latent(4, 16, 8, 24, 24, 40, 19, 0.3, 10000.0), (4, 1, 20)),
         _layer(_attention(6, 2, 24, 0.2, 0.25, 30)), _layer(_latent(3, 20, 8, 16, 32, 40, 37, 0.25, 10000.0, kv_from=1), (5, 3, 16)),
         _layer(_latent(2, 16, 4, 8, 16, 32, 33, 0.35, 500.0), (8, 2, 16)),
-        _layer(_latent(5, 12, 8, 10, 28, 40, 5, 0.3, 10000.0, kv_from=1), (3, 1, 40))]), 3),
+        _layer(_latent(5, 12, 8, 10, 28, 40, 5, 0.3, 10000.0, kv_from=1), (3, 1, 40))]), 10),
     # Sizes that are no multiples of eight anywhere; as many key heads as query heads; every expert chosen.
     "B": (_model(97, 52, 2e-6, 3.5, 1.3, 9.0, [
         _layer(_latent(3, 10, 6, 14, 20, 22, 21, 0.35, 300.0), (5, 1, 10)), _layer(_attention(3, 3, 10, 0.4, 0.5, 7), (3, 3, 14)),

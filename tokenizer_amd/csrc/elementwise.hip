@@ -315,21 +315,6 @@ add_pair_rmsnorm_kernel(float* __restrict__ residual, const T* __restrict__ firs
   }
 }
 
-extern "C" int ta_add_pair_rmsnorm(void* residual, const void* first, const void* second, const void* weight, void* out,
-                                   const void* rows, int n_rows, int hidden, float eps, int store_residual, int dtype,
-                                   hipStream_t stream) {
-  if (n_rows <= 0) return 0;
-  if (hidden <= 0 || hidden > 256 * 32 || !first || !second) return -1;
-#define PAIR(TT, PP) add_pair_rmsnorm_kernel<TT, PP><<<n_rows, 256, 0, stream>>>((float*)residual, (const TT*)first, \
-    (const TT*)second, (const float*)weight, (TT*)out, (const int*)rows, hidden, eps, store_residual)
-#define PAIR_SIZES(TT) if (hidden <= 256) PAIR(TT, 1); else if (hidden <= 1024) PAIR(TT, 4); else if (hidden <= 2048) PAIR(TT, 8); \
-                       else if (hidden <= 4096) PAIR(TT, 16); else PAIR(TT, 32)
-  if (dtype == DT_F32) { PAIR_SIZES(float); } else { PAIR_SIZES(bf16_t); }
-#undef PAIR_SIZES
-#undef PAIR
-  return LAUNCH_STATUS();
-}
-
 // Sub-layers' outputs still to be weighted and added: up to four terms, term k = factor[k] * scale[k][h] * rows[k][r, h]
 // (scale float [hidden] or null).  For output row i, r = rows ? rows[i] : i; x = residual[r] + (the terms' sum), all
 // float; if store_residual: residual[r] = x; out[i] = weight ? x / sqrt(mean(x^2) + eps) * weight : x, in rows of
@@ -392,6 +377,136 @@ add_terms_rmsnorm_kernel(float* __restrict__ residual, SumTerms terms, const flo
   }
 }
 
+// One more term that is a product still in parts: factor * scale[h] * the sum over `count` slabs [n_tokens, hidden] of floats,
+// `stride` floats apart, added in their order.
+struct SlabTerm {
+  const float* slabs;
+  const float* scale;
+  float factor;
+  int count;
+  size_t stride;
+};
+
+// The same for rows of up to 4,096 elements (a multiple of 4) with a norm weight, in pieces of four elements: everything a
+// thread needs (the old residual, the terms, their scales, the norm weights and the first slabs) is asked for at the start,
+// as in add_rmsnorm_vec_kernel.  COUNT terms of rows, all of them with a scale (SCALED) or none; SLABS: and one term in
+// parts behind them.
+template <typename T, int CHUNKS, int COUNT, bool SCALED, bool SLABS>
+__global__ void __launch_bounds__(256)
+add_terms_rmsnorm_vec_kernel(float* __restrict__ residual, SumTerms terms, const float* __restrict__ weight, T* __restrict__ out,
+                             const int* __restrict__ rows, int hidden, float eps, int store_residual, int out_stride,
+                             const float* __restrict__ weight2, float eps2, T* __restrict__ out2, SlabTerm tail) {
+  HELD(residual, weight, out, rows, hidden, eps, store_residual, out_stride, weight2, out2);
+  __shared__ float scratch[16];
+  constexpr int FIRST = CHUNKS == 1 ? 8 : 4;                 // slabs asked for at the start
+  const int i = blockIdx.x;
+  const int r = rows ? scalar_int(rows + i) : i;
+  float* res = residual + (size_t)r * hidden;
+  const float* gain2_at = out2 ? weight2 : weight;           // (without a second output: loaded from a valid place, not used)
+  float4 x[CHUNKS], term[CHUNKS][COUNT], scale[CHUNKS][COUNT], gain[CHUNKS], gain2[CHUNKS];
+  float4 slab[CHUNKS][SLABS ? FIRST : 1], tail_scale[CHUNKS];
+#pragma unroll
+  for (int c = 0; c < CHUNKS; ++c) {
+    const int h = min((c * 256 + (int)threadIdx.x) * 4, hidden - 4);
+    x[c] = ld4(res + h);
+#pragma unroll
+    for (int k = 0; k < COUNT; ++k) {
+      term[c][k] = ld4(reinterpret_cast<const T*>(terms.rows[k]) + (size_t)r * hidden + h);
+      if (SCALED) scale[c][k] = ld4(terms.scale[k] + h);
+    }
+    if (SLABS) {
+      if (SCALED) tail_scale[c] = ld4(tail.scale + h);
+#pragma unroll
+      for (int j = 0; j < FIRST; ++j)                        // (past the last slab: the last one again, not used)
+        slab[c][j] = ld4(tail.slabs + (size_t)min(j, tail.count - 1) * tail.stride + (size_t)r * hidden + h);
+    }
+    gain[c] = ld4(weight + h);
+    gain2[c] = ld4(gain2_at + h);
+  }
+  float sq = 0.f;
+#pragma unroll
+  for (int c = 0; c < CHUNKS; ++c) {
+    const int h = (c * 256 + threadIdx.x) * 4;
+    float4 sum = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+    for (int k = 0; k < COUNT; ++k) {
+      const float f = terms.factor[k];
+      float4 v = make_float4(f * term[c][k].x, f * term[c][k].y, f * term[c][k].z, f * term[c][k].w);
+      if (SCALED) { v.x *= scale[c][k].x; v.y *= scale[c][k].y; v.z *= scale[c][k].z; v.w *= scale[c][k].w; }
+      if (k == 0) sum = v;
+      else { sum.x += v.x; sum.y += v.y; sum.z += v.z; sum.w += v.w; }
+    }
+    if (SLABS) {
+      float4 v = slab[c][0];
+#pragma unroll
+      for (int j = 1; j < FIRST; ++j)
+        if (j < tail.count) { v.x += slab[c][j].x; v.y += slab[c][j].y; v.z += slab[c][j].z; v.w += slab[c][j].w; }
+      for (int j = FIRST; j < tail.count; ++j) {
+        const float4 more = ld4(tail.slabs + (size_t)j * tail.stride + (size_t)r * hidden + min(h, hidden - 4));
+        v.x += more.x; v.y += more.y; v.z += more.z; v.w += more.w;
+      }
+      v.x *= tail.factor; v.y *= tail.factor; v.z *= tail.factor; v.w *= tail.factor;
+      if (SCALED) { v.x *= tail_scale[c].x; v.y *= tail_scale[c].y; v.z *= tail_scale[c].z; v.w *= tail_scale[c].w; }
+      sum.x += v.x; sum.y += v.y; sum.z += v.z; sum.w += v.w;
+    }
+    x[c].x += sum.x; x[c].y += sum.y; x[c].z += sum.z; x[c].w += sum.w;
+    if (h >= hidden) x[c] = make_float4(0.f, 0.f, 0.f, 0.f);
+    else if (store_residual) st4(res + h, x[c]);
+    sq += x[c].x * x[c].x + x[c].y * x[c].y + x[c].z * x[c].z + x[c].w * x[c].w;
+  }
+  const float mean = block_sum(sq, scratch) / (float)hidden;
+  const float inv = 1.0f / sqrtf(mean + eps);
+  T* dst = out + (size_t)i * out_stride;
+#pragma unroll
+  for (int c = 0; c < CHUNKS; ++c) {
+    const int h = (c * 256 + threadIdx.x) * 4;
+    if (h >= hidden) continue;
+    const float4 w = gain[c];
+    st4(dst + h, make_float4(x[c].x * inv * w.x, x[c].y * inv * w.y, x[c].z * inv * w.z, x[c].w * inv * w.w));
+    if (out2) {
+      const float inv2 = 1.0f / sqrtf(mean + eps2);
+      const float4 w2 = gain2[c];
+      st4(out2 + (size_t)i * hidden + h,
+          make_float4(x[c].x * inv2 * w2.x, x[c].y * inv2 * w2.y, x[c].z * inv2 * w2.z, x[c].w * inv2 * w2.w));
+    }
+  }
+}
+
+// The vector form, if these operands have it: 0 or an error of the launch; -2 if not.
+static int launch_terms_vec(void* residual, const SumTerms& terms, const void* weight, float eps, void* out, int out_stride,
+                            const void* weight2, float eps2, void* out2, const void* rows, int n_rows, int hidden,
+                            int store_residual, const SlabTerm& tail, int dtype, hipStream_t stream) {
+  const uintptr_t piece = dtype == DT_F32 ? 15 : 7;
+  if (!weight || hidden % 4 || hidden > 4096 || out_stride % 4 || terms.count < 1 || terms.count > 3 ||
+      (((uintptr_t)out | (uintptr_t)out2) & piece) ||
+      (((uintptr_t)residual | (uintptr_t)weight | (uintptr_t)weight2 | (uintptr_t)tail.slabs | (uintptr_t)tail.scale) & 15))
+    return -2;
+  int scaled = tail.slabs && tail.scale ? 1 : 0;
+  for (int k = 0; k < terms.count; ++k) {
+    if (((uintptr_t)terms.rows[k] & piece) || ((uintptr_t)terms.scale[k] & 15)) return -2;
+    scaled += terms.scale[k] ? 1 : 0;
+  }
+  if (scaled != 0 && scaled != terms.count + (tail.slabs ? 1 : 0)) return -2;
+  if (tail.slabs && (dtype != DT_BF16 || terms.count != 1 || tail.count < 1)) return -2;
+#define GO(TT, CC, NN, SS, LL) add_terms_rmsnorm_vec_kernel<TT, CC, NN, SS, LL><<<n_rows, 256, 0, stream>>>((float*)residual, terms, \
+    (const float*)weight, (TT*)out, (const int*)rows, hidden, eps, store_residual, out_stride, (const float*)weight2, eps2,          \
+    (TT*)out2, tail)
+#define GO_CHUNKS(TT, NN, SS, LL) switch ((hidden + 1023) / 1024) { case 1: GO(TT, 1, NN, SS, LL); break; \
+    case 2: GO(TT, 2, NN, SS, LL); break; case 3: GO(TT, 3, NN, SS, LL); break; default: GO(TT, 4, NN, SS, LL); break; }
+#define GO_SCALED(TT, NN, LL) if (scaled) GO_CHUNKS(TT, NN, true, LL) else GO_CHUNKS(TT, NN, false, LL)
+  if (tail.slabs) { GO_SCALED(bf16_t, 1, true) }
+  else if (dtype == DT_F32) {
+    if (terms.count == 1) { GO_SCALED(float, 1, false) } else if (terms.count == 2) { GO_SCALED(float, 2, false) } else return -2;
+  } else {
+    if (terms.count == 1) { GO_SCALED(bf16_t, 1, false) } else if (terms.count == 2) { GO_SCALED(bf16_t, 2, false) }
+    else { GO_SCALED(bf16_t, 3, false) }
+  }
+#undef GO_SCALED
+#undef GO_CHUNKS
+#undef GO
+  return LAUNCH_STATUS();
+}
+
 extern "C" int ta_add_terms_rmsnorm(void* residual, int count, const void* rows0, const void* rows1, const void* rows2,
                                     const void* rows3, const void* scale0, const void* scale1, const void* scale2,
                                     const void* scale3, float f0, float f1, float f2, float f3, const void* weight,
@@ -405,11 +520,46 @@ extern "C" int ta_add_terms_rmsnorm(void* residual, int count, const void* rows0
                     {f0, f1, f2, f3}, count};
   for (int k = 0; k < count; ++k)
     if (!terms.rows[k]) return -1;
+  const int status = launch_terms_vec(residual, terms, weight, eps, out, out_stride, weight2, eps2, out2, rows, n_rows, hidden,
+                                      store_residual, SlabTerm{nullptr, nullptr, 0.f, 0, 0}, dtype, stream);
+  if (status != -2) return status;
 #define TERMS(TT, PP) add_terms_rmsnorm_kernel<TT, PP><<<n_rows, 256, 0, stream>>>((float*)residual, terms,     (const float*)weight, eps, (TT*)out, out_stride, (const float*)weight2, eps2, (TT*)out2, (const int*)rows, hidden, store_residual)
 #define TERMS_SIZES(TT) if (hidden <= 256) TERMS(TT, 1); else if (hidden <= 1024) TERMS(TT, 4); else if (hidden <= 2048) TERMS(TT, 8);                         else if (hidden <= 4096) TERMS(TT, 16); else TERMS(TT, 32)
   if (dtype == DT_F32) { TERMS_SIZES(float); } else { TERMS_SIZES(bf16_t); }
 #undef TERMS_SIZES
 #undef TERMS
+  return LAUNCH_STATUS();
+}
+
+// One term of rows and one in parts (float slabs [n_slabs, n_tokens, hidden], `stride` floats apart) in bfloat16 mode.  Returns
+// -2 for operands without the vector form (the caller then adds the parts first).
+extern "C" int ta_add_slabs_rmsnorm(void* residual, const void* rows0, const void* scale0, float f0, const void* slabs,
+                                    const void* slab_scale, float slab_factor, int n_slabs, size_t stride, const void* weight,
+                                    float eps, void* out, const void* rows, int n_rows, int hidden, int store_residual,
+                                    hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  if (hidden <= 0 || !rows0 || !slabs || n_slabs < 1 || !weight) return -1;
+  const SumTerms terms = {{rows0, nullptr, nullptr, nullptr}, {(const float*)scale0, nullptr, nullptr, nullptr}, {f0, 0.f, 0.f, 0.f}, 1};
+  return launch_terms_vec(residual, terms, weight, eps, out, hidden, nullptr, 0.f, nullptr, rows, n_rows, hidden, store_residual,
+                          SlabTerm{(const float*)slabs, (const float*)slab_scale, slab_factor, n_slabs, stride}, DT_BF16, stream);
+}
+
+extern "C" int ta_add_pair_rmsnorm(void* residual, const void* first, const void* second, const void* weight, void* out,
+                                   const void* rows, int n_rows, int hidden, float eps, int store_residual, int dtype,
+                                   hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  if (hidden <= 0 || hidden > 256 * 32 || !first || !second) return -1;
+  const SumTerms terms = {{first, second, nullptr, nullptr}, {nullptr, nullptr, nullptr, nullptr}, {1.f, 1.f, 0.f, 0.f}, 2};
+  const int status = launch_terms_vec(residual, terms, weight, eps, out, hidden, nullptr, 0.f, nullptr, rows, n_rows, hidden,
+                                      store_residual, SlabTerm{nullptr, nullptr, 0.f, 0, 0}, dtype, stream);
+  if (status != -2) return status;
+#define PAIR(TT, PP) add_pair_rmsnorm_kernel<TT, PP><<<n_rows, 256, 0, stream>>>((float*)residual, (const TT*)first, \
+    (const TT*)second, (const float*)weight, (TT*)out, (const int*)rows, hidden, eps, store_residual)
+#define PAIR_SIZES(TT) if (hidden <= 256) PAIR(TT, 1); else if (hidden <= 1024) PAIR(TT, 4); else if (hidden <= 2048) PAIR(TT, 8); \
+                       else if (hidden <= 4096) PAIR(TT, 16); else PAIR(TT, 32)
+  if (dtype == DT_F32) { PAIR_SIZES(float); } else { PAIR_SIZES(bf16_t); }
+#undef PAIR_SIZES
+#undef PAIR
   return LAUNCH_STATUS();
 }
 

@@ -161,7 +161,7 @@ class Ops:
                      "ta_add_terms_rmsnorm", "ta_scale_cap", "ta_route_scores", "ta_selective_scan", "ta_route_rows_scores",
                      "ta_rotation_table", "ta_head_norm_rotate_store", "ta_group_norm_add", "ta_relu_gate",
                      "ta_talking_attention_generic", "ta_talking_decode_bf16", "ta_talking_prefill_bf16",
-                     "ta_talking_prefill_parts", "ta_retention_scan", "ta_retention_chunked", "ta_temper_store",
+                     "ta_talking_prefill_parts", "ta_retention_scan", "ta_retention_chunked", "ta_temper_store", "ta_add_slabs_rmsnorm",
                      "ta_expert_gate_slots"):
             getattr(self.lib, name).restype = ctypes.c_int
         self.lib.ta_grouped_gemm_bf16.argtypes = [ctypes.c_void_p, ctypes.c_int, ctypes.c_void_p, ctypes.c_void_p, ctypes.c_int,
@@ -464,6 +464,11 @@ class Ops:
         terms = tuple(terms)
         n_tokens, hidden = residual.shape
         n_rows = n_tokens if rows is None else rows.numel()
+        if any(isinstance(term, PendingSum) for term, _, _ in terms):
+            done = self._add_slabs(residual, terms, weight, eps, out, rows, store_residual, weight2, out2)
+            if done is not None:
+                return done
+            terms = tuple((term.resolve() if isinstance(term, PendingSum) else term, factor, scale) for term, factor, scale in terms)
         _dev(residual, weight, rows, weight2, out2)
         _need(out.is_cuda, "kernel operands must live on the GPU")       # (its rows may lie apart: a half of wider rows)
         _need(len(terms) <= 4, "up to four terms")
@@ -487,6 +492,36 @@ class Ops:
             *[ctypes.c_float(float(t[1])) for t in filled], _ptr(weight), ctypes.c_float(eps), _ptr(out), out.stride(0),
             _ptr(weight2), ctypes.c_float(eps2), _ptr(out2), _ptr(rows), n_rows, hidden, int(bool(store_residual)),
             _code(out.dtype), self._stream()), "add_terms_rmsnorm")
+        return out
+
+    takes_pending_terms = True      # `add_terms_rmsnorm` takes a product still in parts (`PendingSum`) as a term
+
+    def _add_slabs(self, residual, terms, weight, eps, out, rows, store_residual, weight2, out2) -> torch.Tensor | None:
+        """`add_terms_rmsnorm` of one term of rows and, behind it, a product still in parts, which the same kernel adds up;
+        None for other forms (the caller then adds the parts first)."""
+        if len(terms) != 2 or isinstance(terms[0][0], PendingSum) or weight is None or out2 is not None:
+            return None
+        (first, factor, scale), (parts, slab_factor, slab_scale) = terms
+        n_tokens, hidden = residual.shape
+        n_rows = n_tokens if rows is None else rows.numel()
+        if (parts.bias is not None or hidden % 4 or hidden > 4096 or out.dtype != torch.bfloat16 or not out.is_contiguous()
+                or (scale is None) != (slab_scale is None)):
+            return None
+        _dev(residual, first, scale, slab_scale, parts.partial, weight, out, rows)
+        _need(residual.dtype == torch.float32 and weight.dtype == torch.float32 and weight.numel() == hidden
+              and tuple(first.shape) == (n_tokens, hidden) == tuple(parts.shape) and first.dtype == out.dtype
+              and tuple(out.shape) == (n_rows, hidden) and parts.partial.dtype == torch.float32 and parts.partial.is_contiguous(),
+              "terms [T, H] in the output's dtype, a float32 residual stream and norm weight")
+        for each in (scale, slab_scale):
+            _need(each is None or (each.dtype == torch.float32 and each.numel() == hidden), "a term's scale is float32 [H]")
+        _need(rows is None or (rows.dtype == torch.int32 and not store_residual), "rows int32, and a subset stores nothing back")
+        status = self.lib.ta_add_slabs_rmsnorm(
+            _ptr(residual), _ptr(first), _ptr(scale), ctypes.c_float(float(factor)), _ptr(parts.partial), _ptr(slab_scale),
+            ctypes.c_float(float(slab_factor)), parts.partial.shape[0], ctypes.c_size_t(n_tokens * hidden), _ptr(weight),
+            ctypes.c_float(eps), _ptr(out), _ptr(rows), n_rows, hidden, int(bool(store_residual)), self._stream())
+        if status == -2:
+            return None
+        self._check(status, "add_slabs_rmsnorm")
         return out
 
     def scale_cap(self, x: torch.Tensor, scale: float, cap: float) -> torch.Tensor:

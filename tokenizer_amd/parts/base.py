@@ -250,10 +250,12 @@ class ScaledSum:
 
     @classmethod
     def of(cls, ops, value) -> "ScaledSum":
-        """A sub-layer's output as a sum: one itself, or a tensor as its one term."""
+        """A sub-layer's output as a sum: one itself, or a tensor as its one term (a product still in parts stays one where
+        the kernel library's `add_terms_rmsnorm` adds them up)."""
         if isinstance(value, cls):
             return value
-        return cls(ops, () if value is None else ((as_tensor(value), 1.0, None),))
+        kept = hasattr(value, "partial") and getattr(ops, "takes_pending_terms", False)
+        return cls(ops, () if value is None else ((value if kept else as_tensor(value), 1.0, None),))
 
     def scaled_by(self, scale, factor: float = 1.0) -> "ScaledSum":
         """Every term times `factor` and, coordinate by coordinate, `scale` (float32 [H] or None)."""
@@ -268,7 +270,7 @@ class ScaledSum:
         return out
 
     def resolve(self) -> torch.Tensor:
-        rows = self.terms[0][0]
+        rows = as_tensor(self.terms[0][0])
         zero = torch.zeros(rows.shape, dtype=torch.float32, device=rows.device)
         self.ops.add_terms_rmsnorm(zero, self.terms, None, 0.0, torch.empty_like(rows))
         return zero

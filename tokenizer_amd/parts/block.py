@@ -115,7 +115,12 @@ class ScaledParallelBlock(Block):
         h1, h2 = self._normed(residual, delta)
         out = ScaledSum.of(ops, self.mixer.forward(h1, ctx, cache)).scaled_by(self.mixer_scale)
         if self.feed_forward is not None:
-            out = out.plus(ScaledSum.of(ops, self.feed_forward.forward(h2, ctx)).scaled_by(self.ff_scale))
+            # (Behind one term of rows, a feed-forward that can leave its last product in parts may: the next norm adds
+            # them up in its kernel.)
+            run = self.feed_forward.forward
+            if len(out.terms) == 1:
+                run = getattr(self.feed_forward, "forward_pending", run)
+            out = out.plus(ScaledSum.of(ops, run(h2, ctx)).scaled_by(self.ff_scale))
         return out
 
 

@@ -222,6 +222,13 @@ class RoutedExperts(FeedForward):
         return out
 
     def forward(self, x, ctx):
+        return self._run(x, pending=False)
+
+    def forward_pending(self, x, ctx):
+        """As `forward`, but where the last product's K is cut over workgroups its parts may be left for the next norm."""
+        return self._run(x, pending=getattr(self.runtime.ops, "takes_pending_terms", False))
+
+    def _run(self, x, pending: bool):
         ops = self.runtime.ops
         chosen = torch.empty((x.shape[0], self.top_k), dtype=torch.int32, device=x.device)
         weights = torch.empty((x.shape[0], self.top_k), dtype=torch.float32, device=x.device)
@@ -260,7 +267,7 @@ class RoutedExperts(FeedForward):
                             **({"weigh_input": True} if self.weigh_input else {}))
         else:
             ops.expert_act(gate_up, chosen, weights, self.n_experts, self.inner, act)
-        return ops.linear(act, self.w_down)
+        return ops.linear(act, self.w_down, pending=True) if pending else ops.linear(act, self.w_down)
 
     def _sorted(self, x, chosen, weights, shared_weight=None):
         """Tiles of rows that belong to one expert each: gate/up, the activation, down, then a token's experts added up."""
