@@ -411,7 +411,8 @@ class PlainOps:
 
     def paged_attention(self, qkv, out, k_pages, v_pages, positions, entry_of_token, block_table,
                         n_q, n_kv, head_dim, window, scale, max_position=None, batch=None,
-                        value_dim=None, chunk=None, slopes=None, sinks=None, keep_first=0, value_heads=None, softcap=None):
+                        value_dim=None, chunk=None, slopes=None, sinks=None, keep_first=0, value_heads=None, softcap=None,
+                        tied_values=False):
         page_size = k_pages.shape[2]
         group = n_q // n_kv
         share = 1 if value_heads is None else n_kv // value_heads     # key heads that read one value head

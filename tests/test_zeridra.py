@@ -752,3 +752,55 @@ def test_a_term_that_is_a_product_still_in_parts(width, parts, scaled):
         assert float((out.double().cpu() - normed).abs().max()) <= 1e-2 * float(normed.abs().max())
         rough = 2e-6 if width <= 4096 else 1e-2              # (rows too long for that kernel: the parts are added into bfloat16 first)
         assert pick is not None or float((stream.double().cpu() - want).abs().max()) <= rough * float(want.abs().max())
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("d", [16, 32, 48, 64, 80, 96, 112, 128, 160, 192, 224, 256])
+@pytest.mark.parametrize("n_q,n_kv,window,sink,page_size", [(6, 2, None, True, 16), (5, 1, 40, True, 16), (20, 1, None, False, 32), (3, 3, 16, True, 48)])
+def test_single_tokens_over_values_that_are_the_keys_read_once(d, n_q, n_kv, window, sink, page_size):
+    """The kernel that reads keys alone against the one that reads both pages and against the plain op, at every head size;
+    slots that no token wrote hold NaN."""
+    from kernel_refs import PlainOps
+    from tokenizer_amd.kernels import get_ops
+    ops, device, dtype = get_ops(), torch.device("cuda:0"), torch.bfloat16
+    gen = torch.Generator().manual_seed(d + n_q)
+    lengths = [1, 2, 16, 17, 31, 32, 33, 64, 200, 700]
+    pages = [-(-n // page_size) for n in lengths]
+    total = sum(pages) + 3
+    order = torch.randperm(total, generator=gen).tolist()
+    k_pages = torch.full((total, n_kv, page_size, d), float("nan"), dtype=dtype)
+    v_pages = torch.full((total, n_kv, d, page_size), float("nan"), dtype=dtype)
+    table = torch.full((len(lengths), max(pages)), -1, dtype=torch.int32)
+    at = 0
+    for e, n in enumerate(lengths):
+        keys = torch.randn(n, n_kv, d, generator=gen).to(dtype)
+        for j in range(n):
+            page = order[at + j // page_size]
+            table[e, j // page_size] = page
+            k_pages[page, :, j % page_size] = keys[j]
+            v_pages[page, :, :, j % page_size] = keys[j]
+        at += pages[e]
+        if window is not None:                              # pages wholly behind the window are given back
+            for i in range(max(0, n - 1 - window) // page_size):
+                table[e, i] = -1
+    q = torch.randn(len(lengths), n_q * d, generator=gen).to(dtype)
+    positions = torch.tensor([n - 1 for n in lengths], dtype=torch.int32)
+    entries = torch.arange(len(lengths), dtype=torch.int32)
+    sinks = torch.randn(n_q, generator=gen) if sink else None
+    want = torch.empty_like(q)
+    PlainOps(torch.float64).paged_attention(q, want, k_pages, v_pages, positions, entries, table, n_q, n_kv, d, window, 0.2, sinks=sinks)
+    on = lambda t: None if t is None else t.to(device)
+    got = {}
+    before = ops.use_tied_values
+    try:
+        for tied in (False, True):
+            ops.use_tied_values = tied
+            out = torch.empty_like(q, device=device)
+            ops.paged_attention(on(q), out, on(k_pages), on(v_pages), on(positions), on(entries), on(table), n_q, n_kv, d, window, 0.2,
+                                max_position=max(lengths) - 1, sinks=on(sinks), tied_values=True)
+            got[tied] = out.float().cpu()
+    finally:
+        ops.use_tied_values = before
+    for out in got.values():
+        assert float((out - want.float()).abs().max()) <= 2e-2
+    assert float((got[True] - got[False]).abs().max()) <= 2e-2

@@ -32,10 +32,20 @@ __device__ __forceinline__ bf16x8 zero8() {
 // the window) - 1) and leave their partial state beside the others'.  n_v < n_kv: the value pages hold n_v heads and
 // key head g reads value head g / (n_kv / n_v).
 // EXTRA: chunk > 0: only the keys of the token's own run of `chunk` positions (runs counted from position 0) are seen;
-// slopes (float [n_q] or null): head h's score loses slopes[h] per position between token and key; sinks (float [n_q] or
-// null): exp(sinks[h]) joins the softmax's denominator (it rides in the first split's partial sums); softcap > 0: a
+// slopes (float [n_q] or null): head h's score loses slopes[h] per position between token and key; softcap > 0: a
 // score s (scaled, with its distance term) becomes softcap * tanh(s / softcap).
-template <int D, int DEC_WAVES, bool AHEAD, bool EXTRA>
+// sinks (float [n_q] or null): exp(sinks[h]) joins the softmax's denominator (it rides in the first split's partial sums).
+// TIED: the values are the keys, and only the key pages are read: a wave leaves its block of keys in LDS as it came, key by
+// key, and takes the eight keys of a coordinate that the second product wants from there by the transposing LDS read
+// (ds_read_b64_tr_b16: of the 4 x 16 elements that sixteen lanes address, four lanes a row, lane i gets column i).
+template <int D>
+struct KeyStage {                                            // a wave's block of 32 keys in LDS
+  // Rows 3 pieces of sixteen bytes (of eight: mod 8) apart, so that the sixteen rows of a read lie in different banks.
+  static constexpr int ROW = 2 * D + 16 * ((11 - (D / 8) % 8) % 8);
+  static constexpr int BYTES = 32 * ROW;
+};
+
+template <int D, int DEC_WAVES, bool AHEAD, bool EXTRA, bool TIED>
 __global__ void __launch_bounds__(DEC_WAVES * WAVE)
 decode_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out,
                         const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ vt_pages,
@@ -48,8 +58,11 @@ decode_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __re
   constexpr int KS = (D + 31) / 32;   // 32-wide steps over the head size for Q K^T
   constexpr int DB = D / 16;          // 16-row blocks of O^T
   HELD(q, q_stride, out, k_pages, vt_pages, rows, positions, entry_of_token, block_table, table_stride, part_o, part_ml,
-       n_q, n_kv, page_size, window, scale, split_keys, splits);
-  __shared__ float acc_s[DEC_WAVES][D][17];
+       n_q, n_kv, page_size, window, scale, split_keys, splits, sinks);
+  // (The waves' blocks of keys, where they are kept, lie where the waves' sums lie afterwards.)
+  constexpr int SUMS = DEC_WAVES * D * 17 * 4, STAGES = TIED ? DEC_WAVES * KeyStage<D>::BYTES : 0;
+  __shared__ __attribute__((aligned(16))) char shared_s[SUMS > STAGES ? SUMS : STAGES];
+  float (*acc_s)[D][17] = reinterpret_cast<float (*)[D][17]>(shared_s);
   __shared__ float m_s[DEC_WAVES][16], l_s[DEC_WAVES][16];
 
   const int split = blockIdx.x;
@@ -113,7 +126,7 @@ decode_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __re
   // in one (page sizes are multiples of 16).
   struct KeyBlock {
     bf16x8 kf[2][KS];
-    union VFrag { uint4 bits; bf16x8 v; } vf[DB];
+    union VFrag { uint4 bits; bf16x8 v; } vf[TIED ? 1 : DB];
     bool active;
     int left;                                              // this lane's eight keys of the block that exist: 0 .. left
   };
@@ -127,8 +140,10 @@ decode_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __re
     for (int t = 0; t < 2; ++t)
 #pragma unroll
       for (int ks = 0; ks < KS; ++ks) blk.kf[t][ks] = zero8();
+    if (!TIED) {
 #pragma unroll
-    for (int db = 0; db < DB; ++db) blk.vf[db].bits = make_uint4(0, 0, 0, 0);
+      for (int db = 0; db < DB; ++db) blk.vf[db].bits = make_uint4(0, 0, 0, 0);
+    }
     if (blk.active) {
       // The two halves of sixteen keys: a half that holds no key of the range (before `lo`: its page may have been
       // given back; after `last`: it may not exist yet) borrows the other half's page, which is a valid address;
@@ -154,7 +169,7 @@ decode_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __re
           for (int ks = 0; ks < KS; ++ks)
             if (ks * 32 + 8 * g < D) blk.kf[t][ks] = *reinterpret_cast<const bf16x8*>(k_pages + at + t * 4 * D + ks * 32);
       }
-      {
+      if (!TIED) {
         const int half = g >> 1;
         const uint32_t at = ((uint32_t)(half ? page1 : page0) * n_vh + vh) * page_elems + (uint32_t)col * page_size +
                             ((kb + 16 * half) % page_size) + 8 * (g & 1);
@@ -167,7 +182,29 @@ decode_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __re
   };
   // One step of the online softmax over a block that has been brought in.
   auto attend = [&](KeyBlock& blk, int kb) {
-    if (blk.left < 7) {                                      // slots nobody wrote may hold anything: 0 * NaN would poison the sum
+    if (TIED) {
+      if (kb < lo || kb + 31 > last || !blk.active) {        // (the same for the whole wave)
+        // Keys outside lo .. last hold anything (slots nobody wrote, a borrowed page): as values they must be zero.
+#pragma unroll
+        for (int t = 0; t < 2; ++t) {
+          const int key = kb + 8 * (col >> 2) + 4 * t + (col & 3);
+          if (key < lo || key > last) {
+#pragma unroll
+            for (int ks = 0; ks < KS; ++ks) blk.kf[t][ks] = zero8();
+          }
+        }
+      }
+      char* stage = shared_s + wave * KeyStage<D>::BYTES;
+#pragma unroll
+      for (int t = 0; t < 2; ++t)
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks)
+          if (ks * 32 + 8 * g < D)
+            *reinterpret_cast<bf16x8*>(stage + (8 * (col >> 2) + 4 * t + (col & 3)) * KeyStage<D>::ROW + (ks * 4 + g) * 16) = blk.kf[t][ks];
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+    }
+    if (!TIED && blk.left < 7) {                                      // slots nobody wrote may hold anything: 0 * NaN would poison the sum
       const int left = blk.left;
 #pragma unroll
       for (int db = 0; db < DB; ++db) {
@@ -218,8 +255,20 @@ decode_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __re
     for (int db = 0; db < DB; ++db) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) acc[db][r] *= corr;
-      acc[db] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(blk.vf[db].v, pf, acc[db], 0, 0, 0);
+      if constexpr (TIED) {
+        // Keys 8g .. 8g+7 of coordinate db * 16 + col: rows 8g .. 8g+3, then 8g+4 .. 8g+7, sixteen coordinates each.
+        typedef short short4v __attribute__((ext_vector_type(4)));
+        typedef __attribute__((address_space(3))) short4v* stage_t;
+        const char* at = shared_s + wave * KeyStage<D>::BYTES + (8 * g + (col >> 2)) * KeyStage<D>::ROW + db * 32 + (col & 3) * 8;
+        union { short4v part[2]; bf16x8 v; } vf;
+        vf.part[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((stage_t)(at));
+        vf.part[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((stage_t)(at + 4 * KeyStage<D>::ROW));
+        acc[db] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf.v, pf, acc[db], 0, 0, 0);
+      } else {
+        acc[db] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(blk.vf[db].v, pf, acc[db], 0, 0, 0);
+      }
     }
+    if (TIED) __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");   // (the next block is stored behind these reads)
   };
   constexpr int STRIDE = DEC_WAVES * 32;
   int kb = first + wave * 32;
@@ -254,6 +303,7 @@ decode_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __re
   // Sum of the lane groups' partial denominators (the maximum is already common to them).
   l += __shfl_xor(l, 16, WAVE);
   l += __shfl_xor(l, 32, WAVE);
+  if (TIED) __syncthreads();                                // (no wave reads its keys any more)
 #pragma unroll
   for (int db = 0; db < DB; ++db)
 #pragma unroll
@@ -269,7 +319,7 @@ decode_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __re
     for (int w = 0; w < DEC_WAVES; ++w) big = fmaxf(big, m_s[w][h]);
     const int hg = kvh * group + hb * 16 + h;
     float o = 0.f, denom = 0.f;
-    if (EXTRA && sinks && split == 0) {
+    if (sinks && split == 0) {
       const float sink = sinks[hg];
       big = fmaxf(big, sink);
       denom = __expf(sink - big);
@@ -375,17 +425,19 @@ static int launch_decode(const void* q, int q_stride, void* out, const void* k_p
                          const void* block_table, int table_stride, void* part_o, void* part_ml, int n_items,
                          int n_q, int n_kv, int page_size, int window, float scale, int split_keys, int splits,
                          int chunk, const void* slopes, const void* sinks, int keep_first, int kept_splits, int n_v,
-                         float softcap, hipStream_t stream) {
+                         float softcap, int tied, hipStream_t stream) {
   const int group = n_q / n_kv;
   dim3 grid(splits, n_kv * ((group + 15) / 16), n_items);
   constexpr int NW = D > 128 ? 2 : 4;   // keeps the merge buffer within 64 KB of LDS
-#define GO(AHEAD, EE) decode_attention_kernel<D, NW, AHEAD, EE><<<grid, NW * WAVE, 0, stream>>>( \
+#define GO(AHEAD, EE, TT) decode_attention_kernel<D, NW, AHEAD, EE, TT><<<grid, NW * WAVE, 0, stream>>>( \
       (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_pages, (const bf16_t*)vt_pages, (const int*)rows, \
       (const int*)positions, (const int*)entry_of_token, (const int*)block_table, table_stride, (float*)part_o, \
       (float*)part_ml, n_q, n_kv, page_size, window, scale, split_keys, splits, chunk, (const float*)slopes, \
       (const float*)sinks, keep_first, kept_splits, n_v, softcap)
-  if (chunk > 0 || slopes || sinks || kept_splits > 0 || softcap > 0.f || (n_v > 0 && n_v < n_kv)) { if (split_keys <= 32 * NW * 8) GO(true, true); else GO(false, true); }
-  else if (split_keys <= 32 * NW * 8) GO(true, false); else GO(false, false);      // up to eight blocks a wave
+  const bool few = split_keys <= 32 * NW * 8;              // up to eight blocks a wave
+  if (chunk > 0 || slopes || kept_splits > 0 || softcap > 0.f || (n_v > 0 && n_v < n_kv)) { if (few) GO(true, true, false); else GO(false, true, false); }
+  else if (tied) { if (few) GO(true, false, true); else GO(false, false, true); }
+  else if (few) GO(true, false, false); else GO(false, false, false);
 #undef GO
   int status = LAUNCH_STATUS();
   if (status == 0 && splits > 1) {
@@ -409,6 +461,7 @@ extern "C" int ta_attention_merge_tiles(const void* part_o, const void* part_ml,
   return LAUNCH_STATUS();
 }
 
+// tied: the value pages hold what the key pages hold (the kernel may read only one of them).
 // Returns -2 for a head size this kernel has no instance for (the caller then uses the generic kernel).
 extern "C" int ta_decode_attention_bf16(const void* q, int q_stride, void* out, const void* k_pages,
                                         const void* vt_pages, const void* rows, const void* positions,
@@ -416,7 +469,7 @@ extern "C" int ta_decode_attention_bf16(const void* q, int q_stride, void* out, 
                                         void* part_o, void* part_ml, int n_items, int n_q, int n_kv, int d,
                                         int page_size, int window, float scale, int split_keys, int splits,
                                         int chunk, const void* slopes, const void* sinks, int keep_first,
-                                        int kept_splits, int n_v, float softcap, hipStream_t stream) {
+                                        int kept_splits, int n_v, float softcap, int tied, hipStream_t stream) {
   if (n_items <= 0) return 0;
   if (n_kv <= 0 || n_q % n_kv || page_size % 16 || split_keys % 32 || splits < 1) return -1;
   if (n_v <= 0) n_v = n_kv;
@@ -425,7 +478,7 @@ extern "C" int ta_decode_attention_bf16(const void* q, int q_stride, void* out, 
     return -1;
 #define CASE(DD) case DD: return launch_decode<DD>(q, q_stride, out, k_pages, vt_pages, rows, positions, entry_of_token, \
     block_table, table_stride, part_o, part_ml, n_items, n_q, n_kv, page_size, window, scale, split_keys, splits, chunk, \
-    slopes, sinks, keep_first, kept_splits, n_v, softcap, stream);
+    slopes, sinks, keep_first, kept_splits, n_v, softcap, tied, stream);
   switch (d) {
     CASE(16) CASE(32) CASE(48) CASE(64) CASE(80) CASE(96) CASE(112) CASE(128) CASE(160) CASE(192) CASE(224) CASE(256)
     default: return -2;

@@ -1106,10 +1106,14 @@ class Ops:
                         window: int | None, scale: float, max_position: int | None = None,
                         batch=None, value_dim: int | None = None, chunk: int | None = None,
                         slopes: torch.Tensor | None = None, sinks: torch.Tensor | None = None,
-                        keep_first: int = 0, value_heads: int | None = None, softcap: float | None = None) -> torch.Tensor:
+                        keep_first: int = 0, value_heads: int | None = None, softcap: float | None = None,
+                        tied_values: bool = False) -> torch.Tensor:
         """Causal attention of every token over the pages of its request.
 
         `softcap` c: a score (scaled, with its distance term) becomes c tanh(score / c) before the softmax.
+
+        `tied_values`: the value pages hold what the key pages hold (the values are the keys, or both are one latent); a
+        kernel may then read only one of them.
 
         `keep_first` n (with a window): keys at positions below n stay visible behind the window.  `value_heads`
         (a divisor of n_kv): the value pages hold so many heads, and key head g reads value head
@@ -1159,7 +1163,9 @@ class Ops:
                     page_size, window, scale, max_position)
             plain = plain and not softcap
             extras = {} if plain and sinks is None else dict(chunk=chunk, slopes=slopes, sinks=sinks, keep_first=keep_first,
-                                           value_heads=value_heads, softcap=softcap)
+                                                             value_heads=value_heads, softcap=softcap)
+            if tied_values and plain:
+                extras["tied_values"] = True
             if batch is None:
                 return self._decode_attention(*args, **extras)
             if batch.q_tiles.numel() == 0:
@@ -1196,6 +1202,7 @@ class Ops:
         return out
 
     DECODE_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 112, 128, 160, 192, 224, 256)
+    use_tied_values = True        # whether the kernel for single tokens reads tied keys and values once (for comparisons)
     use_fast_attention = True     # tests switch it off to reach the generic kernel in bfloat16
     prefill_waves = 0             # waves that share a tile's keys in the per-wave prompt kernel: 0 lets the launcher choose;
     #                               asking for a number asks for that kernel
@@ -1211,7 +1218,7 @@ class Ops:
     def _decode_attention(self, qkv, out, k_pages, v_pages, positions, entry_of_token, block_table,
                           n_q, n_kv, head_dim, page_size, window, scale, max_position, rows=None,
                           identity_entries=False, chunk=None, slopes=None, sinks=None, keep_first=0, value_heads=None,
-                          softcap=None):
+                          softcap=None, tied_values=False):
         """Matrix-core attention of single tokens with the key range split over workgroups (kept first keys behind a
         window are further splits of their own)."""
         n_items = qkv.shape[0] if rows is None else rows.numel()
@@ -1225,7 +1232,8 @@ class Ops:
             max_keys = min(max_keys, chunk + 32)
         head_blocks = -(-(n_q // n_kv) // 16)
         per_split = max(1, self.target_workgroups // max(1, n_items * n_kv * head_blocks))
-        split_keys = max(self.min_split_keys, -(-max_keys // per_split))
+        # (A block of 32 keys for each of a workgroup's waves; wide heads have two waves.)
+        split_keys = max(self.min_split_keys if head_dim <= 128 else self.min_split_keys // 2, -(-max_keys // per_split))
         split_keys = -(-split_keys // 32) * 32
         splits = max(1, -(-(max_keys + 31) // split_keys))
         kept_splits = -(-int(keep_first) // split_keys) if keep_first and window is not None else 0
@@ -1241,7 +1249,7 @@ class Ops:
             n_q, n_kv, head_dim, page_size, -1 if window is None else int(window), ctypes.c_float(scale),
             split_keys, splits, 0 if chunk is None else int(chunk), _ptr(slopes), _ptr(sinks),
             int(keep_first) if kept_splits else 0, kept_splits, n_kv if value_heads is None else int(value_heads),
-            ctypes.c_float(softcap or 0.0), self._stream()), "decode_attention")
+            ctypes.c_float(softcap or 0.0), int(bool(tied_values) and self.use_tied_values), self._stream()), "decode_attention")
         return out
 
     def talking_attention(self, qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,

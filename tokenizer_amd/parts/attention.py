@@ -160,6 +160,8 @@ class GQAttention(Mixer):
         self.more = {}
         if spec.sink:
             self.more["sinks"] = tensors["sink"].to(torch.float32).contiguous()
+        if self.tied:
+            self.more["tied_values"] = True
         if spec.fixed_sink is not None:
             self.more["sinks"] = torch.full((H * self.maps,), float(spec.fixed_sink), dtype=torch.float32, device=runtime.device)
         if spec.softcap is not None:

@@ -56,7 +56,9 @@ class LatentAttention(Mixer):
             raise ValueError(f"rot_pairs {pairs!r}: known are \"halves\" and \"neighbours\"")
         # (What the kernels take only where a layer has it.)
         self.turns = {"neighbours": True} if pairs == "neighbours" else {}
-        self.more = {"sinks": tensors["sink"].to(torch.float32).contiguous()} if spec.sink else {}
+        self.more = {"tied_values": True}            # (key and value pages hold the same rows)
+        if spec.sink:
+            self.more["sinks"] = tensors["sink"].to(torch.float32).contiguous()
         # One product for the down-projections and the gate; every part starts at a multiple of eight columns
         # (sixteen bytes in bfloat16), filled up with rows of zeros.
         parts, self.offsets, at = [], {}, 0
