@@ -64,7 +64,8 @@ class PlainOps:
                 continue
             page, off = divmod(slot, page_size)
             k_pages[page, 0, off, :] = kept[t]
-            v_pages[page, 0, :, off] = kept[t]
+            if v_pages is not None:
+                v_pages[page, 0, :, off] = kept[t]
 
     def head_linear(self, x, x_offset, x_head_stride, weight, out, out_offset, out_head_stride):
         heads, n, k = weight.shape
@@ -429,7 +430,8 @@ class PlainOps:
             assert all(p >= 0 for p in pages), "attention reads a page that was given back"
             offs = [j % page_size for j in keys]
             k = k_pages[pages, :, offs, :].to(self.work)     # [keys, n_kv, d]
-            v = v_pages[pages, :, :, offs].to(self.work)      # [keys, n_kv, d]
+            assert v_pages is not None or tied_values
+            v = k if v_pages is None else v_pages[pages, :, :, offs].to(self.work)      # [keys, n_kv, d]
             q = qkv[t, :n_q * head_dim].reshape(n_q, head_dim).to(self.work)
             k = k.repeat_interleave(group, dim=1)            # [keys, n_q, d]
             v = v.repeat_interleave(group * share, dim=1)
@@ -608,7 +610,8 @@ class PlainOps:
                 continue
             page, off = divmod(slot, page_size)
             k_pages[page, :, off, :] = keys[t]
-            v_pages[page, :, :, off] = values[t]
+            if v_pages is not None:
+                v_pages[page, :, :, off] = values[t]
 
     def differential_heads(self, mixed, lam, eps, out_scale, n_heads, group, dv, out):
         n_tokens = mixed.shape[0]

@@ -804,3 +804,101 @@ def test_single_tokens_over_values_that_are_the_keys_read_once(d, n_q, n_kv, win
     for out in got.values():
         assert float((out - want.float()).abs().max()) <= 2e-2
     assert float((got[True] - got[False]).abs().max()) <= 2e-2
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("d", [16, 32, 48, 64, 80, 96, 112, 128, 160, 192, 224, 256, 20, 300])
+@pytest.mark.parametrize("n_q,n_kv,window,sink,page_size", [(6, 2, None, True, 16), (5, 1, 40, True, 16), (12, 2, None, False, 32), (3, 3, 100, True, 48)])
+@pytest.mark.parametrize("dtype", ["bfloat16", "float32"])
+def test_portions_over_values_that_are_the_keys(d, n_q, n_kv, window, sink, page_size, dtype):
+    """Ragged portions and single tokens over key pages alone, in every prompt kernel and shape, against the plain op; slots
+    that no token wrote, and pages that were given back and hold another request's keys, hold NaN."""
+    from kernel_refs import PlainOps
+    from tokenizer_amd.cache import CacheManager
+    from tokenizer_amd.engine.batch import StepEntry, build_context
+    from tokenizer_amd.kernels import get_ops
+    from tokenizer_amd.parts import CacheNeed
+    dtype = getattr(torch, dtype)
+    ops, device = get_ops(), torch.device("cuda:0")
+    gen = torch.Generator().manual_seed(d + n_q)
+    need = CacheNeed(kind="full" if window is None else "window", n_kv_heads=n_kv, head_dim=d, window=window, tied_values=True)
+    manager = CacheManager([need], num_pages=60, page_size=page_size, max_requests=5)
+    k_pages = torch.full((60, n_kv, page_size, d), float("nan"), dtype=dtype)
+    counts = {"a": (0, 90), "b": (130, 37), "c": (60, 1), "d": (0, 1), "e": (33, 2)}
+    keys = {rid: torch.randn(before + new, n_kv, d, generator=gen).to(dtype) for rid, (before, new) in counts.items()}
+    entries = []
+    for rid, (before, new) in counts.items():
+        manager.add_request(rid)
+        if before:
+            assert manager.reserve(rid, before)
+            manager.advance(rid, before)
+        assert manager.reserve(rid, before + new)
+        entries.append(StepEntry(rid, [0] * new, []))
+        table = manager.table(rid, 0)
+        for j in range(before + new):
+            if table[j // page_size] >= 0:
+                k_pages[table[j // page_size], :, j % page_size] = keys[rid][j]
+    ctx = build_context(entries, manager, device)
+    n = ctx.n_tokens
+    q = torch.randn(n, n_q * d, generator=gen).to(dtype)
+    sinks = torch.randn(n_q, generator=gen) if sink else None
+    want = torch.zeros_like(q)
+    PlainOps(torch.float64).paged_attention(q, want, k_pages, None, ctx.positions.cpu(), ctx.entry_of_token.cpu(), ctx.block_tables[0].cpu(),
+                                            n_q, n_kv, d, window, 0.2, sinks=sinks, tied_values=True)
+    k_dev, q_dev, sinks_dev = k_pages.to(device), q.to(device), None if sinks is None else sinks.to(device)
+    before = ops.prefill_shared, ops.prefill_shape, ops.prefill_waves
+    shapes = [(0, 0, 0)]
+    if dtype == torch.bfloat16:
+        shapes += [(-1, 0, waves) for waves in (1, 2, 4, 8)] + [(1, shape, 0) for shape in (1, 2, 11, 12)]
+    try:
+        for shape in shapes:
+            ops.prefill_shared, ops.prefill_shape, ops.prefill_waves = shape
+            out = torch.zeros_like(q_dev)
+            ops.paged_attention(q_dev, out, k_dev, None, ctx.positions, ctx.entry_of_token, ctx.block_tables[0], n_q, n_kv, d, window, 0.2,
+                                max_position=ctx.max_position, batch=ctx, sinks=sinks_dev, tied_values=True)
+            real = ctx.entry_of_token >= 0
+            err = (out[real].float().cpu() - want[real.cpu()].float()).abs().max()
+            assert float(err) <= (2e-5 if dtype == torch.float32 else 2e-2), shape
+    finally:
+        ops.prefill_shared, ops.prefill_shape, ops.prefill_waves = before
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("n_q,n_kv,d,new,cached,window", [(14, 2, 64, 40, 4000, None), (14, 1, 128, 30, 3000, None), (28, 4, 128, 16, 6500, None), (14, 1, 128, 20, 3000, 2300)])
+def test_short_portions_far_into_a_request_with_their_keys_in_parts(n_q, n_kv, d, new, cached, window):
+    """A few tiles behind a long context: the tiles' keys are cut over workgroups, and the sink joins one of the parts."""
+    from tokenizer_amd.cache import CacheManager
+    from tokenizer_amd.engine.batch import StepEntry, build_context
+    from tokenizer_amd.kernels import get_ops
+    from tokenizer_amd.parts import CacheNeed
+    ops, device = get_ops(), torch.device("cuda:0")
+    gen = torch.Generator().manual_seed(d + new)
+    need = CacheNeed(kind="full" if window is None else "window", n_kv_heads=n_kv, head_dim=d, window=window, tied_values=True)
+    manager = CacheManager([need], num_pages=420, page_size=16, max_requests=1)
+    manager.add_request("a")
+    manager.reserve("a", cached)
+    manager.advance("a", cached)
+    assert manager.reserve("a", cached + new)
+    ctx = build_context([StepEntry("a", [0] * new, [])], manager, device)
+    keys = torch.randn(cached + new, n_kv, d, generator=gen).to(torch.bfloat16)
+    k_pages = torch.full((420, n_kv, 16, d), float("nan"), dtype=torch.bfloat16)
+    table = manager.table("a", 0)
+    for j in range(cached + new):
+        if table[j // 16] >= 0:
+            k_pages[table[j // 16], :, j % 16] = keys[j]
+    q = torch.randn(ctx.n_tokens, n_q * d, generator=gen).to(torch.bfloat16)
+    sinks = 3.0 + torch.randn(n_q, generator=gen)
+    out = torch.zeros_like(q, device=device)
+    reach = ctx.max_position + 1
+    args = (ctx.q_tiles.shape[0], n_q, n_kv, d, -1 if window is None else window, 0, reach, 0, 0)
+    assert ops.lib.ta_prefill_attention_key_splits(*args) > 1
+    ops.paged_attention(q.to(device), out, k_pages.to(device), None, ctx.positions, ctx.entry_of_token, ctx.block_tables[0], n_q, n_kv, d,
+                        window, d ** -0.5, max_position=ctx.max_position, batch=ctx, sinks=sinks.to(device), tied_values=True)
+    k = keys.double().repeat_interleave(n_q // n_kv, dim=1)
+    for i in range(new):
+        pos = cached + i
+        lo = 0 if window is None else max(0, pos - window)
+        scores = torch.einsum("hd,khd->hk", q[i].double().reshape(n_q, d), k[lo:pos + 1]) * d ** -0.5
+        e = torch.exp(scores)
+        want = torch.einsum("hk,khd->hd", e / (e.sum(-1, keepdim=True) + torch.exp(sinks.double())[:, None]), k[lo:pos + 1]).reshape(-1)
+        assert float((out[i].double().cpu() - want).abs().max()) <= 1e-2

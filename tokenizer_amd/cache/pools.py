@@ -12,7 +12,8 @@ class CachePools:
     """For group g: `pages[g]` of shape [layers in g, num_pages, n_kv, page_size * (d + dv)] elements in the
     compute dtype, a layer's keys first and then its values (d: a key head's size, dv: a value head's, which
     is d unless the mixer says otherwise).  Inside a page keys are laid out [page_size, d] and values
-    transposed, [dv, page_size] (the layout the matrix-core attention kernels read).  For a layer with
+    transposed, [dv, page_size] (the layout the matrix-core attention kernels read).  A group whose values are its keys
+    (`CacheNeed.tied_values`) has key pages alone.  For a layer with
     fixed-size state: `states[layer]` of shape [max_requests, *state_shape]; for a layer whose block keeps
     state of its own: `block_states[layer]`, float32 [max_requests, *block_state_shape]."""
 
@@ -28,7 +29,8 @@ class CachePools:
                                  f"a layer; the kernels address fewer than 2^31 (at most "
                                  f"{(2 ** 31 - 1) // (need.n_kv_heads * manager.page_size * max(need.head_dim, need.v_dim))} pages here)")
             self.pages.append(torch.zeros((len(group.layers), manager.num_pages * manager.page_size
-                                           * (need.n_kv_heads * need.head_dim + need.v_heads * need.v_dim)),
+                                           * (need.n_kv_heads * need.head_dim
+                                              + (0 if need.tied_values else need.v_heads * need.v_dim))),
                                           dtype=dtype, device=device))
         self.states, self.block_states = {}, {}
         for layer, need in enumerate(needs):
@@ -41,7 +43,7 @@ class CachePools:
 
     def layer_pages(self, layer: int):
         """(keys [num_pages, n_kv, page_size, d], values [num_pages, n_v, dv, page_size]) of one layer (n_v = n_kv
-        unless the need names fewer value heads), or (None, None)."""
+        unless the need names fewer value heads; None where the values are the keys), or (None, None)."""
         group = self.manager.group_of_layer[layer]
         if group is None:
             return None, None
@@ -50,6 +52,8 @@ class CachePools:
         pages, page_size = self.pages[group], self.manager.page_size
         shape = (self.manager.num_pages, need.n_kv_heads)
         keys = shape[0] * shape[1] * page_size * need.head_dim
+        if need.tied_values:
+            return pages[index].view(*shape, page_size, need.head_dim), None
         return (pages[index, :keys].view(*shape, page_size, need.head_dim),
                 pages[index, keys:].view(shape[0], need.v_heads, need.v_dim, page_size))
 

@@ -36,15 +36,7 @@ __device__ __forceinline__ bf16x8 zero8() {
 // score s (scaled, with its distance term) becomes softcap * tanh(s / softcap).
 // sinks (float [n_q] or null): exp(sinks[h]) joins the softmax's denominator (it rides in the first split's partial sums).
 // TIED: the values are the keys, and only the key pages are read: a wave leaves its block of keys in LDS as it came, key by
-// key, and takes the eight keys of a coordinate that the second product wants from there by the transposing LDS read
-// (ds_read_b64_tr_b16: of the 4 x 16 elements that sixteen lanes address, four lanes a row, lane i gets column i).
-template <int D>
-struct KeyStage {                                            // a wave's block of 32 keys in LDS
-  // Rows 3 pieces of sixteen bytes (of eight: mod 8) apart, so that the sixteen rows of a read lie in different banks.
-  static constexpr int ROW = 2 * D + 16 * ((11 - (D / 8) % 8) % 8);
-  static constexpr int BYTES = 32 * ROW;
-};
-
+// key, and takes the eight keys of a coordinate that the second product wants from there (`transposed_keys`).
 template <int D, int DEC_WAVES, bool AHEAD, bool EXTRA, bool TIED>
 __global__ void __launch_bounds__(DEC_WAVES * WAVE)
 decode_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out,
@@ -257,13 +249,8 @@ decode_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __re
       for (int r = 0; r < 4; ++r) acc[db][r] *= corr;
       if constexpr (TIED) {
         // Keys 8g .. 8g+7 of coordinate db * 16 + col: rows 8g .. 8g+3, then 8g+4 .. 8g+7, sixteen coordinates each.
-        typedef short short4v __attribute__((ext_vector_type(4)));
-        typedef __attribute__((address_space(3))) short4v* stage_t;
         const char* at = shared_s + wave * KeyStage<D>::BYTES + (8 * g + (col >> 2)) * KeyStage<D>::ROW + db * 32 + (col & 3) * 8;
-        union { short4v part[2]; bf16x8 v; } vf;
-        vf.part[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((stage_t)(at));
-        vf.part[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((stage_t)(at + 4 * KeyStage<D>::ROW));
-        acc[db] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf.v, pf, acc[db], 0, 0, 0);
+        acc[db] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(transposed_keys(at, at + 4 * KeyStage<D>::ROW), pf, acc[db], 0, 0, 0);
       } else {
         acc[db] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(blk.vf[db].v, pf, acc[db], 0, 0, 0);
       }
@@ -435,8 +422,8 @@ static int launch_decode(const void* q, int q_stride, void* out, const void* k_p
       (float*)part_ml, n_q, n_kv, page_size, window, scale, split_keys, splits, chunk, (const float*)slopes, \
       (const float*)sinks, keep_first, kept_splits, n_v, softcap)
   const bool few = split_keys <= 32 * NW * 8;              // up to eight blocks a wave
-  if (chunk > 0 || slopes || kept_splits > 0 || softcap > 0.f || (n_v > 0 && n_v < n_kv)) { if (few) GO(true, true, false); else GO(false, true, false); }
-  else if (tied) { if (few) GO(true, false, true); else GO(false, false, true); }
+  if (chunk > 0 || slopes || kept_splits > 0 || softcap > 0.f || (n_v > 0 && n_v < n_kv)) { if (!vt_pages) return -1; if (few) GO(true, true, false); else GO(false, true, false); }
+  else if (tied || !vt_pages) { if (few) GO(true, false, true); else GO(false, false, true); }
   else if (few) GO(true, false, false); else GO(false, false, false);
 #undef GO
   int status = LAUNCH_STATUS();
@@ -461,7 +448,7 @@ extern "C" int ta_attention_merge_tiles(const void* part_o, const void* part_ml,
   return LAUNCH_STATUS();
 }
 
-// tied: the value pages hold what the key pages hold (the kernel may read only one of them).
+// tied: the value pages hold what the key pages hold, and only the keys are read; vt_pages may then be null.
 // Returns -2 for a head size this kernel has no instance for (the caller then uses the generic kernel).
 extern "C" int ta_decode_attention_bf16(const void* q, int q_stride, void* out, const void* k_pages,
                                         const void* vt_pages, const void* rows, const void* positions,

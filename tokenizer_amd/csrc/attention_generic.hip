@@ -15,6 +15,7 @@
 // sinks (float [n_q] or null): exp(sinks[h]) joins the softmax's denominator (no key, no value, not scaled, no bias).
 // keep_first > 0 (with a window): keys at positions below keep_first stay visible behind the window, at their own positions.
 // n_v (a divisor of n_kv): the value pages hold n_v heads, and key head g reads value head g / (n_kv / n_v).
+// v_pages null: the values are the keys, read from the key pages (n_v = n_kv, dv = d).
 // softcap > 0: a score s (scaled, with its distance term) becomes softcap * tanh(s / softcap) before the softmax.
 template <typename T>
 __global__ void __launch_bounds__(ATT_WAVES * WAVE)
@@ -81,7 +82,17 @@ paged_attention_generic(const T* __restrict__ q, int q_stride, T* __restrict__ o
 #pragma unroll
     for (int r = 0; r < ATT_MAX_D / WAVE; ++r) acc[r] *= corr;
     const int count = min(WAVE, n_keys - base);
-    if (sizeof(T) == 4 && page_size % 4 == 0) {
+    if (!v_pages) {
+      for (int jj = 0; jj < count; ++jj) {
+        const float pj = __shfl(p, jj, WAVE);
+        const T* kr = k_pages + (size_t)__shfl(row, jj, WAVE) * d;
+#pragma unroll
+        for (int r = 0; r < ATT_MAX_D / WAVE; ++r) {
+          const int i = lane + r * WAVE;
+          if (i < dv) acc[r] += pj * ld(kr + i);
+        }
+      }
+    } else if (sizeof(T) == 4 && page_size % 4 == 0) {
       // Values lie transposed inside a page, [d, page_size]: lane i walks row i of the page sixteen bytes (four
       // keys) at a time, so that the wave reads the page as one contiguous block; the keys' weights come through
       // LDS.  (One key at a time, every lane's element would lie a row apart from its neighbour's.)
@@ -167,6 +178,7 @@ extern "C" int ta_paged_attention_generic(const void* q, int q_stride, void* out
   if (dv <= 0) dv = d;
   if (n_v <= 0) n_v = n_kv;
   if (d > ATT_MAX_D || dv > ATT_MAX_D || d <= 0 || n_kv <= 0 || n_q % n_kv || n_kv % n_v || keep_first < 0) return -1;
+  if (!v_pages && (n_v != n_kv || dv != d)) return -1;
   dim3 grid(n_tokens, n_q);
   if (dtype == DT_F32)
     paged_attention_generic<float><<<grid, ATT_WAVES * WAVE, 0, stream>>>((const float*)q, q_stride, (float*)out,

@@ -24,12 +24,14 @@ __device__ __forceinline__ bf16x8 pf_zero8() {
 // Scores stay unscaled; `c` = scale * log2(e) enters in exp2(s*c - m*c).
 // EXTRA: head h's score (still unscaled) loses `slope[h]` (the head's slope over the scale) per position between the
 // token and the key; then, with cap > 0 (the scores' cap over the scale), the score s becomes cap * tanh(s / cap).
-template <int D, int HG, bool FULL, bool EXTRA>
+// TIED (without EXTRA): the values are the keys: the block's keys, as they came, pass through the wave's `stage` in LDS,
+// 32 at a time, and are read back coordinate by coordinate (`transposed_keys`).
+template <int D, int HG, bool FULL, bool EXTRA, bool TIED>
 __device__ __forceinline__ void prefill_block(
     const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ vt_pages, const int* __restrict__ table,
     int kb, int kvh, int n_kv, int page_size, int col, int g, int heads_here, int my_pos, int my_lo, int lo, int hi,
     float c, const bf16x8 (&qf)[HG][(D + 31) / 32], floatx4 (&acc)[HG][D / 16], float (&m)[HG], float (&l)[HG],
-    const float (&slope)[HG], int keep_first = 0, int vh = -1, int n_vh = 0, float cap = 0.f) {
+    const float (&slope)[HG], int keep_first = 0, int vh = -1, int n_vh = 0, float cap = 0.f, char* stage = nullptr) {
   // EXTRA: keep_first > 0: keys below it stay visible (and their pages readable) behind the window; vh >= 0: the
   // value pages hold n_vh heads and this key head reads value head vh.
   if (!EXTRA || vh < 0) { vh = kvh; n_vh = n_kv; }
@@ -74,7 +76,7 @@ __device__ __forceinline__ void prefill_block(
             if (ks * 32 + 8 * g < D)
               kf[2 * u + t][ks] = *reinterpret_cast<const bf16x8*>(k_pages + at + t * 4 * D + ks * 32);
       }
-      {
+      if (!TIED) {
         const int half = g >> 1;
         const uint32_t at = ((uint32_t)(half ? page1 : page0) * n_vh + vh) * page_elems + (uint32_t)col * page_size +
                             ((base_key + 16 * half) % page_size) + 8 * (g & 1);
@@ -87,7 +89,34 @@ __device__ __forceinline__ void prefill_block(
       }
     }
   }
-  if (!FULL) {                                             // slots past the last key may never have been written
+  if (TIED) {
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+#pragma unroll
+      for (int t = 0; t < 2; ++t) {
+        const int key = kb + 32 * u + 8 * (col >> 2) + 4 * t + (col & 3);
+        if (!FULL && (key < lo || key > hi)) {             // such slots hold anything; as values they must be zero
+#pragma unroll
+          for (int ks = 0; ks < KS; ++ks) kf[2 * u + t][ks] = pf_zero8();
+        }
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks)
+          if (ks * 32 + 8 * g < D)
+            *reinterpret_cast<bf16x8*>(stage + (8 * (col >> 2) + 4 * t + (col & 3)) * KeyStage<D>::ROW + (ks * 4 + g) * 16) =
+                kf[2 * u + t][ks];
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+#pragma unroll
+      for (int db = 0; db < DB; ++db) {
+        const char* at = stage + (8 * g + (col >> 2)) * KeyStage<D>::ROW + db * 32 + (col & 3) * 8;
+        vf[u][db].v = transposed_keys(at, at + 4 * KeyStage<D>::ROW);
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");   // (what follows is stored behind these reads)
+      __builtin_amdgcn_wave_barrier();
+    }
+  }
+  if (!FULL && !TIED) {                                    // slots past the last key may never have been written
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
       if (left[u] >= 7) continue;
@@ -161,7 +190,7 @@ __device__ __forceinline__ void prefill_block(
 // tiles: [n_tiles, 2] = (entry, offset of the tile's first token inside the entry's tokens).
 // cu_q[e]: first row of entry e; first_position[e]: position of that row.
 // K pages [n_pages, n_kv, page_size, D]; V^T pages [n_pages, n_kv, D, page_size]; page_size % 16 == 0.
-template <int D, int HG, int NWV, bool EXTRA>
+template <int D, int HG, int NWV, bool EXTRA, bool TIED>
 __global__ void __launch_bounds__(NWV * WAVE, (D <= 64 && HG <= 2) ? 3 : 1)
 prefill_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out,
                          const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ vt_pages,
@@ -174,7 +203,10 @@ prefill_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __r
   constexpr int DB = D / 16;
   HELD(q, q_stride, out, k_pages, vt_pages, tiles, n_tiles, cu_q, first_position, block_table, table_stride, n_q, n_kv,
        page_size, window, scale_log2);
-  __shared__ float merge[NWV > 1 ? NWV - 1 : 1][HG][DB * 4 + 2][WAVE];
+  // (The waves' keys, where they pass through LDS, lie where the waves' states lie afterwards.)
+  constexpr int STATES = (NWV > 1 ? NWV - 1 : 1) * HG * (DB * 4 + 2) * WAVE * 4, STAGES = TIED ? NWV * KeyStage<D>::BYTES : 0;
+  __shared__ __attribute__((aligned(16))) char shared_s[STATES > STAGES ? STATES : STAGES];
+  float (*merge)[HG][DB * 4 + 2][WAVE] = reinterpret_cast<float (*)[HG][DB * 4 + 2][WAVE]>(shared_s);
   const int lane = threadIdx.x & 63, wave = wave_index();
   const int col = lane & 15, g = lane >> 4;
   const int group = n_q / n_kv;
@@ -250,24 +282,26 @@ prefill_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __r
   // A wave's blocks come in three runs: those at the window's edge (some keys masked), those that every token
   // of the tile sees whole, and those on the diagonal.  Each run is a loop of its own over one variant of the
   // block: in one loop over both, the accumulators would be copied between the variants' registers every turn.
+  char* stage = TIED ? shared_s + wave * KeyStage<D>::BYTES : nullptr;
   if (EXTRA && kept > 0) {
     // The kept first keys that lie before the window's first block (those inside the blocks below are let through
     // by the mask there): every token of the tile sees them.
     const int kept_end = min(kept, (lo / 64) * 64);
     for (int k0 = 64 * wave; k0 < kept_end; k0 += 64 * NWV)
-      prefill_block<D, HG, false, EXTRA>(k_pages, vt_pages, table, k0, kvh, n_kv, page_size, col, g, heads_here, my_pos,
-                                  my_lo, lo, hi, scale_log2, qf, acc, m, l, slope, kept, vh, n_vh, softcap * inv_scale);
+      prefill_block<D, HG, false, EXTRA, TIED>(k_pages, vt_pages, table, k0, kvh, n_kv, page_size, col, g, heads_here, my_pos,
+                                  my_lo, lo, hi, scale_log2, qf, acc, m, l, slope, kept, vh, n_vh, softcap * inv_scale, stage);
   }
   int kb = (lo / 64) * 64 + 64 * wave;
   for (; kb <= hi && kb < lo_all; kb += 64 * NWV)
-    prefill_block<D, HG, false, EXTRA>(k_pages, vt_pages, table, kb, kvh, n_kv, page_size, col, g, heads_here, my_pos,
-                                my_lo, lo, hi, scale_log2, qf, acc, m, l, slope, kept, vh, n_vh, softcap * inv_scale);
+    prefill_block<D, HG, false, EXTRA, TIED>(k_pages, vt_pages, table, kb, kvh, n_kv, page_size, col, g, heads_here, my_pos,
+                                my_lo, lo, hi, scale_log2, qf, acc, m, l, slope, kept, vh, n_vh, softcap * inv_scale, stage);
   for (; kb + 63 <= p0; kb += 64 * NWV)
-    prefill_block<D, HG, true, EXTRA>(k_pages, vt_pages, table, kb, kvh, n_kv, page_size, col, g, heads_here, my_pos,
-                               my_lo, lo, hi, scale_log2, qf, acc, m, l, slope, kept, vh, n_vh, softcap * inv_scale);
+    prefill_block<D, HG, true, EXTRA, TIED>(k_pages, vt_pages, table, kb, kvh, n_kv, page_size, col, g, heads_here, my_pos,
+                               my_lo, lo, hi, scale_log2, qf, acc, m, l, slope, kept, vh, n_vh, softcap * inv_scale, stage);
   for (; kb <= hi; kb += 64 * NWV)
-    prefill_block<D, HG, false, EXTRA>(k_pages, vt_pages, table, kb, kvh, n_kv, page_size, col, g, heads_here, my_pos,
-                                my_lo, lo, hi, scale_log2, qf, acc, m, l, slope, kept, vh, n_vh, softcap * inv_scale);
+    prefill_block<D, HG, false, EXTRA, TIED>(k_pages, vt_pages, table, kb, kvh, n_kv, page_size, col, g, heads_here, my_pos,
+                                my_lo, lo, hi, scale_log2, qf, acc, m, l, slope, kept, vh, n_vh, softcap * inv_scale, stage);
+  if (TIED && NWV > 1) __syncthreads();                    // (no wave's keys are read any more)
   if (NWV > 1) {
     // Waves 1.. hand their state to wave 0: maximum, sum and the output accumulators of each head.
     if (wave > 0) {
@@ -311,7 +345,7 @@ prefill_attention_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __r
   for (int h = 0; h < HG; ++h) {
     if (h >= heads_here) break;
     float sink_term = 0.f;
-    if (EXTRA && sinks) {
+    if (sinks) {
       // exp(sink) joins the denominator: under the larger of the running maximum and the sink, so that neither overflows.
       const float sink2 = sinks[head0 + h] * 1.4426950408889634f;
       const float mc = (m[h] == -INFINITY) ? -INFINITY : m[h] * scale_log2;
@@ -348,6 +382,7 @@ struct PrefillExtras {       // what the plain form does not have: see ta_prefil
   int keep_first;            // with a window: keys below this stay visible behind it
   int n_v;                   // value heads in the value pages (0 or n_kv: one a key head)
   float softcap;             // > 0: a scaled score s becomes softcap * tanh(s / softcap)
+  bool tied;                 // the values are the keys: only the key pages are read
 };
 
 template <int D, int HG, int NWV>
@@ -358,12 +393,19 @@ static int launch_prefill_waves(const void* q, int q_stride, void* out, const vo
   const int group = n_q / n_kv;
   const long workgroups = (long)n_tiles * n_kv * ((group + HG - 1) / HG);
   if (workgroups > 0x7fffffffL) return -1;
-#define GO(EE) prefill_attention_kernel<D, HG, NWV, EE><<<(unsigned)workgroups, NWV * WAVE, 0, stream>>>( \
+#define GO(EE, DD) prefill_attention_kernel<D, HG, NWV, EE, DD><<<(unsigned)workgroups, NWV * WAVE, 0, stream>>>( \
       (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_pages, (const bf16_t*)vt_pages, (const int*)tiles, \
       n_tiles, (const int*)cu_q, (const int*)first_position, (const int*)block_table, table_stride, n_q, n_kv, page_size, \
       window, scale * 1.4426950408889634f, extra.chunk, extra.slopes, extra.sinks, 1.0f / scale, extra.keep_first, extra.n_v, extra.softcap)
-  if (extra.chunk > 0 || extra.slopes || extra.sinks || extra.keep_first > 0 || extra.softcap > 0.f || (extra.n_v > 0 && extra.n_v < n_kv)) GO(true);
-  else GO(false);
+  if (extra.chunk > 0 || extra.slopes || extra.keep_first > 0 || extra.softcap > 0.f || (extra.n_v > 0 && extra.n_v < n_kv)) {
+    if (!vt_pages) return -1;
+    GO(true, false);
+  } else if (extra.tied || !vt_pages) {
+    if constexpr (D > 128 && NWV > 2) return -1;           // (the launcher asks for no more waves there)
+    else GO(false, true);
+  } else {
+    GO(false, false);
+  }
 #undef GO
   return LAUNCH_STATUS();
 }
@@ -397,6 +439,7 @@ static int launch_prefill(const void* q, int q_stride, void* out, const void* k_
     // compute unit better than one of four (measured at head sizes 96, 128 and 256, 512 to 8,192 tokens).
     if (D > 64 && waves > 2) waves = 2;
   }
+  if (D > 128 && extra.tied && waves > 2) waves = 2;       // (their keys' LDS)
 #define GO(NWV) launch_prefill_waves<D, HG, NWV>(q, q_stride, out, k_pages, vt_pages, tiles, n_tiles, cu_q, \
     first_position, block_table, table_stride, n_q, n_kv, page_size, window, scale, extra, stream)
   if constexpr (D == 48 || D == 64) {          // (the eight waves' states fit the static LDS at these sizes)
@@ -416,7 +459,7 @@ extern "C" int ta_prefill_attention_shared_bf16(const void* q, int q_stride, voi
                                                 const void* cu_q, const void* first_position,
                                                 const void* block_table, int table_stride, int n_q, int n_kv, int d,
                                                 int page_size, int window, float scale, int shape,
-                                                int key_splits, void* part_o, void* part_ml, const void* sinks,
+                                                int key_splits, void* part_o, void* part_ml, const void* sinks, int tied,
                                                 hipStream_t stream);
 
 // The shape in which the workgroup-shared kernel takes a launch (0: the per-wave kernel takes it), by what the
@@ -450,19 +493,21 @@ extern "C" int ta_prefill_attention_key_splits(int n_tiles, int n_q, int n_kv, i
 // (float [n_q] or null): head h's score loses slopes[h] per position of distance; sinks (float [n_q] or null): exp(sinks[h])
 // joins the softmax's denominator.  keep_first > 0 (with a window): keys at positions below it stay visible behind the
 // window; n_v (a divisor of n_kv): the value pages hold n_v heads, key head g reads value head g / (n_kv / n_v).
-// With any of these but the sinks the per-wave kernel runs, and the keys are not cut.
+// With any of these but the sinks the per-wave kernel runs, and the keys are not cut.  tied (without any of these but the
+// sinks): the value pages hold what the key pages hold, and only the keys are read; vt_pages may then be null.
 extern "C" int ta_prefill_attention_bf16(const void* q, int q_stride, void* out, const void* k_pages,
                                          const void* vt_pages, const void* tiles, int n_tiles, const void* cu_q,
                                          const void* first_position, const void* block_table, int table_stride,
                                          int n_q, int n_kv, int d, int page_size, int window, float scale,
                                          int shared_shape, int max_keys, int waves, int shared,
                                          void* part_o, void* part_ml, int chunk, const void* slopes, const void* sinks,
-                                         int keep_first, int n_v, float softcap, hipStream_t stream) {
+                                         int keep_first, int n_v, float softcap, int tied, hipStream_t stream) {
   if (n_tiles <= 0) return 0;
+  if (!vt_pages) tied = 1;
   if (n_kv <= 0 || n_q % n_kv || page_size % 16 || scale == 0.f) return -1;
   if (n_v <= 0) n_v = n_kv;
   if (n_kv % n_v || keep_first < 0 || (keep_first > 0 && (window < 0 || chunk > 0 || slopes))) return -1;
-  const PrefillExtras extra = {chunk, (const float*)slopes, (const float*)sinks, keep_first, n_v, softcap};
+  const PrefillExtras extra = {chunk, (const float*)slopes, (const float*)sinks, keep_first, n_v, softcap, tied != 0};
   const bool plain = chunk <= 0 && !slopes && keep_first == 0 && n_v == n_kv && !(softcap > 0.f);
   const int shape = plain ? shared_shape_for(n_tiles, n_q, n_kv, d, window, shared_shape, max_keys, waves, shared) : 0;
   if (shape) {
@@ -470,7 +515,8 @@ extern "C" int ta_prefill_attention_bf16(const void* q, int q_stride, void* out,
         ? ta_prefill_attention_shared_key_splits(n_tiles, n_q, n_kv, planned_reach(max_keys, window), shape) : 1;
     const int status = ta_prefill_attention_shared_bf16(q, q_stride, out, k_pages, vt_pages, tiles, n_tiles, cu_q,
                                                         first_position, block_table, table_stride, n_q, n_kv, d,
-                                                        page_size, window, scale, shape, parts, part_o, part_ml, sinks, stream);
+                                                        page_size, window, scale, shape, parts, part_o, part_ml, sinks, tied,
+                                                        stream);
     if (status != -2) return status;
   }
 #define CASE(DD, HG) case DD: return launch_prefill<DD, HG>(q, q_stride, out, k_pages, vt_pages, tiles, n_tiles, cu_q, \

@@ -27,14 +27,16 @@ typedef float floatx4 __attribute__((ext_vector_type(4)));
 extern "C" int ta_attention_merge_tiles(const void* part_o, const void* part_ml, const void* tiles, int n_tiles,
                                         const void* cu_q, void* out, int n_q, int d, int splits, hipStream_t stream);
 
-template <int D>
+// TIED (the values are the keys): a block is its keys alone, and the values' fragments are taken from the key rows by the
+// transposing LDS read (`transposed_keys`): half the bytes from the pages, half the LDS.
+template <int D, bool TIED>
 struct Staged {
   static_assert(D == 64 || D == 128, "a key row must be a power of two of pieces for the swizzle");
   static constexpr int PIECES = D / 8;                      // 16-byte pieces of a key row
   static constexpr int K_ROW = 2 * D;
   static constexpr int K_BYTES = 64 * K_ROW;
   static constexpr int V_RUN = 32 * D;
-  static constexpr int BYTES = K_BYTES + 4 * V_RUN;
+  static constexpr int BYTES = K_BYTES + (TIED ? 0 : 4 * V_RUN);
   static constexpr int KEYS_A_LOAD = 64 / PIECES;           // key rows that one instruction of a wave brings
   static constexpr int K_LOADS = 16 / KEYS_A_LOAD;          // instructions for a run's keys
   static constexpr int V_LOADS = D / 32;                    // and for its values (32 rows of D each)
@@ -68,9 +70,9 @@ struct SharedTile {
 // What a wave brings of every block: one of its four runs of sixteen keys (a run lies inside one page), so
 // that per block a wave looks up one page number and every load is a scalar base plus an offset that the lane
 // worked out once.
-template <int D>
+template <int D, bool TIED>
 struct Carrier {
-  typedef Staged<D> S;
+  typedef Staged<D, TIED> S;
   int run;                                                  // which of a block's runs
   uint32_t k_from[S::K_LOADS];                              // byte offsets of the lane's pieces inside the run's part of its page
   uint32_t v_from;
@@ -135,6 +137,7 @@ struct Carrier {
 #pragma unroll
     for (int j = 0; j < S::K_LOADS; ++j)
       __builtin_amdgcn_global_load_lds((from_t)(k_run + k_from[j]), (to_t)(k_to + j * 1024), 16, 0, 0);
+    if (TIED) return;
 #pragma unroll
     for (int j = 0; j < S::V_LOADS; ++j)
       __builtin_amdgcn_global_load_lds((from_t)(v_run + v_from + (uint32_t)j * 64 * page_size), (to_t)(v_to + j * 1024), 16, 0, 0);
@@ -148,7 +151,7 @@ struct Carrier {
 // row block of V^T that holds ones gives every lane its token's sum over all 64 keys (of the rounded
 // probabilities, the very weights of the product), where sixteen additions a head and two exchanges between
 // lanes at the end stood.
-template <int D, bool FULL>
+template <int D, bool FULL, bool TIED>
 __device__ __forceinline__ void second_product(const char* buf, int kb, int col, int g, int lo, int hi,
                                                const bf16x8 (&pf)[2], floatx4 (&acc)[D / 16], floatx4& l) {
   bf16x8 ones;
@@ -159,8 +162,17 @@ __device__ __forceinline__ void second_product(const char* buf, int kb, int col,
     l = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf[u], l, 0, 0, 0);
 #pragma unroll
     for (int db = 0; db < D / 16; ++db) {
-      bf16x8 vf = *reinterpret_cast<const bf16x8*>(buf + Staged<D>::K_BYTES + (2 * u + (g >> 1)) * Staged<D>::V_RUN +
-                                                   (db * 16 + col) * 32 + (g & 1) * 16);
+      bf16x8 vf;
+      if constexpr (TIED) {
+        // Keys 32 u + 8 g + 0 .. 3 and + 4 .. 7, the sixteen coordinates of db: a lane names half a piece of one row.
+        typedef Staged<D, TIED> S;
+        const int key = 32 * u + 8 * g + (col >> 2), piece = 2 * db + ((col & 3) >> 1);
+        const char* row = buf + key * S::K_ROW + (col & 1) * 8;
+        vf = transposed_keys(row + (piece ^ S::swizzle(key)) * 16, row + 4 * S::K_ROW + (piece ^ S::swizzle(key + 4)) * 16);
+      } else {
+        vf = *reinterpret_cast<const bf16x8*>(buf + Staged<D, TIED>::K_BYTES + (2 * u + (g >> 1)) * Staged<D, TIED>::V_RUN +
+                                              (db * 16 + col) * 32 + (g & 1) * 16);
+      }
       if (!FULL) {
         // A probability of zero times whatever lies in a slot that was never written, or in a borrowed page,
         // must stay zero.
@@ -178,7 +190,7 @@ __device__ __forceinline__ void second_product(const char* buf, int kb, int col,
 // product's instruction t of a half of 32 keys is key 8 (r / 4) + 4 t + r % 4 of the half, whose score then lies
 // in the lane group that holds that key in the second product (lane group g: keys 8g .. 8g+7).
 // lo, hi: the first and last key that any token of the tile sees (unless FULL, values outside them may be anything).
-template <int D, int HG, bool FULL>
+template <int D, int HG, bool FULL, bool TIED>
 __device__ __forceinline__ void shared_block(const char* buf, int kb, int col, int g, int my_pos, int my_lo, int lo, int hi,
                                              float c, const bf16x8 (&qf)[HG][D / 32], floatx4 (&acc)[HG][D / 16],
                                              float (&m)[HG], floatx4 (&l)[HG]) {
@@ -192,7 +204,7 @@ __device__ __forceinline__ void shared_block(const char* buf, int kb, int col, i
     bf16x8 kf[KS];
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks)
-      kf[ks] = *reinterpret_cast<const bf16x8*>(buf + key * Staged<D>::K_ROW + ((ks * 4 + g) ^ turned) * 16);
+      kf[ks] = *reinterpret_cast<const bf16x8*>(buf + key * Staged<D, TIED>::K_ROW + ((ks * 4 + g) ^ turned) * 16);
 #pragma unroll
     for (int h = 0; h < HG; ++h) {
       floatx4 st = (floatx4){0.f, 0.f, 0.f, 0.f};
@@ -240,17 +252,17 @@ __device__ __forceinline__ void shared_block(const char* buf, int kb, int col, i
       pf[h][i >> 3][i & 7] = (__bf16)__builtin_amdgcn_exp2f(fmaf(sh[i], c, -mc));   // masked keys: exp2(-inf) = 0
     // The head's second product follows at once, so that the matrix cores work on it while the vector unit
     // works on the next head's probabilities (the values are read from LDS once per head for that).
-    second_product<D, FULL>(buf, kb, col, g, lo, hi, pf[h], acc[h], l[h]);
+    second_product<D, FULL, TIED>(buf, kb, col, g, lo, hi, pf[h], acc[h], l[h]);
   }
 }
 
 // Arguments as in prefill_attention_kernel (sinks: float [n_q] or null, exp(sinks[h]) joins the softmax's denominator; with
 // the keys cut over workgroups it rides in the first part).  Dynamic LDS: two blocks for each of the KG groups of four waves
-// (2 * KG * Staged<D>::BYTES).
+// (2 * KG * Staged<D, TIED>::BYTES).
 // KG = 2: two groups of four waves, each with the same heads, take the blocks in turn (group i the blocks i,
 // i + 2, ...) and merge their softmax states through LDS at the end: half as many turns for a long walk, for
 // launches that cannot fill the device with workgroups.
-template <int D, int HG, int KG>
+template <int D, int HG, int KG, bool TIED>
 __global__ void __launch_bounds__(SHARED_WAVES * KG * WAVE, 1)
 prefill_attention_shared_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out,
                                 const bf16_t* __restrict__ k_pages, const bf16_t* __restrict__ vt_pages,
@@ -343,9 +355,9 @@ prefill_attention_shared_kernel(const bf16_t* __restrict__ q, int q_stride, bf16
   int kb = first_turn + split * turns_each * STRIDE;       // the turn's first key
   const int end = min(hi, kb + turns_each * STRIDE - 1);   // the last key of this workgroup's turns
   int cur = 0;
-  char* buffers = staged + key_group * 2 * Staged<D>::BYTES;
+  char* buffers = staged + key_group * 2 * Staged<D, TIED>::BYTES;
   const int ahead = 64 * key_group;                        // the group's block within a turn
-  Carrier<D> carrier;
+  Carrier<D, TIED> carrier;
   carrier.plan(head_wave, lane, tile, kb + ahead, STRIDE);
   const auto whole = [&](int turn) { return turn >= lo_all && turn + STRIDE - 1 <= p0; };
   carrier.look_up(tile, kb + ahead, whole(kb));
@@ -356,11 +368,11 @@ prefill_attention_shared_kernel(const bf16_t* __restrict__ q, int q_stride, bf16
 #define TURN(FULL)                                                                                            \
   {                                                                                                           \
     const int next = kb + STRIDE;                                                                             \
-    if (next + ahead <= end) carrier.fetch(tile, buffers + (cur ^ 1) * Staged<D>::BYTES);                     \
+    if (next + ahead <= end) carrier.fetch(tile, buffers + (cur ^ 1) * Staged<D, TIED>::BYTES);               \
     if (next + STRIDE + ahead <= end) carrier.look_up(tile, next + STRIDE + ahead, whole(next + STRIDE));     \
     if (heads_here > 0 && (FULL || kb + ahead <= end))                                                        \
-      shared_block<D, HG, FULL>(buffers + cur * Staged<D>::BYTES, kb + ahead, col, g, my_pos, my_lo, lo, hi,  \
-                                scale_log2, qf, acc, m, l);                                                   \
+      shared_block<D, HG, FULL, TIED>(buffers + cur * Staged<D, TIED>::BYTES, kb + ahead, col, g, my_pos,     \
+                                      my_lo, lo, hi, scale_log2, qf, acc, m, l);                              \
     carrier.landed();                                                                                         \
     __syncthreads();                                                                                          \
     cur ^= 1;                                                                                                 \
@@ -468,7 +480,7 @@ prefill_attention_shared_kernel(const bf16_t* __restrict__ q, int q_stride, bf16
   }
 }
 
-template <int D, int HG, int KG>
+template <int D, int HG, int KG, bool TIED>
 static int launch_shared(const void* q, int q_stride, void* out, const void* k_pages, const void* vt_pages,
                          const void* tiles, int n_tiles, const void* cu_q, const void* first_position,
                          const void* block_table, int table_stride, int n_q, int n_kv, int page_size, int window,
@@ -476,15 +488,16 @@ static int launch_shared(const void* q, int q_stride, void* out, const void* k_p
   const int group = n_q / n_kv;
   const long workgroups = (long)n_tiles * n_kv * ((group + HG * SHARED_WAVES - 1) / (HG * SHARED_WAVES)) * key_splits;
   if (workgroups > 0x7fffffffL) return -1;
-  constexpr int lds = 2 * KG * Staged<D>::BYTES;
+  // (The groups' states are handed over in the blocks' place.)
+  constexpr int blocks = 2 * KG * Staged<D, TIED>::BYTES, states = (KG - 1) * SHARED_WAVES * HG * (D / 4 + 2) * WAVE * 4;
+  constexpr int lds = blocks > states ? blocks : states;
   static_assert(lds <= 160 * 1024, "the blocks must fit a compute unit's LDS");
-  static_assert((KG - 1) * SHARED_WAVES * HG * (D / 4 + 2) * WAVE * 4 <= lds, "the groups' states are handed over in the blocks' place");
   if (lds > 48 * 1024) {
-    hipError_t err = hipFuncSetAttribute(reinterpret_cast<const void*>(&prefill_attention_shared_kernel<D, HG, KG>),
+    hipError_t err = hipFuncSetAttribute(reinterpret_cast<const void*>(&prefill_attention_shared_kernel<D, HG, KG, TIED>),
                                          hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     if (err != hipSuccess) return (int)err;
   }
-  prefill_attention_shared_kernel<D, HG, KG><<<(unsigned)workgroups, SHARED_WAVES * KG * WAVE, lds, stream>>>(
+  prefill_attention_shared_kernel<D, HG, KG, TIED><<<(unsigned)workgroups, SHARED_WAVES * KG * WAVE, lds, stream>>>(
       (const bf16_t*)q, q_stride, (bf16_t*)out, (const bf16_t*)k_pages, (const bf16_t*)vt_pages, (const int*)tiles,
       n_tiles, (const int*)cu_q, (const int*)first_position, (const int*)block_table, table_stride, n_q, n_kv, page_size,
       window, scale * 1.4426950408889634f, key_splits, (float*)part_o, (float*)part_ml,
@@ -572,14 +585,16 @@ extern "C" int ta_prefill_attention_shared_bf16(const void* q, int q_stride, voi
                                                 const void* cu_q, const void* first_position,
                                                 const void* block_table, int table_stride, int n_q, int n_kv, int d,
                                                 int page_size, int window, float scale, int shape,
-                                                int key_splits, void* part_o, void* part_ml, const void* sinks,
+                                                int key_splits, void* part_o, void* part_ml, const void* sinks, int tied,
                                                 hipStream_t stream) {
   if (n_tiles <= 0) return 0;
   const int heads_per_wave = shape % 10, key_groups = shape / 10 + 1;
   if (n_kv <= 0 || n_q % n_kv || page_size % 16 || heads_per_wave < 1 || heads_per_wave > 2 || key_groups > 2) return -1;
   if (key_splits < 1 || key_splits > 64 || (key_splits > 1 && (!part_o || !part_ml))) return -1;
-#define GO(DD, HG, KG) return launch_shared<DD, HG, KG>(q, q_stride, out, k_pages, vt_pages, tiles, n_tiles, cu_q, \
-    first_position, block_table, table_stride, n_q, n_kv, page_size, window, scale, key_splits, part_o, part_ml, sinks, stream);
+#define GO(DD, HG, KG) { if (tied) return launch_shared<DD, HG, KG, true>(q, q_stride, out, k_pages, vt_pages, tiles, n_tiles, cu_q, \
+    first_position, block_table, table_stride, n_q, n_kv, page_size, window, scale, key_splits, part_o, part_ml, sinks, stream); \
+    return launch_shared<DD, HG, KG, false>(q, q_stride, out, k_pages, vt_pages, tiles, n_tiles, cu_q, \
+    first_position, block_table, table_stride, n_q, n_kv, page_size, window, scale, key_splits, part_o, part_ml, sinks, stream); }
 #define SIZE(DD) case DD: if (key_groups == 2) { if (heads_per_wave == 1) GO(DD, 1, 2) GO(DD, 2, 2) } \
     if (heads_per_wave == 1) GO(DD, 1, 1) GO(DD, 2, 1)
   switch (d) {

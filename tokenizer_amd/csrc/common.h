@@ -125,6 +125,25 @@ __device__ __forceinline__ void lines_to_rows(const word4& lower, const word4& u
   second = __builtin_bit_cast(line_bf16x8, b);
 }
 
+// Values that are the keys, taken from a block of keys in LDS by the transposing read (ds_read_b64_tr_b16: of the 4 x 16
+// elements that sixteen lanes address, four lanes a row, lane i gets column i).  A lane names eight bytes of one row of
+// keys 0..3 (`first`) and of keys 4..7 (`second`) and gets the eight keys of its own coordinate.
+typedef short tr_short4 __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ line_bf16x8 transposed_keys(const char* first, const char* second) {
+  typedef __attribute__((address_space(3))) tr_short4* lds_t;
+  union { tr_short4 part[2]; line_bf16x8 v; } got;
+  got.part[0] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_t)first);
+  got.part[1] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_t)second);
+  return got.v;
+}
+
+template <int D>
+struct KeyStage {                                            // a wave's 32 keys in LDS, key by key
+  // Rows 3 pieces of sixteen bytes (of eight: mod 8) apart, so that the sixteen rows of a read lie in different banks.
+  static constexpr int ROW = 2 * D + 16 * ((11 - (D / 8) % 8) % 8);
+  static constexpr int BYTES = 32 * ROW;
+};
+
 // The compute units of the device, asked of the runtime once (the same on every device of a machine); launchers
 // that weigh a launch's workgroups against the device use this, never a number of their own.
 static inline int compute_units() {

@@ -11,7 +11,7 @@
 // coordinates behind it in `rows` with coordinate i < rot / 2 and coordinate i + rot / 2 (neighbours: coordinates 2 i and
 // 2 i + 1) turned by the angle position * rates[i] (float).  It goes into key page [n_pages, 1, page_size, kv_rank + rot] at the token's slot and,
 // transposed inside a page, into value page [n_pages, 1, kv_rank + rot, page_size].  slots null or a negative slot:
-// nothing is stored.  A workgroup a token.
+// nothing is stored; without value pages the row goes into its key page alone.  A workgroup a token.
 template <typename T>
 __global__ void __launch_bounds__(LT_THREADS)
 latent_store_kernel(const T* __restrict__ rows, int row_stride, int q_offset, int q_rank, const float* __restrict__ q_norm,
@@ -37,7 +37,7 @@ latent_store_kernel(const T* __restrict__ rows, int row_stride, int q_offset, in
   for (int i = threadIdx.x; i < kv_rank; i += LT_THREADS) {
     const float c = ld(row + kv_offset + i) * inv_c * kv_norm[i];
     st(k_row + i, c);
-    st(v_col + (size_t)i * page_size, c);
+    if (v_pages) st(v_col + (size_t)i * page_size, c);
   }
   const int half = rot / 2;
   const float position = (float)positions[t];
@@ -50,6 +50,7 @@ latent_store_kernel(const T* __restrict__ rows, int row_stride, int q_offset, in
     const float lo = a * c - b * s, hi = b * c + a * s;
     st(k_row + kv_rank + one, lo);
     st(k_row + kv_rank + other, hi);
+    if (!v_pages) continue;
     st(v_col + (size_t)(kv_rank + one) * page_size, lo);
     st(v_col + (size_t)(kv_rank + other) * page_size, hi);
   }
@@ -224,7 +225,7 @@ extern "C" int ta_latent_store(const void* rows, int row_stride, int q_offset, i
                                const void* slots, void* k_pages, void* v_pages, int page_size, void* latent_q, int n_tokens,
                                int neighbours, int dtype, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
-  if (q_rank <= 0 || kv_rank <= 0 || rot < 0 || (rot & 1) || (rot > 0 && !rates) || (slots && (!k_pages || !v_pages || !kv_norm || page_size <= 0)))
+  if (q_rank <= 0 || kv_rank <= 0 || rot < 0 || (rot & 1) || (rot > 0 && !rates) || (slots && (!k_pages || !kv_norm || page_size <= 0)))
     return -1;
 #define LS(TT) latent_store_kernel<TT><<<n_tokens, LT_THREADS, 0, stream>>>((const TT*)rows, row_stride, q_offset, q_rank, \
     (const float*)q_norm, kv_offset, kv_rank, (const float*)kv_norm, rot, (const float*)rates, eps, (const int*)positions, \

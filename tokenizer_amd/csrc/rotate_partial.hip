@@ -122,7 +122,7 @@ extern "C" int ta_norm_rotate_store(void* qkv, int row_stride, const void* bias,
 }
 
 // Rows of qkv as above without a bias: n_q query heads and n_k key heads of d elements, then n_k value heads of dv (tied: no
-// value heads, the keys are the values too and dv = d).  The query heads are multiplied by
+// value heads, the keys are the values too and dv = d; without v_pages only the keys are stored).  The query heads are multiplied by
 // 1 + coef * ln(floor((position + 1) / every) + 1), formed in float, and go back into their rows; keys and values go into
 // their pages as they are.  A workgroup a token.
 template <typename T>
@@ -144,6 +144,7 @@ temper_store_kernel(T* __restrict__ qkv, int row_stride, const int* __restrict__
   const T* values = tied ? keys : keys + n_k * d;
   for (int i = threadIdx.x; i < n_k * d; i += RP_THREADS)
     k_pages[(((size_t)page * n_k + i / d) * page_size + off) * d + i % d] = keys[i];
+  if (!v_pages) return;
   for (int i = threadIdx.x; i < n_k * dv; i += RP_THREADS)    // head i / dv, coordinate i % dv: one line of a transposed page
     v_pages[((size_t)page * n_k * dv + i) * page_size + off] = values[i];
 }
@@ -181,7 +182,7 @@ temper_store_vec_kernel(bf16_t* __restrict__ qkv, int row_stride, const int* __r
     const int j = i - q_size;
     *reinterpret_cast<uint4*>(k_pages + (((size_t)page * n_k + j / d) * page_size + off) * d + j % d) = raw;
   }
-  if (!key || tied) {
+  if ((!key || tied) && v_pages) {
     const int j = i - q_size - (tied ? 0 : k_size);           // head j / dv, coordinate j % dv
     bf16_t* to = v_pages + ((size_t)page * n_k * dv + j) * page_size + off;
     const uint32_t in[4] = {raw.x, raw.y, raw.z, raw.w};
@@ -195,7 +196,7 @@ extern "C" int ta_temper_store(void* qkv, int row_stride, const void* positions,
                                int tied, int dtype, hipStream_t stream) {
   if (n_tokens <= 0) return 0;
   if (every < 1 || d <= 0 || dv <= 0 || n_q <= 0 || n_k < 0 || page_size <= 0 || (tied && dv != d) ||
-      (slots && (!k_pages || !v_pages)))
+      (slots && (!k_pages || (!v_pages && !tied))))
     return -1;
   const int used = (n_q + n_k) * d + (tied ? 0 : n_k * dv);
   if (used > row_stride) return -1;

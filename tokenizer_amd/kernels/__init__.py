@@ -308,7 +308,7 @@ class Ops:
         kv_offset : + kv_rank]) * kv_norm | the rot_dim coordinates behind them, coordinate i with i + rot_dim / 2 turned by
         positions[t] * rates[i]], goes into key pages [n_pages, 1, page_size, kv_rank + rot_dim] at slots[t] and,
         transposed within a page, into value pages [n_pages, 1, kv_rank + rot_dim, page_size] (slots None: nothing is
-        stored, and the rows need no such part: kv_norm may be None).  `neighbours`: coordinate 2i turns with 2i + 1.  Norms
+        stored, and the rows need no such part: kv_norm may be None; v_pages None: into the key pages alone).  `neighbours`: coordinate 2i turns with 2i + 1.  Norms
         and angles are float32."""
         _dev(rows, q_norm, kv_norm, rates, positions, slots, k_pages, v_pages, latent_q)
         n_tokens = rows.shape[0]
@@ -326,7 +326,7 @@ class Ops:
         page_size = 0
         if slots is not None:
             _need(slots.dtype == torch.int32 and slots.numel() == n_tokens, "slots must be int32 [T]")
-            _need(k_pages is not None and v_pages is not None and k_pages.dtype == rows.dtype == v_pages.dtype,
+            _need(k_pages is not None and k_pages.dtype == rows.dtype and (v_pages is None or v_pages.dtype == rows.dtype),
                   "pages must have the rows' dtype")
             page_size = self._page_size(k_pages, v_pages, 1, kv_rank + rot_dim)
         self._check(self.lib.ta_latent_store(_ptr(rows), rows.shape[1], q_offset, q_rank, _ptr(q_norm), kv_offset, kv_rank,
@@ -744,7 +744,7 @@ class Ops:
         """In place on rows of `qkv` ([T, >= (n_q + n_k) d + n_k dv]: query heads, key heads, value heads; `tied`: no value
         heads, the keys are the values and dv = d): the query heads times 1 + coef ln(floor((position + 1) / every) + 1), a
         float32 factor; keys and values written as they are at `slots` into key pages [n_pages, n_k, page_size, d] and
-        value pages [n_pages, n_k, dv, page_size]."""
+        value pages [n_pages, n_k, dv, page_size] (`tied` and v_pages None: the keys alone)."""
         _dev(positions, slots, k_pages, v_pages)
         _need(qkv.is_cuda, "kernel operands must live on the GPU")
         n_tokens, width = qkv.shape
@@ -754,8 +754,8 @@ class Ops:
         page_size = 1
         if slots is not None:
             _need(slots.dtype == torch.int32 and slots.numel() == n_tokens, "slots must be int32 [T]")
-            _need(k_pages is not None and v_pages is not None, "slots without pages")
-            _need(k_pages.dtype == qkv.dtype and v_pages.dtype == qkv.dtype, "pages must have the dtype of qkv")
+            _need(k_pages is not None and (tied or v_pages is not None), "slots without pages")
+            _need(k_pages.dtype == qkv.dtype and (v_pages is None or v_pages.dtype == qkv.dtype), "pages must have the dtype of qkv")
             page_size = self._page_size(k_pages, v_pages, n_k, d, dv)
         self._check(self.lib.ta_temper_store(
             _ptr(qkv), qkv.stride(0), _ptr(positions), ctypes.c_float(coef), int(every), _ptr(slots),
@@ -1088,20 +1088,24 @@ class Ops:
                                            head_dim, page_size, _code(qkv.dtype), value_dim, self._stream()), "rope_store")
 
     @staticmethod
-    def _page_size(k_pages: torch.Tensor, v_pages: torch.Tensor, n_kv: int, head_dim: int,
+    def _page_size(k_pages: torch.Tensor, v_pages: torch.Tensor | None, n_kv: int, head_dim: int,
                    value_dim: int | None = None, value_heads: int | None = None) -> int:
+        """(`v_pages` None: the values are the keys, and there are no pages of their own.)"""
         value_dim = head_dim if value_dim is None else value_dim
         _need(k_pages.dim() == 4 and k_pages.shape[1] == n_kv and k_pages.shape[3] == head_dim,
               "key pages must be [n_pages, n_kv, page_size, d]")
         page_size = k_pages.shape[2]
-        _need(tuple(v_pages.shape) == (k_pages.shape[0], n_kv if value_heads is None else value_heads, value_dim, page_size),
-              "value pages must be [n_pages, n_kv, dv, page_size]")
-        _need(k_pages.numel() < 2 ** 31 and v_pages.numel() < 2 ** 31, "a layer's pages must hold fewer than 2^31 elements")
+        if v_pages is None:
+            _need(value_dim == head_dim and value_heads in (None, n_kv), "values that are the keys have their number and size")
+        else:
+            _need(tuple(v_pages.shape) == (k_pages.shape[0], n_kv if value_heads is None else value_heads, value_dim, page_size),
+                  "value pages must be [n_pages, n_kv, dv, page_size]")
+        _need(k_pages.numel() < 2 ** 31 and (v_pages is None or v_pages.numel() < 2 ** 31), "a layer's pages must hold fewer than 2^31 elements")
         return page_size
 
     # ------------------------------------------------------------------ attention
     def paged_attention(self, qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor,
-                        v_pages: torch.Tensor, positions: torch.Tensor, entry_of_token: torch.Tensor,
+                        v_pages: torch.Tensor | None, positions: torch.Tensor, entry_of_token: torch.Tensor,
                         block_table: torch.Tensor, n_q: int, n_kv: int, head_dim: int,
                         window: int | None, scale: float, max_position: int | None = None,
                         batch=None, value_dim: int | None = None, chunk: int | None = None,
@@ -1112,8 +1116,8 @@ class Ops:
 
         `softcap` c: a score (scaled, with its distance term) becomes c tanh(score / c) before the softmax.
 
-        `tied_values`: the value pages hold what the key pages hold (the values are the keys, or both are one latent); a
-        kernel may then read only one of them.
+        `tied_values`: the values are the keys (or both are one latent): there are no value pages (v_pages None), or they
+        hold what the key pages hold.
 
         `keep_first` n (with a window): keys at positions below n stay visible behind the window.  `value_heads`
         (a divisor of n_kv): the value pages hold so many heads, and key head g reads value head
@@ -1144,7 +1148,8 @@ class Ops:
         _need(value_heads > 0 and n_kv % value_heads == 0 and keep_first >= 0, "value heads divide the key heads")
         _need(qkv.shape[1] >= n_q * head_dim, "qkv is narrower than the query heads")
         _need(tuple(out.shape) == (n_tokens, n_q * value_dim) and out.dtype == qkv.dtype, "attention output shape")
-        _need(k_pages.dtype == qkv.dtype and v_pages.dtype == qkv.dtype, "pages must have the dtype of qkv")
+        _need(k_pages.dtype == qkv.dtype and (v_pages is None or v_pages.dtype == qkv.dtype), "pages must have the dtype of qkv")
+        _need(v_pages is not None or tied_values, "values that are not the keys need pages of their own")
         page_size = self._page_size(k_pages, v_pages, n_kv, head_dim, value_dim, value_heads)
         _need(positions.dtype == torch.int32 and positions.numel() == n_tokens, "positions must be int32 [T]")
         _need(entry_of_token.dtype == torch.int32 and entry_of_token.numel() == n_tokens, "entry_of_token must be int32 [T]")
@@ -1158,13 +1163,15 @@ class Ops:
         plain = plain and keep_first == 0 and value_heads == n_kv
         if (value_dim == head_dim and qkv.dtype == torch.bfloat16 and head_dim in self.DECODE_HEAD_DIMS and page_size % 16 == 0
                 and qkv.shape[1] % 8 == 0 and self.use_fast_attention
-                and (keep_first == 0 or (chunk is None and slopes is None))):
+                and (keep_first == 0 or (chunk is None and slopes is None))
+                and (v_pages is not None or (plain and not softcap))):
             args = (qkv, out, k_pages, v_pages, positions, entry_of_token, block_table, n_q, n_kv, head_dim,
                     page_size, window, scale, max_position)
             plain = plain and not softcap
             extras = {} if plain and sinks is None else dict(chunk=chunk, slopes=slopes, sinks=sinks, keep_first=keep_first,
                                                              value_heads=value_heads, softcap=softcap)
-            if tied_values and plain:
+            tied = v_pages is None or (tied_values and plain and self.use_tied_values)
+            if tied:
                 extras["tied_values"] = True
             if batch is None:
                 return self._decode_attention(*args, **extras)
@@ -1189,7 +1196,7 @@ class Ops:
                 n_tiles, _ptr(batch.cu_q), _ptr(batch.first_position), _ptr(block_table),
                 block_table.shape[1], n_q, n_kv, head_dim, page_size, choice[0], ctypes.c_float(scale), *choice[1:],
                 _ptr(part_o), _ptr(part_ml), 0 if chunk is None else int(chunk), _ptr(slopes), _ptr(sinks),
-                keep_first, value_heads, ctypes.c_float(softcap or 0.0), self._stream()), "prefill_attention")
+                keep_first, value_heads, ctypes.c_float(softcap or 0.0), int(tied), self._stream()), "prefill_attention")
             if batch.decode_rows.numel():
                 self._decode_attention(*args, rows=batch.decode_rows, **extras)
             return out
@@ -1202,7 +1209,7 @@ class Ops:
         return out
 
     DECODE_HEAD_DIMS = (16, 32, 48, 64, 80, 96, 112, 128, 160, 192, 224, 256)
-    use_tied_values = True        # whether the kernel for single tokens reads tied keys and values once (for comparisons)
+    use_tied_values = True        # whether tied keys and values that both have pages are read once (tests compare the two)
     use_fast_attention = True     # tests switch it off to reach the generic kernel in bfloat16
     prefill_waves = 0             # waves that share a tile's keys in the per-wave prompt kernel: 0 lets the launcher choose;
     #                               asking for a number asks for that kernel
@@ -1249,7 +1256,7 @@ class Ops:
             n_q, n_kv, head_dim, page_size, -1 if window is None else int(window), ctypes.c_float(scale),
             split_keys, splits, 0 if chunk is None else int(chunk), _ptr(slopes), _ptr(sinks),
             int(keep_first) if kept_splits else 0, kept_splits, n_kv if value_heads is None else int(value_heads),
-            ctypes.c_float(softcap or 0.0), int(bool(tied_values) and self.use_tied_values), self._stream()), "decode_attention")
+            ctypes.c_float(softcap or 0.0), int(bool(tied_values)), self._stream()), "decode_attention")
         return out
 
     def talking_attention(self, qkv: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,

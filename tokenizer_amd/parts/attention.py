@@ -113,7 +113,7 @@ class GQAttention(Mixer):
             raise ValueError("norms of single heads and changed values do not combine with biases, differential maps or a norm "
                              "over the whole projection")
         self.tied = spec.tied_values
-        if self.tied and (self.head_wise or spec.differential is not None or spec.qk_norm is not None or spec.qkv_bias
+        if self.tied and (spec.talking or self.head_wise or spec.differential is not None or spec.qk_norm is not None or spec.qkv_bias
                           or self.dv != self.d or (spec.position is not None and spec.position.kind != "query_temperature")):
             raise ValueError("values that are the keys do not combine with biases, norms, differential maps, a rotation or "
                              "value heads of another size")
@@ -225,7 +225,7 @@ class GQAttention(Mixer):
             return CacheNeed(kind=kind, n_kv_heads=2 * spec.n_kv_heads, head_dim=spec.head_dim, window=spec.window,
                              value_dim=spec.value_dim or 0, n_value_heads=spec.n_kv_heads)
         return CacheNeed(kind=kind, n_kv_heads=spec.n_kv_heads, head_dim=spec.head_dim, window=spec.window,
-                         value_dim=spec.value_dim or 0, keep_first=int(spec.keep_first) if spec.window is not None else 0)
+                         tied_values=spec.tied_values, value_dim=spec.value_dim or 0, keep_first=int(spec.keep_first) if spec.window is not None else 0)
 
     def repeatable(self):
         position = repeatable_of(self.position)

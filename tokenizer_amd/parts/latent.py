@@ -56,7 +56,7 @@ class LatentAttention(Mixer):
             raise ValueError(f"rot_pairs {pairs!r}: known are \"halves\" and \"neighbours\"")
         # (What the kernels take only where a layer has it.)
         self.turns = {"neighbours": True} if pairs == "neighbours" else {}
-        self.more = {"tied_values": True}            # (key and value pages hold the same rows)
+        self.more = {"tied_values": True}
         if spec.sink:
             self.more["sinks"] = tensors["sink"].to(torch.float32).contiguous()
         # One product for the down-projections and the gate; every part starts at a multiple of eight columns
@@ -97,19 +97,19 @@ class LatentAttention(Mixer):
 
     @staticmethod
     def cache_need(spec: MixerSpec) -> CacheNeed:
-        # One key head of kv_rank + rot_dim coordinates; the same rows, transposed within a page, as the value head.
+        # One key head of kv_rank + rot_dim coordinates; the same rows serve as values.
         if not spec.own_kv:
             return CacheNeed()                  # it reads the pages of the layer it is pointed at
         window = spec.options["kept_window"] if "kept_window" in spec.options else spec.window
         return CacheNeed(kind="full" if window is None else "window", n_kv_heads=1, head_dim=spec.kv_rank + spec.rot_dim,
-                         window=window)
+                         window=window, tied_values=True)
 
     def forward(self, x, ctx, cache):
         ops, H, D = self.runtime.ops, self.heads, self.key_dim
         n_tokens = x.shape[0]
         rows = ops.linear(x, self.w_in)
         latent_q = torch.empty((n_tokens, self.q_rank), dtype=x.dtype, device=x.device)
-        # Both latents' norms, the rotation of the shared key part and the store of [c | rot(k_rot)] as key and as value.
+        # Both latents' norms, the rotation of the shared key part and the store of [c | rot(k_rot)].
         ops.latent_store(rows, self.offsets["dq"], self.q_rank, self.q_norm, self.offsets.get("dkv", 0), self.rank, self.kv_norm,
                          self.rot, self.rates, self.eps, ctx.positions,
                          ctx.slots[cache.group] if cache.writes and self.own_kv else None, cache.k_pages, cache.v_pages, latent_q,

@@ -53,6 +53,7 @@ class CacheNeed:
     `keep_first`: with a window, the first so many positions of a sequence stay readable for every later query.
     `n_value_heads`: the number of value heads where it is not the number of key heads (several key heads, the
     maps of one differential head, read the same values).
+    `tied_values`: the values are the keys: there are no value pages.
     """
     kind: str = "none"
     n_kv_heads: int = 0
@@ -64,6 +65,7 @@ class CacheNeed:
     block_state_shape: tuple[int, ...] | None = None
     keep_first: int = 0           # kind "window": the pages of the first so many positions are never given back
     n_value_heads: int = 0        # value heads where several key heads read one value head (0: as many as key heads)
+    tied_values: bool = False     # no value pages: whoever reads keys finds the values in them
 
     @property
     def v_dim(self) -> int:
@@ -75,7 +77,8 @@ class CacheNeed:
 
     def page_key(self) -> tuple:
         """Layers with equal keys share one group of pages and one block table."""
-        return (self.kind, self.n_kv_heads, self.head_dim, self.window, self.v_dim, self.keep_first, self.v_heads)
+        return (self.kind, self.n_kv_heads, self.head_dim, self.window, self.v_dim, self.keep_first, self.v_heads,
+                self.tied_values)
 
 
 @dataclasses.dataclass(frozen=True)
