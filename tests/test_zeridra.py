@@ -627,7 +627,8 @@ def test_the_router_whose_scores_are_the_weights(backend, experts, top, width, t
 
 @pytest.mark.parametrize("backend", BACKENDS)
 @pytest.mark.parametrize("experts,top,inner,width,tokens", [(6, 2, 24, 64, 37), (1, 1, 10, 52, 9), (12, 1, 32, 128, 50), (8, 3, 16, 64, 3), (16, 1, 40, 64, 600),
-                                                            (8, 4, 32, 64, 300), (24, 1, 16, 64, 1), (24, 2, 48, 64, 16), (5, 2, 12, 40, 200)])
+                                                            (8, 4, 32, 64, 300), (24, 1, 16, 64, 1), (24, 2, 48, 64, 16), (5, 2, 12, 40, 200),
+                                                            (12, 1, 24, 64, 44)])
 def test_the_routed_experts_with_weighted_inputs(backend, experts, top, inner, width, tokens):
     """In the form that multiplies every expert, over sorted tokens, and for few rows; a weight on the output instead of the input
     would give other rows (checked in the oracle)."""
@@ -902,3 +903,47 @@ def test_short_portions_far_into_a_request_with_their_keys_in_parts(n_q, n_kv, d
         e = torch.exp(scores)
         want = torch.einsum("hk,khd->hd", e / (e.sum(-1, keepdim=True) + torch.exp(sinks.double())[:, None]), k[lo:pos + 1]).reshape(-1)
         assert float((out[i].double().cpu() - want).abs().max()) <= 1e-2
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("gated,weigh_input", [(True, True), (True, False), (False, False)])
+@pytest.mark.parametrize("experts,top,inner,width,tokens", [(8, 2, 48, 64, 1), (2, 1, 40, 1032, 50), (3, 3, 1032, 72, 40), (64, 4, 16, 128, 16),
+                                                            (300, 1, 8, 8, 200), (5, 2, 24, 4096, 9), (1, 1, 104, 40, 33)])
+def test_the_chosen_experts_of_few_rows(experts, top, inner, width, tokens, gated, weigh_input):
+    """Experts that nobody chose hold NaN; more rows than one block choose the same expert; a row that names one expert twice
+    (as a row of NaN does that only fills a batch up) stays a row of its own."""
+    from tokenizer_amd.kernels import get_ops
+    ops, device, dtype = get_ops(), torch.device("cuda:0"), torch.bfloat16
+    gen = torch.Generator().manual_seed(experts * 10 + tokens)
+    rand = lambda *shape: torch.randn(*shape, generator=gen, dtype=torch.float64)
+    halves = 2 if gated else 1
+    first = rounded(rand(experts, halves, inner, width) / width ** 0.5 * 2, dtype)
+    second = rounded(rand(width, experts, inner) / inner ** 0.5, dtype)
+    x = rounded(rand(tokens, width), dtype)
+    chosen = torch.stack([torch.randperm(experts, generator=gen)[:top] for _ in range(tokens)]).to(torch.int32)
+    if experts > 40:
+        chosen = chosen % 40
+    if top > 1:
+        chosen[-1] = chosen[-1, 0]
+    weights = (0.2 + torch.rand(tokens, top, generator=gen)).float()
+    for e in range(experts):
+        if not bool((chosen == e).any()):
+            first[e], second[:, e] = float("nan"), float("nan")
+    want = torch.zeros(top, tokens, width, dtype=torch.float64)
+    for t in range(tokens):
+        for k in range(top):
+            e, w = int(chosen[t, k]), float(weights[t, k])
+            row = w * x[t] if weigh_input else x[t]
+            if gated:
+                inside = plain.silu(first[e, 0] @ row) * (first[e, 1] @ row) * (1.0 if weigh_input else w)
+            else:
+                inside = w * torch.relu(first[e, 0] @ row) ** 2
+            want[k, t] = second[:, e] @ inside
+    on = lambda t: t.to(dtype).to(device).contiguous()
+    fill = torch.full((width, 8), float("nan"), dtype=torch.float64)                   # columns behind the experts' own
+    parts = ops.experts_few(on(x), chosen.to(device), weights.to(device), experts, on(first.reshape(-1, width)), gated, inner,
+                            on(torch.cat([second.reshape(width, -1), fill], dim=1)), weigh_input=weigh_input)
+    assert parts is not None and tuple(parts.partial.shape) == (top, tokens, width)
+    bound = 1.5e-2 * float(want.abs().max())
+    assert float((parts.partial.double().cpu() - want).abs().max()) <= bound
+    assert float((parts.resolve().double().cpu() - want.sum(0)).abs().max()) <= 2 * bound

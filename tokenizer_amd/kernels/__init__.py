@@ -161,7 +161,7 @@ class Ops:
                      "ta_add_terms_rmsnorm", "ta_scale_cap", "ta_route_scores", "ta_selective_scan", "ta_route_rows_scores",
                      "ta_rotation_table", "ta_head_norm_rotate_store", "ta_group_norm_add", "ta_relu_gate",
                      "ta_talking_attention_generic", "ta_talking_decode_bf16", "ta_talking_prefill_bf16",
-                     "ta_talking_prefill_parts", "ta_retention_scan", "ta_retention_chunked", "ta_temper_store", "ta_add_slabs_rmsnorm",
+                     "ta_talking_prefill_parts", "ta_retention_scan", "ta_retention_chunked", "ta_temper_store", "ta_add_slabs_rmsnorm", "ta_experts_few",
                      "ta_expert_gate_slots"):
             getattr(self.lib, name).restype = ctypes.c_int
         self.lib.ta_grouped_gemm_bf16.argtypes = [ctypes.c_void_p, ctypes.c_int, ctypes.c_void_p, ctypes.c_void_p, ctypes.c_int,
@@ -1016,6 +1016,34 @@ class Ops:
         self._check(self.lib.ta_expert_gate_slots(_ptr(gate_up), _ptr(slot_of), _ptr(weights), weights.numel(), inner, _ptr(out),
                                                   _code(out.dtype), self._stream()), "expert_gate_slots")
         return out
+
+    FEW_PAIRS = 256             # (row, pick) pairs up to which `experts_few` runs
+
+    def experts_few(self, x: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor, n_experts: int, w_first: torch.Tensor,
+                    gated: bool, inner: int, w_second: torch.Tensor, weigh_input: bool = False) -> "PendingSum | None":
+        """The chosen experts of few rows, reading no others: x bfloat16 [T, H]; w_first [experts (2) inner, H] (an expert's gate
+        rows, then its up rows; `gated` False: up rows alone, squared ReLU), w_second [H, >= experts inner].  The weights
+        multiply the activation (`weigh_input`: what the gated expert is handed).  The result is left in `top` parts
+        (float32, a row's k-th pick in part k).  None for sizes the kernels do not take."""
+        _dev(chosen, weights, w_first, w_second)
+        n_tokens, hidden = x.shape
+        top, halves = chosen.shape[1], 2 if gated else 1
+        if x.dtype != torch.bfloat16 or n_tokens * top > self.FEW_PAIRS:
+            return None
+        _need(x.is_cuda and x.stride(1) == 1 and w_first.dtype == x.dtype == w_second.dtype, "bfloat16 rows and matrices")
+        _need(tuple(w_first.shape) == (n_experts * halves * inner, hidden) and w_second.shape[0] == hidden
+              and w_second.shape[1] >= n_experts * inner, "the experts' matrices do not fit")
+        _need(chosen.dtype == torch.int32 and weights.dtype == torch.float32 and tuple(chosen.shape) == (n_tokens, top) == tuple(weights.shape)
+              and chosen.is_contiguous() and weights.is_contiguous(), "chosen int32 and weights float32 [T, top]")
+        act = torch.empty((n_tokens * top, inner), dtype=x.dtype, device=x.device)
+        partial = torch.empty((top, n_tokens, hidden), dtype=torch.float32, device=x.device)
+        status = self.lib.ta_experts_few(_ptr(x), x.stride(0) if n_tokens > 1 else hidden, _ptr(chosen), _ptr(weights), n_tokens, top,
+                                         n_experts, _ptr(w_first), halves, inner, hidden, int(bool(weigh_input)), _ptr(act),
+                                         _ptr(w_second), w_second.shape[1], _ptr(partial), self._stream())
+        if status == -2:
+            return None
+        self._check(status, "experts_few")
+        return PendingSum(self, partial, None, x.dtype)
 
     def side_gate(self, gate: torch.Tensor, table: torch.Tensor, token_ids: torch.Tensor, offset: int, dim: int,
                   out: torch.Tensor) -> torch.Tensor:
