@@ -676,6 +676,7 @@ def test_routed_layers_over_sorted_tokens(experts, top, inner, shared, width, to
     monkeypatch.setattr(cls, "GROUPED_FROM", 1)
     sorted_form = part.forward(x, None).double().cpu()
     monkeypatch.setattr(cls, "GROUPED_FROM", 1 << 30)
+    monkeypatch.setattr(cls, "GROUPED_ROWS", 1 << 30)
     every_expert = part.forward(x, None).double().cpu()
     # (A token whose last chosen and best unchosen logit are nearly equal may go either way in either form: the two
     # forms form the logits with the same kernel, so they agree with each other; the plain function may not.)

@@ -130,9 +130,10 @@ class RoutedExperts(FeedForward):
     products whatever the routing: between them a kernel turns gate and up into weight * silu(gate) * up for the
     experts a token chose and into zero for the others (the shared expert counts as chosen with weight 1), and the
     second product then adds the chosen experts' outputs up in its own sum.  That multiplies every token with every
-    expert, which is right while the weights bound the step (few rows: every expert is read anyway).  Steps with
-    `GROUPED_FROM` or more (token, expert) pairs in bfloat16 sort the pairs by expert on the device into tiles of rows
-    that belong to one expert each, multiply every tile with its expert's matrices alone, and add a token's experts
+    expert, which is right while the weights bound the step and nearly every expert is somebody's.  Steps of fewer
+    rows (`FEW_ROWS`, `FEW_AN_EXPERT`; bfloat16, no shared expert) read the chosen experts alone (`ops.experts_few`).  Steps
+    with `GROUPED_FROM` or more (token, expert) pairs, or `GROUPED_ROWS` or more rows, in bfloat16 sort the pairs by expert on
+    the device into tiles of rows that belong to one expert each, multiply every tile with its expert's matrices alone, and add a token's experts
     up at the end (the shared expert runs as a dense one).  Either way the routing stays on the device, so the step's
     launches do not depend on it.
 
@@ -152,7 +153,11 @@ class RoutedExperts(FeedForward):
     gives back is added as it is.  Logits, scores and weights are float32.
     """
     graph_safe = True
-    GROUPED_FROM = 1024        # (token, expert) pairs from which the sorted form runs
+    # The sorted form runs from so many (token, expert) pairs or rows on.  (Measured, us a layer, all experts | sorted: width 896,
+    # 2 of 8 experts of 2,432: 96 rows 60 | 60, 256 rows 86 | 68, 512 rows 149 | 83; width 3,584, 2 of 8 of 9,472: 96 rows 435 |
+    # 378; width 1,536, 4 of 64 of 768: 96 rows 162 | 144, 768 rows 477 | 162; 1 of 12 of 4,480: 96 rows 168 | 149, 768 rows 466 | 184.)
+    GROUPED_FROM = 1024
+    GROUPED_ROWS = 96
     # Only the chosen experts are read, by kernels of their own, for up to FEW_ROWS rows, and for more rows while an expert
     # is chosen by FEW_AN_EXPERT of them on average (beyond that nearly every expert is somebody's, and products over all
     # of them read the rows less often).  Measured, us a layer, all experts | the chosen ones: width 896, 2 of 8 gated experts of
@@ -263,7 +268,8 @@ class RoutedExperts(FeedForward):
             fused = getattr(ops, "route_rows", None)      # the router's product and the choice in one kernel, where there is one
             if fused is None or not fused(x, self.w_router, chosen, weights):
                 ops.route_top(ops.linear(x, self.w_router, out_dtype=torch.float32), chosen, weights)
-        if self.groupable and x.shape[0] * self.top_k >= self.GROUPED_FROM and hasattr(ops, "grouped_linear"):
+        if (self.groupable and (x.shape[0] * self.top_k >= self.GROUPED_FROM or x.shape[0] >= self.GROUPED_ROWS)
+                and hasattr(ops, "grouped_linear")):
             return self._sorted(x, chosen, weights, shared_weight)
         if (not self.shared and x.shape[0] <= max(self.FEW_ROWS, self.FEW_AN_EXPERT * self.n_experts // self.top_k)
                 and hasattr(ops, "experts_few")):
