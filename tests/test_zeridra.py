@@ -947,3 +947,32 @@ def test_the_chosen_experts_of_few_rows(experts, top, inner, width, tokens, gate
     bound = 1.5e-2 * float(want.abs().max())
     assert float((parts.partial.double().cpu() - want).abs().max()) <= bound
     assert float((parts.resolve().double().cpu() - want.sum(0)).abs().max()) <= 2 * bound
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("n_q,n_kv,d,width,rows", [(4, 2, 32, 64, 8), (14, 2, 64, 896, 1), (5, 1, 96, 72, 16), (3, 3, 128, 1032, 3), (28, 4, 128, 3584, 8),
+                                                   (2, 1, 256, 40, 16)])
+@pytest.mark.parametrize("coef,every", [(0.4, 7), (0.0, 3), (1.2, 1)])
+def test_the_projection_with_the_temperature_and_the_store_in_its_epilogue(n_q, n_kv, d, width, rows, coef, every):
+    from tokenizer_amd.kernels import get_ops
+    ops, device, dtype = get_ops(), torch.device("cuda:0"), torch.bfloat16
+    gen = torch.Generator().manual_seed(n_q * 100 + d + rows)
+    x = torch.randn(rows, width, generator=gen).to(dtype)
+    weight = (torch.randn((n_q + n_kv) * d, width, generator=gen) / width ** 0.5).to(dtype)
+    positions = torch.randint(0, 5000, (rows,), generator=gen, dtype=torch.int32)
+    positions[0] = every - 1
+    slots = torch.randperm(64, generator=gen)[:rows].to(torch.int32)
+    if rows > 2:
+        slots[2] = -1
+    k_pages = torch.full((4, n_kv, 16, d), 7.0, dtype=dtype, device=device)
+    q = ops.fused_qk_temper(x.to(device), weight.to(device), positions.to(device), coef, every, slots.to(device), k_pages, n_q, n_kv, d)
+    both = x.double() @ weight.double().T
+    want_q = both[:, :n_q * d] * plain.temperature(positions.long(), coef, every)[:, None]
+    assert float((q.double().cpu() - want_q).abs().max()) <= 6e-3 * float(want_q.abs().max())
+    want_k = torch.full((4, n_kv, 16, d), 7.0, dtype=torch.float64)
+    for t, slot in enumerate(slots.tolist()):
+        if slot >= 0:
+            want_k[slot // 16, :, slot % 16] = both[t, n_q * d:].reshape(n_kv, d)
+    assert float((k_pages.double().cpu() - want_k).abs().max()) <= 6e-3 * float(want_k.abs().max())
+    untouched = want_k == 7.0
+    assert torch.equal(k_pages.double().cpu()[untouched], want_k[untouched])

@@ -30,6 +30,7 @@ struct FusedArgs {
   // EPI_ROPE_STORE
   const int* positions; const float* cos_sin; const int* slots;
   bf16_t* k_pages; bf16_t* v_pages; int n_q, n_kv, d, page_size;
+  float temper_coef; int temper_every;                     // temper_every > 0: query heads times 1 + coef ln(floor((p + 1) / every) + 1)
 };
 
 __device__ __forceinline__ bf16x8 fz8() {
@@ -74,7 +75,7 @@ __global__ void __launch_bounds__(NW * WAVE)
 fused_decode_kernel(const bf16_t* w, const void* rows_in, void* result, const float* norm_weight,
                     int m, int n, int k, int rows, int lda, float eps, const float* bias,
                     const int* positions, const float* cos_sin, const int* slots, bf16_t* k_pages, bf16_t* v_pages,
-                    int n_q, int n_kv, int d, int page_size) {
+                    int n_q, int n_kv, int d, int page_size, float temper_coef, int temper_every) {
   HELD(w, rows_in, result, norm_weight, m, n, k, rows, lda, eps);          // (the fourteen words that are there)
   if constexpr (EPI == EPI_ROPE_STORE) HELD(n_q, n_kv, d, page_size);      // (where a tile's rows lie)
   FusedArgs p;
@@ -147,6 +148,11 @@ fused_decode_kernel(const bf16_t* w, const void* rows_in, void* result, const fl
         pre_cos[r] = cs[r];
         pre_sin[r] = cs[p.d / 2 + r];
       }
+    } else if (temper_every > 0 && row0 < p.n_q * p.d) {      // the factor stands where a rotation's cosine would
+      const int steps = (p.positions[col] + 1) / temper_every;
+      const float factor = 1.f + temper_coef * logf((float)steps + 1.f);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) pre_cos[r] = factor;
     }
   }
 
@@ -418,7 +424,7 @@ static int launch_kernel(const FusedArgs& args, int tiles, hipStream_t stream) {
       args.w, from_residual ? (const void*)args.residual_in : (const void*)args.a,
       EPI == EPI_RESIDUAL ? (void*)args.residual_out : (void*)args.out, args.norm_weight, args.m, args.n,
       args.k, args.rows, args.lda, args.eps, args.bias, args.positions, args.cos_sin, args.slots, args.k_pages, args.v_pages,
-      args.n_q, args.n_kv, args.d, args.page_size);
+      args.n_q, args.n_kv, args.d, args.page_size, args.temper_coef, args.temper_every);
   return LAUNCH_STATUS();
 }
 
@@ -470,14 +476,14 @@ static int launch_rows(const FusedArgs& args, int tiles, int waves, hipStream_t 
 // the bytes the busiest compute unit has to ask for: rounds of workgroups x (prologue + its weight rows + what a
 // unit could have streamed during the trips to memory that every workgroup begins with; without that last term one
 // row of 3,584 took three rounds of four weight rows, 17.7 us, where one round of sixteen takes 14.0).
-static int rows_per_tile(int n_q, int n_kv, int d, int m, int k, bool norm, int rows_override) {
+static int rows_per_tile(int n_q, int n_kv, int n_v, int d, int m, int k, bool norm, int rows_override) {
   if (rows_override == 16 || rows_override == 8 || rows_override == 4) return rows_override;
   const long units = compute_units();
   const long prologue = (long)m * k * (norm ? 8 : 2);       // float rows and the norm weight per row, or bfloat16 rows
   int best = 16;
   long best_cost = -1;
   for (int r = 16; r >= 4; r /= 2) {
-    const long tiles = (long)(n_q + n_kv) * (d / 2 / r) + (long)n_kv * d / r;
+    const long tiles = (long)(n_q + n_kv) * (d / 2 / r) + (long)n_v * d / r;
     const long cost = ((tiles + units - 1) / units) * (prologue + 2L * r * k * 2 + 64 * 1024);
     if (best_cost < 0 || cost < best_cost) { best = r; best_cost = cost; }
   }
@@ -523,16 +529,18 @@ static bool stage_rows(int m, int k) { return (size_t)m * (k + 8) * sizeof(uint1
 
 static int fused_qkv_rope(const FusedArgs& base, bool norm, const void* w, const void* bias, void* q_out,
                           const void* positions, const void* cos_sin, const void* slots, void* k_pages, void* v_pages,
-                          int m, int k, int n_q, int n_kv, int d, int page_size, int rows, int waves, hipStream_t stream) {
+                          int m, int k, int n_q, int n_kv, int d, int page_size, int rows, int waves, hipStream_t stream,
+                          bool tied = false) {
   if (m <= 0) return 0;
   if (m > 16 || (k & 7) || (d & 31)) return -1;
   FusedArgs a = base;
-  a.w = (const bf16_t*)w; a.bias = (const float*)bias; a.m = m; a.n = (n_q + 2 * n_kv) * d; a.k = k;
+  const int n_v = tied ? 0 : n_kv;                           // (values that are the keys have no rows and no pages of their own)
+  a.w = (const bf16_t*)w; a.bias = (const float*)bias; a.m = m; a.n = (n_q + n_kv + n_v) * d; a.k = k;
   a.out = (bf16_t*)q_out; a.ldc = n_q * d;
   a.positions = (const int*)positions; a.cos_sin = (const float*)cos_sin; a.slots = (const int*)slots;
   a.k_pages = (bf16_t*)k_pages; a.v_pages = (bf16_t*)v_pages; a.n_q = n_q; a.n_kv = n_kv; a.d = d; a.page_size = page_size;
-  a.rows = rows_per_tile(n_q, n_kv, d, m, k, norm, rows);
-  const int tiles = (n_q + n_kv) * (d / 2 / a.rows) + n_kv * d / a.rows;
+  a.rows = rows_per_tile(n_q, n_kv, n_v, d, m, k, norm, rows);
+  const int tiles = (n_q + n_kv) * (d / 2 / a.rows) + n_v * d / a.rows;
   if (norm || stage_rows(m, k)) return launch_rows<EPI_ROPE_STORE, true>(a, tiles, waves, stream);
   return launch_rows<EPI_ROPE_STORE, false>(a, tiles, waves, stream);
 }
@@ -561,6 +569,18 @@ extern "C" int ta_fused_qkv_rope(const void* x, int lda, const void* w, const vo
   a.a = (const bf16_t*)x; a.lda = lda;
   return fused_qkv_rope(a, false, w, bias, q_out, positions, cos_sin, slots, k_pages, v_pages, m, k, n_q, n_kv, d,
                         page_size, rows, waves, stream);
+}
+
+// The projection of queries and of keys that are the values too, from rows that are normalised already: query heads times
+// 1 + coef ln(floor((position + 1) / every) + 1) (coef 0: as they are), keys into the key pages.
+extern "C" int ta_fused_qk_temper(const void* x, int lda, const void* w, void* q_out, const void* positions, float coef, int every,
+                                  const void* slots, void* k_pages, int m, int k, int n_q, int n_kv, int d, int page_size,
+                                  int rows, int waves, hipStream_t stream) {
+  if ((lda & 7) || every < 1 || !positions) return -1;
+  FusedArgs a = {};
+  a.a = (const bf16_t*)x; a.lda = lda; a.temper_coef = coef; a.temper_every = coef == 0.f ? 0 : every;
+  return fused_qkv_rope(a, false, w, nullptr, q_out, positions, nullptr, slots, k_pages, nullptr, m, k, n_q, n_kv, d, page_size,
+                        rows, waves, stream, true);
 }
 
 // out [m, n/2] = silu(x Wg^T) * (x Wu^T), x = the normalised residual rows, W = [Wg; Wu] of shape [n, k].

@@ -162,6 +162,7 @@ class Ops:
                      "ta_rotation_table", "ta_head_norm_rotate_store", "ta_group_norm_add", "ta_relu_gate",
                      "ta_talking_attention_generic", "ta_talking_decode_bf16", "ta_talking_prefill_bf16",
                      "ta_talking_prefill_parts", "ta_retention_scan", "ta_retention_chunked", "ta_temper_store", "ta_add_slabs_rmsnorm", "ta_experts_few",
+                     "ta_fused_qk_temper",
                      "ta_expert_gate_slots"):
             getattr(self.lib, name).restype = ctypes.c_int
         self.lib.ta_grouped_gemm_bf16.argtypes = [ctypes.c_void_p, ctypes.c_int, ctypes.c_void_p, ctypes.c_void_p, ctypes.c_int,
@@ -1638,6 +1639,30 @@ class Ops:
         else:
             status = self.lib.ta_fused_norm_qkv_rope(_ptr(residual), _ptr(norm_weight), ctypes.c_float(eps), *tail)
         self._check(status, "fused_norm_qkv_rope")
+        return q
+
+    def fused_qk_temper(self, x, weight, positions, coef: float, every: int, slots, k_pages, n_q: int, n_kv: int,
+                        head_dim: int) -> torch.Tensor:
+        """q, k = x @ weight.T for up to sixteen normalised bfloat16 rows; q times 1 + coef ln(floor((position + 1) / every) + 1) in
+        float32 before it is rounded; k, which is the values too, stored into its key pages (when `slots` is given); returns
+        q [M, n_q * d]."""
+        _dev(weight, positions, slots, k_pages)
+        m, k = x.shape
+        _need(x.is_cuda and x.dtype == torch.bfloat16 and x.stride(1) == 1 and (m == 1 or x.stride(0) % 8 == 0) and x.data_ptr() % 16 == 0,
+              "normalised rows are bfloat16 with 16-byte aligned rows")
+        _need(weight.dtype == torch.bfloat16 and tuple(weight.shape) == ((n_q + n_kv) * head_dim, k), "the joined q/k matrix has the wrong shape")
+        _need(k % 8 == 0 and head_dim % 32 == 0 and 0 < m <= self.FUSED_ROWS and every >= 1, "sizes the fused projection does not take")
+        _need(positions.dtype == torch.int32 and positions.numel() == m, "positions must be int32 [M]")
+        page_size = 1
+        if slots is not None:
+            _need(slots.dtype == torch.int32 and slots.numel() == m and k_pages is not None and k_pages.dtype == torch.bfloat16,
+                  "slots int32 [M] and bfloat16 pages")
+            page_size = self._page_size(k_pages, None, n_kv, head_dim)
+        q = torch.empty((m, n_q * head_dim), dtype=torch.bfloat16, device=x.device)
+        self._check(self.lib.ta_fused_qk_temper(
+            _ptr(x), x.stride(0) if m > 1 else k, _ptr(weight), _ptr(q), _ptr(positions), ctypes.c_float(coef), int(every), _ptr(slots),
+            _ptr(k_pages if slots is not None else None), m, k, n_q, n_kv, head_dim, page_size, self.fused_rows, self.fused_waves,
+            self._stream()), "fused_qk_temper")
         return q
 
     ROPE_STORE_WEIGHT = 2 ** 22   # joined q/k/v matrices up to this many elements take the route below at 17-64 rows

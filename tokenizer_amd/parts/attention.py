@@ -274,6 +274,13 @@ class GQAttention(Mixer):
         output product."""
         ops = self.runtime.ops
         heads, key_heads = self.n_q * self.maps, self.n_kv * self.maps
+        temper = getattr(self.position, "temper", None) if self.tied and cache.group is not None and not self.head_gate else None
+        if (temper is not None and self.d % 32 == 0 and x.shape[1] % 8 == 0 and hasattr(ops, "fused_qk_temper")
+                and _can_fuse(ops, x, self.runtime.dtype)):
+            # Up to sixteen rows: the queries' factor and the keys' store ride in the projection's epilogue.
+            qkv = ops.fused_qk_temper(x, self.w_qkv, ctx.positions, *temper, ctx.slots[cache.group] if cache.writes else None,
+                                      cache.k_pages, heads, key_heads, self.d)
+            return self._attend(qkv, x, ctx, cache, heads, key_heads)
         qkv = ops.linear(x, self.w_qkv, self.b_qkv)           # bias joins the float accumulator
         if self.head_wise:
             take = None
@@ -294,6 +301,11 @@ class GQAttention(Mixer):
                                   ctx.block_tables[cache.group], heads, key_heads, self.d, self.dv, self.scale, self.talk,
                                   max_position=ctx.max_position, batch=ctx)
             return ops.linear(mixed, self.w_o)
+        return self._attend(qkv, x, ctx, cache, heads, key_heads)
+
+    def _attend(self, qkv, x, ctx, cache, heads: int, key_heads: int):
+        """From the rows whose query heads stand first to the mixer's output; the keys and values are in their pages."""
+        ops = self.runtime.ops
         mixed = torch.empty((x.shape[0], heads * self.dv), dtype=x.dtype, device=x.device)
         ops.paged_attention(qkv, mixed, cache.k_pages, cache.v_pages, ctx.positions, ctx.entry_of_token,
                             ctx.block_tables[cache.group], heads, key_heads, self.d, self.window, self.scale,

@@ -125,6 +125,7 @@ class QueryTemperature(PositionEncoding):
 
     def __init__(self, spec: PositionSpec, runtime: Runtime):
         self.runtime, self.coef, self.every = runtime, float(spec.options["coef"]), int(spec.options["every"])
+        self.temper = (self.coef, self.every)        # for projections that apply it in their epilogue
         if self.every < 1:
             raise ValueError(f"a query temperature that steps every {self.every} positions")
 
