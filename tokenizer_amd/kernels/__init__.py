@@ -1268,8 +1268,7 @@ class Ops:
             max_keys = min(max_keys, chunk + 32)
         head_blocks = -(-(n_q // n_kv) // 16)
         per_split = max(1, self.target_workgroups // max(1, n_items * n_kv * head_blocks))
-        # (A block of 32 keys for each of a workgroup's waves; wide heads have two waves.)
-        split_keys = max(self.min_split_keys if head_dim <= 128 else self.min_split_keys // 2, -(-max_keys // per_split))
+        split_keys = max(self.min_split_keys, -(-max_keys // per_split))
         split_keys = -(-split_keys // 32) * 32
         splits = max(1, -(-(max_keys + 31) // split_keys))
         kept_splits = -(-int(keep_first) // split_keys) if keep_first and window is not None else 0
