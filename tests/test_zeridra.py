@@ -428,7 +428,7 @@ def test_a_layer_that_reads_anothers_latents(backend, cut, own_window, window):
 
 @pytest.mark.parametrize("backend", BACKENDS)
 @pytest.mark.parametrize("cut", list(CUTS))
-@pytest.mark.parametrize("window", [2, 16, 17, 31, 64, 72 + 9])
+@pytest.mark.parametrize("window", [2, 16, 17, 31, 64, 81])
 def test_one_latent_made_to_stand_out_just_inside_and_just_outside_the_window(backend, cut, window):
     """The mixer's input is [a query part | a key part]: the query latent reads the first half, the key latent the
     second, and both go up through the same matrix, so a query whose first half is the second half of a chosen token
